@@ -26,21 +26,27 @@ void kva_set_error(const char *fmt, ...) {
 // (the token a sampling kernel left in row r of its output), so a decode step can be launched
 // before the host has seen the token it continues from.
 template <typename TW, typename TO>
-__global__ void embed_gather_kernel(TO *__restrict__ out, const TW *__restrict__ table,
+__global__ void embed_gather_kernel(TO *__restrict__ out, TO *__restrict__ copy, const TW *__restrict__ table,
                                     const int *__restrict__ ids, const int *__restrict__ feedback,
-                                    int width, int table_rows) {
+                                    int width, int table_rows, float scale) {
     const int row = blockIdx.x;
     int id = ids[row];
     if (id < 0) id = feedback[-1 - id];
     id = id < 0 ? 0 : (id >= table_rows ? table_rows - 1 : id);      // whatever a kernel left there: inside the table
     const TW *src = table + (size_t)id * width;
     TO *dst = out + (size_t)row * width;
-    for (int i = threadIdx.x; i < width; i += blockDim.x) dst[i] = from_float<TO>(to_float(src[i]));
+    TO *second = copy ? copy + (size_t)row * width : nullptr;
+    for (int i = threadIdx.x; i < width; i += blockDim.x) {
+        const TO v = from_float<TO>(to_float(src[i]) * scale);
+        dst[i] = v;
+        if (second) second[i] = v;
+    }
 }
 
-// feedback may be null when no id is negative (the caller checks the ids it uploads).
-extern "C" int kva_embed_gather(void *out, const void *table, const int *ids, const int *feedback,
-                                int rows, int width, int table_rows, int table_dtype, int out_dtype,
+// feedback may be null when no id is negative (the caller checks the ids it uploads).  The rows are taken
+// times `scale`; `copy` (optional) receives them a second time.
+extern "C" int kva_embed_gather(void *out, void *copy, const void *table, const int *ids, const int *feedback,
+                                int rows, int width, int table_rows, int table_dtype, int out_dtype, float scale,
                                 hipStream_t stream) {
     KVA_REQUIRE(rows >= 0 && width > 0 && table_rows > 0, "embed_gather: bad sizes rows=%d width=%d table rows=%d",
                 rows, width, table_rows);
@@ -48,7 +54,7 @@ extern "C" int kva_embed_gather(void *out, const void *table, const int *ids, co
     dim3 grid(rows), block(256);
 #define LAUNCH(TW, TO)                                                                    \
     hipLaunchKernelGGL((embed_gather_kernel<TW, TO>), grid, block, 0, stream, (TO *)out, \
-                       (const TW *)table, ids, feedback, width, table_rows)
+                       (TO *)copy, (const TW *)table, ids, feedback, width, table_rows, scale)
     if (table_dtype == KVA_F32 && out_dtype == KVA_F32) LAUNCH(float, float);
     else if (table_dtype == KVA_BF16 && out_dtype == KVA_BF16) LAUNCH(bf16_t, bf16_t);
     else if (table_dtype == KVA_F32 && out_dtype == KVA_BF16) LAUNCH(float, bf16_t);

@@ -241,11 +241,13 @@ __device__ inline void rotate_pair(const T *src, T *dst, int i, int rot, int int
     dst[b] = from_float<T>(v * co + u * si);
 }
 
-// y row: [H heads of (plain_dim + rot) | ... ] with the compressed entry (rank + rot) at kv_off.
+// y row: [H heads of (plain_dim + rot) | ... ] with the compressed entry (rank + rot) at kv_off; or, for
+// queries that come from a latent of their own (q_rank > 0, heads = 0), [q_rank query latent | ... ]: the
+// first q_rank elements, RMS-normed with q_weight, go to c_q [T, q_rank].
 template <typename T, typename TW>
 __global__ void __launch_bounds__(256)
 latent_encode_cache_kernel(const T *__restrict__ y, int row_stride, int kv_off, T *__restrict__ q_lat,
-                           T *__restrict__ cache, T *__restrict__ cache_t, int page_size,
+                           T *__restrict__ c_q, const TW *__restrict__ q_weight, int q_rank, T *__restrict__ cache, T *__restrict__ cache_t, int page_size,
                            const TW *__restrict__ norm_weight, float eps,
                            const float *__restrict__ cos_table, const float *__restrict__ sin_table,
                            const int *__restrict__ positions, const int *__restrict__ slot_mapping, int heads,
@@ -260,6 +262,16 @@ latent_encode_cache_kernel(const T *__restrict__ y, int row_stride, int kv_off, 
         const int h = w / half, i = w % half;
         rotate_pair(row + (size_t)h * (plain_dim + rot) + plain_dim, q_lat + ((size_t)t * heads + h) * kd + rank, i, rot,
                     interleaved, cs, sn);
+    }
+    if (q_rank > 0) {
+        float qs = 0.f;
+        for (int j = threadIdx.x; j < q_rank; j += blockDim.x) {
+            const float v = to_float(row[j]);
+            qs += v * v;
+        }
+        const float qi = 1.0f / sqrtf(block_sum(qs, red_s, blockDim.x / KVA_WAVE) / (float)q_rank + eps);
+        for (int j = threadIdx.x; j < q_rank; j += blockDim.x)
+            c_q[(size_t)t * q_rank + j] = from_float<T>(to_float(row[j]) * qi * to_float(q_weight[j]));
     }
     const int slot = slot_mapping ? slot_mapping[t] : -1;       // uniform over the workgroup
     if (slot < 0) return;
@@ -281,15 +293,18 @@ latent_encode_cache_kernel(const T *__restrict__ y, int row_stride, int kv_off, 
     for (int i = threadIdx.x; i < half; i += blockDim.x) rotate_pair(c + rank, dst + rank, i, rot, interleaved, cs, sn);
 }
 
-extern "C" int kva_latent_encode_cache(const void *y, int row_stride, int kv_off, void *q_lat, void *cache,
+extern "C" int kva_latent_encode_cache(const void *y, int row_stride, int kv_off, void *q_lat, void *c_q,
+                                       const void *q_weight, int q_rank, void *cache,
                                        void *cache_t, int page_size, const void *norm_weight, int weight_dtype, float eps, const float *cos_table,
                                        const float *sin_table, const int *positions, const int *slot_mapping,
                                        int tokens, int heads, int plain_dim, int rank, int rot, int interleaved,
                                        int dtype, hipStream_t stream) {
-    KVA_REQUIRE(tokens >= 0 && heads > 0 && plain_dim > 0 && rank > 0, "latent_encode_cache: bad sizes");
+    KVA_REQUIRE(tokens >= 0 && heads >= 0 && plain_dim > 0 && rank > 0, "latent_encode_cache: bad sizes");
+    KVA_REQUIRE(heads > 0 ? (q_lat && q_rank == 0) : (c_q && q_weight && q_rank > 0),
+                "latent_encode_cache: rows start with the query heads or with a query latent");
     KVA_REQUIRE(rot > 0 && rot % 2 == 0 && cos_table && sin_table,
                 "latent_encode_cache: %d rotated elements must be even and positive, with both tables", rot);
-    KVA_REQUIRE(kv_off >= heads * (plain_dim + rot) && row_stride >= kv_off + rank + rot,
+    KVA_REQUIRE(kv_off >= heads * (plain_dim + rot) && kv_off >= q_rank && row_stride >= kv_off + rank + rot,
                 "latent_encode_cache: the row layout [queries | entry] does not fit its stride");
     KVA_REQUIRE(!slot_mapping || cache, "latent_encode_cache: cache write asked for without a cache");
     KVA_REQUIRE(!cache_t || page_size > 0, "latent_encode_cache: the transposed copy needs the page size");
@@ -297,7 +312,7 @@ extern "C" int kva_latent_encode_cache(const void *y, int row_stride, int kv_off
     if (tokens == 0) return KVA_OK;
 #define LAUNCH_LE(T, TW)                                                                                        \
     hipLaunchKernelGGL((latent_encode_cache_kernel<T, TW>), dim3(tokens), dim3(256), 0, stream, (const T *)y,   \
-                       row_stride, kv_off, (T *)q_lat, (T *)cache, (T *)cache_t, page_size,                     \
+                       row_stride, kv_off, (T *)q_lat, (T *)c_q, (const TW *)q_weight, q_rank, (T *)cache, (T *)cache_t, page_size,                     \
                        (const TW *)norm_weight, eps, cos_table,                                                 \
                        sin_table, positions, slot_mapping, heads, plain_dim, rank, rot, interleaved)
     if (dtype == KVA_F32 && weight_dtype == KVA_F32) LAUNCH_LE(float, float);

@@ -796,7 +796,7 @@ extern "C" int kva_gemm_skinny(void *Y, const void *X, const void *W, int M, int
     const int act = mode >> 4;
     mode &= 15;
     KVA_REQUIRE(mode >= 0 && mode <= 3, "gemm_skinny: unknown mode %d", mode);
-    KVA_REQUIRE(act >= 0 && act <= KVA_ACT_GELU_TANH && (act == 0 || mode == 2), "gemm_skinny: unknown activation %d", act);
+    KVA_REQUIRE(kva_plain_activation(act) && (act == 0 || mode == 2), "gemm_skinny: unknown activation %d", act);
     KVA_REQUIRE(ldx >= K && ldx % 8 == 0, "gemm_skinny: X row stride %d must be a multiple of 8 and >= K", ldx);
     KVA_REQUIRE(mode != 2 || N % 2 == 0, "gemm_skinny: a joined [gate; up] matrix needs an even row count");
     KVA_REQUIRE(sumsq == nullptr || (sumsq_parts >= 1 && norm_width >= 1),

@@ -534,7 +534,7 @@ extern "C" int kva_gemv(void *Y, const void *X, const void *W, int M, int N, int
     a.act = mode >> 4;
     mode &= 15;
     KVA_REQUIRE(mode >= 0 && mode <= 3, "gemv: unknown mode %d", mode);
-    KVA_REQUIRE(a.act >= 0 && a.act <= KVA_ACT_GELU_TANH && (a.act == 0 || mode == 2), "gemv: unknown activation %d", a.act);
+    KVA_REQUIRE(kva_plain_activation(a.act) && (a.act == 0 || mode == 2), "gemv: unknown activation %d", a.act);
     if (mode == 3) {
         KVA_REQUIRE(hidden && scaled_out && sumsq_out, "gemv: the residual epilogue needs hidden, scaled_out and sumsq_out");
         a.hidden = (bf16_t *)hidden; a.next_w = next_w; a.next_w_f32 = next_w_f32;

@@ -5,7 +5,50 @@
 // stride and a head stride each, so both may be column ranges of wider buffers.  Operands are
 // fp32 or bf16; sums are fp32 with k ascending into one accumulator per output, so a row's result
 // does not depend on the other rows of the launch.
+//
+// Two things may ride on the launch.  A sigmoid gate in the epilogue, one number a head or one an output
+// element.  And a rotation (HeadsRotate): heads whose product covers only their first elements (queries with
+// a rotated part behind the unrotated one) have the rest rotated into place by workgroups of their own.
 #include "common.h"
+#include <math.h>
+
+// out *= sigmoid(p[row * row_stride + head * head_stride (+ n)])
+struct HeadsGate {
+    const void *p;
+    int row, head, per_element;
+};
+
+template <typename T>
+__device__ inline float heads_gate(const HeadsGate &g, size_t m, int h, int n) {
+    const T *p = reinterpret_cast<const T *>(g.p);
+    return 1.0f / (1.0f + expf(-to_float(p[m * g.row + (size_t)h * g.head + (g.per_element ? n : 0)])));
+}
+
+// dst[row, head, 0..rot) = the rotation of src[row, head, 0..rot) by the row's position: pair i is (2 i, 2 i + 1)
+// (`interleaved`) or (i, i + rot / 2); cos and sin are fp32 [positions, rot / 2]
+struct HeadsRotate {
+    const void *src;
+    void *dst;
+    const float *cos_table, *sin_table;
+    const int *positions;
+    int src_row, src_head, dst_row, dst_head, rot, interleaved;
+};
+
+template <typename T>
+__device__ inline void heads_rotate(const HeadsRotate &ro, int h, int row0, int row1) {
+    const int half = ro.rot / 2;
+    for (int w = threadIdx.x; w < (row1 - row0) * half; w += blockDim.x) {
+        const int m = row0 + w / half, i = w % half;
+        const size_t at = (size_t)ro.positions[m] * half + i;
+        const float co = ro.cos_table[at], si = ro.sin_table[at];
+        const int a = ro.interleaved ? 2 * i : i, b = ro.interleaved ? 2 * i + 1 : i + half;
+        const T *src = reinterpret_cast<const T *>(ro.src) + (size_t)m * ro.src_row + (size_t)h * ro.src_head;
+        T *dst = reinterpret_cast<T *>(ro.dst) + (size_t)m * ro.dst_row + (size_t)h * ro.dst_head;
+        const float u = to_float(src[a]), v = to_float(src[b]);
+        dst[a] = from_float<T>(u * co - v * si);
+        dst[b] = from_float<T>(v * co + u * si);
+    }
+}
 
 #define HM_BM 64
 #define HM_BN 64
@@ -14,7 +57,11 @@
 template <typename T>
 __global__ void __launch_bounds__(256)
 heads_matmul_kernel(T *__restrict__ out, int o_row, int o_head, const T *__restrict__ x, int x_row, int x_head,
-                    const T *__restrict__ w, int M, int N, int K, const T *__restrict__ gate, int g_row) {
+                    const T *__restrict__ w, int M, int N, int K, HeadsGate gate, HeadsRotate ro) {
+    if (ro.rot > 0 && blockIdx.x == gridDim.x - 1) {            // the last column of workgroups rotates
+        heads_rotate<T>(ro, blockIdx.z, blockIdx.y * HM_BM, min(M, (int)(blockIdx.y + 1) * HM_BM));
+        return;
+    }
     __shared__ float Xs[HM_BK][HM_BM + 4];
     __shared__ float Ws[HM_BK][HM_BN + 4];
     const int h = blockIdx.z;
@@ -59,31 +106,60 @@ heads_matmul_kernel(T *__restrict__ out, int o_row, int o_head, const T *__restr
     for (int i = 0; i < 4; ++i) {
         const int m = m0 + ty * 4 + i;
         if (m >= M) continue;
-        // (optional) the head's gate: the row's outputs of head h times sigmoid(gate[m, h])
-        const float gmul = gate ? 1.0f / (1.0f + expf(-to_float(gate[(size_t)m * g_row + h]))) : 1.0f;
+        const float gmul = gate.p && !gate.per_element ? heads_gate<T>(gate, m, h, 0) : 1.0f;
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
             const int n = n0 + tx * 4 + j;
-            if (n < N) out[(size_t)m * o_row + (size_t)h * o_head + n] = from_float<T>(acc[i][j] * gmul);
+            if (n >= N) continue;
+            const float g = gate.per_element ? heads_gate<T>(gate, m, h, n) : gmul;
+            out[(size_t)m * o_row + (size_t)h * o_head + n] = from_float<T>(acc[i][j] * g);
         }
     }
 }
 
+static int heads_options(HeadsGate &gate, HeadsRotate &ro, const void *g, int g_row, int g_head, int g_per_element,
+                         const void *r_src, int r_src_row, int r_src_head, void *r_dst, int r_dst_row, int r_dst_head,
+                         const float *cos_table, const float *sin_table, const int *positions, int rot, int interleaved,
+                         int heads, int N) {
+    KVA_REQUIRE(!g || (g_head >= (g_per_element ? N : 1) && g_row >= (heads - 1) * g_head + (g_per_element ? N : 1)),
+                "heads_matmul: the gate's strides do not fit %d heads of %d", heads, N);
+    KVA_REQUIRE(rot >= 0 && rot % 2 == 0 && (rot == 0 || (r_src && r_dst && cos_table && sin_table && positions)),
+                "heads_matmul: a rotation of %d elements (an even number) needs source, target, tables and positions", rot);
+    KVA_REQUIRE(rot == 0 || (r_src_head >= rot && r_dst_head >= rot && r_src_row >= (heads - 1) * r_src_head + rot &&
+                             r_dst_row >= (heads - 1) * r_dst_head + rot),
+                "heads_matmul: the rotation's strides do not fit %d heads of %d elements", heads, rot);
+    gate = HeadsGate{g, g_row, g_head, g ? g_per_element : 0};
+    ro = HeadsRotate{r_src, r_dst, cos_table, sin_table, positions, r_src_row, r_src_head, r_dst_row, r_dst_head, rot, interleaved};
+    return KVA_OK;
+}
+
+#define HEADS_OPTION_ARGS                                                                                              \
+    const void *gate_p, int g_row, int g_head, int g_per_element, const void *r_src, int r_src_row, int r_src_head,     \
+        void *r_dst, int r_dst_row, int r_dst_head, const float *cos_table, const float *sin_table, const int *positions, \
+        int rot, int interleaved
+#define HEADS_OPTIONS(gate, ro)                                                                                        \
+    HeadsGate gate;                                                                                                    \
+    HeadsRotate ro;                                                                                                    \
+    if (const int bad = heads_options(gate, ro, gate_p, g_row, g_head, g_per_element, r_src, r_src_row, r_src_head, r_dst, \
+                                      r_dst_row, r_dst_head, cos_table, sin_table, positions, rot, interleaved, heads, N)) \
+        return bad
+
 extern "C" int kva_heads_matmul(void *out, int o_row, int o_head, const void *x, int x_row, int x_head,
-                                const void *w, int rows, int heads, int N, int K, const void *gate, int g_row,
-                                int dtype, hipStream_t stream) {
+                                const void *w, int rows, int heads, int N, int K, HEADS_OPTION_ARGS, int dtype,
+                                hipStream_t stream) {
     KVA_REQUIRE(rows >= 0 && heads > 0 && heads <= 65535 && N > 0 && K > 0, "heads_matmul: bad sizes");
     KVA_REQUIRE(x_head >= K && o_head >= N && x_row >= (heads - 1) * x_head + K && o_row >= (heads - 1) * o_head + N,
                 "heads_matmul: strides do not fit %d heads of %d -> %d", heads, K, N);
+    HEADS_OPTIONS(gate, ro);
     if (rows == 0) return KVA_OK;
-    dim3 grid((N + HM_BN - 1) / HM_BN, (rows + HM_BM - 1) / HM_BM, heads), block(256);
+    dim3 grid((N + HM_BN - 1) / HM_BN + (rot > 0 ? 1 : 0), (rows + HM_BM - 1) / HM_BM, heads), block(256);
     KVA_REQUIRE(grid.y <= 65535, "heads_matmul: %d rows are too many for one launch", rows);
     if (dtype == KVA_F32)
         hipLaunchKernelGGL(heads_matmul_kernel<float>, grid, block, 0, stream, (float *)out, o_row, o_head,
-                           (const float *)x, x_row, x_head, (const float *)w, rows, N, K, (const float *)gate, g_row);
+                           (const float *)x, x_row, x_head, (const float *)w, rows, N, K, gate, ro);
     else if (dtype == KVA_BF16)
         hipLaunchKernelGGL(heads_matmul_kernel<bf16_t>, grid, block, 0, stream, (bf16_t *)out, o_row, o_head,
-                           (const bf16_t *)x, x_row, x_head, (const bf16_t *)w, rows, N, K, (const bf16_t *)gate, g_row);
+                           (const bf16_t *)x, x_row, x_head, (const bf16_t *)w, rows, N, K, gate, ro);
     else KVA_REQUIRE(false, "heads_matmul: unsupported dtype %d", dtype);
     KVA_CHECK_LAUNCH("heads_matmul");
     return KVA_OK;
@@ -100,8 +176,13 @@ extern "C" int kva_heads_matmul(void *out, int o_row, int o_head, const void *x,
 template <int NKS, int NT>
 __global__ void __launch_bounds__(KVA_WAVE)
 heads_matmul_mfma_kernel(bf16_t *__restrict__ out, int o_row, int o_head, const bf16_t *__restrict__ x, int x_row,
-                         int x_head, const bf16_t *__restrict__ w, int M, int N, int tiles_per_wave,
-                         const bf16_t *__restrict__ gate, int g_row) {
+                         int x_head, const bf16_t *__restrict__ w, int M, int N, int tiles_per_wave, HeadsGate gate,
+                         HeadsRotate ro) {
+    if (ro.rot > 0 && blockIdx.x == gridDim.x - 1) {            // the last column of workgroups rotates
+        heads_rotate<bf16_t>(ro, blockIdx.y, min(M, (int)blockIdx.z * tiles_per_wave * 16),
+                             min(M, (int)(blockIdx.z + 1) * tiles_per_wave * 16));
+        return;
+    }
     // NT neighbouring tiles of 16 outputs a wavefront: every fragment of x it loads serves NT products
     // (many rows: what a wavefront takes in per product is what bounds it); NT = 1 for few rows,
     // where more wavefronts matter more
@@ -124,7 +205,7 @@ heads_matmul_mfma_kernel(bf16_t *__restrict__ out, int o_row, int o_head, const 
 #pragma unroll
         for (int ks = 0; ks < NKS; ++ks) xf[ks].u4 = *reinterpret_cast<const uint4 *>(xrow + 32 * ks);
         float gmul = 1.f;
-        if (gate) gmul = 1.0f / (1.0f + expf(-to_float(gate[(size_t)t * g_row + h])));
+        if (gate.p && !gate.per_element) gmul = heads_gate<bf16_t>(gate, t, h, 0);
 #pragma unroll
         for (int nt = 0; nt < NT; ++nt) {
             const int n0 = n_first + 16 * nt;
@@ -135,22 +216,37 @@ heads_matmul_mfma_kernel(bf16_t *__restrict__ out, int o_row, int o_head, const 
             // lane (row t = r, group g) holds outputs n0 + 4 g .. + 3 of its row
             if (tile * 16 + r < M) {
                 bf16_t *o = out + (size_t)t * o_row + (size_t)h * o_head + n0 + 4 * g;
+                float mul[4] = {gmul, gmul, gmul, gmul};
+                if (gate.per_element) {
+                    const bf16_t *gp = reinterpret_cast<const bf16_t *>(gate.p) + (size_t)t * gate.row + (size_t)h * gate.head + n0 + 4 * g;
+                    Frag4 gv;
+                    gv.u2 = make_uint2(0u, 0u);
+                    if (n0 + 4 * g + 3 < N && ((reinterpret_cast<uintptr_t>(gp) & 7) == 0)) {
+                        gv.u2 = *reinterpret_cast<const uint2 *>(gp);
+                    } else {
+#pragma unroll
+                        for (int i = 0; i < 4; ++i)
+                            if (n0 + 4 * g + i < N) gv.h[i] = gp[i].bits;
+                    }
+#pragma unroll
+                    for (int i = 0; i < 4; ++i) mul[i] = 1.0f / (1.0f + expf(-bf16_bits_to_float(gv.h[i])));
+                }
                 if (n0 + 4 * g + 3 < N && ((o_row | o_head) % 4 == 0)) {
                     Frag4 v;
 #pragma unroll
-                    for (int i = 0; i < 4; ++i) v.h[i] = float_to_bf16_bits(acc[i] * gmul);
+                    for (int i = 0; i < 4; ++i) v.h[i] = float_to_bf16_bits(acc[i] * mul[i]);
                     *reinterpret_cast<uint2 *>(o) = v.u2;
                 } else {
 #pragma unroll
                     for (int i = 0; i < 4; ++i)
-                        if (n0 + 4 * g + i < N) o[i].bits = float_to_bf16_bits(acc[i] * gmul);
+                        if (n0 + 4 * g + i < N) o[i].bits = float_to_bf16_bits(acc[i] * mul[i]);
                 }
             }
         }
     }
 }
 
-#define HM_INSTANCES(X) X(1) X(2) X(3) X(4) X(6) X(8) X(12) X(16)
+#define HM_INSTANCES(X) X(1) X(2) X(3) X(4) X(5) X(6) X(8) X(10) X(12) X(16)
 
 extern "C" int kva_heads_matmul_mfma_supported(int K, int x_row, int x_head) {
     if (K % 32 || x_row % 8 || x_head % 8) return 0;
@@ -161,13 +257,14 @@ extern "C" int kva_heads_matmul_mfma_supported(int K, int x_row, int x_head) {
 }
 
 extern "C" int kva_heads_matmul_mfma(void *out, int o_row, int o_head, const void *x, int x_row, int x_head,
-                                     const void *w, int rows, int heads, int N, int K, const void *gate, int g_row,
+                                     const void *w, int rows, int heads, int N, int K, HEADS_OPTION_ARGS,
                                      hipStream_t stream) {
     KVA_REQUIRE(rows >= 0 && heads > 0 && heads <= 65535 && N > 0, "heads_matmul_mfma: bad sizes");
     KVA_REQUIRE(kva_heads_matmul_mfma_supported(K, x_row, x_head),
                 "heads_matmul_mfma: no instance for K = %d with strides %d / %d", K, x_row, x_head);
     KVA_REQUIRE(x_head >= K && o_head >= N && x_row >= (heads - 1) * x_head + K && o_row >= (heads - 1) * o_head + N,
                 "heads_matmul_mfma: strides do not fit %d heads of %d -> %d", heads, K, N);
+    HEADS_OPTIONS(gate, ro);
     if (rows == 0) return KVA_OK;
     const int row_tiles = (rows + 15) / 16;
     const int n_tiles = (N + 15) / 16;
@@ -182,12 +279,12 @@ extern "C" int kva_heads_matmul_mfma(void *out, int o_row, int o_head, const voi
         /* enough wavefronts to fill the chip before a wavefront takes more than one row tile */                 \
         int per_wave = 1;                                                                                        \
         while (per_wave < 8 && (long long)groups * heads * ((row_tiles + per_wave - 1) / per_wave) > 4096) per_wave *= 2; \
-        dim3 grid(groups, heads, (row_tiles + per_wave - 1) / per_wave), block(KVA_WAVE);                        \
+        dim3 grid(groups + (rot > 0 ? 1 : 0), heads, (row_tiles + per_wave - 1) / per_wave), block(KVA_WAVE);                        \
         KVA_REQUIRE(grid.z <= 65535, "heads_matmul_mfma: %d rows are too many for one launch", rows);            \
         auto kernel = wide ? heads_matmul_mfma_kernel<NKS, NTW> : heads_matmul_mfma_kernel<NKS, 1>;              \
         hipLaunchKernelGGL(kernel, grid, block, 0, stream, (bf16_t *)out, o_row, o_head,                         \
                            (const bf16_t *)x, x_row, x_head, (const bf16_t *)w, rows, N, per_wave,               \
-                           (const bf16_t *)gate, g_row);                                                         \
+                           gate, ro);                                                                            \
         done = true;                                                                                             \
     }
     HM_INSTANCES(LAUNCH_ONE)

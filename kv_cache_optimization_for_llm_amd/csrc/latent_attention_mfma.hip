@@ -259,7 +259,7 @@ latent_merge_kernel(bf16_t *__restrict__ out, const float *__restrict__ part_o, 
 }
 
 // The (rank, row size) pairs with an instance.
-#define LAT_INSTANCES(X) X(4, 3) X(4, 4) X(8, 5) X(8, 6) X(16, 9) X(16, 10) X(32, 18) X(24, 14)
+#define LAT_INSTANCES(X) X(4, 3) X(4, 4) X(6, 4) X(8, 5) X(8, 6) X(10, 6) X(12, 7) X(16, 9) X(16, 10) X(32, 18) X(24, 14)
 
 extern "C" int kva_latent_attention_mfma_supported(int rank, int key_dim, int page_size) {
     if (page_size <= 0 || page_size % 16) return 0;

@@ -7,7 +7,9 @@
 //    Or (`over_chosen`) the largest logits are chosen and the weights are the softmax over them alone.
 //  * kva_moe_align:  the (token, choice) slots of real experts sorted by expert into a list padded
 //    so that every tile of 16 rows belongs to one expert (`sorted_slot`, -1 = padding), with the
-//    expert of every tile (`tile_expert`, -1 = unused tile).
+//    expert of every tile (`tile_expert`, -1 = unused tile).  Without a router (`table`): the experts of a
+//    token are the entries of its id's row in an integer table, all with one weight; the same launch looks
+//    them up.
 //  * kva_moe_expert_rows: one product per tile against its expert's matrix.  Mode 0 ("up"): rows of
 //    x gathered by slot / top, activation applied (a gated expert: act(gate) * up, its gate and up rows
 //    interleaved in one matrix), written at the sorted position.  Mode 1 ("down"):
@@ -29,6 +31,7 @@
 
 __device__ inline float moe_activate(float z, int act) {
     if (act == 3) return 0.5f * z * (1.0f + erff(z * 0.70710678118654752f));       // exact gelu
+    if (act == 5) return kva_activate(z, KVA_ACT_RELU2);
     return kva_activate(z, act);
 }
 
@@ -177,10 +180,29 @@ extern "C" int kva_moe_route(int *idx, float *wgt, const float *logits, const fl
 }
 
 // ---- slots sorted by expert --------------------------------------------------------------
+// experts by token id: idx[t, k] = table[id_t, k] and wgt[t, k] = weight.  A negative id -1 - r stands for
+// feedback[r], as in the embedding gather.
+struct MoeTable {
+    const int *table, *ids, *feedback;
+    int rows, top;
+    float weight;
+    float *wgt;
+};
+
 __global__ void __launch_bounds__(1024)
-moe_align_kernel(int *__restrict__ sorted_slot, int *__restrict__ tile_expert, const int *__restrict__ idx, int slots,
-                 int experts, int capacity, int max_tiles) {
+moe_align_kernel(int *__restrict__ sorted_slot, int *__restrict__ tile_expert, int *idx, int slots, int experts, int capacity,
+                 int max_tiles, MoeTable tab) {
     __shared__ int count[MOE_MAX_EXPERTS], start[MOE_MAX_EXPERTS];
+    if (tab.table) {
+        // (a slot is written and later read by the same thread)
+        for (int s = threadIdx.x; s < slots; s += blockDim.x) {
+            int id = tab.ids[s / tab.top];
+            if (id < 0) id = tab.feedback[-1 - id];
+            id = id < 0 ? 0 : (id >= tab.rows ? tab.rows - 1 : id);
+            idx[s] = tab.table[(size_t)id * tab.top + s % tab.top];
+            tab.wgt[s] = tab.weight;
+        }
+    }
     for (int e = threadIdx.x; e < experts; e += blockDim.x) count[e] = 0;
     for (int p = threadIdx.x; p < capacity; p += blockDim.x) sorted_slot[p] = -1;
     for (int i = threadIdx.x; i < max_tiles; i += blockDim.x) tile_expert[i] = -1;
@@ -207,17 +229,32 @@ moe_align_kernel(int *__restrict__ sorted_slot, int *__restrict__ tile_expert, c
     }
 }
 
-extern "C" int kva_moe_align(int *sorted_slot, int *tile_expert, const int *idx, int slots, int experts, int capacity,
-                             int max_tiles, hipStream_t stream) {
+static int moe_align_launch(int *sorted_slot, int *tile_expert, int *idx, int slots, int experts, int capacity, int max_tiles,
+                            const MoeTable &tab, hipStream_t stream) {
     KVA_REQUIRE(sorted_slot && tile_expert && idx, "moe_align: missing operand");
     KVA_REQUIRE(experts > 0 && experts <= MOE_MAX_EXPERTS, "moe_align: %d experts (at most %d)", experts, MOE_MAX_EXPERTS);
     KVA_REQUIRE(capacity == max_tiles * MOE_TILE && capacity >= slots + experts * (MOE_TILE - 1),
                 "moe_align: a list of %d places cannot hold %d slots of %d experts in tiles of %d", capacity, slots,
                 experts, MOE_TILE);
     hipLaunchKernelGGL(moe_align_kernel, dim3(1), dim3(1024), 0, stream, sorted_slot, tile_expert, idx, slots, experts,
-                       capacity, max_tiles);
+                       capacity, max_tiles, tab);
     KVA_CHECK_LAUNCH("moe_align");
     return KVA_OK;
+}
+
+extern "C" int kva_moe_align(int *sorted_slot, int *tile_expert, const int *idx, int slots, int experts, int capacity,
+                             int max_tiles, hipStream_t stream) {
+    // (without a table the kernel only reads idx)
+    return moe_align_launch(sorted_slot, tile_expert, const_cast<int *>(idx), slots, experts, capacity, max_tiles,
+                            MoeTable{nullptr, nullptr, nullptr, 0, 1, 0.f, nullptr}, stream);
+}
+
+extern "C" int kva_moe_table_align(int *sorted_slot, int *tile_expert, int *idx, float *wgt, const int *table, int table_rows,
+                                   const int *ids, const int *feedback, int tokens, int top, float weight, int experts,
+                                   int capacity, int max_tiles, hipStream_t stream) {
+    KVA_REQUIRE(wgt && table && ids && table_rows > 0 && tokens >= 0 && top > 0, "moe_table_align: missing operand or bad sizes");
+    return moe_align_launch(sorted_slot, tile_expert, idx, tokens * top, experts, capacity, max_tiles,
+                            MoeTable{table, ids, feedback, table_rows, top, weight, wgt}, stream);
 }
 
 // ---- one product per tile ------------------------------------------------------------------
@@ -404,7 +441,7 @@ extern "C" int kva_moe_expert_rows(void *out, int out_dtype, const void *x, cons
     KVA_REQUIRE(mode == 0 || (mode == 1 && slot_weight && out_dtype == KVA_F32),
                 "moe_expert_rows: mode 1 writes fp32 rows times a weight per slot");
     KVA_REQUIRE(mode == 1 || out_dtype == dtype, "moe_expert_rows: mode 0 writes rows of the operands' type");
-    KVA_REQUIRE(N > 0 && K > 0 && top > 0 && act >= 0 && act <= 4, "moe_expert_rows: bad sizes or activation");
+    KVA_REQUIRE(N > 0 && K > 0 && top > 0 && act >= 0 && act <= 5, "moe_expert_rows: bad sizes or activation");
     KVA_REQUIRE(max_tiles >= 0 && max_tiles <= 65535, "moe_expert_rows: %d tiles are too many for one launch", max_tiles);
     if (max_tiles == 0) return KVA_OK;
     MoeRows a{sorted_slot, tile_expert, slot_weight, top, N, K, mode, act, gated, limit};

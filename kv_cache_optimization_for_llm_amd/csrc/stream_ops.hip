@@ -143,7 +143,7 @@ __global__ void act_mul_vec_kernel(uint4 *__restrict__ out, const uint4 *__restr
 extern "C" int kva_act_mul(void *out, const void *gate_up, int rows, int inter, int act, float limit, int dtype,
                            hipStream_t stream) {
     KVA_REQUIRE(rows >= 0 && rows <= 65535 && inter > 0, "act_mul: bad sizes");
-    KVA_REQUIRE(act >= KVA_ACT_SILU && act <= KVA_ACT_SWISH_CLAMPED, "act_mul: unknown activation %d", act);
+    KVA_REQUIRE(act >= KVA_ACT_SILU && act <= KVA_ACT_RELU2, "act_mul: unknown activation %d", act);
     if (rows == 0) return KVA_OK;
     if (dtype == KVA_BF16 && inter % 8 == 0) {
         hipLaunchKernelGGL(act_mul_vec_kernel, dim3((inter / 8 + 255) / 256, rows), dim3(256), 0, stream, (uint4 *)out,
@@ -326,7 +326,7 @@ extern "C" int kva_table_gate(void *out, const void *z, int dtype, const void *t
     KVA_REQUIRE(out && z && table && ids && rows >= 0 && dim > 0 && table_rows > 0, "table_gate: missing operand or bad sizes");
     KVA_REQUIRE(col0 >= 0 && col0 + dim <= table_width, "table_gate: columns %d..%d lie outside a table row of %d", col0,
                 col0 + dim, table_width);
-    KVA_REQUIRE(act >= KVA_ACT_SILU && act <= KVA_ACT_GELU_TANH, "table_gate: unknown activation %d", act);
+    KVA_REQUIRE(kva_plain_activation(act), "table_gate: unknown activation %d", act);
     if (rows == 0) return KVA_OK;
     const size_t n = (size_t)rows * dim;
     hipLaunchKernelGGL(table_gate_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, stream, out, z, dtype, table,
@@ -345,12 +345,33 @@ __global__ void bias_act_kernel(void *__restrict__ out, const void *__restrict__
     st_from_float(out, dtype, i, kva_activate(z, act));
 }
 
+// bf16 without a bias, a count that is a multiple of 8: a thread takes 8 neighbouring elements
+__global__ void act_vec_kernel(uint4 *__restrict__ out, const uint4 *__restrict__ x, int act, size_t n8) {
+    const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+    if (i >= n8) return;
+    const uint4 v = x[i];
+    const uint32_t w[4] = {v.x, v.y, v.z, v.w};
+    uint32_t o[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+        o[j] = (uint32_t)float_to_bf16_bits(kva_activate(__uint_as_float(w[j] << 16), act)) |
+               ((uint32_t)float_to_bf16_bits(kva_activate(__uint_as_float(w[j] & 0xffff0000u), act)) << 16);
+    out[i] = make_uint4(o[0], o[1], o[2], o[3]);
+}
+
 extern "C" int kva_bias_act(void *out, const void *x, int dtype, const float *bias, int rows, int width, int act,
                             hipStream_t stream) {
     KVA_REQUIRE(out && x && rows >= 0 && width > 0, "bias_act: missing operand or bad sizes");
-    KVA_REQUIRE(act >= KVA_ACT_SILU && act <= KVA_ACT_GELU_TANH, "bias_act: unknown activation %d", act);
+    KVA_REQUIRE(kva_plain_activation(act), "bias_act: unknown activation %d", act);
     if (rows == 0) return KVA_OK;
     const size_t n = (size_t)rows * width;
+    if (dtype == KVA_BF16 && !bias && n % 8 == 0 &&
+        ((reinterpret_cast<uintptr_t>(out) | reinterpret_cast<uintptr_t>(x)) & 15) == 0) {
+        hipLaunchKernelGGL(act_vec_kernel, dim3((unsigned)((n / 8 + 255) / 256)), dim3(256), 0, stream, (uint4 *)out,
+                           (const uint4 *)x, act, n / 8);
+        KVA_CHECK_LAUNCH("bias_act");
+        return KVA_OK;
+    }
     hipLaunchKernelGGL(bias_act_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, stream, out, x, dtype, bias, width,
                        act, n);
     KVA_CHECK_LAUNCH("bias_act");
@@ -618,5 +639,194 @@ extern "C" int kva_hyper_fill(float *x, const void *first, int dtype, int stream
     hipLaunchKernelGGL(hyper_fill_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, stream, x, first, dtype, streams,
                        width, n);
     KVA_CHECK_LAUNCH("hyper_fill");
+    return KVA_OK;
+}
+
+// ---- norms on both sides of a branch ---------------------------------------------------------------
+// The residual stream x [rows, width] fp32; a branch reads a norm of it and enters it under another norm:
+//     x <- x + n_post(y) (+ addend),    out = n_pre(x).
+// One launch does what lies between two branches, a workgroup a row: the branch output y that is still to
+// enter goes through its norm into the stream, an optional second addend (fp32, as it is) follows it, and
+// the new row is normed for the next branch.  n(v) = (v - mean) / sqrt(mean((v - mean)^2) + eps) * w (+ b);
+// without `center` the mean is not taken off.  Without a post weight y enters as it is; without `out` the
+// stream is only updated.  With row_idx only the named rows are read, and nothing is written back: the
+// model's last norm.
+struct SideNorm {
+    const void *w, *b;
+    int w_dtype, center;
+    float eps;
+};
+
+__global__ void __launch_bounds__(256)
+sandwich_step_kernel(float *__restrict__ x, const void *__restrict__ y, int y_dtype, SideNorm post,
+                     const float *__restrict__ addend, SideNorm pre, void *__restrict__ out, int out_dtype,
+                     const int *__restrict__ row_idx, int width) {
+    extern __shared__ float row_s[];
+    __shared__ float red_s[4];
+    const int r = blockIdx.x, waves = blockDim.x / KVA_WAVE;
+    const size_t row = (size_t)(row_idx ? row_idx[r] : r) * width;
+    float mean = 0.f, inv = 1.f;
+    if (y && post.w) {
+        float sum = 0.f;
+        for (int j = threadIdx.x; j < width; j += blockDim.x) sum += ld_as_float(y, y_dtype, row + j);
+        if (post.center) mean = block_sum(sum, red_s, waves) / (float)width;
+        float sq = 0.f;
+        for (int j = threadIdx.x; j < width; j += blockDim.x) {
+            const float d = ld_as_float(y, y_dtype, row + j) - mean;
+            sq += d * d;
+        }
+        inv = 1.0f / sqrtf(block_sum(sq, red_s, waves) / (float)width + post.eps);
+    }
+    float sum = 0.f;
+    for (int j = threadIdx.x; j < width; j += blockDim.x) {
+        float v = x[row + j];
+        if (y) {
+            const float yv = ld_as_float(y, y_dtype, row + j);
+            v += post.w ? (yv - mean) * inv * ld_as_float(post.w, post.w_dtype, j) + (post.b ? ld_as_float(post.b, post.w_dtype, j) : 0.f)
+                        : yv;
+        }
+        if (addend) v += addend[row + j];
+        if (!row_idx && (y || addend)) x[row + j] = v;
+        row_s[j] = v;
+        sum += v;
+    }
+    if (!out) return;
+    mean = 0.f;
+    if (pre.center) mean = block_sum(sum, red_s, waves) / (float)width;
+    float sq = 0.f;
+    for (int j = threadIdx.x; j < width; j += blockDim.x) {
+        const float d = row_s[j] - mean;
+        sq += d * d;
+    }
+    inv = 1.0f / sqrtf(block_sum(sq, red_s, waves) / (float)width + pre.eps);
+    for (int j = threadIdx.x; j < width; j += blockDim.x)
+        st_from_float(out, out_dtype, (size_t)r * width + j,
+                      (row_s[j] - mean) * inv * ld_as_float(pre.w, pre.w_dtype, j) + (pre.b ? ld_as_float(pre.b, pre.w_dtype, j) : 0.f));
+}
+
+// The same with a row's elements in registers (a width that is a multiple of 4): a thread takes 4
+// neighbouring columns ITERS times, and every load - stream, branch output, addend, both norms' weights and
+// biases - is asked for before the first sum.
+template <int THREADS, int ITERS>
+__global__ void __launch_bounds__(THREADS)
+sandwich_step_vec_kernel(float *__restrict__ x, const void *__restrict__ y, int y_dtype, SideNorm post,
+                         const float *__restrict__ addend, SideNorm pre, void *__restrict__ out, int out_dtype,
+                         const int *__restrict__ row_idx, int width) {
+    constexpr int WAVES = THREADS / KVA_WAVE;
+    __shared__ float red_s[WAVES];
+    const int r = blockIdx.x;
+    const size_t row = (size_t)(row_idx ? row_idx[r] : r) * width;
+    float v[ITERS][4], yv[ITERS][4], av[ITERS][4], pw[ITERS][4], pb[ITERS][4], nw[ITERS][4], nb[ITERS][4];
+    const bool norm_y = y && post.w;
+#pragma unroll
+    for (int it = 0; it < ITERS; ++it) {
+        const int j = (threadIdx.x + it * THREADS) * 4;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[it][e] = yv[it][e] = av[it][e] = pw[it][e] = pb[it][e] = nw[it][e] = nb[it][e] = 0.f;
+        if (j >= width) continue;
+        hyper_ld4(x, KVA_F32, row + j, v[it]);
+        if (y) hyper_ld4(y, y_dtype, row + j, yv[it]);
+        if (addend) hyper_ld4(addend, KVA_F32, row + j, av[it]);
+        if (norm_y) hyper_ld4(post.w, post.w_dtype, j, pw[it]);
+        if (norm_y && post.b) hyper_ld4(post.b, post.w_dtype, j, pb[it]);
+        if (out) hyper_ld4(pre.w, pre.w_dtype, j, nw[it]);
+        if (out && pre.b) hyper_ld4(pre.b, pre.w_dtype, j, nb[it]);
+    }
+    if (norm_y) {
+        float mean = 0.f;
+        if (post.center) {
+            float sum = 0.f;
+#pragma unroll
+            for (int it = 0; it < ITERS; ++it) sum += (yv[it][0] + yv[it][1]) + (yv[it][2] + yv[it][3]);
+            mean = block_sum(sum, red_s, WAVES) / (float)width;
+        }
+        float sq = 0.f;
+#pragma unroll
+        for (int it = 0; it < ITERS; ++it) {
+            const bool on = (threadIdx.x + it * THREADS) * 4 < width;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                yv[it][e] = on ? yv[it][e] - mean : 0.f;
+                sq += yv[it][e] * yv[it][e];
+            }
+        }
+        const float inv = 1.0f / sqrtf(block_sum(sq, red_s, WAVES) / (float)width + post.eps);
+#pragma unroll
+        for (int it = 0; it < ITERS; ++it)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) yv[it][e] = yv[it][e] * inv * pw[it][e] + pb[it][e];
+    }
+    float sum = 0.f;
+#pragma unroll
+    for (int it = 0; it < ITERS; ++it) {
+        const int j = (threadIdx.x + it * THREADS) * 4;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            v[it][e] = (v[it][e] + yv[it][e]) + av[it][e];
+            sum += v[it][e];
+        }
+        if (!row_idx && (y || addend) && j < width)
+            *reinterpret_cast<float4 *>(x + row + j) = make_float4(v[it][0], v[it][1], v[it][2], v[it][3]);
+    }
+    if (!out) return;
+    float mean = 0.f;
+    if (pre.center) mean = block_sum(sum, red_s, WAVES) / (float)width;
+    float sq = 0.f;
+#pragma unroll
+    for (int it = 0; it < ITERS; ++it) {
+        const bool on = (threadIdx.x + it * THREADS) * 4 < width;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            v[it][e] = on ? v[it][e] - mean : 0.f;
+            sq += v[it][e] * v[it][e];
+        }
+    }
+    const float inv = 1.0f / sqrtf(block_sum(sq, red_s, WAVES) / (float)width + pre.eps);
+#pragma unroll
+    for (int it = 0; it < ITERS; ++it) {
+        const int j = (threadIdx.x + it * THREADS) * 4;
+        if (j >= width) continue;
+        float o[4];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) o[e] = v[it][e] * inv * nw[it][e] + nb[it][e];
+        if (out_dtype == KVA_F32)
+            *reinterpret_cast<float4 *>(reinterpret_cast<float *>(out) + (size_t)r * width + j) = make_float4(o[0], o[1], o[2], o[3]);
+        else
+            *reinterpret_cast<uint2 *>(reinterpret_cast<uint16_t *>(out) + (size_t)r * width + j) =
+                make_uint2((uint32_t)float_to_bf16_bits(o[0]) | ((uint32_t)float_to_bf16_bits(o[1]) << 16),
+                           (uint32_t)float_to_bf16_bits(o[2]) | ((uint32_t)float_to_bf16_bits(o[3]) << 16));
+    }
+}
+
+extern "C" int kva_sandwich_step(float *x, const void *y, int y_dtype, const void *post_w, const void *post_b, int post_dtype,
+                                 int post_center, float post_eps, const float *addend, const void *pre_w, const void *pre_b,
+                                 int pre_dtype, int pre_center, float pre_eps, void *out, int out_dtype, const int *row_idx,
+                                 int rows, int width, hipStream_t stream) {
+    KVA_REQUIRE(x && rows >= 0 && width > 0 && width <= 16000, "sandwich_step: width %d must lie in 1..16000", width);
+    KVA_REQUIRE(y || (!post_w && !post_b), "sandwich_step: a norm without the branch output it norms");
+    KVA_REQUIRE(!post_b || post_w, "sandwich_step: a norm's bias without its weight");
+    KVA_REQUIRE(!out || (pre_w && pre_eps >= 0.f), "sandwich_step: the read-out needs a norm");
+    KVA_REQUIRE(post_eps >= 0.f, "sandwich_step: negative eps");
+    KVA_REQUIRE(y || addend || out, "sandwich_step: nothing to do");
+    KVA_REQUIRE(!row_idx || out, "sandwich_step: rows are gathered for the read-out only");
+    if (rows == 0) return KVA_OK;
+    const SideNorm post{post_w, post_b, post_dtype, post_center, post_eps}, pre{pre_w, pre_b, pre_dtype, pre_center, pre_eps};
+    // (which kernel runs depends on width and alignment alone, never on the rows: a row's numbers are the same in any batch)
+    const bool aligned = aligned16(x) && aligned16(y) && aligned16(post_w) && aligned16(post_b) && aligned16(addend) &&
+                         aligned16(pre_w) && aligned16(pre_b) && aligned16(out);
+    if (width % 4 == 0 && width <= 8192 && aligned) {
+#define KVA_SANDWICH(THREADS, ITERS)                                                                                     \
+    hipLaunchKernelGGL((sandwich_step_vec_kernel<THREADS, ITERS>), dim3(rows), dim3(THREADS), 0, stream, x, y, y_dtype,  \
+                       post, addend, pre, out, out_dtype, row_idx, width)
+        if (width <= 1024) KVA_SANDWICH(256, 1);
+        else if (width <= 2048) KVA_SANDWICH(512, 1);
+        else if (width <= 4096) KVA_SANDWICH(512, 2);
+        else KVA_SANDWICH(1024, 2);
+#undef KVA_SANDWICH
+    } else {
+        hipLaunchKernelGGL(sandwich_step_kernel, dim3(rows), dim3(256), (size_t)width * sizeof(float), stream, x, y, y_dtype, post,
+                           addend, pre, out, out_dtype, row_idx, width);
+    }
+    KVA_CHECK_LAUNCH("sandwich_step");
     return KVA_OK;
 }

@@ -12,10 +12,11 @@ from . import gadopel as _gadopel   # noqa: F401  (registers Gadopel)
 from . import radilix as _radilix   # noqa: F401  (registers Radilix)
 from . import lomodra as _lomodra   # noqa: F401  (registers Lomodra)
 from . import bonusun as _bonusun   # noqa: F401  (registers Bonusun)
+from . import bilolorn as _bilolorn   # noqa: F401  (registers Bilolorn)
 from ..config.registry import (BLOCKS, FEED_FORWARDS, MIXERS, NORMS, STREAM_OPS, architecture_for)
 from ..models.spec import LayerCall, ModelSpec, TensorSpec
 from ..ops import kernels as K
-from ..parts.base import Block, KVCacheSpec, KVView, MixerContext, NormedRows, StateSpec, StreamCopy
+from ..parts.base import Block, KVCacheSpec, KVView, MixerContext, NormedRows, PendingNorm, StateSpec, StreamCopy
 from ..parts.linear import Linear
 
 
@@ -235,7 +236,7 @@ class Model:
         S = int(self.spec.streams)
         hidden = torch.empty((T, S * self.spec.hidden_size), dtype=self.stream_dtype, device=self.device)
         delta = None
-        first = None            # the embedding output in the compute type, for operations that read it again
+        first = {}              # the embedding output once more, for operations between layers that read it
         first_norm = self.blocks[self.calls[0][0].layer].first_norm() if self.calls else self.final_norm
         prep = first_norm.prepared_by_product() if first_norm is not None else None
         if (T <= self.GATHER_PREP_MAX_ROWS and prep is not None and prep[1] == self.spec.hidden_size
@@ -254,33 +255,35 @@ class Model:
             if self.stream_ops:
                 raise TypeError("operations between layers take a stream of one copy")
             one = torch.empty((T, self.spec.hidden_size), dtype=self.stream_dtype, device=self.device)
-            K.embed_gather(self.embedding, batch.token_ids, one, getattr(batch, "feedback", None))
-            if self.spec.embedding_scale != 1.0:
-                K.scale_softcap(one, self.spec.embedding_scale)
+            K.embed_gather(self.embedding, batch.token_ids, one, getattr(batch, "feedback", None), self.spec.embedding_scale)
             K.hyper_fill(hidden, one, S)
         else:
-            K.embed_gather(self.embedding, batch.token_ids, hidden, getattr(batch, "feedback", None))
-            if self.spec.embedding_scale != 1.0:
-                K.scale_softcap(hidden, self.spec.embedding_scale)
-            if self.stream_ops:
-                if self.stream_dtype == self.dtype:
-                    first = hidden.clone()
-                else:
-                    first = torch.empty((T, self.spec.hidden_size), dtype=self.dtype, device=self.device)
-                    K.embed_gather(self.embedding, batch.token_ids, first, getattr(batch, "feedback", None))
-                    if self.spec.embedding_scale != 1.0:
-                        K.scale_softcap(first, self.spec.embedding_scale)
+            copies = {}
+            for op in self.stream_ops:
+                kind = self.stream_dtype if getattr(op, "first_in_stream_type", False) else self.dtype
+                if kind not in copies:
+                    copies[kind] = torch.empty((T, self.spec.hidden_size), dtype=kind, device=self.device)
+                first[id(op)] = copies[kind]
+            feedback, scale = getattr(batch, "feedback", None), self.spec.embedding_scale
+            K.embed_gather(self.embedding, batch.token_ids, hidden, feedback, scale, copies.pop(self.stream_dtype, None))
+            for rows in copies.values():
+                K.embed_gather(self.embedding, batch.token_ids, rows, feedback, scale)
         for i, (call, slot) in enumerate(self.calls):
             block = self.blocks[call.layer]
             if call.before is not None:
+                op = self.stream_ops[call.before]
                 if isinstance(delta, StreamCopy):
                     delta = None                    # the stream holds everything already
                 if isinstance(delta, NormedRows):
                     raise TypeError("an operation between layers takes the stream, not rows prepared for a norm")
-                if getattr(delta, "scale", 1.0) != 1.0:
-                    raise TypeError("an operation between layers adds pending branch outputs as they are, not times a constant")
-                pending = () if delta is None else (tuple(delta) if isinstance(delta, (tuple, list)) else (delta,))
-                hidden, delta = self.stream_ops[call.before].forward(hidden, pending, first), None
+                if getattr(op, "defers", False):
+                    hidden, delta = op.defer(hidden, delta, first[id(op)])
+                else:
+                    if getattr(delta, "scale", 1.0) != 1.0 or isinstance(delta, PendingNorm):
+                        raise TypeError("an operation between layers adds pending branch outputs as they are, not times "
+                                        "a constant or under a norm")
+                    pending = () if delta is None else (tuple(delta) if isinstance(delta, (tuple, list)) else (delta,))
+                    hidden, delta = op.forward(hidden, pending, first[id(op)]), None
             # the norm that reads the residual stream after this block
             if i + 1 == len(self.calls):
                 next_norm = self.final_norm

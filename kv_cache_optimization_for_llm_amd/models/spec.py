@@ -18,13 +18,15 @@ class TensorSpec:
     """One tensor a part reads from the checkpoint.
 
     ``init`` names the random-weights rule: ``"normal"`` (N(0, 0.02)), ``"norm"``
-    (1 + U(-0.1, 0.1)), ``"eye"`` (a square matrix: the identity + U(-0.1, 0.1)) or ``"zeros"``.  ``role`` is ``"matrix"`` (takes the engine's compute
+    (1 + U(-0.1, 0.1)), ``"eye"`` (a square matrix: the identity + U(-0.1, 0.1)) or ``"zeros"``, for tables ``"distinct"`` (every row so
+    many different integers below ``bound``).  ``role`` is ``"matrix"`` (takes the engine's compute
     dtype unless stored in 32-bit), ``"vector"`` (same rule) or ``"table"`` (integers, int32).
     """
 
     shape: Tuple[Optional[int], ...]
     init: str = "normal"
     role: str = "matrix"
+    bound: int = 0
 
 
 @dataclass(frozen=True)

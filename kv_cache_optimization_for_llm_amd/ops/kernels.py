@@ -96,8 +96,10 @@ def check_cache_shapes(what: str, k_cache: torch.Tensor, v_cache: torch.Tensor, 
 
 # --------------------------------------------------------------------------------------
 def embed_gather(table: torch.Tensor, ids: torch.Tensor, out: torch.Tensor,
-                 feedback: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """out[t, :] = table[ids[t], :], converted to out's dtype.  A negative id ``-1 - r`` stands
+                 feedback: Optional[torch.Tensor] = None, scale: float = 1.0,
+                 copy: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """out[t, :] = table[ids[t], :] * scale, converted to out's dtype; ``copy`` (out's shape and dtype)
+    receives the rows a second time.  A negative id ``-1 - r`` stands
     for ``feedback[r]`` (a token still on the device); the caller guarantees ``r`` is inside
     ``feedback`` and that no id is negative when there is none.  An id outside the table (only
     what a kernel left in ``feedback`` can be: the host checks the ids it uploads) reads the
@@ -106,10 +108,12 @@ def embed_gather(table: torch.Tensor, ids: torch.Tensor, out: torch.Tensor,
     if table.dim() != 2 or table.shape[1] != width or ids.shape != (rows,):
         raise KernelError(f"embed_gather: shapes table {tuple(table.shape)} ids {tuple(ids.shape)} "
                           f"out {tuple(out.shape)} do not fit")
-    check(hip_lib().kva_embed_gather(_dev(out, "out"), _dev(table, "table"),
+    if copy is not None and (copy.shape != out.shape or copy.dtype != out.dtype):
+        raise KernelError("embed_gather: the second copy has out's shape and dtype")
+    check(hip_lib().kva_embed_gather(_dev(out, "out"), _opt(copy, "copy"), _dev(table, "table"),
                                      _dev(ids, "ids", torch.int32),
                                      _opt(feedback, "feedback", torch.int32), rows, width, table.shape[0],
-                                     dtype_code(table.dtype), dtype_code(out.dtype), _stream()),
+                                     dtype_code(table.dtype), dtype_code(out.dtype), float(scale), _stream()),
           "embed_gather")
     return out
 
@@ -582,7 +586,7 @@ def norm_into_stream(x: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, eps
     return x
 
 
-ACTIVATIONS = {"silu": 0, "relu": 1, "gelu_tanh": 2}
+ACTIVATIONS = {"silu": 0, "relu": 1, "gelu_tanh": 2, "relu2": 4}        # relu2: the square of relu
 # gated forms only: act(gate) * up with "swish_clamped" = g sigmoid(1.702 g) (u + 1), g = min(gate, limit),
 # u = clamp(up, -limit, limit)
 GATED_ACTIVATIONS = dict(ACTIVATIONS, swish_clamped=3)
@@ -678,6 +682,44 @@ def hyper_fill(x: torch.Tensor, first: torch.Tensor, streams: int) -> torch.Tens
     return x
 
 
+def sandwich_step(x: torch.Tensor, *, y: Optional[torch.Tensor] = None, post=None, addend: Optional[torch.Tensor] = None,
+                  pre=None, out: Optional[torch.Tensor] = None, row_idx: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
+    """What lies between two branches that have norms on both sides, over a residual stream ``x`` fp32 ``[T,
+    width]``: ``x += n_post(y) (+ addend)``, then ``out = n_pre(x)``.  ``post`` and ``pre`` are ``(weight, bias or
+    None, eps, center)``: ``(v - mean) / sqrt(var + eps) * weight + bias``, without ``center`` the mean is not taken
+    off.  Without ``post`` the branch output enters as it is; ``addend`` (fp32) always does.  ``row_idx``: only
+    these rows are read out, and nothing is written back."""
+    T, width = x.shape
+    if x.dim() != 2 or x.dtype != torch.float32:
+        raise KernelError(f"sandwich_step: x {tuple(x.shape)} is not an fp32 [T, width] stream")
+    if (y is not None and y.shape != x.shape) or (addend is not None and (addend.shape != x.shape or addend.dtype != torch.float32)):
+        raise KernelError("sandwich_step: the branch output and the addend (fp32) have the stream's shape")
+    for norm in (post, pre):
+        if norm is not None and (norm[0].shape != (width,) or (norm[1] is not None and (
+                norm[1].shape != (width,) or norm[1].dtype != norm[0].dtype))):
+            raise KernelError("sandwich_step: a norm has a weight [width] and a bias of its shape and type, or none")
+    if (post is not None and y is None) or (out is None) != (pre is None):
+        raise KernelError("sandwich_step: the first norm goes with a branch output, the second with an output")
+    rows = T
+    if out is not None:
+        rows = T if row_idx is None else row_idx.shape[0]
+        if out.shape != (rows, width):
+            raise KernelError(f"sandwich_step: out {tuple(out.shape)} is not [{rows}, {width}]")
+    elif row_idx is not None:
+        raise KernelError("sandwich_step: rows are gathered for the read-out only")
+
+    def args(norm, name):
+        if norm is None:
+            return None, None, 0, 0, 0.0
+        w, b, eps, center = norm
+        return _dev(w, name), _opt(b, name), dtype_code(w.dtype), 1 if center else 0, float(eps)
+    check(hip_lib().kva_sandwich_step(
+        _dev(x, "x"), _opt(y, "y"), dtype_code(y.dtype) if y is not None else 0, *args(post, "post norm"), _opt(addend, "addend"),
+        *args(pre, "pre norm"), _opt(out, "out"), dtype_code(out.dtype) if out is not None else 0,
+        _opt(row_idx, "row_idx", torch.int32), rows, width, _stream()), "sandwich_step")
+    return out
+
+
 def head_gate(x: torch.Tensor, gates: torch.Tensor, heads: int) -> torch.Tensor:
     """In place: head h of row t of ``x`` ``[T, heads * d]`` times ``sigmoid(gates[t, h])``; ``gates``
     is a ``[T, heads]`` view whose rows may be columns of a wider buffer."""
@@ -744,18 +786,32 @@ def qk_encode_cache(qkv: torch.Tensor, positions: torch.Tensor, num_q_heads: int
         1 if norm_first else 0, _stream()), "qk_encode_cache")
 
 
-def latent_encode_cache(y: torch.Tensor, kv_off: int, q_lat: torch.Tensor, cache: Optional[torch.Tensor],
+def latent_encode_cache(y: torch.Tensor, kv_off: int, q_lat: Optional[torch.Tensor], cache: Optional[torch.Tensor],
                         norm_weight: torch.Tensor, eps: float, cos: torch.Tensor, sin: torch.Tensor,
                         positions: torch.Tensor, slot_mapping: Optional[torch.Tensor], heads: int, plain_dim: int,
-                        rank: int, interleaved: bool = False, cache_t: Optional[torch.Tensor] = None) -> None:
+                        rank: int, interleaved: bool = False, cache_t: Optional[torch.Tensor] = None,
+                        c_q: Optional[torch.Tensor] = None, q_norm_weight: Optional[torch.Tensor] = None) -> None:
     """From a projection row ``y[t] = [heads x (plain_dim + rot) | ... rank + rot at kv_off ...]``:
     the rotated part of every query head goes to ``q_lat[t, h, rank:]``; the entry's first ``rank``
     elements, RMS-normed with ``norm_weight``, and its rotated last ``rot`` go to row
     ``slot_mapping[t]`` of ``cache`` ``[pages, page_size, rank + rot]`` - and the normed latent a
-    second time into ``cache_t`` ``[pages, rank, page_size]`` where that is given."""
+    second time into ``cache_t`` ``[pages, rank, page_size]`` where that is given.
+
+    With ``c_q`` ``[T, q_rank]`` (and without ``q_lat``) the rows start with a query latent instead of the
+    query heads, ``y[t] = [q_rank | ... rank + rot at kv_off ...]``: it is RMS-normed with ``q_norm_weight`` (and
+    the same eps) into ``c_q``, and the query heads are somebody else's to rotate."""
     tokens = y.shape[0]
     rot = 2 * cos.shape[1]
-    if y.dim() != 2 or q_lat.shape != (tokens, heads, rank + rot) or q_lat.dtype != y.dtype or positions.shape != (tokens,):
+    if (q_lat is None) == (c_q is None):
+        raise KernelError("latent_encode_cache: rows start with the query heads or with a query latent")
+    if c_q is not None:
+        heads = 0
+        if c_q.dim() != 2 or c_q.shape[0] != tokens or c_q.dtype != y.dtype or q_norm_weight is None \
+                or q_norm_weight.shape != (c_q.shape[1],) or q_norm_weight.dtype != norm_weight.dtype:
+            raise KernelError("latent_encode_cache: the query latent [T, q_rank] of y's dtype has a norm weight [q_rank]")
+    if y.dim() != 2 or positions.shape != (tokens,):
+        raise KernelError(f"latent_encode_cache: y {tuple(y.shape)} does not fit one position per token")
+    if q_lat is not None and (q_lat.shape != (tokens, heads, rank + rot) or q_lat.dtype != y.dtype):
         raise KernelError(f"latent_encode_cache: y {tuple(y.shape)} and q_lat {tuple(q_lat.shape)} do not fit")
     if cos.shape != sin.shape or norm_weight.shape != (rank,):
         raise KernelError("latent_encode_cache: tables [positions, rot / 2] and a norm weight [rank] are needed")
@@ -766,7 +822,8 @@ def latent_encode_cache(y: torch.Tensor, kv_off: int, q_lat: torch.Tensor, cache
     if cache_t is not None and write and (cache_t.shape != (cache.shape[0], rank, cache.shape[1]) or cache_t.dtype != y.dtype):
         raise KernelError("latent_encode_cache: the transposed copy must be [pages, rank, page_size] of y's dtype")
     check(hip_lib().kva_latent_encode_cache(
-        _dev(y, "y"), y.shape[1], int(kv_off), _dev(q_lat, "q_lat"), _opt(cache if write else None, "cache"),
+        _dev(y, "y"), y.shape[1], int(kv_off), _opt(q_lat, "q_lat"), _opt(c_q, "c_q"), _opt(q_norm_weight, "q_norm_weight"),
+        c_q.shape[1] if c_q is not None else 0, _opt(cache if write else None, "cache"),
         _opt(cache_t if write else None, "cache_t"), cache.shape[1] if write else 0,
         _dev(norm_weight, "norm_weight"), dtype_code(norm_weight.dtype), float(eps),
         _dev(cos, "cos", torch.float32), _dev(sin, "sin", torch.float32), _dev(positions, "positions", torch.int32),
@@ -774,37 +831,56 @@ def latent_encode_cache(y: torch.Tensor, kv_off: int, q_lat: torch.Tensor, cache
         1 if interleaved else 0, dtype_code(y.dtype), _stream()), "latent_encode_cache")
 
 
-def heads_matmul(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, gates: Optional[torch.Tensor] = None) -> torch.Tensor:
+def heads_matmul(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, gates: Optional[torch.Tensor] = None,
+                 rotate: Optional[tuple] = None) -> torch.Tensor:
     """``out[t, h, :] = w[h] @ x[t, h, :]`` for ``w`` ``[heads, N, K]``.  ``x`` ``[T, heads, K]`` and
     ``out`` ``[T, heads, N]`` may be views into wider buffers (unit stride along the last axis).
     With ``gates`` (``[T, heads]``, a column range of another buffer) head h of row t is multiplied
-    by ``sigmoid(gates[t, h])``."""
+    by ``sigmoid(gates[t, h])``; gates ``[T, heads, N]`` multiply every output element by its own.
+
+    ``rotate = (src, dst, cos, sin, positions, interleaved)``: in the same launch the rows ``src`` ``[T, heads,
+    rot]`` are rotated by their positions into ``dst`` (views like ``x`` and ``out``; pair i is ``(2i, 2i + 1)`` when
+    ``interleaved``, else ``(i, i + rot / 2)``; fp32 tables ``[positions, rot / 2]``)."""
     heads, n, k = w.shape
     rows = x.shape[0]
-    g_row = 0
+
+    def strides(t, last):
+        """(row, head) strides of a [T, heads, last] view, also where T or heads is 1 and they are arbitrary"""
+        head = t.stride(1) if heads > 1 else max(t.stride(1), last)
+        row = t.stride(0) if rows > 1 else max(t.stride(0), (heads - 1) * head + last)
+        return row, head
+    options = [None, 0, 0, 0]
     if gates is not None:
-        if gates.shape != (rows, heads) or gates.dtype != x.dtype or gates.stride(1) != 1:
+        elementwise = gates.dim() == 3
+        if gates.shape != ((rows, heads, n) if elementwise else (rows, heads)) or gates.dtype != x.dtype or gates.stride(-1) != 1:
             raise KernelError(f"heads_matmul: gates {tuple(gates.shape)} do not fit {rows} rows of {heads} heads")
-        g_row = gates.stride(0) if rows > 1 else heads
+        g_row, g_head = strides(gates, n) if elementwise else (gates.stride(0) if rows > 1 else heads, 1)
+        options = [_dev(gates, "gates", contiguous=False), g_row, g_head, 1 if elementwise else 0]
+    if rotate is None:
+        options += [None, 0, 0, None, 0, 0, None, None, None, 0, 0]
+    else:
+        src, dst, cos, sin, positions, interleaved = rotate
+        rot = src.shape[2]
+        if src.shape != (rows, heads, rot) or dst.shape != src.shape or src.stride(2) != 1 or dst.stride(2) != 1 \
+                or src.dtype != x.dtype or dst.dtype != x.dtype or cos.shape != sin.shape or cos.dim() != 2 \
+                or 2 * cos.shape[1] != rot or positions.shape != (rows,):
+            raise KernelError(f"heads_matmul: the rotated rows {tuple(src.shape)} -> {tuple(dst.shape)} do not fit")
+        options += [_dev(src, "rotate source", contiguous=False), *strides(src, rot), _dev(dst, "rotate target", contiguous=False),
+                    *strides(dst, rot), _dev(cos, "cos", torch.float32), _dev(sin, "sin", torch.float32),
+                    _dev(positions, "positions", torch.int32), rot, 1 if interleaved else 0]
     if x.shape != (rows, heads, k) or out.shape != (rows, heads, n) or x.stride(2) != 1 or out.stride(2) != 1 \
             or not (x.dtype == w.dtype == out.dtype):
         raise KernelError(f"heads_matmul: x {tuple(x.shape)}, w {tuple(w.shape)}, out {tuple(out.shape)} do not fit")
-    xr, xh = (x.stride(0), x.stride(1)) if rows > 1 else (max(x.stride(0), (heads - 1) * x.stride(1) + k), x.stride(1))
-    orr, oh = (out.stride(0), out.stride(1)) if rows > 1 else (max(out.stride(0), (heads - 1) * out.stride(1) + n), out.stride(1))
-    if heads == 1:
-        xh, oh = max(xh, k), max(oh, n)
+    (xr, xh), (orr, oh) = strides(x, k), strides(out, n)
     if x.dtype == torch.bfloat16 and x.data_ptr() % 16 == 0 and out.data_ptr() % 8 == 0 \
             and hip_lib().kva_heads_matmul_mfma_supported(k, xr, xh):
         # bf16 with a K that has an instance: the matrix cores
         check(hip_lib().kva_heads_matmul_mfma(_dev(out, "out", contiguous=False), orr, oh, _dev(x, "x", contiguous=False),
-                                              xr, xh, _dev(w, "w"), rows, heads, n, k,
-                                              None if gates is None else _dev(gates, "gates", contiguous=False), g_row,
-                                              _stream()), "heads_matmul_mfma")
+                                              xr, xh, _dev(w, "w"), rows, heads, n, k, *options, _stream()),
+              "heads_matmul_mfma")
         return out
     check(hip_lib().kva_heads_matmul(_dev(out, "out", contiguous=False), orr, oh, _dev(x, "x", contiguous=False), xr, xh,
-                                     _dev(w, "w"), rows, heads, n, k,
-                                     None if gates is None else _dev(gates, "gates", contiguous=False), g_row,
-                                     dtype_code(x.dtype), _stream()), "heads_matmul")
+                                     _dev(w, "w"), rows, heads, n, k, *options, dtype_code(x.dtype), _stream()), "heads_matmul")
     return out
 
 
@@ -1693,7 +1769,7 @@ def head_norm_gate(x: torch.Tensor, weight: Optional[torch.Tensor], eps: float, 
 # --------------------------------------------------------------------------------------
 # Routed experts.
 MOE_TILE = 16
-EXPERT_ACTIVATIONS = {"silu": 0, "relu": 1, "gelu_tanh": 2, "gelu": 3, "swish_clamped": 4}     # the last one gated only, with a limit
+EXPERT_ACTIVATIONS = {"silu": 0, "relu": 1, "gelu_tanh": 2, "gelu": 3, "swish_clamped": 4, "relu2": 5}     # swish_clamped: gated only, with a limit
 
 
 def moe_route(logits: torch.Tensor, correction: Optional[torch.Tensor], top: int, idx: torch.Tensor,
@@ -1738,6 +1814,24 @@ def moe_align(idx: torch.Tensor, experts: int, sorted_slot: torch.Tensor, tile_e
     check(hip_lib().kva_moe_align(_dev(sorted_slot, "sorted_slot", torch.int32), _dev(tile_expert, "tile_expert", torch.int32),
                                   _dev(idx, "idx", torch.int32), slots, int(experts), tiles * MOE_TILE, tiles,
                                   _stream()), "moe_align")
+
+
+def moe_table_align(table: torch.Tensor, ids: torch.Tensor, idx: torch.Tensor, wgt: torch.Tensor, experts: int,
+                    sorted_slot: torch.Tensor, tile_expert: torch.Tensor, feedback: Optional[torch.Tensor] = None) -> None:
+    """Experts by token id, without a router: ``idx[t] = table[ids[t]]`` (int32 ``[rows, top]``) with equal
+    weights ``wgt[t, k] = 1 / top``, and the slots sorted by expert as :func:`moe_align` does, in one launch.  A
+    negative id ``-1 - r`` stands for ``feedback[r]`` as in :func:`embed_gather`."""
+    tokens, top = idx.shape
+    tiles = tile_expert.shape[0]
+    if table.dim() != 2 or table.shape[1] != top or ids.shape != (tokens,) or wgt.shape != (tokens, top):
+        raise KernelError(f"moe_table_align: table {tuple(table.shape)}, ids {tuple(ids.shape)}, idx {tuple(idx.shape)} do not fit")
+    if sorted_slot.shape != (tiles * MOE_TILE,) or tiles < moe_tiles(tokens * top, experts):
+        raise KernelError(f"moe_table_align: {tiles} tiles cannot hold {tokens * top} slots of {experts} experts")
+    check(hip_lib().kva_moe_table_align(
+        _dev(sorted_slot, "sorted_slot", torch.int32), _dev(tile_expert, "tile_expert", torch.int32), _dev(idx, "idx", torch.int32),
+        _dev(wgt, "wgt", torch.float32), _dev(table, "table", torch.int32), table.shape[0], _dev(ids, "ids", torch.int32),
+        _opt(feedback, "feedback", torch.int32), tokens, top, 1.0 / top, int(experts), tiles * MOE_TILE, tiles,
+        _stream()), "moe_table_align")
 
 
 def moe_expert_rows(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, sorted_slot: torch.Tensor,
@@ -1850,10 +1944,10 @@ KERNEL_CLASSES = {
     "sample": "sampling", "mark_tokens": "sampling",
     "causal_conv_act": "recurrent mixers", "gated_delta_rule": "recurrent mixers",
     "gated_linear_attention": "recurrent mixers", "head_norm_gate": "elementwise",
-    "moe_route": "routed experts", "moe_align": "routed experts", "moe_expert_rows": "routed experts",
+    "moe_route": "routed experts", "moe_align": "routed experts", "moe_table_align": "routed experts", "moe_expert_rows": "routed experts",
     "moe_combine": "routed experts", "small_product_f32": "small fp32 products",
     "norm_into_stream": "norm", "table_gate": "elementwise",
-    "hyper_step": "norm", "hyper_fill": "embedding", "bias_act": "activation",
+    "hyper_step": "norm", "sandwich_step": "norm", "hyper_fill": "embedding", "bias_act": "activation",
     "block_gates": "recurrent mixers", "linear_scan_gate": "recurrent mixers", "matrix_memory": "recurrent mixers",
 }
 

@@ -32,7 +32,7 @@ LL = c_longlong
 U = c_uint
 
 _HIP_SIGNATURES = {
-    "kva_embed_gather": [P, P, P, P, I, I, I, I, I, P],
+    "kva_embed_gather": [P, P, P, P, P, I, I, I, I, I, F, P],
     "kva_embed_gather_prep": [P, P, P, P, P, P, P, I, I, I, I, P],
     "kva_rmsnorm": [P, P, P, P, P, I, I, F, I, I, P, I, I, P],
     "kva_residual_add": [P, P, LL, I, P],
@@ -50,14 +50,14 @@ _HIP_SIGNATURES = {
     "kva_act_mul": [P, P, I, I, I, F, I, P],
     "kva_head_gate": [P, P, I, I, I, I, I, P],
     "kva_qk_encode_cache": [P, I, I, I, P, P, P, P, P, P, I, I, I, I, I, I, I, F, I, I, P, P, P, I, P],
-    "kva_latent_encode_cache": [P, I, I, P, P, P, I, P, I, F, P, P, P, P, I, I, I, I, I, I, I, P],
+    "kva_latent_encode_cache": [P, I, I, P, P, P, I, P, P, I, P, I, F, P, P, P, P, I, I, I, I, I, I, I, P],
     "kva_latent_attention_mfma_supported": [I, I, I],
     "kva_attention_rows_mfma_supported": [I, I, I],
     "kva_attention_rows_mfma": [P, P, P, P, I, P, P, P, I, P, P, P, P, P, I, I, I, I, I, I, I, F, I, I, I, P, I, I, I, P],
     "kva_latent_attention_mfma": [P, P, P, P, P, P, P, I, P, P, P, P, P, I, I, I, I, I, I, F, I, I, P, I, I, P],
-    "kva_heads_matmul": [P, I, I, P, I, I, P, I, I, I, I, P, I, I, P],
+    "kva_heads_matmul": [P, I, I, P, I, I, P, I, I, I, I, P, I, I, I, P, I, I, P, I, I, P, P, P, I, I, I, P],
     "kva_heads_matmul_mfma_supported": [I, I, I],
-    "kva_heads_matmul_mfma": [P, I, I, P, I, I, P, I, I, I, I, P, I, P],
+    "kva_heads_matmul_mfma": [P, I, I, P, I, I, P, I, I, I, I, P, I, I, I, P, I, I, P, I, I, P, P, P, I, I, P],
     "kva_attention_mfma": [P, P, P, P, I, P, P, P, I, P, P, P, I, I, P, P, P, I, I, I, I, I, F, I, I, I, I, I, I, I, P],
     "kva_attention_mfma_rope": [P, P, P, P, I, P, P, P, I, P, I, I, I, I, I, I, F, I, I, I, I, P, P, P, I, P],
     "kva_attention_mfma_rope_supported": [I, I, I],
@@ -97,6 +97,7 @@ _HIP_SIGNATURES = {
     "kva_head_norm_gate": [P, I, I, I, P, I, P, F, P, I, I, I, I, I, I, I, F, I, P],
     "kva_moe_route": [P, P, P, P, I, I, I, I, I, I, I, I, I, F, F, I, P],
     "kva_moe_align": [P, P, P, I, I, I, I, P],
+    "kva_moe_table_align": [P, P, P, P, P, I, P, P, I, I, F, I, I, I, P],
     "kva_moe_expert_rows": [P, I, P, P, I, P, P, P, I, I, I, I, I, I, I, F, P],
     "kva_moe_combine": [P, P, I, P, P, P, P, P, I, I, I, I, I, P],
     "kva_small_product_f32": [P, P, I, I, P, I, I, I, I, P, F, P, I, P],
@@ -104,6 +105,7 @@ _HIP_SIGNATURES = {
     "kva_table_gate": [P, P, I, P, I, I, I, I, P, P, I, I, I, P],
     "kva_bias_act": [P, P, I, P, I, I, I, P],
     "kva_hyper_step": [P, I, P, I, P, P, F, P, P, P, I, F, P, I, P, I, I, P],
+    "kva_sandwich_step": [P, P, I, P, P, I, I, F, P, P, P, I, I, F, P, I, P, I, I, P],
     "kva_hyper_fill": [P, P, I, I, I, I, P],
     "kva_block_gates": [P, P, P, I, I, I, P, P, I, P, P, P, P],
     "kva_linear_scan_gate": [P, I, I, I, P, P, I, P, I, I, I, P, P, LL, I, P, P, I, F, P],

@@ -208,6 +208,18 @@ class PendingMix:
 
 
 @dataclass
+class PendingNorm:
+    """A branch output that has not entered the residual stream yet and does so under a norm of its own
+    (``x <- x + norm(y)``), with ``addend`` (fp32, the stream's shape; optional) behind it: whoever reads the
+    stream next lets both in, in the pass that reads (``ops.kernels.sandwich_step``).  ``norm`` None: ``y`` enters
+    as it is; ``y`` None: only the addend does."""
+
+    y: Optional[torch.Tensor]
+    norm: object = None
+    addend: Optional[torch.Tensor] = None
+
+
+@dataclass
 class BranchTail:
     """What is to happen to a branch's output: it is added to ``hidden`` (the residual stream, in
     place) and the sum is handed to ``norm``, the norm that reads the stream next.  A mixer or

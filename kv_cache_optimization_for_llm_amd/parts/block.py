@@ -15,7 +15,7 @@ from ..config.registry import BLOCKS, LAYER_INPUTS
 from ..models.spec import PartSpec
 from ..ops import kernels as K
 from ..models.spec import TensorSpec
-from .base import Block, BranchTail, MixerContext, Norm, NormedRows, Part, PendingMix, PendingSum, StreamCopy
+from .base import Block, BranchTail, MixerContext, Norm, NormedRows, Part, PendingMix, PendingNorm, PendingSum, StreamCopy
 
 
 @BLOCKS.register("pre_norm")
@@ -158,6 +158,44 @@ class PostNormBlock(Block):
         if self.layer_input is not None:
             h = self._into_stream(hidden, self.layer_input.forward(h, ctx), self.layer_input)
         return hidden, (StreamCopy(h) if h is not hidden else None)
+
+
+@BLOCKS.register("sandwich_norm")
+class SandwichNormBlock(Block):
+    """A norm in front of every branch and another on its output: ``h += norm_mo(mixer(norm_m(h))); h +=
+    norm_fo(ffn(norm_f(h)))``, over a residual stream kept in 32-bit.  The norms are of kind ``"layernorm"``
+    (weight, optional bias, with or without the mean taken off).  What lies between two branches - the
+    output's norm, the sum, the next branch's norm - is one launch: the block hands its last output on as
+    :class:`~.base.PendingNorm`, and whoever reads the stream next lets it in in its own pass.  A layer without
+    a feed-forward (``"none"``) names only the mixer's two norms."""
+
+    graph_safe = True
+    NORM_NAMES = ("mixer", "mixer_out", "feed_forward", "feed_forward_out")
+
+    def __init__(self, mixer, feed_forward, norms):
+        self.has_ffn = not getattr(feed_forward, "absent", False)
+        if not self.has_ffn:
+            self.NORM_NAMES = ("mixer", "mixer_out")
+        super().__init__(mixer, feed_forward, norms)
+        for name, norm in self.norms.items():
+            if not hasattr(norm, "pass_args"):
+                raise ValueError(f"this arrangement runs its norms inside its own pass; {name!r} is a {type(norm).__name__}")
+
+    def first_norm(self) -> Optional[Norm]:
+        return None
+
+    def forward(self, hidden: torch.Tensor, delta, ctx: MixerContext, next_norm: Optional[Norm] = None):
+        if delta is None:
+            delta = PendingNorm(None)
+        if not isinstance(delta, PendingNorm) or hidden.dtype != torch.float32:
+            raise TypeError("this arrangement takes a 32-bit stream and a pending output with the norm it enters under")
+        n = self.norms
+        a = self.mixer.forward(n["mixer"].forward(hidden, delta=delta), ctx)
+        delta = PendingNorm(a, n["mixer_out"])
+        if self.has_ffn:
+            f = self.feed_forward.forward(n["feed_forward"].forward(hidden, delta=delta), ctx)
+            delta = PendingNorm(f, n["feed_forward_out"])
+        return hidden, delta
 
 
 class HyperConnection(Part):

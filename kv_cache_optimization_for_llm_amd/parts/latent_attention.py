@@ -17,9 +17,10 @@ behind the attention, ``sum_j p U_v c_j = U_v (sum_j p c_j)``.  What a step cost
 is then independent of the number of heads' key and value sizes, and a prompt cut anywhere
 continues from the rows alone.
 
-Options: a softmax sink per head (``exp(sink_h)`` added to the denominator; no key, no value,
-not scaled), a sigmoid output gate per head read from the mixer's input, a window with kept first
-positions.  Softmax, the latent's norm and the rotation are fp32.
+Options: queries through a latent of their own (``c_q = RMSnorm(W_dq x)``, ``q = W_uq c_q``), a softmax sink
+per head (``exp(sink_h)`` added to the denominator; no key, no value, not scaled), a sigmoid output
+gate read from the mixer's input (one number a head, or one an element of the concatenated heads), a
+window with kept first positions.  Softmax, the latents' norms and the rotation are fp32.
 """
 from __future__ import annotations
 
@@ -52,20 +53,25 @@ class LatentAttention(Mixer):
 
     def __init__(self, prefix: str, *, hidden_size: int, num_heads: int, head_dim: int, rot_dim: int,
                  value_dim: int, rank: int, scale: float, norm_eps: float, position: PartSpec, sink: bool = False,
-                 gate: bool = False, window: int = 0, keep_first: int = 0,
+                 gate=False, window: int = 0, keep_first: int = 0, q_rank: int = 0,
                  tensor_names: Optional[Dict[str, str]] = None):
         """``head_dim``: unrotated query/key elements per head; ``rot_dim``: rotated ones (the
         ``position`` encoding must rotate exactly these); ``rank``: size of the latent.
-        ``tensor_names`` maps ``q``, ``down``, ``down_norm``, ``up_k``, ``up_v``, ``sink``, ``gate``,
-        ``o`` to the tensors' names behind ``prefix``."""
+        ``q_rank`` > 0: queries come from a latent of that size, normed with a weight and ``norm_eps``.
+        ``gate``: False, True or "head" (one number a head), "element" (one an element of the concatenated heads).
+        ``tensor_names`` maps ``q`` (with ``q_rank``: the matrix behind the latent), ``q_down``, ``q_norm``,
+        ``down``, ``down_norm``, ``up_k``, ``up_v``, ``sink``, ``gate``, ``o`` to the tensors' names behind ``prefix``."""
         super().__init__(prefix)
         self.hidden_size, self.num_heads, self.head_dim = int(hidden_size), int(num_heads), int(head_dim)
         self.rot_dim, self.value_dim, self.rank = int(rot_dim), int(value_dim), int(rank)
         self.scale, self.norm_eps = float(scale), float(norm_eps)
-        self.has_sink, self.has_gate = bool(sink), bool(gate)
+        if gate not in (False, True, "head", "element"):
+            raise ValueError(f"{prefix}: gate {gate!r} is not one of False, 'head', 'element'")
+        self.has_sink, self.has_gate, self.gate_elements = bool(sink), bool(gate), gate == "element"
+        self.q_rank = int(q_rank)
         self.window = int(window)
         self.keep_first = int(keep_first) if self.window > 0 else 0
-        names = dict(q="q_proj.weight", down="kv_down.weight", down_norm="kv_norm.weight", up_k="k_up.weight",
+        names = dict(q="q_proj.weight", q_down="q_down.weight", q_norm="q_norm.weight", down="kv_down.weight", down_norm="kv_norm.weight", up_k="k_up.weight",
                      up_v="v_up.weight", sink="sinks", gate="gate.weight", o="o_proj.weight")
         names.update(tensor_names or {})
         self.names = {key: prefix + name for key, name in names.items()}
@@ -73,34 +79,43 @@ class LatentAttention(Mixer):
         if getattr(self.position, "rotary_dim", None) != self.rot_dim or getattr(self.position, "unit_norm_eps", None) is not None:
             raise ValueError("latent attention needs a rotary encoding over exactly its rot_dim elements")
         self.key_dim = self.rank + self.rot_dim
-        self.proj: Optional[Linear] = None          # [q ; down ; gate] joined
+        self.proj: Optional[Linear] = None          # [q or its latent ; down ; gate] joined
+        self.q_up: Optional[Linear] = None          # the queries from their latent
         self.o: Optional[Linear] = None
-        self.up_k_t = self.up_v = self.norm_weight = self.sinks = None
+        self.up_k_t = self.up_v = self.norm_weight = self.q_norm_weight = self.sinks = None
 
     def tensor_specs(self) -> Dict[str, TensorSpec]:
         n, H, W = self.names, self.num_heads, self.hidden_size
         specs = {
-            n["q"]: TensorSpec((H * (self.head_dim + self.rot_dim), W)),
+            n["q"]: TensorSpec((H * (self.head_dim + self.rot_dim), self.q_rank or W)),
             n["down"]: TensorSpec((self.key_dim, W)),
             n["down_norm"]: TensorSpec((self.rank,), init="norm", role="vector"),
             n["up_k"]: TensorSpec((H * self.head_dim, self.rank)),
             n["up_v"]: TensorSpec((H * self.value_dim, self.rank)),
             n["o"]: TensorSpec((W, H * self.value_dim)),
         }
+        if self.q_rank:
+            specs[n["q_down"]] = TensorSpec((self.q_rank, W))
+            specs[n["q_norm"]] = TensorSpec((self.q_rank,), init="norm", role="vector")
         if self.has_sink:
             specs[n["sink"]] = TensorSpec((H,), init="normal", role="vector")
         if self.has_gate:
-            specs[n["gate"]] = TensorSpec((H, W))
+            specs[n["gate"]] = TensorSpec((self._gates(), W))
         return specs
+
+    def _gates(self) -> int:
+        return self.num_heads * (self.value_dim if self.gate_elements else 1)
 
     def load(self, tensors: Dict[str, torch.Tensor]) -> None:
         n, H = self.names, self.num_heads
-        mats = [tensors[n["q"]], tensors[n["down"]]] + ([tensors[n["gate"]]] if self.has_gate else [])
+        mats = [tensors[n["q_down" if self.q_rank else "q"]], tensors[n["down"]]] + ([tensors[n["gate"]]] if self.has_gate else [])
         if len({m.dtype for m in mats}) != 1:
             raise ValueError(f"{self.prefix}: the input projections are stored in different dtypes")
         self.proj = Linear(torch.cat(mats, dim=0))
-        self.kv_off = H * (self.head_dim + self.rot_dim)
+        self.kv_off = self.q_rank or H * (self.head_dim + self.rot_dim)
         self.gate_off = self.kv_off + self.key_dim
+        self.q_up = Linear(tensors[n["q"]]) if self.q_rank else None
+        self.q_norm_weight = tensors[n["q_norm"]].contiguous() if self.q_rank else None
         self.o = Linear(tensors[n["o"]])
         # U_k per head, transposed: the query-side product reads [heads, rank, dim]
         self.up_k_t = tensors[n["up_k"]].view(H, self.head_dim, self.rank).transpose(1, 2).contiguous()
@@ -119,7 +134,7 @@ class LatentAttention(Mixer):
     def activation_elements(self) -> int:
         H = self.num_heads
         return (self.proj.out_features if self.proj is not None else 0) + H * (self.key_dim + self.rank + self.value_dim) \
-            + self.hidden_size
+            + (self.q_rank + H * (self.head_dim + self.rot_dim) if self.q_rank else 0) + self.hidden_size
 
     def forward(self, x, ctx: MixerContext, tail=None):
         if isinstance(x, NormedRows):
@@ -128,21 +143,28 @@ class LatentAttention(Mixer):
         if kv is None:
             raise K.KernelError("latent attention: the mixer has no cache view")
         T, H = x.shape[0], self.num_heads
-        y = self.proj(x)                                                    # [T, q | entry | gates]
+        y = self.proj(x)                                                    # [T, q or its latent | entry | gates]
         q_lat = torch.empty((T, H, self.key_dim), dtype=x.dtype, device=x.device)
         cos, sin = self.position.tables(x.device)
+        interleaved = self.position.pairing == "interleaved"
         write = kv.writes
-        K.latent_encode_cache(y, self.kv_off, q_lat, kv.arrays["latent"] if write else None, self.norm_weight,
-                              self.norm_eps, cos, sin, batch.positions, kv.slot_mapping if write else None, H,
-                              self.head_dim, self.rank, interleaved=self.position.pairing == "interleaved",
-                              cache_t=kv.arrays.get(lat_ops.TRANSPOSED) if write else None)
+        c_q = torch.empty((T, self.q_rank), dtype=x.dtype, device=x.device) if self.q_rank else None
+        K.latent_encode_cache(y, self.kv_off, None if self.q_rank else q_lat, kv.arrays["latent"] if write else None,
+                              self.norm_weight, self.norm_eps, cos, sin, batch.positions,
+                              kv.slot_mapping if write else None, H, self.head_dim, self.rank, interleaved=interleaved,
+                              cache_t=kv.arrays.get(lat_ops.TRANSPOSED) if write else None, c_q=c_q,
+                              q_norm_weight=self.q_norm_weight)
+        q = (self.q_up(c_q) if self.q_rank else y[:, :self.kv_off]).view(T, H, self.head_dim + self.rot_dim)
+        # queries from a latent exist only now: their rotated parts are turned in the expansion's launch
+        rotate = (q[:, :, self.head_dim:], q_lat[:, :, self.rank:], cos, sin, batch.positions, interleaved) if self.q_rank else None
         # the key expansion on the query side: q_lat[:, h, :rank] = U_k[h]^T q_p[h]
-        q_plain = y[:, :self.kv_off].view(T, H, self.head_dim + self.rot_dim)[:, :, :self.head_dim]
-        lat_ops.heads_product(q_plain, self.up_k_t, q_lat[:, :, :self.rank])
+        lat_ops.heads_product(q[:, :, :self.head_dim], self.up_k_t, q_lat[:, :, :self.rank], rotate=rotate)
         o_lat = torch.empty((T, H, self.rank), dtype=x.dtype, device=x.device)
         lat_ops.latent_attention(q_lat, o_lat, kv, batch, self.scale, self.window, self.keep_first, self.sinks)
         out = torch.empty((T, H * self.value_dim), dtype=x.dtype, device=x.device)
-        # the value expansion behind the attention, the head's output gate in the same pass
-        lat_ops.heads_product(o_lat, self.up_v, out.view(T, H, self.value_dim),
-                              gates=y[:, self.gate_off:self.gate_off + H] if self.has_gate else None)
+        # the value expansion behind the attention, the output gate in the same pass
+        gates = y[:, self.gate_off:self.gate_off + self._gates()] if self.has_gate else None
+        if self.gate_elements:
+            gates = gates.unflatten(1, (H, self.value_dim))
+        lat_ops.heads_product(o_lat, self.up_v, out.view(T, H, self.value_dim), gates=gates)
         return self.o(out)

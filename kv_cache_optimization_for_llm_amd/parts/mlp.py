@@ -107,7 +107,7 @@ class SwiGLU(FeedForward):
 @FEED_FORWARDS.register("mlp")
 class PlainMLP(FeedForward):
     """A feed-forward that is not gated: ``down(act(up(x)))`` without biases; ``act`` one of silu, relu,
-    gelu_tanh, applied by its own kernel between the two products."""
+    gelu_tanh, relu2 (the square of relu), applied by its own kernel between the two products."""
 
     graph_safe = True
 

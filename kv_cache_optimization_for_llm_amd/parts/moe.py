@@ -9,6 +9,8 @@ are chosen; their weights are the plain scores (``renormalise``: divided by thei
 largest logits are chosen and the weights are the softmax over the chosen logits alone.
 ``gated``: an expert is ``W_down (act(W_gate x) * (W_up x))``; its gate and up matrices are stacked
 row by row in turns at load time, so that one product's epilogue has both halves of every output.
+``router="table"``: no router at all; an integer table ``[token ids, top]`` names every token id's
+experts (distinct in a row), each with weight ``1 / top``.
 ``shared_intermediate``: one more expert of that width (its tensors behind ``shared.``) that every
 token uses with weight 1; it runs as an ordinary gated feed-forward and is added to the sum.
 
@@ -43,8 +45,8 @@ class RoutedExperts(FeedForward):
                  gated: bool = False, router_bias: bool = False, softmax_over: str = "all",
                  shared_intermediate: int = 0, scores: str = "softmax", groups: int = 1, keep_groups: int = 1,
                  group_top: int = 2, weight_scale: float = 1.0, sum_eps: float = 0.0, limit: float = 0.0,
-                 shared_limit: Optional[float] = None, shared_gate: bool = False,
-                 tensor_names: Optional[Dict[str, str]] = None):
+                 shared_limit: Optional[float] = None, shared_gate: bool = False, router: str = "learned",
+                 table_rows: int = 0, tensor_names: Optional[Dict[str, str]] = None):
         """``scores="sigmoid"``: every router output's score is its own sigmoid.  ``groups`` > 1: the outputs
         form so many equal runs of neighbours, a run's score is the sum of its ``group_top`` largest choice
         scores (score + correction), and only outputs of the ``keep_groups`` best runs can be chosen.
@@ -53,7 +55,8 @@ class RoutedExperts(FeedForward):
         (u + 1)``, ``g = min(gate, limit)``, ``u = clamp(up, -limit, limit)``; ``shared_limit``: the limit of the
         expert every token uses (default: ``limit``).  ``shared_gate``: that expert's result enters times
         ``sigmoid(w . x)``, one number a token, ``w`` stored as ``[1, hidden]``.
-        ``tensor_names`` maps ``router``, ``router_bias``, ``correction``, ``gate``, ``up``, ``down``,
+        ``router="table"``: experts by token id (``table``, int32 ``[table_rows, top]``).
+        ``tensor_names`` maps ``router``, ``table``, ``router_bias``, ``correction``, ``gate``, ``up``, ``down``,
         ``shared`` (a prefix) and ``shared_gate`` to names behind ``prefix``; the experts' names hold ``{e}`` for
         the expert's number."""
         super().__init__(prefix)
@@ -78,7 +81,12 @@ class RoutedExperts(FeedForward):
         if activation not in K.EXPERT_ACTIVATIONS:
             raise ValueError(f"activation {activation!r} is not one of {sorted(K.EXPERT_ACTIVATIONS)}")
         self.activation, self.has_correction, self.renormalise = activation, bool(correction), bool(renormalise)
-        names = dict(router="router", router_bias="router.b", correction="correction", gate="e{e}.gate", up="e{e}.up",
+        if router not in ("learned", "table"):
+            raise ValueError(f"{prefix}: router {router!r} is neither 'learned' nor 'table'")
+        self.by_table, self.table_rows = router == "table", int(table_rows)
+        if self.by_table and (correction or router_bias or shared_gate or identity or self.table_rows <= 0):
+            raise ValueError(f"{prefix}: a table of experts has its rows, and nothing a router's logits would need")
+        names = dict(router="router", table="table", router_bias="router.b", correction="correction", gate="e{e}.gate", up="e{e}.up",
                      down="e{e}.down", shared="shared.", shared_gate="shared.sg")
         names.update(tensor_names or {})
         self.names = {key: prefix + name for key, name in names.items()}
@@ -96,7 +104,10 @@ class RoutedExperts(FeedForward):
 
     def tensor_specs(self) -> Dict[str, TensorSpec]:
         n, W, I = self.names, self.hidden_size, self.intermediate_size
-        specs = {n["router"]: TensorSpec((self.outputs, W))}
+        if self.by_table:
+            specs = {n["table"]: TensorSpec((self.table_rows, self.top), init="distinct", role="table", bound=self.experts)}
+        else:
+            specs = {n["router"]: TensorSpec((self.outputs, W))}
         if self.has_correction:
             specs[n["correction"]] = TensorSpec((self.outputs,), init="zeros", role="vector")
         if self.has_router_bias:
@@ -114,7 +125,12 @@ class RoutedExperts(FeedForward):
 
     def load(self, tensors: Dict[str, torch.Tensor]) -> None:
         n = self.names
-        self.router = tensors[n["router"]].contiguous()             # its logits are formed in 32-bit (ops.kernels.small_product_f32)
+        self.table = None
+        if self.by_table:
+            self.table = tensors[n["table"]].contiguous()
+            if int(self.table.min()) < 0 or int(self.table.max()) >= self.experts:
+                raise ValueError(f"{n['table']}: entries must name one of {self.experts} experts")
+        self.router = None if self.by_table else tensors[n["router"]].contiguous()             # its logits are formed in 32-bit (ops.kernels.small_product_f32)
         self.correction = tensors[n["correction"]].float().contiguous() if self.has_correction else None
         self.router_bias = tensors[n["router_bias"]].float().contiguous() if self.has_router_bias else None
         if self.shared is not None:
@@ -143,32 +159,46 @@ class RoutedExperts(FeedForward):
         return self.outputs + self.top * (2 * self.intermediate_size + 2 * self.hidden_size) + self.hidden_size \
             + (self.shared.activation_elements() + self.hidden_size if self.shared is not None else 0)
 
-    def forward(self, x, ctx: MixerContext, tail=None):
+    def _sorted(self, slots: int, dev):
+        """(sorted slots, tiles' experts), still to be filled"""
+        tiles = K.moe_tiles(slots, self.experts)
+        return torch.empty(tiles * K.MOE_TILE, dtype=torch.int32, device=dev), torch.empty(tiles, dtype=torch.int32, device=dev)
+
+    def _route(self, x, idx, wgt):
+        """Fills ``idx`` and ``wgt`` from the router's logits; returns the shared expert's gate (a column, or None)."""
         T, dev = x.shape[0], x.device
         cols = self.router.shape[0]              # the router's outputs, and the shared expert's gate behind them
         product = K.small_product_f32(x, self.router, torch.empty((T, cols), dtype=torch.float32, device=dev),
                                       bias=self.router_bias)
         logits = product[:, :self.outputs]
-        idx = torch.empty((T, self.top), dtype=torch.int32, device=dev)
-        wgt = torch.empty((T, self.top), dtype=torch.float32, device=dev)
         K.moe_route(logits, self.correction, self.top, idx, wgt, self.renormalise, over_chosen=self.over_chosen,
                     scores=self.scores, groups=self.groups, keep_groups=self.keep_groups, group_top=self.group_top,
                     weight_scale=self.weight_scale, sum_eps=self.sum_eps)
+        # the shared expert's gate: one number a token, in 32-bit; its sigmoid is taken where the rows are added
+        return product[:, self.outputs] if self.shared_gate is not None else None
+
+    def forward(self, x, ctx: MixerContext, tail=None):
+        T, dev = x.shape[0], x.device
+        idx = torch.empty((T, self.top), dtype=torch.int32, device=dev)
+        wgt = torch.empty((T, self.top), dtype=torch.float32, device=dev)
+        slots, gate = T * self.top, None
+        if self.by_table:
+            sorted_slot, tile_expert = self._sorted(slots, dev)
+            K.moe_table_align(self.table, ctx.batch.token_ids, idx, wgt, self.experts, sorted_slot, tile_expert,
+                              getattr(ctx.batch, "feedback", None))
+        else:
+            gate = self._route(x, idx, wgt)
         if RoutedExperts.on_route is not None and not torch.cuda.is_current_stream_capturing():
             RoutedExperts.on_route(self, idx)
-        slots = T * self.top
         rows = torch.empty((slots, self.hidden_size), dtype=torch.float32, device=dev)
         if self.experts:
-            tiles = K.moe_tiles(slots, self.experts)
-            sorted_slot = torch.empty(tiles * K.MOE_TILE, dtype=torch.int32, device=dev)
-            tile_expert = torch.empty(tiles, dtype=torch.int32, device=dev)
-            K.moe_align(idx, self.experts, sorted_slot, tile_expert)
-            act = torch.empty((tiles * K.MOE_TILE, self.intermediate_size), dtype=x.dtype, device=dev)
+            if not self.by_table:
+                sorted_slot, tile_expert = self._sorted(slots, dev)
+                K.moe_align(idx, self.experts, sorted_slot, tile_expert)
+            act = torch.empty((sorted_slot.shape[0], self.intermediate_size), dtype=x.dtype, device=dev)
             K.moe_expert_rows(x, self.w_up, act, sorted_slot, tile_expert, self.top, activation=self.activation,
                               gated=self.gated, limit=self.limit)
             K.moe_expert_rows(act, self.w_down, rows, sorted_slot, tile_expert, self.top, slot_weight=wgt)
         out = torch.empty_like(x)
         extra = self.shared.forward(x, ctx) if self.shared is not None else None
-        # one number a token, in 32-bit; its sigmoid is taken where the rows are added
-        gate = product[:, self.outputs] if self.shared_gate is not None else None
         return K.moe_combine(x, rows, idx, wgt, self.experts, out, extra=extra, extra_gate=gate)

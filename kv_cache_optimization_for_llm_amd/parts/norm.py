@@ -12,7 +12,7 @@ import torch
 from ..config.registry import NORMS
 from ..models.spec import TensorSpec
 from ..ops import kernels as K
-from .base import Norm, PendingMix
+from .base import Norm, PendingMix, PendingNorm
 
 
 @NORMS.register("rmsnorm")
@@ -70,7 +70,8 @@ class LayerNorm(Norm):
         ``bias_name``: the norm has a bias, ``... * w + b``.  ``streams``: the rows it reads hold so
         many copies of the stream side by side (32-bit), and what is normed is their sum; a pending
         :class:`~.base.PendingMix` enters the copies first.  A norm with a bias or over several copies
-        reads a 32-bit stream (``ops.kernels.hyper_step``)."""
+        reads a 32-bit stream (``ops.kernels.hyper_step``).  A pending :class:`~.base.PendingNorm` enters a
+        32-bit stream of one copy under the branch's own norm first (``ops.kernels.sandwich_step``)."""
         super().__init__(prefix)
         self.width, self.eps = int(width), float(eps)
         self.weight_name = prefix + weight_name
@@ -118,8 +119,17 @@ class LayerNorm(Norm):
         # the products behind a norm take the weights' type; a 32-bit stream of a bf16 model is normalised into bf16
         return torch.empty((rows, self.width), dtype=self.out_dtype or self.weight.dtype, device=x.device)
 
+    def pass_args(self) -> tuple:
+        """``(weight, bias, eps, center)`` as a kernel that norms inside its own pass takes them."""
+        return self.weight, self.bias, self.eps, self.center
+
     def forward(self, x, out=None, delta=None, row_idx=None):
         out = self._out(x, row_idx) if out is None else out
+        if isinstance(delta, PendingNorm):
+            if self.streams > 1:
+                raise TypeError(f"{self.prefix}: a branch output under a norm enters a stream of one copy")
+            return K.sandwich_step(x, y=delta.y, post=delta.norm.pass_args() if delta.norm is not None else None,
+                                   addend=delta.addend, pre=self.pass_args(), out=out, row_idx=row_idx)
         if self.bias is not None or self.streams > 1 or isinstance(delta, PendingMix):
             if delta is not None and not isinstance(delta, PendingMix):
                 raise TypeError(f"{self.prefix}: this norm takes a pending output with its way into the stream's copies")

@@ -2,7 +2,7 @@
 configuration and a seed.
 
 Matrices are N(0, 0.02), norm weights 1 + U(-0.1, 0.1), matrices that mix copies of the stream the identity
-+ U(-0.1, 0.1).  With a ``gain`` a matrix ``[out, in]``
++ U(-0.1, 0.1), tables of choices rows of different integers.  With a ``gain`` a matrix ``[out, in]``
 is N(0, gain / sqrt(in)) instead: its products of unit-size inputs are of size ``gain`` at any
 width, so attention scores spread and a tied model's best next token is not its input token -
 what tests of generation need from random weights.  Each tensor's generator is seeded from
@@ -31,11 +31,20 @@ def _generator(seed: int, name: str) -> torch.Generator:
     return g
 
 
+def _random_table(spec: TensorSpec, g: torch.Generator, device) -> torch.Tensor:
+    """Integers: zeros, or (``"distinct"``) every row a random choice of different integers below ``bound``."""
+    if spec.init != "distinct":
+        return torch.zeros(spec.shape, dtype=torch.int32, device=device)
+    rows, k = spec.shape
+    order = torch.rand((rows, spec.bound), generator=g, device=device).argsort(dim=-1)
+    return order[:, :k].to(torch.int32).contiguous()
+
+
 def random_tensor(name: str, spec: TensorSpec, seed: int, dtype: torch.dtype,
                   gain: Optional[float] = None) -> torch.Tensor:
     g = _generator(seed, name)
     if spec.role == "table":
-        return torch.zeros(spec.shape, dtype=torch.int32)
+        return _random_table(spec, g, "cpu")
     if spec.init == "normal":
         std = 0.02 if gain is None or len(spec.shape) != 2 else float(gain) / float(spec.shape[1]) ** 0.5
         t = torch.randn(spec.shape, generator=g, dtype=torch.float32) * std
@@ -64,7 +73,7 @@ def random_tensors_on_device(specs: Mapping[str, TensorSpec], seed: int, dtype: 
     for i, (name, spec) in enumerate(specs.items()):
         g.manual_seed((int(seed) * 1000003 + i) & ((1 << 63) - 1))
         if spec.role == "table":
-            out[name] = torch.zeros(spec.shape, dtype=torch.int32, device=device)
+            out[name] = _random_table(spec, g, device)
         elif spec.init == "normal":
             t = torch.empty(spec.shape, dtype=torch.float32, device=device).normal_(0.0, 0.02, generator=g)
             out[name] = t.to(dtype)
