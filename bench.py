@@ -15,7 +15,7 @@ tokens, each with its step time, bytes and fraction of the HBM peak, and the ser
 (``kclass_...``; ``--no-kernel-classes`` leaves them out) and, for the serving runs, pages reused,
 preemptions and fragmentation failures.
 
-    python bench.py --design gadopel|radilix|lomodra|bonusun [--layers 8]
+    python bench.py --design gadopel|radilix|lomodra|bonusun|bilolorn [--layers 8]
 
 is another measurement with a JSON line of its own (the default run above is untouched): prefill
 and decode throughput of a Gadopel model at layer sizes of a served model (random weights), beside
@@ -73,17 +73,19 @@ def prefill_flops(cfg, T):
 # --design gadopel: layers of width 2,048 with a feed-forward of 8,192.  Latent layers with 16
 # heads of 128 + 64 query/key elements over rows of 512 + 64, windowed layers with 32 heads of 64
 # over 8 kv heads and a window of 1,024 that keeps 64 first positions, in turn; the Llama beside it
-# has 32 heads of 64 over 8 kv heads in every layer.
-def gadopel_config(layers: int, vocab: int) -> dict:
-    latent = {"type": "latent_attention", "mlp": {"kind": "dense", "ff": 8192},
-              "mixer": {"heads": 16, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 512, "scale": 192 ** -0.5,
-                        "rot": {"base": 10000.0, "dims": 64}}}
-    windowed = {"type": "attention", "mlp": {"kind": "dense", "ff": 8192},
-                "mixer": {"heads": 32, "kv_heads": 8, "dim": 64, "vdim": 64, "scale": 1.0,
+# has 32 heads of 64 over 8 kv heads in every layer.  At another width W head counts and feed-forward scale
+# with it (W / 128 latent heads over rows of min(512, W / 4) + 64, W / 64 windowed heads over W / 256).
+def gadopel_config(layers: int, vocab: int, width: int = 2048) -> dict:
+    W = width
+    latent = {"type": "latent_attention", "mlp": {"kind": "dense", "ff": 4 * W},
+              "mixer": {"heads": W // 128, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": min(512, W // 4),
+                        "scale": 192 ** -0.5, "rot": {"base": 10000.0, "dims": 64}}}
+    windowed = {"type": "attention", "mlp": {"kind": "dense", "ff": 4 * W},
+                "mixer": {"heads": W // 64, "kv_heads": W // 256, "dim": 64, "vdim": 64, "scale": 1.0,
                           "mask": {"size": 1024, "keep_first": 64},
                           "rot": {"base": 500000.0, "dims": 64,
                                   "scaling": {"factor": 16.0, "original": 4096, "fast": 16.0, "slow": 2.0}}}}
-    return {"architecture": "Gadopel", "vocab": vocab, "width": 2048, "norm": {"eps": 1e-6},
+    return {"architecture": "Gadopel", "vocab": vocab, "width": W, "norm": {"eps": 1e-6},
             "layers": [latent if i % 2 == 0 else windowed for i in range(layers)], "max_positions": 8192}
 
 
@@ -157,6 +159,22 @@ def bonusun_config(layers: int, vocab: int, width: int = 2048) -> dict:
             "layers": [kinds[i % 4] for i in range(layers)], "max_positions": 8192}
 
 
+# --design bilolorn: layers of width W of latent attention - W / 128 heads of 128 + 64 query/key elements over
+# rows of min(512, W / 4) + 64, queries through a latent of 3 W / 8, a sink a head, a gate an element - between
+# layer norms on both sides.  The first layer has a dense feed-forward of 4 W, the others 16 gated experts of
+# width 3 W / 8 picked by token id, 4 a token, and one more expert of that width that every token uses.
+# Beside it run the closest designs, Gadopel (latent attention in every second layer) and Bonusun (layer norms
+# with biases, experts of the same sizes), and the Llama model, all at the same width.
+def bilolorn_config(layers: int, vocab: int, width: int = 2048) -> dict:
+    W = width
+    mixer = {"heads": W // 128, "dim": 128, "rot_dim": 64, "vdim": 128, "q_rank": 3 * W // 8, "kv_rank": min(512, W // 4),
+             "scale": 192 ** -0.5, "rot": {"base": 10000.0, "dims": 64}}
+    moe = {"kind": "moe", "expert": {"ff": 3 * W // 8}, "router": {"experts": 16, "top": 4}, "shared": {"ff": 3 * W // 8}}
+    return {"architecture": "Bilolorn", "vocab": vocab, "width": W, "norm": {"eps": 1e-6}, "embedding": {"scale": 4.0},
+            "layers": [{"type": "latent_attention", "mixer": mixer, "mlp": moe if i else {"kind": "dense", "ff": 4 * W}}
+                       for i in range(layers)], "max_positions": 8192}
+
+
 def design_comparison(args) -> int:
     import torch
     from kv_cache_optimization_for_llm_amd.engine.batch import StepEntry
@@ -167,8 +185,8 @@ def design_comparison(args) -> int:
     llama = dict(CONFIG_1B, num_hidden_layers=layers, vocab_size=vocab, tie_word_embeddings=False)
     design, width = args.design, args.width
     if width != 2048:
-        if design not in ("radilix", "lomodra", "bonusun") or width % 512 or not 512 <= width <= 8192:
-            print("--width: a multiple of 512 from 512 to 8192, for --design radilix, lomodra or bonusun")
+        if width % 512 or not 512 <= width <= 8192:
+            print("--width: a multiple of 512 from 512 to 8192")
             return 2
         llama.update(hidden_size=width, intermediate_size=4 * width, num_attention_heads=width // 64,
                      num_key_value_heads=width // 256)
@@ -176,10 +194,13 @@ def design_comparison(args) -> int:
         configs = {design: lomodra_config(layers, vocab, width), "radilix": radilix_config(layers, vocab, width), "llama": llama}
     elif design == "bonusun":
         configs = {design: bonusun_config(layers, vocab, width), "radilix": radilix_config(layers, vocab, width), "llama": llama}
+    elif design == "bilolorn":
+        configs = {design: bilolorn_config(layers, vocab, width), "gadopel": gadopel_config(layers, vocab, width),
+                   "bonusun": bonusun_config(layers, vocab, width), "llama": llama}
     elif design == "radilix":
         configs = {design: radilix_config(layers, vocab, width), "llama": llama}
     else:
-        configs = {design: gadopel_config(layers, vocab), "llama": llama}
+        configs = {design: gadopel_config(layers, vocab, width), "llama": llama}
     shapes = [(8, 4096), (32, 2048)]            # (requests, context) of the decode runs
     gen = torch.Generator().manual_seed(0)
     out = {}
@@ -216,7 +237,8 @@ def design_comparison(args) -> int:
             for rid in ids:
                 for lo in range(0, len(base), 4096):
                     engine.step([StepEntry(rid, base[lo:lo + 4096], [])])
-            step = [StepEntry(rid, [7], [0]) for rid in ids]
+            # (a token id of its own per request: experts picked by token id spread like routed ones)
+            step = [StepEntry(rid, [(7 + 911 * i) % vocab], [0]) for i, rid in enumerate(ids)]
             for _ in range(args.warmup + 2):
                 engine.step(step)
             torch.cuda.synchronize()
@@ -263,10 +285,10 @@ def design_comparison(args) -> int:
 
 def main():
     ap = argparse.ArgumentParser()
-    ap.add_argument("--design", choices=["gadopel", "radilix", "lomodra", "bonusun"], default=None,
+    ap.add_argument("--design", choices=["gadopel", "radilix", "lomodra", "bonusun", "bilolorn"], default=None,
                     help="another measurement (its own JSON line): a model of this design at the layer sizes of a "
                          "served model beside a Llama model of equal size; the default run is left as it is")
-    ap.add_argument("--width", type=int, default=2048, help="--design radilix, lomodra or bonusun: the models' width (head counts and "
+    ap.add_argument("--width", type=int, default=2048, help="--design: the models' width (head counts and "
                     "feed-forward sizes scale with it)")
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=128)

@@ -13,6 +13,9 @@ Notation.  ``x`` [T, W] is the residual stream of one sequence, positions 0..T-1
 * looping:  layers ``start..stop-1`` run ``times`` times; in front of every pass but the first
             ``x <- x + x0``
 * head:     ``logits = W_head LN_final(x)``
+
+``r`` is what is done to every value that an engine with 16-bit products would store in 16 bits (the
+identity by default; a rounding, to see what rounding alone does to a row of logits).
 """
 from __future__ import annotations
 
@@ -57,48 +60,52 @@ def causal_softmax(scores: torch.Tensor, sink: torch.Tensor) -> torch.Tensor:
     return e / (e.sum(dim=-1, keepdim=True) + torch.exp(sink[:, None, None] - m))
 
 
-def latent_attention(h: torch.Tensor, w: Mapping[str, torch.Tensor], p: str, mc: Mapping, eps: float) -> torch.Tensor:
+def same(t: torch.Tensor) -> torch.Tensor:
+    return t
+
+
+def latent_attention(h: torch.Tensor, w: Mapping[str, torch.Tensor], p: str, mc: Mapping, eps: float, r_=same) -> torch.Tensor:
     T = h.shape[0]
     H, d, r, dv, rank, base = mc["heads"], mc["dim"], mc["rot_dim"], mc["vdim"], mc["kv_rank"], mc["rot"]["base"]
-    c_q = rms_norm(h @ w[p + "dq"].T, w[p + "dq.norm"], eps)
-    q = (c_q @ w[p + "uq"].T).view(T, H, d + r)
-    q = torch.cat([q[..., :d], rotate_pairs(q[..., d:], base)], dim=-1)
-    down = h @ w[p + "dkv"].T
-    c = rms_norm(down[:, :rank], w[p + "dkv.norm"], eps)
-    k_rot = rotate_pairs(down[:, rank:], base)                                   # one for all heads
+    c_q = r_(rms_norm(r_(h @ w[p + "dq"].T), w[p + "dq.norm"], eps))
+    q = r_(c_q @ w[p + "uq"].T).view(T, H, d + r)
+    q = torch.cat([q[..., :d], r_(rotate_pairs(q[..., d:], base))], dim=-1)
+    down = r_(h @ w[p + "dkv"].T)
+    c = r_(rms_norm(down[:, :rank], w[p + "dkv.norm"], eps))
+    k_rot = r_(rotate_pairs(down[:, rank:], base))                                   # one for all heads
     k = torch.cat([(c @ w[p + "uk"].T).view(T, H, d), k_rot[:, None, :].expand(T, H, r)], dim=-1)
     v = (c @ w[p + "uv"].T).view(T, H, dv)
     out = torch.empty(T, H, dv, dtype=h.dtype)
     for a in range(H):
         s = (q[:, a] @ k[:, a].T * mc["scale"])[None]
         out[:, a] = causal_softmax(s, w[p + "sink"][a:a + 1])[0] @ v[:, a]
-    gate = torch.sigmoid(h @ w[p + "g"].T)                                       # [T, H dv], one number an element
-    return (out.reshape(T, H * dv) * gate) @ w[p + "o"].T
+    gate = torch.sigmoid(r_(h @ w[p + "g"].T))                                   # [T, H dv], one number an element
+    return r_(r_(out.reshape(T, H * dv) * gate) @ w[p + "o"].T)
 
 
-def squared_relu_mlp(h: torch.Tensor, w: Mapping[str, torch.Tensor], p: str) -> torch.Tensor:
-    return torch.clamp(h @ w[p + "up"].T, min=0.0) ** 2 @ w[p + "down"].T
+def squared_relu_mlp(h: torch.Tensor, w: Mapping[str, torch.Tensor], p: str, r_=same) -> torch.Tensor:
+    return r_(r_(torch.clamp(r_(h @ w[p + "up"].T), min=0.0) ** 2) @ w[p + "down"].T)
 
 
-def silu_glu(h: torch.Tensor, w: Mapping[str, torch.Tensor], p: str) -> torch.Tensor:
+def silu_glu(h: torch.Tensor, w: Mapping[str, torch.Tensor], p: str, r_=same) -> torch.Tensor:
     g = h @ w[p + "gate"].T
-    return (g * torch.sigmoid(g) * (h @ w[p + "up"].T)) @ w[p + "down"].T
+    return r_(g * torch.sigmoid(g) * (h @ w[p + "up"].T)) @ w[p + "down"].T
 
 
-def table_experts(h: torch.Tensor, tokens: torch.Tensor, w: Mapping[str, torch.Tensor], p: str, mlp: Mapping) -> torch.Tensor:
+def table_experts(h: torch.Tensor, tokens: torch.Tensor, w: Mapping[str, torch.Tensor], p: str, mlp: Mapping, r_=same) -> torch.Tensor:
     """Every token id's row of the table names its experts; their outputs are averaged."""
     top = mlp["router"]["top"]
     out = torch.zeros_like(h)
     for t in range(h.shape[0]):
         for e in w[p + "table"][int(tokens[t])].tolist():
-            out[t] += silu_glu(h[t:t + 1], w, f"{p}e{int(e)}.")[0] / top
+            out[t] += silu_glu(h[t:t + 1], w, f"{p}e{int(e)}.", r_)[0] / top
     if mlp.get("shared"):
-        out = out + silu_glu(h, w, p + "shared.")
-    return out
+        out = out + r_(silu_glu(h, w, p + "shared.", r_))
+    return r_(out)
 
 
-def feed_forward(h, tokens, w, p: str, mlp: Mapping) -> torch.Tensor:
-    return squared_relu_mlp(h, w, p) if mlp["kind"] == "dense" else table_experts(h, tokens, w, p, mlp)
+def feed_forward(h, tokens, w, p: str, mlp: Mapping, r_=same) -> torch.Tensor:
+    return squared_relu_mlp(h, w, p, r_) if mlp["kind"] == "dense" else table_experts(h, tokens, w, p, mlp, r_)
 
 
 def run_order(cfg: Mapping) -> List[tuple]:
@@ -115,7 +122,7 @@ def run_order(cfg: Mapping) -> List[tuple]:
 
 
 def forward(cfg: Mapping, weights: Mapping[str, torch.Tensor], tokens, dtype=torch.float64,
-            residuals: Optional[list] = None) -> torch.Tensor:
+            residuals: Optional[list] = None, r_=same) -> torch.Tensor:
     """Logits [T, vocab] of one whole sequence; ``residuals`` collects the stream after every layer run."""
     w: Dict[str, torch.Tensor] = {k: (v.to(dtype) if v.is_floating_point() else v) for k, v in weights.items()}
     eps = cfg["norm"]["eps"]
@@ -129,9 +136,9 @@ def forward(cfg: Mapping, weights: Mapping[str, torch.Tensor], tokens, dtype=tor
 
         def norm(name, z):
             return layer_norm(z, w[p + name], w[p + name + ".b"], eps)
-        x = x + norm("norm1b", latent_attention(norm("norm1", x), w, p + "mix.", layer["mixer"], eps))
+        x = x + norm("norm1b", latent_attention(r_(norm("norm1", x)), w, p + "mix.", layer["mixer"], eps, r_))
         if layer.get("mlp"):
-            x = x + norm("norm2b", feed_forward(norm("norm2", x), ids, w, p + "mlp.", layer["mlp"]))
+            x = x + norm("norm2b", feed_forward(r_(norm("norm2", x)), ids, w, p + "mlp.", layer["mlp"], r_))
         if residuals is not None:
             residuals.append(x)
-    return layer_norm(x, w["final.norm"], w["final.norm.b"], eps) @ w["head"].T
+    return r_(layer_norm(x, w["final.norm"], w["final.norm.b"], eps)) @ w["head"].T
