@@ -402,9 +402,10 @@ def paged_attention(qkv: torch.Tensor, out: torch.Tensor, kv, batch, num_q_heads
             tiles = 2 if (head_dim <= 128 and value_dim <= 128
                           and batch.num_tokens * group * num_kv_heads >= _ROWS_TWO_TILES) else 1
             item_entry, item_row0, _ = batch.attention_items(group, tiles, "all")
-            # (with a window most ranges of a long context hold no visible key: their wavefronts end at once)
+            # (workgroups of one wavefront: four a compute unit;
+            # with a window most ranges of a long context hold no visible key: their wavefronts end at once)
             ranges, per = choose_ranges(item_entry.shape[0] * num_kv_heads, batch.max_context,
-                                        window + keep_first if window > 0 else chunk)
+                                        window + keep_first if window > 0 else chunk, workgroups=1024)
             return K.attention_rows_mfma(qkv, stride, out, kv.k_cache, kv.v_cache, kv.block_table, item_entry,
                                          item_row0, batch.entry_seat, batch.entry_q_start, batch.entry_start_pos,
                                          num_q_heads, num_kv_heads, head_dim, scale, window, keep_first, sinks,

@@ -50,11 +50,11 @@ _HIP_SIGNATURES = {
     "kva_act_mul": [P, P, I, I, I, F, I, P],
     "kva_head_gate": [P, P, I, I, I, I, I, P],
     "kva_qk_encode_cache": [P, I, I, I, P, P, P, P, P, P, I, I, I, I, I, I, I, F, I, I, P, P, P, I, P],
-    "kva_latent_encode_cache": [P, I, I, P, P, P, I, P, P, I, P, I, F, P, P, P, P, I, I, I, I, I, I, I, P],
+    "kva_latent_encode_cache": [P, I, I, P, P, P, I, P, P, I, F, P, P, P, P, I, I, I, I, I, I, I, P],
     "kva_latent_attention_mfma_supported": [I, I, I],
     "kva_attention_rows_mfma_supported": [I, I, I],
     "kva_attention_rows_mfma": [P, P, P, P, I, P, P, P, I, P, P, P, P, P, I, I, I, I, I, I, I, F, I, I, I, P, I, I, I, P],
-    "kva_latent_attention_mfma": [P, P, P, P, P, P, P, I, P, P, P, P, P, I, I, I, I, I, I, F, I, I, P, I, I, P],
+    "kva_latent_attention_mfma": [P, P, P, P, P, P, I, P, P, P, P, P, I, I, I, I, I, I, F, I, I, P, I, I, P],
     "kva_heads_matmul": [P, I, I, P, I, I, P, I, I, I, I, P, I, I, I, P, I, I, P, I, I, P, P, P, I, I, I, P],
     "kva_heads_matmul_mfma_supported": [I, I, I],
     "kva_heads_matmul_mfma": [P, I, I, P, I, I, P, I, I, I, I, P, I, I, I, P, I, I, P, I, I, P, P, P, I, I, P],
@@ -105,6 +105,7 @@ _HIP_SIGNATURES = {
     "kva_table_gate": [P, P, I, P, I, I, I, I, P, P, I, I, I, P],
     "kva_bias_act": [P, P, I, P, I, I, I, P],
     "kva_hyper_step": [P, I, P, I, P, P, F, P, P, P, I, F, P, I, P, I, I, P],
+    "kva_latent_attention_merge": [P, P, P, P, I, I, I, I, P],
     "kva_sandwich_step": [P, P, I, P, P, I, I, F, P, P, P, I, I, F, P, I, P, I, I, P],
     "kva_hyper_fill": [P, P, I, I, I, I, P],
     "kva_block_gates": [P, P, P, I, I, I, P, P, I, P, P, P, P],

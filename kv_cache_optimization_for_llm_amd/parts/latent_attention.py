@@ -36,14 +36,9 @@ from .base import CacheArray, KVCacheSpec, Mixer, MixerContext, NormedRows
 from .linear import Linear
 
 
-def latent_cache_spec(rank: int, rot_dim: int, kind: str = "full", window: int = 0, keep_first: int = 0,
-                      transposed: bool = False) -> KVCacheSpec:
-    """One row ``[latent (rank) ; rotated key part (rot_dim)]`` per token, pages ``[page_size, rank +
-    rot_dim]``; with ``transposed`` the latent a second time in pages ``[rank, page_size]``, the
-    layout in which the matrix-core kernel reads it as the values' operand."""
+def latent_cache_spec(rank: int, rot_dim: int, kind: str = "full", window: int = 0, keep_first: int = 0) -> KVCacheSpec:
+    """One row ``[latent (rank) ; rotated key part (rot_dim)]`` per token, pages ``[page_size, rank + rot_dim]``."""
     arrays = (CacheArray("latent", (int(rank) + int(rot_dim),), token_axis=0),)
-    if transposed:
-        arrays += (CacheArray(lat_ops.TRANSPOSED, (int(rank),), token_axis=1),)
     return KVCacheSpec(arrays, kind, int(window), int(keep_first) if kind == "window" else 0)
 
 
@@ -124,12 +119,8 @@ class LatentAttention(Mixer):
         self.sinks = tensors[n["sink"]].to(torch.float32).contiguous() if self.has_sink else None
 
     def kv_cache_spec(self) -> KVCacheSpec:
-        # a bf16 model at sizes the matrix-core kernel has an instance for keeps the transposed copy
-        # it reads (asked after load(): the weights' type is the compute type)
-        fast = self.proj is not None and self.proj.weight.dtype == torch.bfloat16 and self.proj.weight.is_cuda \
-            and lat_ops.mfma_supported(self.rank, self.key_dim)
         return latent_cache_spec(self.rank, self.rot_dim, kind="window" if self.window > 0 else "full",
-                                 window=self.window, keep_first=self.keep_first, transposed=fast)
+                                 window=self.window, keep_first=self.keep_first)
 
     def activation_elements(self) -> int:
         H = self.num_heads
@@ -152,8 +143,7 @@ class LatentAttention(Mixer):
         K.latent_encode_cache(y, self.kv_off, None if self.q_rank else q_lat, kv.arrays["latent"] if write else None,
                               self.norm_weight, self.norm_eps, cos, sin, batch.positions,
                               kv.slot_mapping if write else None, H, self.head_dim, self.rank, interleaved=interleaved,
-                              cache_t=kv.arrays.get(lat_ops.TRANSPOSED) if write else None, c_q=c_q,
-                              q_norm_weight=self.q_norm_weight)
+                              c_q=c_q, q_norm_weight=self.q_norm_weight)
         q = (self.q_up(c_q) if self.q_rank else y[:, :self.kv_off]).view(T, H, self.head_dim + self.rot_dim)
         # queries from a latent exist only now: their rotated parts are turned in the expansion's launch
         rotate = (q[:, :, self.head_dim:], q_lat[:, :, self.rank:], cos, sin, batch.positions, interleaved) if self.q_rank else None

@@ -144,18 +144,15 @@ def test_query_latent_norm_beside_the_cache_write(q_rank, rank, rot, dtype, gpu)
     cos, sin = RotaryEncoding(head_dim=rot, max_positions=64, theta=90.0, frequencies="plain_f64", pairing="interleaved").tables(gpu)
     slots = torch.from_numpy(np.random.default_rng(1).permutation(48)[:T].astype(np.int32))
     cache = torch.zeros((3, page, rank + rot), dtype=DT[dtype], device=gpu)
-    cache_t = torch.zeros((3, rank, page), dtype=DT[dtype], device=gpu)
     c_q = torch.empty((T, q_rank), dtype=DT[dtype], device=gpu)
     K.latent_encode_cache(y.to(gpu), q_rank, None, cache, kw.to(gpu), eps, cos, sin, torch.arange(T, dtype=torch.int32, device=gpu),
-                          slots.to(gpu), 4, 12, rank, interleaved=True, cache_t=cache_t, c_q=c_q, q_norm_weight=qw.to(gpu))
+                          slots.to(gpu), 4, 12, rank, interleaved=True, c_q=c_q, q_norm_weight=qw.to(gpu))
     src = y.double()
     close(c_q, plain.rms_norm(src[:, :q_rank], qw.double(), eps), TOL[dtype], "query latent")
     got = cache.view(48, rank + rot)[slots.long().to(gpu)]
     c = plain.rms_norm(src[:, q_rank:q_rank + rank], kw.double(), eps)
     close(got[:, :rank], c, TOL[dtype], "latent")
     close(got[:, rank:], plain.rotate_pairs(src[:, q_rank + rank:q_rank + rank + rot], 90.0), TOL[dtype], "rotated part")
-    sl = slots.long()
-    assert torch.equal(cache_t.cpu()[sl // page, :, sl % page], got[:, :rank].cpu())
     # without a cache (a layer call that only reads) the query latent is still made
     again = torch.empty_like(c_q)
     K.latent_encode_cache(y.to(gpu), q_rank, None, None, kw.to(gpu), eps, cos, sin, torch.arange(T, dtype=torch.int32, device=gpu),
@@ -243,17 +240,73 @@ def test_a_far_key_that_stands_out_and_a_sink_over_low_rank_rows(heads, rank, ro
                 K.latent_attention_rowwise(q.to(gpu), out, cache, table.to(gpu), seat, p, scale, 0, 0, sinks.to(gpu))
                 close(out, want, TOL[dtype], f"key {key}")
                 continue
-            cache_t = cache[:, :, :rank].transpose(1, 2).contiguous()
-            items = (n * heads + 15) // 16
-            entry = torch.zeros(items, dtype=torch.int32, device=gpu)
-            row0 = (16 * torch.arange(items)).to(torch.int32).to(gpu)
             i32 = dict(dtype=torch.int32, device=gpu)
-            for splits, per in ((1, 0), (2, 352), (6, 128), (22, 32)):
-                out.fill_(float("nan"))
-                K.latent_attention_mfma(q.to(gpu), out, cache, cache_t, table.to(gpu), entry, row0, torch.tensor([1], **i32),
-                                        torch.tensor([0, n], **i32), torch.tensor([q_pos[0]], **i32), scale, 0, 0, sinks.to(gpu),
-                                        splits, per)
-                close(out, want, TOL[dtype], f"key {key}, {splits} ranges")
+            for item_rows in (16, 64):
+                items = (n * heads + item_rows - 1) // item_rows
+                entry = torch.zeros(items, dtype=torch.int32, device=gpu)
+                row0 = (item_rows * torch.arange(items)).to(torch.int32).to(gpu)
+                for splits, per in ((1, 0), (2, 352), (6, 128), (22, 32)):
+                    out.fill_(float("nan"))
+                    K.latent_attention_mfma(q.to(gpu), out, cache, table.to(gpu), entry, row0, torch.tensor([1], **i32),
+                                            torch.tensor([0, n], **i32), torch.tensor([q_pos[0]], **i32), scale, 0, 0, sinks.to(gpu),
+                                            splits, per, item_rows)
+                    close(out, want, TOL[dtype], f"key {key}, items of {item_rows} rows, {splits} ranges")
+
+
+@pytest.mark.parametrize("heads, rank, rot, page", [(5, 64, 32, 16), (16, 128, 32, 32), (4, 512, 64, 16), (3, 96, 32, 48), (33, 192, 32, 16),
+                                                    (8, 256, 64, 16), (6, 384, 64, 16), (7, 160, 32, 64)])
+@pytest.mark.parametrize("window, keep_first", [(0, 0), (50, 0), (37, 5), (1, 3)])
+def test_rows_of_several_entries_in_items_of_both_sizes(heads, rank, rot, page, window, keep_first, gpu):
+    """Prompt portions and decoded tokens of several requests in one call, pages that hold garbage (NaN) behind
+    every request's newest token and where a window has let pages go, keys in one range and in several."""
+    key_dim, scale = rank + rot, 0.15
+    starts, lens = [0, 75, 130, 9], [40, 1, 23, 2]
+    seats, blocks = [2, 0, 3, 1], 12
+    pool = sum((s + n + page - 1) // page for s, n in zip(starts, lens)) + 2
+    perm = torch.from_numpy(np.random.default_rng(heads).permutation(pool).astype(np.int32))
+    cache = torch.full((pool, page, key_dim), float("nan"), dtype=torch.bfloat16)
+    table = torch.full((4, blocks), -1, dtype=torch.int32)
+    rows, at = [], 0
+    for s, n, seat in zip(starts, lens, seats):
+        r = rnd((s + n, key_dim), 10 + s, torch.bfloat16)
+        rows.append(r)
+        need = (s + n + page - 1) // page
+        for b in range(need):
+            # a page that lies wholly behind the window of the entry's first token, and past the kept positions, is gone
+            if window > 0 and (b + 1) * page <= s - window + 1 and b * page >= keep_first:
+                continue
+            table[seat, b] = perm[at + b]
+            part = r[b * page:(b + 1) * page]
+            cache[perm[at + b], :part.shape[0]] = part
+        at += need
+    q_start = np.concatenate([[0], np.cumsum(lens)]).astype(np.int32)
+    T = int(q_start[-1])
+    q = rnd((T, heads, key_dim), 3, torch.bfloat16, 0.4)
+    sinks = torch.linspace(-1, 2, heads)
+    want = torch.empty((T, heads, rank), dtype=torch.float64)
+    for e, (s, n) in enumerate(zip(starts, lens)):
+        k = rows[e].double()
+        sc = torch.einsum("ihk,jk->hij", q[q_start[e]:q_start[e + 1]].double(), k) * scale
+        i, j = torch.arange(s, s + n)[:, None], torch.arange(s + n)[None, :]
+        seen = (j <= i) & ((i - j < window) | (j < keep_first) if window > 0 else torch.ones_like(j <= i))
+        sc = sc.masked_fill(~seen[None], float("-inf"))
+        p = torch.softmax(torch.cat([sc, sinks.double()[:, None, None].expand(heads, n, 1)], -1), -1)[..., :-1]
+        want[q_start[e]:q_start[e + 1]] = torch.einsum("hij,jk->ihk", p, k[:, :rank])
+    dev, i32 = cache.to(gpu), dict(dtype=torch.int32, device=gpu)
+
+    def items(rows_per_item, entries):
+        ent = [e for e in entries for _ in range(0, lens[e] * heads, rows_per_item)]
+        row0 = [r for e in entries for r in range(0, lens[e] * heads, rows_per_item)]
+        return torch.tensor(ent, **i32), torch.tensor(row0, **i32), rows_per_item
+    few = [e for e in range(4) if lens[e] <= 2]
+    many = [e for e in range(4) if e not in few]
+    for first, more in ((items(16, range(4)), ()), (items(64, range(4)), ()), (items(64, many), (items(16, few),))):
+        for splits, per in ((1, 0), (3, 64), (5, 32)):            # (the longest request has 153 keys)
+            out = torch.full((T, heads, rank), float("nan"), dtype=torch.bfloat16, device=gpu)
+            K.latent_attention_mfma(q.to(gpu), out, dev, table.to(gpu), first[0], first[1], torch.tensor(seats, **i32),
+                                    torch.from_numpy(q_start).to(gpu), torch.tensor(starts, **i32), scale, window, keep_first,
+                                    sinks.to(gpu), splits, per, first[2], more)
+            close(out, want, 2e-2, f"items of {first[2]} rows, {splits} ranges of {per}")
 
 
 # ---------------------------------------------------------------- feed-forwards
