@@ -14,8 +14,8 @@
 //    x gathered by slot / top, activation applied (a gated expert: act(gate) * up, its gate and up rows
 //    interleaved in one matrix), written at the sorted position.  Mode 1 ("down"):
 //    rows at the sorted position, times the slot's routing weight, written at the slot (fp32).
-//    bf16 with K % 32 == 0 runs on the matrix cores, everything else (fp32 too) on a plain tiled
-//    kernel that adds k ascending.
+//    bf16 with K % 32 == 0 runs on the matrix cores (with many rows an expert through LDS, in groups of
+//    tiles), everything else (fp32 too) on a plain tiled kernel that adds k ascending.
 //  * kva_moe_combine: out[t] = sum over the token's choices of the slot's row, or, for a router
 //    output past the real experts (an identity expert), weight * x[t].
 //
@@ -189,71 +189,114 @@ struct MoeTable {
     float *wgt;
 };
 
+// `group` tiles form a group that belongs to one expert (its last tiles may be padding): what a kernel that
+// takes several tiles at once walks over.  One workgroup; a thread keeps up to MOE_SLOTS_IN_REGISTERS slots
+// and their places in their experts' runs in registers (all its loads in flight at once, one pass of
+// counters); more slots than that are read and counted twice.
+#define MOE_SLOTS_IN_REGISTERS 16
+__device__ inline int moe_slot_expert(int *idx, int s, const MoeTable &tab) {
+    if (!tab.table) return idx[s];
+    int id = tab.ids[s / tab.top];
+    if (id < 0) id = tab.feedback[-1 - id];
+    id = id < 0 ? 0 : (id >= tab.rows ? tab.rows - 1 : id);
+    return tab.table[(size_t)id * tab.top + s % tab.top];
+}
+
 __global__ void __launch_bounds__(1024)
 moe_align_kernel(int *__restrict__ sorted_slot, int *__restrict__ tile_expert, int *idx, int slots, int experts, int capacity,
-                 int max_tiles, MoeTable tab) {
+                 int max_tiles, int group, MoeTable tab) {
     __shared__ int count[MOE_MAX_EXPERTS], start[MOE_MAX_EXPERTS];
-    if (tab.table) {
-        // (a slot is written and later read by the same thread)
-        for (int s = threadIdx.x; s < slots; s += blockDim.x) {
-            int id = tab.ids[s / tab.top];
-            if (id < 0) id = tab.feedback[-1 - id];
-            id = id < 0 ? 0 : (id >= tab.rows ? tab.rows - 1 : id);
-            idx[s] = tab.table[(size_t)id * tab.top + s % tab.top];
-            tab.wgt[s] = tab.weight;
+    const bool in_registers = slots <= (int)blockDim.x * MOE_SLOTS_IN_REGISTERS;
+    int ex[MOE_SLOTS_IN_REGISTERS], at[MOE_SLOTS_IN_REGISTERS];
+#pragma unroll
+    for (int j = 0; j < MOE_SLOTS_IN_REGISTERS; ++j) ex[j] = -1;
+    if (in_registers) {
+#pragma unroll
+        for (int j = 0; j < MOE_SLOTS_IN_REGISTERS; ++j) {
+            const int s = threadIdx.x + j * blockDim.x;
+            if (j * (int)blockDim.x >= slots) break;
+            ex[j] = s < slots ? moe_slot_expert(idx, s, tab) : -1;
         }
     }
     for (int e = threadIdx.x; e < experts; e += blockDim.x) count[e] = 0;
     for (int p = threadIdx.x; p < capacity; p += blockDim.x) sorted_slot[p] = -1;
     for (int i = threadIdx.x; i < max_tiles; i += blockDim.x) tile_expert[i] = -1;
     __syncthreads();
-    for (int s = threadIdx.x; s < slots; s += blockDim.x) {
-        const int e = idx[s];
-        if (e >= 0 && e < experts) atomicAdd(&count[e], 1);
-    }
-    __syncthreads();
-    if (threadIdx.x == 0) {
-        int at = 0;
-        for (int e = 0; e < experts; ++e) {
-            start[e] = at;
-            const int tiles = (count[e] + MOE_TILE - 1) / MOE_TILE;
-            for (int i = 0; i < tiles; ++i) tile_expert[at / MOE_TILE + i] = e;
-            at += tiles * MOE_TILE;
-            count[e] = 0;               // from here on: the next free place of the expert's run
+    if (in_registers) {
+#pragma unroll
+        for (int j = 0; j < MOE_SLOTS_IN_REGISTERS; ++j)
+            if (ex[j] >= 0 && ex[j] < experts) at[j] = atomicAdd(&count[ex[j]], 1);
+    } else {
+        for (int s = threadIdx.x; s < slots; s += blockDim.x) {
+            const int e = moe_slot_expert(idx, s, tab);
+            if (e >= 0 && e < experts) atomicAdd(&count[e], 1);
         }
     }
     __syncthreads();
+    if (threadIdx.x == 0) {
+        int first = 0;
+        for (int e = 0; e < experts; ++e) {
+            start[e] = first;
+            const int tiles = (count[e] + MOE_TILE - 1) / MOE_TILE;
+            first += (tiles + group - 1) / group * group * MOE_TILE;
+        }
+    }
+    __syncthreads();
+    for (int e = threadIdx.x; e < experts; e += blockDim.x) {
+        const int tiles = (count[e] + MOE_TILE - 1) / MOE_TILE;
+        for (int i = 0; i < tiles; ++i) tile_expert[start[e] / MOE_TILE + i] = e;
+        count[e] = 0;                   // from here on: the next free place of the expert's run
+    }
+    if (in_registers) {
+#pragma unroll
+        for (int j = 0; j < MOE_SLOTS_IN_REGISTERS; ++j) {
+            const int s = threadIdx.x + j * blockDim.x;
+            if (s >= slots) continue;
+            if (ex[j] >= 0 && ex[j] < experts) sorted_slot[start[ex[j]] + at[j]] = s;
+            if (tab.table) {
+                idx[s] = ex[j];
+                tab.wgt[s] = tab.weight;
+            }
+        }
+        return;
+    }
+    __syncthreads();
     for (int s = threadIdx.x; s < slots; s += blockDim.x) {
-        const int e = idx[s];
+        const int e = moe_slot_expert(idx, s, tab);
         if (e >= 0 && e < experts) sorted_slot[start[e] + atomicAdd(&count[e], 1)] = s;
+        if (tab.table) {
+            idx[s] = e;
+            tab.wgt[s] = tab.weight;
+        }
     }
 }
 
 static int moe_align_launch(int *sorted_slot, int *tile_expert, int *idx, int slots, int experts, int capacity, int max_tiles,
-                            const MoeTable &tab, hipStream_t stream) {
+                            int group, const MoeTable &tab, hipStream_t stream) {
+    KVA_REQUIRE(group >= 1 && max_tiles % group == 0, "moe_align: %d tiles do not come in groups of %d", max_tiles, group);
     KVA_REQUIRE(sorted_slot && tile_expert && idx, "moe_align: missing operand");
     KVA_REQUIRE(experts > 0 && experts <= MOE_MAX_EXPERTS, "moe_align: %d experts (at most %d)", experts, MOE_MAX_EXPERTS);
-    KVA_REQUIRE(capacity == max_tiles * MOE_TILE && capacity >= slots + experts * (MOE_TILE - 1),
+    KVA_REQUIRE(capacity == max_tiles * MOE_TILE && capacity >= slots + experts * (MOE_TILE * group - 1),
                 "moe_align: a list of %d places cannot hold %d slots of %d experts in tiles of %d", capacity, slots,
                 experts, MOE_TILE);
     hipLaunchKernelGGL(moe_align_kernel, dim3(1), dim3(1024), 0, stream, sorted_slot, tile_expert, idx, slots, experts,
-                       capacity, max_tiles, tab);
+                       capacity, max_tiles, group, tab);
     KVA_CHECK_LAUNCH("moe_align");
     return KVA_OK;
 }
 
 extern "C" int kva_moe_align(int *sorted_slot, int *tile_expert, const int *idx, int slots, int experts, int capacity,
-                             int max_tiles, hipStream_t stream) {
+                             int max_tiles, int group, hipStream_t stream) {
     // (without a table the kernel only reads idx)
-    return moe_align_launch(sorted_slot, tile_expert, const_cast<int *>(idx), slots, experts, capacity, max_tiles,
+    return moe_align_launch(sorted_slot, tile_expert, const_cast<int *>(idx), slots, experts, capacity, max_tiles, group,
                             MoeTable{nullptr, nullptr, nullptr, 0, 1, 0.f, nullptr}, stream);
 }
 
 extern "C" int kva_moe_table_align(int *sorted_slot, int *tile_expert, int *idx, float *wgt, const int *table, int table_rows,
                                    const int *ids, const int *feedback, int tokens, int top, float weight, int experts,
-                                   int capacity, int max_tiles, hipStream_t stream) {
+                                   int capacity, int max_tiles, int group, hipStream_t stream) {
     KVA_REQUIRE(wgt && table && ids && table_rows > 0 && tokens >= 0 && top > 0, "moe_table_align: missing operand or bad sizes");
-    return moe_align_launch(sorted_slot, tile_expert, idx, tokens * top, experts, capacity, max_tiles,
+    return moe_align_launch(sorted_slot, tile_expert, idx, tokens * top, experts, capacity, max_tiles, group,
                             MoeTable{table, ids, feedback, table_rows, top, weight, wgt}, stream);
 }
 
@@ -262,6 +305,7 @@ struct MoeRows {
     const int *sorted_slot, *tile_expert;
     const float *slot_weight;       // mode 1
     int top, N, K, mode, act;
+    int tiled;                      // the matrices lie in operand order: [N / 16][K / 32][lane][8] (lane = 16 (k % 32 / 8) + n % 16)
     int gated;                      // mode 0: rows 2 j and 2 j + 1 of the matrix are output j's gate and up rows
     float limit;                    // activation 4 (clamped swish): gate and up are cut off at this value
 };
@@ -353,9 +397,11 @@ __device__ inline void moe_tiles_product(const MoeRows &a, void *__restrict__ ou
         xrow[rt] = x + src * a.K + 8 * g;
     }
     const bf16_t *wrow[NT];
+    const int wstep = a.tiled ? 16 * 32 : 32;       // from one step of 32 to the next
 #pragma unroll
     for (int nt = 0; nt < NT; ++nt)
-        wrow[nt] = w + ((size_t)e * a.N + min(n_first + 16 * nt + r, a.N - 1)) * a.K + 8 * g;
+        wrow[nt] = w + (a.tiled ? ((size_t)e * a.N + min(n_first + 16 * nt, a.N - 16)) * a.K + 8 * lane
+                                : ((size_t)e * a.N + min(n_first + 16 * nt + r, a.N - 1)) * a.K + 8 * g);
     f32x4 acc[NT][RT];
 #pragma unroll
     for (int nt = 0; nt < NT; ++nt)
@@ -363,14 +409,15 @@ __device__ inline void moe_tiles_product(const MoeRows &a, void *__restrict__ ou
         for (int rt = 0; rt < RT; ++rt) acc[nt][rt] = f32x4{0.f, 0.f, 0.f, 0.f};
     const int steps = a.K / 32, per = (steps + 3) / 4;
     const int s0 = wave * per, s1 = min(steps, s0 + per);
-#pragma unroll 2
+    constexpr int AHEAD = NT * RT == 1 ? 8 : 2;         // a tile of its own: as many loads in flight as there are products
+#pragma unroll AHEAD
     for (int s = s0; s < s1; ++s) {
         const int k0 = 32 * s;
         Frag8 xf[RT], wf[NT];
 #pragma unroll
         for (int rt = 0; rt < RT; ++rt) xf[rt].u4 = *reinterpret_cast<const uint4 *>(xrow[rt] + k0);
 #pragma unroll
-        for (int nt = 0; nt < NT; ++nt) wf[nt].u4 = *reinterpret_cast<const uint4 *>(wrow[nt] + k0);
+        for (int nt = 0; nt < NT; ++nt) wf[nt].u4 = *reinterpret_cast<const uint4 *>(wrow[nt] + (size_t)s * wstep);
 #pragma unroll
         for (int nt = 0; nt < NT; ++nt)
 #pragma unroll
@@ -431,10 +478,125 @@ moe_expert_rows_mfma_kernel(MoeRows a, void *__restrict__ out, int out_dtype, co
     }
 }
 
+// matrix cores, many rows an expert: a workgroup takes a group of 2 RT tiles of one expert (32 RT rows) and 128
+// outputs, a wavefront half of either.  64 elements of K of both operands go through LDS at a time, two deep
+// (the next ones' loads are in flight while these are multiplied), in rows padded so that a fragment's 16
+// lanes lie on banks of their own.  K is added in ascending order.  Workgroups that follow each other in the
+// work list run on one of the 8 dies (the hardware deals them out in turn), so that a die reads few experts.
+#define MOE_LDS_K 64
+#define MOE_LDS_STRIDE 72
+#define MOE_LDS_N 128
+template <int RT>
+__global__ void __launch_bounds__(256)
+moe_expert_rows_lds_kernel(MoeRows a, void *__restrict__ out, int out_dtype, const bf16_t *__restrict__ x,
+                           const bf16_t *__restrict__ w, int n_blocks) {
+    constexpr int ROWS = 32 * RT, XI = ROWS * MOE_LDS_K / 8 / 256, WI = MOE_LDS_N * MOE_LDS_K / 8 / 256;
+    __shared__ __align__(16) bf16_t xs[2][ROWS * MOE_LDS_STRIDE], ws[2][MOE_LDS_N * MOE_LDS_STRIDE];
+    const int total = gridDim.x, die = blockIdx.x % 8, q = total / 8, rem = total % 8;
+    const int id = die * q + min(die, rem) + (int)blockIdx.x / 8;
+    const int first = (id / n_blocks) * 2 * RT, n0 = (id % n_blocks) * MOE_LDS_N;
+    const int e = a.tile_expert[first];
+    if (e < 0) return;
+    const int lane = threadIdx.x % KVA_WAVE, wave = threadIdx.x / KVA_WAVE, r = lane & 15, g = lane >> 4;
+    const int wr = wave & 1, wn = wave >> 1;
+    // 16 bytes at a time: thread t takes elements 8 (t % 8) .. of rows t / 8 + 32 i
+    const int kc = 8 * (threadIdx.x % 8), srow = threadIdx.x / 8;
+    const bf16_t *xp[XI], *wp[WI];
+#pragma unroll
+    for (int i = 0; i < XI; ++i) {
+        const int place = first * MOE_TILE + srow + 32 * i, slot = a.sorted_slot[place];
+        xp[i] = x + (a.mode == 0 ? (size_t)(slot < 0 ? 0 : slot / a.top) : (size_t)place) * a.K + kc;
+    }
+    // ... and of a matrix in operand order the piece of lane t % 64 of one of its tiles of 16 x 32, which is neighbouring bytes
+    int wat[WI], wkc[WI];               // where a piece goes in LDS, and its first element of the 64
+#pragma unroll
+    for (int i = 0; i < WI; ++i) {
+        const int f = wave + 4 * i, nt = f >> 1;
+        const int row = a.tiled ? 16 * nt + r : srow + 32 * i;
+        wkc[i] = a.tiled ? 32 * (f & 1) + 8 * g : kc;
+        wat[i] = row * MOE_LDS_STRIDE + wkc[i];
+        wp[i] = w + (a.tiled ? ((size_t)e * a.N + min(n0 + 16 * nt, a.N - 16)) * a.K + (f & 1) * 16 * 32 + 8 * lane
+                             : ((size_t)e * a.N + min(n0 + row, a.N - 1)) * a.K + kc);
+    }
+    const int wmul = a.tiled ? 16 : 1;  // elements of a matrix's storage a step of one element of K moves on by
+    uint4 xv[XI], wv[WI];
+#define MOE_LDS_LOAD(K0)                                                                                              \
+    {                                                                                                                 \
+        const bool in = (K0) + kc < a.K;                                                                              \
+        _Pragma("unroll") for (int i = 0; i < XI; ++i)                                                                \
+            xv[i] = in ? *reinterpret_cast<const uint4 *>(xp[i] + (K0)) : make_uint4(0u, 0u, 0u, 0u);                  \
+        _Pragma("unroll") for (int i = 0; i < WI; ++i)                                                                \
+            wv[i] = (K0) + wkc[i] < a.K ? *reinterpret_cast<const uint4 *>(wp[i] + (K0) * wmul) : make_uint4(0u, 0u, 0u, 0u); \
+    }
+    f32x4 acc[4][RT];
+#pragma unroll
+    for (int nt = 0; nt < 4; ++nt)
+#pragma unroll
+        for (int rt = 0; rt < RT; ++rt) acc[nt][rt] = f32x4{0.f, 0.f, 0.f, 0.f};
+    MOE_LDS_LOAD(0)
+    int buf = 0;
+    for (int k0 = 0; k0 < a.K; k0 += MOE_LDS_K, buf ^= 1) {
+#pragma unroll
+        for (int i = 0; i < XI; ++i) *reinterpret_cast<uint4 *>(&xs[buf][(srow + 32 * i) * MOE_LDS_STRIDE + kc]) = xv[i];
+#pragma unroll
+        for (int i = 0; i < WI; ++i) *reinterpret_cast<uint4 *>(&ws[buf][wat[i]]) = wv[i];
+        __syncthreads();                // (a buffer was read last two turns ago: every wavefront has passed the barrier between)
+        if (k0 + MOE_LDS_K < a.K) MOE_LDS_LOAD(k0 + MOE_LDS_K)
+        const bf16_t *xr = &xs[buf][(wr * 16 * RT + r) * MOE_LDS_STRIDE + 8 * g], *wrow = &ws[buf][(wn * 64 + r) * MOE_LDS_STRIDE + 8 * g];
+        Frag8 xf[2][RT], wf[2][4];
+#pragma unroll
+        for (int ks = 0; ks < 2; ++ks) {
+#pragma unroll
+            for (int nt = 0; nt < 4; ++nt) wf[ks][nt].u4 = *reinterpret_cast<const uint4 *>(wrow + nt * 16 * MOE_LDS_STRIDE + 32 * ks);
+#pragma unroll
+            for (int rt = 0; rt < RT; ++rt) xf[ks][rt].u4 = *reinterpret_cast<const uint4 *>(xr + rt * 16 * MOE_LDS_STRIDE + 32 * ks);
+        }
+        __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+        for (int ks = 0; ks < 2; ++ks)
+#pragma unroll
+            for (int nt = 0; nt < 4; ++nt)
+#pragma unroll
+                for (int rt = 0; rt < RT; ++rt)
+                    acc[nt][rt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[ks][nt].v, xf[ks][rt].v, acc[nt][rt], 0, 0, 0);
+    }
+#undef MOE_LDS_LOAD
+    // lane (row r, group g) holds outputs 4 g .. 4 g + 3 of tile nt, of its row of tile rt
+#pragma unroll
+    for (int rt = 0; rt < RT; ++rt) {
+        const int place = first * MOE_TILE + (wr * RT + rt) * 16 + r, slot = a.sorted_slot[place];
+        if (slot < 0) continue;
+        const float weight = a.mode == 1 ? a.slot_weight[slot] : 1.f;
+#pragma unroll
+        for (int nt = 0; nt < 4; ++nt) {
+            const int n = n0 + wn * 64 + nt * 16 + 4 * g;
+            const f32x4 v = acc[nt][rt];
+            if (a.mode == 1 && a.N % 4 == 0) {
+                if (n < a.N)
+                    *reinterpret_cast<float4 *>(reinterpret_cast<float *>(out) + (size_t)slot * a.N + n) =
+                        make_float4(v[0] * weight, v[1] * weight, v[2] * weight, v[3] * weight);
+            } else if (a.gated) {
+                if (n + 1 < a.N) moe_store_gated(a, out, out_dtype, place, n, v[0], v[1]);
+                if (n + 3 < a.N) moe_store_gated(a, out, out_dtype, place, n + 2, v[2], v[3]);
+            } else {
+#pragma unroll
+                for (int i = 0; i < 4; ++i)
+                    if (n + i < a.N) moe_store(a, out, out_dtype, place, slot, n + i, v[i]);
+            }
+        }
+    }
+}
+
+// groups of so many tiles of 16 rows have a kernel of their own (for operands in bf16 whose K is a multiple of 32)
+extern "C" int kva_moe_group_supported(int group, int K) { return (group == 4 || group == 8) && K > 0 && K % 32 == 0; }
+
 extern "C" int kva_moe_expert_rows(void *out, int out_dtype, const void *x, const void *w, int dtype,
                                    const int *sorted_slot, const int *tile_expert, const float *slot_weight,
                                    int max_tiles, int top, int N, int K, int mode, int act, int gated, float limit,
-                                   hipStream_t stream) {
+                                   int group, int tiled, hipStream_t stream) {
+    KVA_REQUIRE(!tiled || (dtype == KVA_BF16 && K % 32 == 0 && N % 16 == 0), "moe_expert_rows: no operand order for %d x %d", N, K);
+    KVA_REQUIRE(group == 1 || (dtype == KVA_BF16 && kva_moe_group_supported(group, K) && max_tiles % group == 0),
+                "moe_expert_rows: no kernel for groups of %d tiles, %d of them, with K = %d", group, max_tiles, K);
     KVA_REQUIRE(act != 4 || gated, "moe_expert_rows: the clamped activation is a gated one");
     KVA_REQUIRE(!gated || (mode == 0 && N % 2 == 0), "moe_expert_rows: gate and up rows come in pairs, in the first product");
     KVA_REQUIRE(out && x && w && sorted_slot && tile_expert, "moe_expert_rows: missing operand");
@@ -444,8 +606,18 @@ extern "C" int kva_moe_expert_rows(void *out, int out_dtype, const void *x, cons
     KVA_REQUIRE(N > 0 && K > 0 && top > 0 && act >= 0 && act <= 5, "moe_expert_rows: bad sizes or activation");
     KVA_REQUIRE(max_tiles >= 0 && max_tiles <= 65535, "moe_expert_rows: %d tiles are too many for one launch", max_tiles);
     if (max_tiles == 0) return KVA_OK;
-    MoeRows a{sorted_slot, tile_expert, slot_weight, top, N, K, mode, act, gated, limit};
-    if (dtype == KVA_BF16 && K % 32 == 0) {
+    MoeRows a{sorted_slot, tile_expert, slot_weight, top, N, K, mode, act, tiled, gated, limit};
+    if (group > 1) {
+        const int n_blocks = (N + MOE_LDS_N - 1) / MOE_LDS_N;
+        const long long blocks = (long long)n_blocks * (max_tiles / group);
+        KVA_REQUIRE(blocks <= 0x7fffffff, "moe_expert_rows: too many workgroups");
+        if (group == 8)
+            hipLaunchKernelGGL((moe_expert_rows_lds_kernel<4>), dim3((unsigned)blocks), dim3(256), 0, stream, a, out, out_dtype,
+                               (const bf16_t *)x, (const bf16_t *)w, n_blocks);
+        else
+            hipLaunchKernelGGL((moe_expert_rows_lds_kernel<2>), dim3((unsigned)blocks), dim3(256), 0, stream, a, out, out_dtype,
+                               (const bf16_t *)x, (const bf16_t *)w, n_blocks);
+    } else if (dtype == KVA_BF16 && K % 32 == 0) {
         // few tiles: 16 outputs a workgroup, so that enough of them stream the matrices; many: 64 outputs and
         // four row tiles, which share what they load
         if ((long long)max_tiles * ((N + 15) / 16) <= 8192)

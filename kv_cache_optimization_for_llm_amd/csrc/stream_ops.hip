@@ -706,14 +706,26 @@ sandwich_step_kernel(float *__restrict__ x, const void *__restrict__ y, int y_dt
 
 // The same with a row's elements in registers (a width that is a multiple of 4): a thread takes 4
 // neighbouring columns ITERS times, and every load - stream, branch output, addend, both norms' weights and
-// biases - is asked for before the first sum.
+// biases - is asked for before the first sum.  Sums over the workgroup go through the vector ALU inside a
+// wavefront and meet in a line of LDS of their own: one barrier a sum.
+template <int WAVES>
+__device__ inline float sandwich_sum(float v, float *line) {
+    v = wave_sum_valu(v);
+    if (threadIdx.x % KVA_WAVE == 0) line[threadIdx.x / KVA_WAVE] = v;
+    __syncthreads();
+    float total = 0.f;
+#pragma unroll
+    for (int w = 0; w < WAVES; ++w) total += line[w];
+    return total;
+}
+
 template <int THREADS, int ITERS>
 __global__ void __launch_bounds__(THREADS)
 sandwich_step_vec_kernel(float *__restrict__ x, const void *__restrict__ y, int y_dtype, SideNorm post,
                          const float *__restrict__ addend, SideNorm pre, void *__restrict__ out, int out_dtype,
                          const int *__restrict__ row_idx, int width) {
     constexpr int WAVES = THREADS / KVA_WAVE;
-    __shared__ float red_s[WAVES];
+    __shared__ float red_s[4][WAVES];
     const int r = blockIdx.x;
     const size_t row = (size_t)(row_idx ? row_idx[r] : r) * width;
     float v[ITERS][4], yv[ITERS][4], av[ITERS][4], pw[ITERS][4], pb[ITERS][4], nw[ITERS][4], nb[ITERS][4];
@@ -738,7 +750,7 @@ sandwich_step_vec_kernel(float *__restrict__ x, const void *__restrict__ y, int 
             float sum = 0.f;
 #pragma unroll
             for (int it = 0; it < ITERS; ++it) sum += (yv[it][0] + yv[it][1]) + (yv[it][2] + yv[it][3]);
-            mean = block_sum(sum, red_s, WAVES) / (float)width;
+            mean = sandwich_sum<WAVES>(sum, red_s[0]) / (float)width;
         }
         float sq = 0.f;
 #pragma unroll
@@ -750,7 +762,7 @@ sandwich_step_vec_kernel(float *__restrict__ x, const void *__restrict__ y, int 
                 sq += yv[it][e] * yv[it][e];
             }
         }
-        const float inv = 1.0f / sqrtf(block_sum(sq, red_s, WAVES) / (float)width + post.eps);
+        const float inv = 1.0f / sqrtf(sandwich_sum<WAVES>(sq, red_s[1]) / (float)width + post.eps);
 #pragma unroll
         for (int it = 0; it < ITERS; ++it)
 #pragma unroll
@@ -770,7 +782,7 @@ sandwich_step_vec_kernel(float *__restrict__ x, const void *__restrict__ y, int 
     }
     if (!out) return;
     float mean = 0.f;
-    if (pre.center) mean = block_sum(sum, red_s, WAVES) / (float)width;
+    if (pre.center) mean = sandwich_sum<WAVES>(sum, red_s[2]) / (float)width;
     float sq = 0.f;
 #pragma unroll
     for (int it = 0; it < ITERS; ++it) {
@@ -781,7 +793,7 @@ sandwich_step_vec_kernel(float *__restrict__ x, const void *__restrict__ y, int 
             sq += v[it][e] * v[it][e];
         }
     }
-    const float inv = 1.0f / sqrtf(block_sum(sq, red_s, WAVES) / (float)width + pre.eps);
+    const float inv = 1.0f / sqrtf(sandwich_sum<WAVES>(sq, red_s[3]) / (float)width + pre.eps);
 #pragma unroll
     for (int it = 0; it < ITERS; ++it) {
         const int j = (threadIdx.x + it * THREADS) * 4;

@@ -1801,25 +1801,42 @@ def moe_route(logits: torch.Tensor, correction: Optional[torch.Tensor], top: int
                                   logits.stride(0) if tokens > 1 else outputs, _stream()), "moe_route")
 
 
-def moe_tiles(slots: int, experts: int) -> int:
-    """Tiles of 16 rows that hold ``slots`` (token, choice) pairs sorted by expert, whatever the split."""
-    return (int(slots) + int(experts) * (MOE_TILE - 1) + MOE_TILE - 1) // MOE_TILE
+def moe_tiles(slots: int, experts: int, group: int = 1) -> int:
+    """Tiles of 16 rows that hold ``slots`` (token, choice) pairs sorted by expert, whatever the split, every
+    expert's run a multiple of ``group`` tiles."""
+    rows = MOE_TILE * int(group)
+    return (int(slots) + int(experts) * (rows - 1) + rows - 1) // rows * int(group)
 
 
-def moe_align(idx: torch.Tensor, experts: int, sorted_slot: torch.Tensor, tile_expert: torch.Tensor) -> None:
+# (token, choice) pairs an expert gets on average from which on its products go through LDS in groups of tiles
+MOE_GROUPS = ((160, 8), (56, 4))
+
+
+def moe_group(slots: int, experts: int, dtype: torch.dtype, *inner: int) -> int:
+    """How many tiles of 16 rows the experts' products take at once (``group`` below) for products over
+    ``inner`` elements: decided by sizes alone."""
+    if dtype == torch.bfloat16:
+        for least, group in MOE_GROUPS:
+            if slots >= least * experts and all(hip_lib().kva_moe_group_supported(group, int(k)) for k in inner):
+                return group
+    return 1
+
+
+def moe_align(idx: torch.Tensor, experts: int, sorted_slot: torch.Tensor, tile_expert: torch.Tensor, group: int = 1) -> None:
     """The slots ``idx.view(-1)`` that name one of the first ``experts`` router outputs, sorted by
     expert into ``sorted_slot`` (every tile of 16 places belongs to one expert, -1 pads) with the
-    tiles' experts in ``tile_expert`` (-1: unused)."""
+    tiles' experts in ``tile_expert`` (-1: unused).  ``group``: an expert's run starts at a multiple of so many tiles."""
     slots, tiles = idx.numel(), tile_expert.shape[0]
-    if sorted_slot.shape != (tiles * MOE_TILE,) or tiles < moe_tiles(slots, experts):
+    if sorted_slot.shape != (tiles * MOE_TILE,) or tiles < moe_tiles(slots, experts, group):
         raise KernelError(f"moe_align: {tiles} tiles cannot hold {slots} slots of {experts} experts")
     check(hip_lib().kva_moe_align(_dev(sorted_slot, "sorted_slot", torch.int32), _dev(tile_expert, "tile_expert", torch.int32),
                                   _dev(idx, "idx", torch.int32), slots, int(experts), tiles * MOE_TILE, tiles,
-                                  _stream()), "moe_align")
+                                  int(group), _stream()), "moe_align")
 
 
 def moe_table_align(table: torch.Tensor, ids: torch.Tensor, idx: torch.Tensor, wgt: torch.Tensor, experts: int,
-                    sorted_slot: torch.Tensor, tile_expert: torch.Tensor, feedback: Optional[torch.Tensor] = None) -> None:
+                    sorted_slot: torch.Tensor, tile_expert: torch.Tensor, feedback: Optional[torch.Tensor] = None,
+                    group: int = 1) -> None:
     """Experts by token id, without a router: ``idx[t] = table[ids[t]]`` (int32 ``[rows, top]``) with equal
     weights ``wgt[t, k] = 1 / top``, and the slots sorted by expert as :func:`moe_align` does, in one launch.  A
     negative id ``-1 - r`` stands for ``feedback[r]`` as in :func:`embed_gather`."""
@@ -1827,24 +1844,40 @@ def moe_table_align(table: torch.Tensor, ids: torch.Tensor, idx: torch.Tensor, w
     tiles = tile_expert.shape[0]
     if table.dim() != 2 or table.shape[1] != top or ids.shape != (tokens,) or wgt.shape != (tokens, top):
         raise KernelError(f"moe_table_align: table {tuple(table.shape)}, ids {tuple(ids.shape)}, idx {tuple(idx.shape)} do not fit")
-    if sorted_slot.shape != (tiles * MOE_TILE,) or tiles < moe_tiles(tokens * top, experts):
+    if sorted_slot.shape != (tiles * MOE_TILE,) or tiles < moe_tiles(tokens * top, experts, group):
         raise KernelError(f"moe_table_align: {tiles} tiles cannot hold {tokens * top} slots of {experts} experts")
     check(hip_lib().kva_moe_table_align(
         _dev(sorted_slot, "sorted_slot", torch.int32), _dev(tile_expert, "tile_expert", torch.int32), _dev(idx, "idx", torch.int32),
         _dev(wgt, "wgt", torch.float32), _dev(table, "table", torch.int32), table.shape[0], _dev(ids, "ids", torch.int32),
         _opt(feedback, "feedback", torch.int32), tokens, top, 1.0 / top, int(experts), tiles * MOE_TILE, tiles,
-        _stream()), "moe_table_align")
+        int(group), _stream()), "moe_table_align")
+
+
+def moe_can_tile(w: torch.Tensor) -> bool:
+    """Whether experts' matrices ``[experts, N, K]`` can be stored in operand order."""
+    return w.is_cuda and w.dtype == torch.bfloat16 and w.shape[1] % 16 == 0 and w.shape[2] % 32 == 0
+
+
+def moe_tiled_weight(w: torch.Tensor) -> torch.Tensor:
+    """Experts' matrices ``[experts, N, K]`` in operand order: every tile of 16 x 32 elements, which a
+    wavefront loads at once, is 1 KiB of neighbouring bytes (``[experts, N / 16, K / 32, k % 32 / 8, n % 16,
+    8]``); the shape is left as it was."""
+    e, n, k = w.shape
+    return w.view(e, n // 16, 16, k // 32, 4, 8).permute(0, 1, 3, 4, 2, 5).contiguous().view(e, n, k)
 
 
 def moe_expert_rows(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, sorted_slot: torch.Tensor,
                     tile_expert: torch.Tensor, top: int, *, activation: Optional[str] = None,
-                    slot_weight: Optional[torch.Tensor] = None, gated: bool = False, limit: float = 0.0) -> torch.Tensor:
+                    slot_weight: Optional[torch.Tensor] = None, gated: bool = False, limit: float = 0.0,
+                    group: int = 1, tiled: bool = False) -> torch.Tensor:
     """One product per tile against its expert's matrix ``w[e]`` ``[N, K]``.  With an ``activation``
     (the first product): row ``slot // top`` of ``x`` ``[T, K]``, activated, goes to the slot's sorted
     place of ``out`` ``[places, N]`` (x's type).  With ``slot_weight`` (the second): the row at the
     sorted place of ``x`` ``[places, K]``, times the slot's weight, goes to row ``slot`` of ``out`` fp32
     ``[slots, N]``.  ``gated`` (first product): rows ``2 j`` and ``2 j + 1`` of an expert's matrix are
-    output j's gate and up rows, and ``out`` ``[places, N / 2]`` gets ``act(gate) * up``."""
+    output j's gate and up rows, and ``out`` ``[places, N / 2]`` gets ``act(gate) * up``.  ``group`` (as the list
+    was sorted, :func:`moe_group`): so many tiles at a time, through LDS.  ``tiled``: the matrices are
+    stored in operand order (:func:`moe_tiled_weight`)."""
     tiles = tile_expert.shape[0]
     n_out = w.shape[1] // 2 if gated else w.shape[1]
     if gated and (activation is None or w.shape[1] % 2):
@@ -1867,7 +1900,8 @@ def moe_expert_rows(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, sorted_
         _dev(out, "out"), dtype_code(out.dtype), _dev(x, "x"), _dev(w, "w"), dtype_code(x.dtype),
         _dev(sorted_slot, "sorted_slot", torch.int32), _dev(tile_expert, "tile_expert", torch.int32),
         _opt(slot_weight, "slot_weight"), tiles, int(top), w.shape[1], w.shape[2], 0 if activation is not None else 1,
-        EXPERT_ACTIVATIONS.get(activation, 0), 1 if gated else 0, float(limit), _stream()), "moe_expert_rows")
+        EXPERT_ACTIVATIONS.get(activation, 0), 1 if gated else 0, float(limit), int(group), 1 if tiled else 0, _stream()),
+        "moe_expert_rows")
     return out
 
 

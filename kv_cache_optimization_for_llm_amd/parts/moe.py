@@ -19,7 +19,7 @@ Everything from the router's logits to the sum stays on the device (``csrc/moe.h
 product of every tile with its activation, a second the other product times the slot's weight,
 and a third adds a token's rows up - no count of tokens per expert reaches the host, so a step
 with this layer can be captured into a graph.  The experts' matrices are stacked at load time
-(``[experts, ff, hidden]`` and ``[experts, hidden, ff]``).
+(``[experts, ff, hidden]`` and ``[experts, hidden, ff]``; for the matrix-core kernels in operand order).
 """
 from __future__ import annotations
 
@@ -154,14 +154,18 @@ class RoutedExperts(FeedForward):
             self.w_down = torch.stack([tensors[n["down"].format(e=e)] for e in range(self.experts)]).contiguous()
         else:
             self.w_up = self.w_down = None
+        # matrices of the matrix-core kernels lie in operand order: what a wavefront loads at once is one run of bytes
+        self.tiled = self.experts > 0 and K.moe_can_tile(self.w_up) and K.moe_can_tile(self.w_down)
+        if self.tiled:
+            self.w_up, self.w_down = K.moe_tiled_weight(self.w_up), K.moe_tiled_weight(self.w_down)
 
     def activation_elements(self) -> int:
         return self.outputs + self.top * (2 * self.intermediate_size + 2 * self.hidden_size) + self.hidden_size \
             + (self.shared.activation_elements() + self.hidden_size if self.shared is not None else 0)
 
-    def _sorted(self, slots: int, dev):
+    def _sorted(self, slots: int, group: int, dev):
         """(sorted slots, tiles' experts), still to be filled"""
-        tiles = K.moe_tiles(slots, self.experts)
+        tiles = K.moe_tiles(slots, self.experts, group)
         return torch.empty(tiles * K.MOE_TILE, dtype=torch.int32, device=dev), torch.empty(tiles, dtype=torch.int32, device=dev)
 
     def _route(self, x, idx, wgt):
@@ -182,10 +186,11 @@ class RoutedExperts(FeedForward):
         idx = torch.empty((T, self.top), dtype=torch.int32, device=dev)
         wgt = torch.empty((T, self.top), dtype=torch.float32, device=dev)
         slots, gate = T * self.top, None
+        group = K.moe_group(slots, self.experts, x.dtype, self.hidden_size, self.intermediate_size) if self.experts else 1
         if self.by_table:
-            sorted_slot, tile_expert = self._sorted(slots, dev)
+            sorted_slot, tile_expert = self._sorted(slots, group, dev)
             K.moe_table_align(self.table, ctx.batch.token_ids, idx, wgt, self.experts, sorted_slot, tile_expert,
-                              getattr(ctx.batch, "feedback", None))
+                              getattr(ctx.batch, "feedback", None), group)
         else:
             gate = self._route(x, idx, wgt)
         if RoutedExperts.on_route is not None and not torch.cuda.is_current_stream_capturing():
@@ -193,12 +198,13 @@ class RoutedExperts(FeedForward):
         rows = torch.empty((slots, self.hidden_size), dtype=torch.float32, device=dev)
         if self.experts:
             if not self.by_table:
-                sorted_slot, tile_expert = self._sorted(slots, dev)
-                K.moe_align(idx, self.experts, sorted_slot, tile_expert)
+                sorted_slot, tile_expert = self._sorted(slots, group, dev)
+                K.moe_align(idx, self.experts, sorted_slot, tile_expert, group)
             act = torch.empty((sorted_slot.shape[0], self.intermediate_size), dtype=x.dtype, device=dev)
             K.moe_expert_rows(x, self.w_up, act, sorted_slot, tile_expert, self.top, activation=self.activation,
-                              gated=self.gated, limit=self.limit)
-            K.moe_expert_rows(act, self.w_down, rows, sorted_slot, tile_expert, self.top, slot_weight=wgt)
+                              gated=self.gated, limit=self.limit, group=group, tiled=self.tiled)
+            K.moe_expert_rows(act, self.w_down, rows, sorted_slot, tile_expert, self.top, slot_weight=wgt, group=group,
+                              tiled=self.tiled)
         out = torch.empty_like(x)
         extra = self.shared.forward(x, ctx) if self.shared is not None else None
         return K.moe_combine(x, rows, idx, wgt, self.experts, out, extra=extra, extra_gate=gate)

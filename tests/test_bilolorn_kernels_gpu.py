@@ -343,8 +343,9 @@ def test_squared_relu_as_a_gate_and_in_a_products_epilogue(gpu):
             close(out, want, 2e-2, "epilogue")
 
 
-@pytest.mark.parametrize("rows, experts, top", [(1, 1, 1), (5, 3, 2), (40, 24, 5), (900, 7, 7), (700, 300, 3), (2049, 16, 4)])
-def test_experts_by_token_id_and_their_sorted_tiles(rows, experts, top, gpu):
+@pytest.mark.parametrize("group", [1, 4, 8])
+@pytest.mark.parametrize("rows, experts, top", [(1, 1, 1), (5, 3, 2), (40, 24, 5), (900, 7, 7), (700, 300, 3), (2049, 16, 4), (6000, 5, 3)])
+def test_experts_by_token_id_and_their_sorted_tiles(rows, experts, top, group, gpu):
     vocab = 97
     g = torch.Generator().manual_seed(rows)
     table = torch.rand((vocab, experts), generator=g).argsort(-1)[:, :top].to(torch.int32).contiguous()
@@ -355,10 +356,10 @@ def test_experts_by_token_id_and_their_sorted_tiles(rows, experts, top, gpu):
         ids[1], ids[2], real[1], real[2] = -1, -2, 5, 96              # ids that are still on the device
     idx = torch.full((rows, top), -9, dtype=torch.int32, device=gpu)
     wgt = torch.empty((rows, top), dtype=torch.float32, device=gpu)
-    tiles = K.moe_tiles(rows * top, experts)
+    tiles = K.moe_tiles(rows * top, experts, group)
     slot = torch.empty(tiles * K.MOE_TILE, dtype=torch.int32, device=gpu)
     tile_expert = torch.empty(tiles, dtype=torch.int32, device=gpu)
-    K.moe_table_align(table.to(gpu), ids.to(gpu), idx, wgt, experts, slot, tile_expert, feedback.to(gpu))
+    K.moe_table_align(table.to(gpu), ids.to(gpu), idx, wgt, experts, slot, tile_expert, feedback.to(gpu), group)
     assert torch.equal(idx.cpu(), table[real])
     assert torch.allclose(wgt.cpu(), torch.full((rows, top), 1.0 / top))
     slot, tile_expert = slot.cpu().view(tiles, K.MOE_TILE), tile_expert.cpu()
@@ -369,6 +370,58 @@ def test_experts_by_token_id_and_their_sorted_tiles(rows, experts, top, gpu):
         for s in slot[t][slot[t] >= 0].tolist():
             assert flat[s] == tile_expert[t]
     assert ((tile_expert >= 0) == (slot >= 0).any(-1)).all()
+    groups = tile_expert.view(-1, group)                              # a group belongs to one expert, from its first tile on
+    assert ((groups == groups[:, :1]) | (groups < 0)).all()
+    # the same list from choices that are there already
+    again, again_expert = torch.empty_like(slot, device=gpu).view(-1), torch.empty_like(tile_expert, device=gpu)
+    K.moe_align(idx, experts, again, again_expert, group)
+    assert torch.equal(again_expert.cpu(), tile_expert)
+    for t in range(tiles):
+        assert sorted(again.cpu().view(tiles, -1)[t].tolist()) == sorted(slot[t].tolist()) or tile_expert[t] >= 0
+
+
+@pytest.mark.parametrize("group", [1, 4, 8])
+@pytest.mark.parametrize("rows, width, ff, experts, top, gated", [(7, 64, 96, 5, 2, True), (300, 64, 96, 5, 2, True), (90, 96, 160, 3, 3, False), (700, 128, 36, 9, 4, True),
+                                                                  (513, 32, 64, 2, 1, True), (1500, 288, 200, 8, 3, False)])
+def test_experts_products_in_tiles_and_in_groups_of_tiles(rows, width, ff, experts, top, gated, group, gpu):
+    """Both products alone: outputs that are no multiples of the kernel's 128, inner sizes of one step of 32
+    and of odd numbers of them, experts without a token, runs that end inside a group."""
+    g = torch.Generator().manual_seed(rows)
+    idx = torch.rand((rows, experts), generator=g).argsort(-1)[:, :top].to(torch.int32).contiguous()
+    if experts > 4:
+        idx[idx == 3] = experts                                       # (an expert nobody chose; those slots name none)
+    x = rnd((rows, width), 1, torch.bfloat16)
+    up = rnd((experts, (2 if gated else 1) * ff, width), 2, torch.bfloat16, width ** -0.5)
+    ff_pad = (ff + 31) // 32 * 32
+    down = torch.zeros((experts, width, ff_pad), dtype=torch.bfloat16)
+    down[:, :, :ff] = rnd((experts, width, ff), 3, torch.bfloat16, ff ** -0.5)
+    wgt = torch.rand((rows, top), generator=g)
+    tiles = K.moe_tiles(rows * top, experts, group)
+    slot = torch.empty(tiles * K.MOE_TILE, dtype=torch.int32, device=gpu)
+    tile_expert = torch.empty(tiles, dtype=torch.int32, device=gpu)
+    K.moe_align(idx.to(gpu), experts, slot, tile_expert, group)
+    flat, xd = idx.view(-1).long(), x.double().repeat_interleave(top, 0)
+    want_act, want = torch.zeros(rows * top, ff, dtype=torch.float64), torch.zeros(rows * top, width, dtype=torch.float64)
+    for e in range(experts):
+        m = flat == e
+        z = xd[m] @ up[e].double().T
+        h = torch.nn.functional.silu(z[:, 0::2]) * z[:, 1::2] if gated else torch.clamp(z, min=0) ** 2
+        want_act[m] = h
+        want[m] = h @ down[e, :, :ff].double().T * wgt.view(-1)[m].double()[:, None]
+    sl = slot.cpu().long()
+    used = sl >= 0
+    # the matrices row by row, and - where outputs come in whole tiles - in operand order
+    for tiled in (False, True)[:2 if up.shape[1] % 16 == 0 else 1]:
+        lay = K.moe_tiled_weight if tiled else (lambda w: w)
+        act = torch.full((tiles * K.MOE_TILE, ff), float("nan"), dtype=torch.bfloat16, device=gpu)
+        K.moe_expert_rows(x.to(gpu), lay(up.to(gpu)), act, slot, tile_expert, top, activation="silu" if gated else "relu2", gated=gated,
+                          group=group, tiled=tiled)
+        wide = torch.zeros((tiles * K.MOE_TILE, ff_pad), dtype=torch.bfloat16, device=gpu)
+        wide[:, :ff] = act
+        out = torch.zeros((rows * top, width), dtype=torch.float32, device=gpu)
+        K.moe_expert_rows(wide, lay(down.to(gpu)), out, slot, tile_expert, top, slot_weight=wgt.to(gpu), group=group, tiled=tiled)
+        close(act.cpu()[used], want_act[sl[used]], 2e-2, "first product")
+        close(out, want, 3e-2, "second product")
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
