@@ -173,6 +173,36 @@ extern "C" int kva_heads_matmul(void *out, int o_row, int o_head, const void *x,
 // bytes of its row.  K = 32 NKS.  blockIdx: (n tile, head, group of row tiles).
 #include "attention_frag.h"
 
+// outputs n .. n + 3 of row t, head h, under the gate
+__device__ __forceinline__ void heads_store4(bf16_t *o, const f32x4 &acc, float gmul, const HeadsGate &gate, int t, int h, int n, int N,
+                                             bool aligned) {
+    float mul[4] = {gmul, gmul, gmul, gmul};
+    if (gate.per_element) {
+        const bf16_t *gp = reinterpret_cast<const bf16_t *>(gate.p) + (size_t)t * gate.row + (size_t)h * gate.head + n;
+        Frag4 gv;
+        gv.u2 = make_uint2(0u, 0u);
+        if (n + 3 < N && ((reinterpret_cast<uintptr_t>(gp) & 7) == 0)) {
+            gv.u2 = *reinterpret_cast<const uint2 *>(gp);
+        } else {
+#pragma unroll
+            for (int i = 0; i < 4; ++i)
+                if (n + i < N) gv.h[i] = gp[i].bits;
+        }
+#pragma unroll
+        for (int i = 0; i < 4; ++i) mul[i] = 1.0f / (1.0f + expf(-bf16_bits_to_float(gv.h[i])));
+    }
+    if (n + 3 < N && aligned) {
+        Frag4 v;
+#pragma unroll
+        for (int i = 0; i < 4; ++i) v.h[i] = float_to_bf16_bits(acc[i] * mul[i]);
+        *reinterpret_cast<uint2 *>(o) = v.u2;
+    } else {
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+            if (n + i < N) o[i].bits = float_to_bf16_bits(acc[i] * mul[i]);
+    }
+}
+
 template <int NKS, int NT>
 __global__ void __launch_bounds__(KVA_WAVE)
 heads_matmul_mfma_kernel(bf16_t *__restrict__ out, int o_row, int o_head, const bf16_t *__restrict__ x, int x_row,
@@ -215,37 +245,68 @@ heads_matmul_mfma_kernel(bf16_t *__restrict__ out, int o_row, int o_head, const 
             for (int ks = 0; ks < NKS; ++ks) acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[nt][ks].v, xf[ks].v, acc, 0, 0, 0);
             // lane (row t = r, group g) holds outputs n0 + 4 g .. + 3 of its row
             if (tile * 16 + r < M) {
-                bf16_t *o = out + (size_t)t * o_row + (size_t)h * o_head + n0 + 4 * g;
-                float mul[4] = {gmul, gmul, gmul, gmul};
-                if (gate.per_element) {
-                    const bf16_t *gp = reinterpret_cast<const bf16_t *>(gate.p) + (size_t)t * gate.row + (size_t)h * gate.head + n0 + 4 * g;
-                    Frag4 gv;
-                    gv.u2 = make_uint2(0u, 0u);
-                    if (n0 + 4 * g + 3 < N && ((reinterpret_cast<uintptr_t>(gp) & 7) == 0)) {
-                        gv.u2 = *reinterpret_cast<const uint2 *>(gp);
-                    } else {
-#pragma unroll
-                        for (int i = 0; i < 4; ++i)
-                            if (n0 + 4 * g + i < N) gv.h[i] = gp[i].bits;
-                    }
-#pragma unroll
-                    for (int i = 0; i < 4; ++i) mul[i] = 1.0f / (1.0f + expf(-bf16_bits_to_float(gv.h[i])));
-                }
-                if (n0 + 4 * g + 3 < N && ((o_row | o_head) % 4 == 0)) {
-                    Frag4 v;
-#pragma unroll
-                    for (int i = 0; i < 4; ++i) v.h[i] = float_to_bf16_bits(acc[i] * mul[i]);
-                    *reinterpret_cast<uint2 *>(o) = v.u2;
-                } else {
-#pragma unroll
-                    for (int i = 0; i < 4; ++i)
-                        if (n0 + 4 * g + i < N) o[i].bits = float_to_bf16_bits(acc[i] * mul[i]);
-                }
+                heads_store4(out + (size_t)t * o_row + (size_t)h * o_head + n0 + 4 * g, acc, gmul, gate, t, h, n0 + 4 * g, N,
+                             (o_row | o_head) % 4 == 0);
             }
         }
     }
 }
 
+// Many rows: a workgroup takes 32 RT rows and 128 outputs of one head, operands through LDS (lds_product.h).
+#include "lds_product.h"
+
+template <int RT>
+__global__ void __launch_bounds__(256)
+heads_matmul_lds_kernel(bf16_t *__restrict__ out, int o_row, int o_head, const bf16_t *__restrict__ x, int x_row, int x_head,
+                        const bf16_t *__restrict__ w, int M, int N, int K, int n_blocks, int m_blocks, HeadsGate gate, HeadsRotate ro) {
+    __shared__ __align__(16) typename LdsProduct<RT>::Shared shared;
+    constexpr int ROWS = LdsProduct<RT>::ROWS;
+    const int cols = n_blocks + (ro.rot > 0 ? 1 : 0);           // the last column of workgroups rotates
+    const int id = die_order(blockIdx.x, gridDim.x);
+    const int h = id / (cols * m_blocks), m0 = (id / cols) % m_blocks * ROWS, col = id % cols;
+    if (col == n_blocks) {
+        heads_rotate<bf16_t>(ro, h, m0, min(M, m0 + ROWS));
+        return;
+    }
+    const int n0 = col * LDSP_N;
+    const int lane = threadIdx.x % KVA_WAVE, wave = threadIdx.x / KVA_WAVE, r = lane & 15, g = lane >> 4;
+    LdsProduct<RT> p;
+#pragma unroll
+    for (int i = 0; i < LdsProduct<RT>::XI; ++i)
+        p.xp[i] = x + (size_t)min(m0 + p.row() + 32 * i, M - 1) * x_row + (size_t)h * x_head + p.element();
+    p.plain_w(w + (size_t)h * N * K, N, K, n0);
+    f32x4 acc[4][RT];
+    p.run(shared, K, acc);
+    // Results go out 16 bytes a lane, 256 neighbouring bytes a row: through LDS, where the operands were (a lane
+    // holds 4 outputs of a row).  Rows that are not aligned for that are written as they are.
+    constexpr int OUT_STRIDE = LDSP_N + 8;
+    static_assert(sizeof(shared) >= ROWS * OUT_STRIDE * sizeof(bf16_t), "the results fit where the operands were");
+    const bool through = (o_row | o_head | N) % 8 == 0 && (reinterpret_cast<uintptr_t>(out) & 15) == 0;
+    bf16_t *tile = shared.x[0];
+    if (through) __syncthreads();                               // nobody reads the operands any more
+#pragma unroll
+    for (int rt = 0; rt < RT; ++rt) {
+        const int row = (wave & 1) * 16 * RT + 16 * rt + r, t = m0 + row;
+        if (t >= M) continue;
+        const float gmul = gate.p && !gate.per_element ? heads_gate<bf16_t>(gate, t, h, 0) : 1.f;
+#pragma unroll
+        for (int nt = 0; nt < 4; ++nt) {
+            const int c = 64 * (wave >> 1) + 16 * nt + 4 * g, n = n0 + c;
+            if (n >= N) continue;
+            bf16_t *o = through ? tile + row * OUT_STRIDE + c : out + (size_t)t * o_row + (size_t)h * o_head + n;
+            heads_store4(o, acc[nt][rt], gmul, gate, t, h, n, N, through || (o_row | o_head) % 4 == 0);
+        }
+    }
+    if (!through) return;
+    __syncthreads();
+    const int c = 8 * (threadIdx.x % 16);
+    if (n0 + c >= N) return;
+    for (int row = threadIdx.x / 16; row < ROWS && m0 + row < M; row += 16)
+        *reinterpret_cast<uint4 *>(out + (size_t)(m0 + row) * o_row + (size_t)h * o_head + n0 + c) =
+            *reinterpret_cast<const uint4 *>(tile + row * OUT_STRIDE + c);
+}
+
+#define HM_LDS_ROWS 128         // more rows than this go through LDS
 #define HM_INSTANCES(X) X(1) X(2) X(3) X(4) X(5) X(6) X(8) X(10) X(12) X(16)
 
 extern "C" int kva_heads_matmul_mfma_supported(int K, int x_row, int x_head) {
@@ -266,6 +327,19 @@ extern "C" int kva_heads_matmul_mfma(void *out, int o_row, int o_head, const voi
                 "heads_matmul_mfma: strides do not fit %d heads of %d -> %d", heads, K, N);
     HEADS_OPTIONS(gate, ro);
     if (rows == 0) return KVA_OK;
+    if (rows > HM_LDS_ROWS && N >= 64) {
+        const int n_blocks = (N + LDSP_N - 1) / LDSP_N, cols = n_blocks + (rot > 0 ? 1 : 0);
+        // the smaller tile where the larger would leave compute units without work
+        const bool small = (long long)n_blocks * heads * ((rows + 127) / 128) < 512;
+        const int tile = small ? 64 : 128, m_blocks = (rows + tile - 1) / tile;
+        const long long blocks = (long long)cols * m_blocks * heads;
+        KVA_REQUIRE(blocks <= 0x7fffffff, "heads_matmul_mfma: too many workgroups");
+        auto kernel = small ? heads_matmul_lds_kernel<2> : heads_matmul_lds_kernel<4>;
+        hipLaunchKernelGGL(kernel, dim3((unsigned)blocks), dim3(256), 0, stream, (bf16_t *)out, o_row, o_head, (const bf16_t *)x, x_row,
+                           x_head, (const bf16_t *)w, rows, N, K, n_blocks, m_blocks, gate, ro);
+        KVA_CHECK_LAUNCH("heads_matmul_mfma");
+        return KVA_OK;
+    }
     const int row_tiles = (rows + 15) / 16;
     const int n_tiles = (N + 15) / 16;
     // many rows: several output tiles a wavefront (at most 32 fragments of W in its registers)

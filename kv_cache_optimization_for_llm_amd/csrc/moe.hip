@@ -23,6 +23,7 @@
 // share its tile: the same token gives the same numbers in any batch.
 #include "common.h"
 #include "attention_frag.h"
+#include "lds_product.h"
 #include <math.h>
 
 #define MOE_TILE 16
@@ -479,88 +480,29 @@ moe_expert_rows_mfma_kernel(MoeRows a, void *__restrict__ out, int out_dtype, co
 }
 
 // matrix cores, many rows an expert: a workgroup takes a group of 2 RT tiles of one expert (32 RT rows) and 128
-// outputs, a wavefront half of either.  64 elements of K of both operands go through LDS at a time, two deep
-// (the next ones' loads are in flight while these are multiplied), in rows padded so that a fragment's 16
-// lanes lie on banks of their own.  K is added in ascending order.  Workgroups that follow each other in the
-// work list run on one of the 8 dies (the hardware deals them out in turn), so that a die reads few experts.
-#define MOE_LDS_K 64
-#define MOE_LDS_STRIDE 72
-#define MOE_LDS_N 128
+// outputs, operands through LDS (lds_product.h).  A die reads few experts.
 template <int RT>
 __global__ void __launch_bounds__(256)
 moe_expert_rows_lds_kernel(MoeRows a, void *__restrict__ out, int out_dtype, const bf16_t *__restrict__ x,
                            const bf16_t *__restrict__ w, int n_blocks) {
-    constexpr int ROWS = 32 * RT, XI = ROWS * MOE_LDS_K / 8 / 256, WI = MOE_LDS_N * MOE_LDS_K / 8 / 256;
-    __shared__ __align__(16) bf16_t xs[2][ROWS * MOE_LDS_STRIDE], ws[2][MOE_LDS_N * MOE_LDS_STRIDE];
-    const int total = gridDim.x, die = blockIdx.x % 8, q = total / 8, rem = total % 8;
-    const int id = die * q + min(die, rem) + (int)blockIdx.x / 8;
-    const int first = (id / n_blocks) * 2 * RT, n0 = (id % n_blocks) * MOE_LDS_N;
+    __shared__ __align__(16) typename LdsProduct<RT>::Shared shared;
+    const int id = die_order(blockIdx.x, gridDim.x);
+    const int first = (id / n_blocks) * 2 * RT, n0 = (id % n_blocks) * LDSP_N;
     const int e = a.tile_expert[first];
     if (e < 0) return;
     const int lane = threadIdx.x % KVA_WAVE, wave = threadIdx.x / KVA_WAVE, r = lane & 15, g = lane >> 4;
     const int wr = wave & 1, wn = wave >> 1;
-    // 16 bytes at a time: thread t takes elements 8 (t % 8) .. of rows t / 8 + 32 i
-    const int kc = 8 * (threadIdx.x % 8), srow = threadIdx.x / 8;
-    const bf16_t *xp[XI], *wp[WI];
+    LdsProduct<RT> p;
 #pragma unroll
-    for (int i = 0; i < XI; ++i) {
-        const int place = first * MOE_TILE + srow + 32 * i, slot = a.sorted_slot[place];
-        xp[i] = x + (a.mode == 0 ? (size_t)(slot < 0 ? 0 : slot / a.top) : (size_t)place) * a.K + kc;
+    for (int i = 0; i < LdsProduct<RT>::XI; ++i) {
+        const int place = first * MOE_TILE + p.row() + 32 * i, slot = a.sorted_slot[place];
+        p.xp[i] = x + (a.mode == 0 ? (size_t)(slot < 0 ? 0 : slot / a.top) : (size_t)place) * a.K + p.element();
     }
-    // ... and of a matrix in operand order the piece of lane t % 64 of one of its tiles of 16 x 32, which is neighbouring bytes
-    int wat[WI], wkc[WI];               // where a piece goes in LDS, and its first element of the 64
-#pragma unroll
-    for (int i = 0; i < WI; ++i) {
-        const int f = wave + 4 * i, nt = f >> 1;
-        const int row = a.tiled ? 16 * nt + r : srow + 32 * i;
-        wkc[i] = a.tiled ? 32 * (f & 1) + 8 * g : kc;
-        wat[i] = row * MOE_LDS_STRIDE + wkc[i];
-        wp[i] = w + (a.tiled ? ((size_t)e * a.N + min(n0 + 16 * nt, a.N - 16)) * a.K + (f & 1) * 16 * 32 + 8 * lane
-                             : ((size_t)e * a.N + min(n0 + row, a.N - 1)) * a.K + kc);
-    }
-    const int wmul = a.tiled ? 16 : 1;  // elements of a matrix's storage a step of one element of K moves on by
-    uint4 xv[XI], wv[WI];
-#define MOE_LDS_LOAD(K0)                                                                                              \
-    {                                                                                                                 \
-        const bool in = (K0) + kc < a.K;                                                                              \
-        _Pragma("unroll") for (int i = 0; i < XI; ++i)                                                                \
-            xv[i] = in ? *reinterpret_cast<const uint4 *>(xp[i] + (K0)) : make_uint4(0u, 0u, 0u, 0u);                  \
-        _Pragma("unroll") for (int i = 0; i < WI; ++i)                                                                \
-            wv[i] = (K0) + wkc[i] < a.K ? *reinterpret_cast<const uint4 *>(wp[i] + (K0) * wmul) : make_uint4(0u, 0u, 0u, 0u); \
-    }
+    const bf16_t *we = w + (size_t)e * a.N * a.K;
+    if (a.tiled) p.tiled_w(we, a.N, a.K, n0);
+    else p.plain_w(we, a.N, a.K, n0);
     f32x4 acc[4][RT];
-#pragma unroll
-    for (int nt = 0; nt < 4; ++nt)
-#pragma unroll
-        for (int rt = 0; rt < RT; ++rt) acc[nt][rt] = f32x4{0.f, 0.f, 0.f, 0.f};
-    MOE_LDS_LOAD(0)
-    int buf = 0;
-    for (int k0 = 0; k0 < a.K; k0 += MOE_LDS_K, buf ^= 1) {
-#pragma unroll
-        for (int i = 0; i < XI; ++i) *reinterpret_cast<uint4 *>(&xs[buf][(srow + 32 * i) * MOE_LDS_STRIDE + kc]) = xv[i];
-#pragma unroll
-        for (int i = 0; i < WI; ++i) *reinterpret_cast<uint4 *>(&ws[buf][wat[i]]) = wv[i];
-        __syncthreads();                // (a buffer was read last two turns ago: every wavefront has passed the barrier between)
-        if (k0 + MOE_LDS_K < a.K) MOE_LDS_LOAD(k0 + MOE_LDS_K)
-        const bf16_t *xr = &xs[buf][(wr * 16 * RT + r) * MOE_LDS_STRIDE + 8 * g], *wrow = &ws[buf][(wn * 64 + r) * MOE_LDS_STRIDE + 8 * g];
-        Frag8 xf[2][RT], wf[2][4];
-#pragma unroll
-        for (int ks = 0; ks < 2; ++ks) {
-#pragma unroll
-            for (int nt = 0; nt < 4; ++nt) wf[ks][nt].u4 = *reinterpret_cast<const uint4 *>(wrow + nt * 16 * MOE_LDS_STRIDE + 32 * ks);
-#pragma unroll
-            for (int rt = 0; rt < RT; ++rt) xf[ks][rt].u4 = *reinterpret_cast<const uint4 *>(xr + rt * 16 * MOE_LDS_STRIDE + 32 * ks);
-        }
-        __builtin_amdgcn_sched_barrier(0);
-#pragma unroll
-        for (int ks = 0; ks < 2; ++ks)
-#pragma unroll
-            for (int nt = 0; nt < 4; ++nt)
-#pragma unroll
-                for (int rt = 0; rt < RT; ++rt)
-                    acc[nt][rt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[ks][nt].v, xf[ks][rt].v, acc[nt][rt], 0, 0, 0);
-    }
-#undef MOE_LDS_LOAD
+    p.run(shared, a.K, acc);
     // lane (row r, group g) holds outputs 4 g .. 4 g + 3 of tile nt, of its row of tile rt
 #pragma unroll
     for (int rt = 0; rt < RT; ++rt) {
@@ -608,7 +550,7 @@ extern "C" int kva_moe_expert_rows(void *out, int out_dtype, const void *x, cons
     if (max_tiles == 0) return KVA_OK;
     MoeRows a{sorted_slot, tile_expert, slot_weight, top, N, K, mode, act, tiled, gated, limit};
     if (group > 1) {
-        const int n_blocks = (N + MOE_LDS_N - 1) / MOE_LDS_N;
+        const int n_blocks = (N + LDSP_N - 1) / LDSP_N;
         const long long blocks = (long long)n_blocks * (max_tiles / group);
         KVA_REQUIRE(blocks <= 0x7fffffff, "moe_expert_rows: too many workgroups");
         if (group == 8)

@@ -176,6 +176,25 @@ def test_per_head_products_with_a_gate_per_element(heads, n, k, rows, dtype, gpu
     close(out.view(rows, heads, n), want, TOL[dtype], "gate per head")
 
 
+@pytest.mark.parametrize("heads, n, k, rot", [(36, 264, 96, 0), (36, 260, 32, 0), (40, 130, 64, 6), (130, 128, 160, 4)])
+def test_per_head_products_of_many_rows_and_heads(heads, n, k, rot, gpu):
+    """Enough work for the larger of the two tiles: rows and outputs that end inside one, outputs whose rows are
+    not aligned for 16 bytes, a rotation in the same launch, and rows cut from a wider buffer."""
+    rows = 517
+    x, w = rnd((rows, heads, k + 8), 1, torch.bfloat16), rnd((heads, n, k), 2, torch.bfloat16, k ** -0.5)
+    out = torch.full((rows + 1, heads, n + rot), float("nan"), dtype=torch.bfloat16, device=gpu)
+    dev, turn = x.to(gpu), None
+    if rot:
+        cos, sin = RotaryEncoding(head_dim=rot, max_positions=600, theta=60.0, frequencies="plain_f64", pairing="interleaved").tables(gpu)
+        turn = (dev[:, :, k:k + rot], out[:rows, :, n:], cos, sin, torch.arange(rows, dtype=torch.int32, device=gpu), True)
+    lat_ops.heads_product(dev[:, :, :k], w.to(gpu), out[:rows, :, :n], rotate=turn)
+    want = torch.matmul(x[..., :k].double().transpose(0, 1).contiguous(), w.double().transpose(1, 2).contiguous()).transpose(0, 1)
+    close(out[:rows, :, :n], want, TOL["bfloat16"], "product")
+    if rot:
+        close(out[:rows, :, n:], plain.rotate_pairs(x[..., k:k + rot].double(), 60.0), TOL["bfloat16"], "rotation")
+    assert out[rows].isnan().all()                                  # nothing behind the last row
+
+
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 @pytest.mark.parametrize("interleaved", [True, False])
 @pytest.mark.parametrize("rows, heads, plain_dim, rot, rank", [(1, 3, 12, 8, 40), (1, 1, 32, 2, 16), (37, 5, 64, 32, 96),
