@@ -13,7 +13,8 @@
 //  * kva_moe_expert_rows: one product per tile against its expert's matrix.  Mode 0 ("up"): rows of
 //    x gathered by slot / top, activation applied (a gated expert: act(gate) * up, its gate and up rows
 //    interleaved in one matrix), written at the sorted position.  Mode 1 ("down"):
-//    rows at the sorted position, times the slot's routing weight, written at the slot (fp32).
+//    rows at the sorted position, times the slot's routing weight, written at the slot (fp32).  The weight may
+//    stand on the expert's input instead: it then multiplies the first product's rows, before the activation.
 //    bf16 with K % 32 == 0 runs on the matrix cores (with many rows an expert through LDS, in groups of
 //    tiles), everything else (fp32 too) on a plain tiled kernel that adds k ascending.
 //  * kva_moe_combine: out[t] = sum over the token's choices of the slot's row, or, for a router
@@ -304,7 +305,7 @@ extern "C" int kva_moe_table_align(int *sorted_slot, int *tile_expert, int *idx,
 // ---- one product per tile ------------------------------------------------------------------
 struct MoeRows {
     const int *sorted_slot, *tile_expert;
-    const float *slot_weight;       // mode 1
+    const float *slot_weight;       // mode 1: of the row that is written; mode 0 (optional): of the row that is read
     int top, N, K, mode, act;
     int tiled;                      // the matrices lie in operand order: [N / 16][K / 32][lane][8] (lane = 16 (k % 32 / 8) + n % 16)
     int gated;                      // mode 0: rows 2 j and 2 j + 1 of the matrix are output j's gate and up rows
@@ -312,7 +313,12 @@ struct MoeRows {
 };
 
 // mode 0 of a gated expert: outputs n (even) and n + 1 of the product are one output of the layer
-__device__ inline void moe_store_gated(const MoeRows &a, void *out, int out_dtype, int place, int n, float gate, float up) {
+// (a weight on the expert's input multiplies both of them in front of the activation: W (w x) = w (W x))
+__device__ inline void moe_store_gated(const MoeRows &a, void *out, int out_dtype, int place, int slot, int n, float gate, float up) {
+    if (a.slot_weight) {
+        gate *= a.slot_weight[slot];
+        up *= a.slot_weight[slot];
+    }
     const float v = a.act == 4 ? kva_gated_activate(gate, up, KVA_ACT_SWISH_CLAMPED, a.limit) : moe_activate(gate, a.act) * up;
     const size_t at = (size_t)place * (a.N / 2) + n / 2;
     if (out_dtype == KVA_BF16) reinterpret_cast<uint16_t *>(out)[at] = float_to_bf16_bits(v);
@@ -321,11 +327,12 @@ __device__ inline void moe_store_gated(const MoeRows &a, void *out, int out_dtyp
 
 __device__ inline void moe_store(const MoeRows &a, void *out, int out_dtype, int place, int slot, int n, float v) {
     if (a.mode == 0) {
+        if (a.slot_weight) v *= a.slot_weight[slot];
         v = moe_activate(v, a.act);
         if (out_dtype == KVA_BF16) reinterpret_cast<uint16_t *>(out)[(size_t)place * a.N + n] = float_to_bf16_bits(v);
         else reinterpret_cast<float *>(out)[(size_t)place * a.N + n] = v;
     } else {
-        reinterpret_cast<float *>(out)[(size_t)slot * a.N + n] = v * a.slot_weight[slot];
+        reinterpret_cast<float *>(out)[(size_t)slot * a.N + n] = a.slot_weight ? v * a.slot_weight[slot] : v;
     }
 }
 
@@ -365,7 +372,7 @@ moe_expert_rows_kernel(MoeRows a, void *__restrict__ out, int out_dtype, const T
 #pragma unroll
         for (int j = 0; j < 4; j += 2) {
             const int n = n0 + 4 * cx + j;
-            if (n + 1 < a.N) moe_store_gated(a, out, out_dtype, place, n, acc[j], acc[j + 1]);
+            if (n + 1 < a.N) moe_store_gated(a, out, out_dtype, place, slot, n, acc[j], acc[j + 1]);
         }
         return;
     }
@@ -448,8 +455,8 @@ __device__ inline void moe_tiles_product(const MoeRows &a, void *__restrict__ ou
                        + red[(2 * NT + nt) * RT + rt][lane][i];
             const int n = n_first + 16 * nt + 4 * g;
             if (a.gated) {
-                if (n + 1 < a.N) moe_store_gated(a, out, out_dtype, place[rt], n, v[0], v[1]);
-                if (n + 3 < a.N) moe_store_gated(a, out, out_dtype, place[rt], n + 2, v[2], v[3]);
+                if (n + 1 < a.N) moe_store_gated(a, out, out_dtype, place[rt], slot[rt], n, v[0], v[1]);
+                if (n + 3 < a.N) moe_store_gated(a, out, out_dtype, place[rt], slot[rt], n + 2, v[2], v[3]);
             } else {
 #pragma unroll
                 for (int i = 0; i < 4; ++i)
@@ -508,7 +515,7 @@ moe_expert_rows_lds_kernel(MoeRows a, void *__restrict__ out, int out_dtype, con
     for (int rt = 0; rt < RT; ++rt) {
         const int place = first * MOE_TILE + (wr * RT + rt) * 16 + r, slot = a.sorted_slot[place];
         if (slot < 0) continue;
-        const float weight = a.mode == 1 ? a.slot_weight[slot] : 1.f;
+        const float weight = a.mode == 1 && a.slot_weight ? a.slot_weight[slot] : 1.f;
 #pragma unroll
         for (int nt = 0; nt < 4; ++nt) {
             const int n = n0 + wn * 64 + nt * 16 + 4 * g;
@@ -518,8 +525,8 @@ moe_expert_rows_lds_kernel(MoeRows a, void *__restrict__ out, int out_dtype, con
                     *reinterpret_cast<float4 *>(reinterpret_cast<float *>(out) + (size_t)slot * a.N + n) =
                         make_float4(v[0] * weight, v[1] * weight, v[2] * weight, v[3] * weight);
             } else if (a.gated) {
-                if (n + 1 < a.N) moe_store_gated(a, out, out_dtype, place, n, v[0], v[1]);
-                if (n + 3 < a.N) moe_store_gated(a, out, out_dtype, place, n + 2, v[2], v[3]);
+                if (n + 1 < a.N) moe_store_gated(a, out, out_dtype, place, slot, n, v[0], v[1]);
+                if (n + 3 < a.N) moe_store_gated(a, out, out_dtype, place, slot, n + 2, v[2], v[3]);
             } else {
 #pragma unroll
                 for (int i = 0; i < 4; ++i)
@@ -542,8 +549,8 @@ extern "C" int kva_moe_expert_rows(void *out, int out_dtype, const void *x, cons
     KVA_REQUIRE(act != 4 || gated, "moe_expert_rows: the clamped activation is a gated one");
     KVA_REQUIRE(!gated || (mode == 0 && N % 2 == 0), "moe_expert_rows: gate and up rows come in pairs, in the first product");
     KVA_REQUIRE(out && x && w && sorted_slot && tile_expert, "moe_expert_rows: missing operand");
-    KVA_REQUIRE(mode == 0 || (mode == 1 && slot_weight && out_dtype == KVA_F32),
-                "moe_expert_rows: mode 1 writes fp32 rows times a weight per slot");
+    // slot_weight: in mode 1 of the row that is written, in mode 0 of the row that is read; absent: 1
+    KVA_REQUIRE(mode == 0 || (mode == 1 && out_dtype == KVA_F32), "moe_expert_rows: mode 1 writes fp32 rows");
     KVA_REQUIRE(mode == 1 || out_dtype == dtype, "moe_expert_rows: mode 0 writes rows of the operands' type");
     KVA_REQUIRE(N > 0 && K > 0 && top > 0 && act >= 0 && act <= 5, "moe_expert_rows: bad sizes or activation");
     KVA_REQUIRE(max_tiles >= 0 && max_tiles <= 65535, "moe_expert_rows: %d tiles are too many for one launch", max_tiles);

@@ -707,10 +707,21 @@ extern "C" int kva_gated_linear_attention(float *out, float *state, long long se
 // ---- per-head norm and gate ----------------------------------------------------------------
 // out[t, out_off + h dv + j] = (x[t, h, j] / sqrt(mean_j x^2 + eps) * w[j], or x as it is without a
 // weight) * act(gate[t, gate_off + h dv + j]) * mul;  act: 0 silu, 1 sigmoid.  One wavefront a head.
+// gate_first: the gate multiplies what is normed, n(x * act(gate)), instead of the norm's result.
+struct HeadGate {
+    const void *p;
+    int dtype, stride, off, act, first;
+    __device__ float at(size_t t, int i) const {
+        if (!p) return 1.f;
+        const float g = rec_ld(p, dtype, t * stride + off + i);
+        return act == 1 ? rec_sigmoid(g) : rec_silu(g);
+    }
+};
+
 __global__ void __launch_bounds__(256)
 head_norm_gate_kernel(void *__restrict__ out, int out_dtype, int out_stride, int out_off, const void *__restrict__ x,
-                      int x_dtype, const float *__restrict__ w, float eps, const void *__restrict__ gate,
-                      int gate_dtype, int gate_stride, int gate_off, int heads, int dv, int act, float mul, int w_stride) {
+                      int x_dtype, const float *__restrict__ w, float eps, HeadGate gate, int heads, int dv, float mul,
+                      int w_stride) {
     const size_t t = blockIdx.x;
     const int lane = threadIdx.x % KVA_WAVE, wave = threadIdx.x / KVA_WAVE, waves = blockDim.x / KVA_WAVE;
     for (int h = wave; h < heads; h += waves) {
@@ -719,18 +730,18 @@ head_norm_gate_kernel(void *__restrict__ out, int out_dtype, int out_stride, int
         if (w) {
             float sq = 0.f;
             for (int j = lane; j < dv; j += KVA_WAVE) {
-                const float v = rec_ld(x, x_dtype, base + j);
+                float v = rec_ld(x, x_dtype, base + j);
+                if (gate.first) v *= gate.at(t, h * dv + j);
                 sq += v * v;
             }
             inv = 1.0f / sqrtf(wave_sum(sq) / (float)dv + eps);
         }
         for (int j = lane; j < dv; j += KVA_WAVE) {
             float v = rec_ld(x, x_dtype, base + j);
+            const float g = gate.at(t, h * dv + j);
+            if (gate.first) v *= g;
             if (w) v = v * inv * w[(size_t)h * w_stride + j];
-            if (gate) {
-                const float g = rec_ld(gate, gate_dtype, t * gate_stride + gate_off + h * dv + j);
-                v *= (act == 1 ? rec_sigmoid(g) : rec_silu(g));
-            }
+            if (!gate.first) v *= g;
             v *= mul;
             rec_st(out, out_dtype, t * out_stride + out_off + h * dv + j, v);
         }
@@ -741,8 +752,8 @@ head_norm_gate_kernel(void *__restrict__ out, int out_dtype, int out_stride, int
 // all its wavefronts on each; the sum of squares is taken in a fixed order.
 __global__ void __launch_bounds__(256)
 head_norm_gate_wide_kernel(void *__restrict__ out, int out_dtype, int out_stride, int out_off, const void *__restrict__ x,
-                           int x_dtype, const float *__restrict__ w, float eps, const void *__restrict__ gate,
-                           int gate_dtype, int gate_stride, int gate_off, int heads, int dv, int act, float mul, int w_stride) {
+                           int x_dtype, const float *__restrict__ w, float eps, HeadGate gate, int heads, int dv, float mul,
+                           int w_stride) {
     __shared__ float red_s[4];
     const size_t t = blockIdx.x;
     for (int h = 0; h < heads; ++h) {
@@ -751,18 +762,18 @@ head_norm_gate_wide_kernel(void *__restrict__ out, int out_dtype, int out_stride
         if (w) {
             float sq = 0.f;
             for (int j = threadIdx.x; j < dv; j += blockDim.x) {
-                const float v = rec_ld(x, x_dtype, base + j);
+                float v = rec_ld(x, x_dtype, base + j);
+                if (gate.first) v *= gate.at(t, h * dv + j);
                 sq += v * v;
             }
             inv = 1.0f / sqrtf(block_sum(sq, red_s, blockDim.x / KVA_WAVE) / (float)dv + eps);
         }
         for (int j = threadIdx.x; j < dv; j += blockDim.x) {
             float v = rec_ld(x, x_dtype, base + j);
+            const float g = gate.at(t, h * dv + j);
+            if (gate.first) v *= g;
             if (w) v = v * inv * w[(size_t)h * w_stride + j];
-            if (gate) {
-                const float g = rec_ld(gate, gate_dtype, t * gate_stride + gate_off + h * dv + j);
-                v *= (act == 1 ? rec_sigmoid(g) : rec_silu(g));
-            }
+            if (!gate.first) v *= g;
             v *= mul;
             rec_st(out, out_dtype, t * out_stride + out_off + h * dv + j, v);
         }
@@ -771,19 +782,21 @@ head_norm_gate_wide_kernel(void *__restrict__ out, int out_dtype, int out_stride
 
 extern "C" int kva_head_norm_gate(void *out, int out_dtype, int out_stride, int out_off, const void *x, int x_dtype,
                                   const float *w, float eps, const void *gate, int gate_dtype, int gate_stride,
-                                  int gate_off, int rows, int heads, int dv, int act, float mul, int w_stride,
+                                  int gate_off, int rows, int heads, int dv, int act, int gate_first, float mul, int w_stride,
                                   hipStream_t stream) {
     // w_stride: 0 - one weight of dv elements shared by the heads; dv - a weight of heads * dv elements.  gate may be absent.
     KVA_REQUIRE(out && x && heads > 0 && dv > 0 && rows >= 0, "head_norm_gate: missing operand or bad sizes");
     KVA_REQUIRE(w_stride == 0 || w_stride == dv, "head_norm_gate: a weight is shared by the heads or has all heads' size");
     KVA_REQUIRE(act == 0 || act == 1, "head_norm_gate: activation %d is neither silu (0) nor sigmoid (1)", act);
+    KVA_REQUIRE(!gate_first || gate, "head_norm_gate: a gate in front of the norm needs the gate");
     if (rows == 0) return KVA_OK;
+    const HeadGate hg{gate, gate_dtype, gate_stride, gate_off, act, gate_first};
     if (heads < 4 && dv >= 256)
         hipLaunchKernelGGL(head_norm_gate_wide_kernel, dim3(rows), dim3(256), 0, stream, out, out_dtype, out_stride, out_off,
-                           x, x_dtype, w, eps, gate, gate_dtype, gate_stride, gate_off, heads, dv, act, mul, w_stride);
+                           x, x_dtype, w, eps, hg, heads, dv, mul, w_stride);
     else
         hipLaunchKernelGGL(head_norm_gate_kernel, dim3(rows), dim3(256), 0, stream, out, out_dtype, out_stride, out_off, x,
-                           x_dtype, w, eps, gate, gate_dtype, gate_stride, gate_off, heads, dv, act, mul, w_stride);
+                           x_dtype, w, eps, hg, heads, dv, mul, w_stride);
     KVA_CHECK_LAUNCH("head_norm_gate");
     return KVA_OK;
 }

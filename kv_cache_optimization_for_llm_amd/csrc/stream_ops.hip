@@ -842,3 +842,168 @@ extern "C" int kva_sandwich_step(float *x, const void *y, int y_dtype, const voi
     KVA_CHECK_LAUNCH("sandwich_step");
     return KVA_OK;
 }
+
+// ---- tanh norms on both sides of a branch ------------------------------------------------------------
+// A norm without statistics, n(v) = tanh(alpha v) w + b with one number alpha: what lies between two branches is
+// then element by element,
+//     x <- x + n_post(y + y_bias),    out = n_pre(x),
+// over the residual stream x [rows, width] fp32; y_bias (fp32, optional) is the bias of the product that made y.
+// Without y the stream is only read; without `out` it is only updated.  With row_idx only the named rows are
+// read, and nothing is written back: the model's last norm.  A thread takes 4 neighbouring elements of a row
+// (VEC) or one.
+struct TanhNorm {
+    const void *w, *b;
+    int dtype;
+    float alpha;
+};
+
+template <bool VEC>
+__global__ void __launch_bounds__(256)
+tanh_step_kernel(float *__restrict__ x, const void *__restrict__ y, int y_dtype, const float *__restrict__ y_bias,
+                 TanhNorm post, TanhNorm pre, void *__restrict__ out, int out_dtype, const int *__restrict__ row_idx,
+                 int width, size_t n) {
+    constexpr int W = VEC ? 4 : 1;
+    const size_t i = ((size_t)blockIdx.x * blockDim.x + threadIdx.x) * W;
+    if (i >= n) return;
+    const size_t r = i / width;
+    const int j = (int)(i % width);
+    const size_t at = row_idx ? (size_t)row_idx[r] * width + j : i;
+    float v[W], yv[W], yb[W], pw[W], pb[W], nw[W], nb[W];
+    auto load = [&](const void *p, int dtype, size_t k, float (&f)[W]) {
+        if constexpr (VEC) hyper_ld4(p, dtype, k, f);
+        else f[0] = ld_as_float(p, dtype, k);
+    };
+#pragma unroll
+    for (int e = 0; e < W; ++e) yv[e] = yb[e] = pw[e] = pb[e] = nw[e] = nb[e] = 0.f;
+    load(x, KVA_F32, at, v);
+    if (y) {
+        load(y, y_dtype, at, yv);
+        if (y_bias) load(y_bias, KVA_F32, j, yb);
+        if (post.w) {
+            load(post.w, post.dtype, j, pw);
+            load(post.b, post.dtype, j, pb);
+        }
+    }
+    if (out) {
+        load(pre.w, pre.dtype, j, nw);
+        load(pre.b, pre.dtype, j, nb);
+    }
+    if (y) {
+#pragma unroll
+        for (int e = 0; e < W; ++e) v[e] += post.w ? tanhf(post.alpha * (yv[e] + yb[e])) * pw[e] + pb[e] : yv[e] + yb[e];
+        if (!row_idx) {
+            if constexpr (VEC) *reinterpret_cast<float4 *>(x + at) = make_float4(v[0], v[1], v[2], v[3]);
+            else x[at] = v[0];
+        }
+    }
+    if (!out) return;
+    float o[W];
+#pragma unroll
+    for (int e = 0; e < W; ++e) o[e] = tanhf(pre.alpha * v[e]) * nw[e] + nb[e];
+    if constexpr (VEC) {
+        if (out_dtype == KVA_F32)
+            *reinterpret_cast<float4 *>(reinterpret_cast<float *>(out) + i) = make_float4(o[0], o[1], o[2], o[3]);
+        else
+            *reinterpret_cast<uint2 *>(reinterpret_cast<uint16_t *>(out) + i) =
+                make_uint2((uint32_t)float_to_bf16_bits(o[0]) | ((uint32_t)float_to_bf16_bits(o[1]) << 16),
+                           (uint32_t)float_to_bf16_bits(o[2]) | ((uint32_t)float_to_bf16_bits(o[3]) << 16));
+    } else {
+        st_from_float(out, out_dtype, i, o[0]);
+    }
+}
+
+extern "C" int kva_tanh_step(float *x, const void *y, int y_dtype, const float *y_bias, const void *post_w, const void *post_b,
+                             int post_dtype, float post_alpha, const void *pre_w, const void *pre_b, int pre_dtype,
+                             float pre_alpha, void *out, int out_dtype, const int *row_idx, int rows, int width,
+                             hipStream_t stream) {
+    KVA_REQUIRE(x && rows >= 0 && width > 0, "tanh_step: missing operand or bad sizes");
+    KVA_REQUIRE(y || (!post_w && !y_bias), "tanh_step: a norm or a bias without the branch output it goes with");
+    KVA_REQUIRE((post_w == nullptr) == (post_b == nullptr) && (pre_w == nullptr) == (pre_b == nullptr),
+                "tanh_step: a norm has a weight and a bias");
+    KVA_REQUIRE(!out || pre_w, "tanh_step: the read-out needs a norm");
+    KVA_REQUIRE(y || out, "tanh_step: nothing to do");
+    KVA_REQUIRE(!row_idx || out, "tanh_step: rows are gathered for the read-out only");
+    if (rows == 0) return KVA_OK;
+    const TanhNorm post{post_w, post_b, post_dtype, post_alpha}, pre{pre_w, pre_b, pre_dtype, pre_alpha};
+    const size_t n = (size_t)rows * width;
+    const bool vec = width % 4 == 0 && aligned16(x) && aligned16(y) && aligned16(y_bias) && aligned16(post_w) &&
+                     aligned16(post_b) && aligned16(pre_w) && aligned16(pre_b) && aligned16(out);
+    if (vec)
+        hipLaunchKernelGGL(tanh_step_kernel<true>, dim3((unsigned)((n / 4 + 255) / 256)), dim3(256), 0, stream, x, y, y_dtype,
+                           y_bias, post, pre, out, out_dtype, row_idx, width, n);
+    else
+        hipLaunchKernelGGL(tanh_step_kernel<false>, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, stream, x, y, y_dtype,
+                           y_bias, post, pre, out, out_dtype, row_idx, width, n);
+    KVA_CHECK_LAUNCH("tanh_step");
+    return KVA_OK;
+}
+
+// ---- an embedding of tokens and of pairs of tokens -------------------------------------------------------
+// x[t] = n(table[id] * scale + pairs[row]), row = (previous id * mul_prev + id * mul_cur) mod buckets, or `buckets`
+// (the table's last row) for a sequence's first token; n is a tanh norm or absent, the pair table is optional.
+// The id in front of an entry's first token is the seat's state: one integer, 0 for none, else id + 1; the
+// workgroup of an entry's first token reads it and leaves the entry's last id there.  A negative id -1 - r
+// stands for feedback[r].  Workgroup: a token.
+struct PairTable {
+    const void *p;
+    int dtype, buckets;
+    long long mul_prev, mul_cur;
+};
+
+__device__ inline int pair_token(const int *ids, const int *feedback, int t, int table_rows) {
+    int id = ids[t];
+    if (id < 0) id = feedback[-1 - id];
+    return id < 0 ? 0 : (id >= table_rows ? table_rows - 1 : id);
+}
+
+__global__ void __launch_bounds__(256)
+pair_embed_kernel(float *__restrict__ x, const void *__restrict__ table, int table_dtype, int table_rows, float scale,
+                  PairTable pairs, TanhNorm norm, const int *__restrict__ ids, const int *__restrict__ feedback,
+                  int *__restrict__ state, int state_stride, const int *__restrict__ entry_q_start,
+                  const int *__restrict__ entry_seat, int entries, int width) {
+    __shared__ int entry_s, prev_s;
+    const int t = blockIdx.x;
+    if (threadIdx.x == 0) entry_s = -1;
+    __syncthreads();
+    for (int e = threadIdx.x; e < entries; e += blockDim.x)
+        if (entry_q_start[e] == t && entry_q_start[e + 1] > t) entry_s = e;      // (one entry at most starts here)
+    __syncthreads();
+    if (threadIdx.x == 0) {
+        const int e = entry_s;
+        if (e < 0) {
+            prev_s = pair_token(ids, feedback, t - 1, table_rows);
+        } else {
+            int *seat = state + (size_t)entry_seat[e] * state_stride;
+            prev_s = *seat - 1;
+            *seat = pair_token(ids, feedback, entry_q_start[e + 1] - 1, table_rows) + 1;
+        }
+    }
+    __syncthreads();
+    const int id = pair_token(ids, feedback, t, table_rows), prev = prev_s;
+    const int row = prev < 0 ? pairs.buckets : (int)((prev * pairs.mul_prev + id * pairs.mul_cur) % pairs.buckets);
+    for (int j = threadIdx.x; j < width; j += blockDim.x) {
+        float v = ld_as_float(table, table_dtype, (size_t)id * width + j) * scale;
+        if (pairs.p) v += ld_as_float(pairs.p, pairs.dtype, (size_t)row * width + j);
+        if (norm.w) v = tanhf(norm.alpha * v) * ld_as_float(norm.w, norm.dtype, j) + ld_as_float(norm.b, norm.dtype, j);
+        x[(size_t)t * width + j] = v;
+    }
+}
+
+extern "C" int kva_pair_embed(float *x, const void *table, int table_dtype, int table_rows, float scale, const void *pair_table,
+                              int pair_dtype, int buckets, int mul_prev, int mul_cur, const void *norm_w, const void *norm_b,
+                              int norm_dtype, float norm_alpha, const int *ids, const int *feedback, int *state,
+                              int state_stride, const int *entry_q_start, const int *entry_seat, int entries, int tokens,
+                              int width, hipStream_t stream) {
+    KVA_REQUIRE(x && table && ids && state && entry_q_start && entry_seat && tokens >= 0 && entries >= 0,
+                "pair_embed: missing operand");
+    KVA_REQUIRE(table_rows > 0 && width > 0 && state_stride > 0 && buckets > 0 && mul_prev >= 0 && mul_cur >= 0,
+                "pair_embed: bad sizes or negative multipliers");
+    KVA_REQUIRE((norm_w == nullptr) == (norm_b == nullptr), "pair_embed: a norm has a weight and a bias");
+    if (tokens == 0) return KVA_OK;
+    hipLaunchKernelGGL(pair_embed_kernel, dim3(tokens), dim3(256), 0, stream, x, table, table_dtype, table_rows, scale,
+                       PairTable{pair_table, pair_dtype, buckets, mul_prev, mul_cur},
+                       TanhNorm{norm_w, norm_b, norm_dtype, norm_alpha}, ids, feedback, state, state_stride, entry_q_start,
+                       entry_seat, entries, width);
+    KVA_CHECK_LAUNCH("pair_embed");
+    return KVA_OK;
+}

@@ -13,7 +13,8 @@ from . import radilix as _radilix   # noqa: F401  (registers Radilix)
 from . import lomodra as _lomodra   # noqa: F401  (registers Lomodra)
 from . import bonusun as _bonusun   # noqa: F401  (registers Bonusun)
 from . import bilolorn as _bilolorn   # noqa: F401  (registers Bilolorn)
-from ..config.registry import (BLOCKS, FEED_FORWARDS, MIXERS, NORMS, STREAM_OPS, architecture_for)
+from . import gokinex as _gokinex   # noqa: F401  (registers Gokinex)
+from ..config.registry import (BLOCKS, EMBEDDINGS, FEED_FORWARDS, MIXERS, NORMS, STREAM_OPS, architecture_for)
 from ..models.spec import LayerCall, ModelSpec, TensorSpec
 from ..ops import kernels as K
 from ..parts.base import Block, KVCacheSpec, KVView, MixerContext, NormedRows, PendingNorm, StateSpec, StreamCopy
@@ -40,8 +41,14 @@ def build_stream_ops(spec: ModelSpec) -> list:
     return [STREAM_OPS.get(ps.kind)(**ps.params) for ps in spec.stream_ops]
 
 
-def model_tensor_specs(spec: ModelSpec, blocks: List[Block], final_norm, stream_ops=()) -> Dict[str, TensorSpec]:
+def build_embedding(spec: ModelSpec):
+    return None if spec.embedding is None else EMBEDDINGS.get(spec.embedding.kind)(**spec.embedding.params)
+
+
+def model_tensor_specs(spec: ModelSpec, blocks: List[Block], final_norm, stream_ops=(), embedding=None) -> Dict[str, TensorSpec]:
     out: Dict[str, TensorSpec] = {spec.embedding_name: TensorSpec((spec.vocab_size, spec.hidden_size))}
+    if embedding is not None:
+        out.update(embedding.tensor_specs())
     groups = [b.parts() for b in blocks] + [tuple(stream_ops)]
     for parts in groups:
         for part in parts:
@@ -60,7 +67,7 @@ def tensor_specs_for_config(config_dict: Mapping[str, Any]) -> Dict[str, TensorS
     _, spec = spec_for_config(config_dict)
     blocks = build_blocks(spec)
     final_norm = NORMS.get(spec.final_norm.kind)(**spec.final_norm.params)
-    return model_tensor_specs(spec, blocks, final_norm, build_stream_ops(spec))
+    return model_tensor_specs(spec, blocks, final_norm, build_stream_ops(spec), build_embedding(spec))
 
 
 def resolve_order(spec: ModelSpec) -> List[Tuple[LayerCall, int]]:
@@ -97,6 +104,14 @@ class Model:
         if int(spec.streams) < 1 or (int(spec.streams) > 1 and self.stream_dtype != torch.float32):
             raise ValueError("several copies of the stream are kept in 32-bit (residual_dtype='float32')")
         self.calls = resolve_order(spec)
+        self.token_input = build_embedding(spec)
+        if self.token_input is not None:
+            if spec.stream_ops or int(spec.streams) > 1:
+                raise ValueError("an embedding part fills a stream of one copy, without operations between layers")
+            if self.token_input.table_name != spec.embedding_name:
+                raise ValueError(f"the embedding part reads {self.token_input.table_name!r}, the model names {spec.embedding_name!r}")
+        # what the embedding keeps per request lies behind the calls' slots
+        self.token_input_slot = 1 + max((slot for _, slot in self.calls), default=-1)
         self.embedding: Optional[torch.Tensor] = None
         self.head: Optional[Linear] = None
 
@@ -130,6 +145,8 @@ class Model:
                 if slot in states and states[slot] != st:
                     raise ValueError(f"state slot {slot} is shared by mixers with different state")
                 states[slot] = st
+        if self.token_input is not None and self.token_input.state_spec() is not None:
+            states[self.token_input_slot] = self.token_input.state_spec()
         for slot, has_writer in slot_writer.items():
             if not has_writer:
                 raise ValueError(f"cache slot {slot} is read but no layer call writes it")
@@ -152,7 +169,7 @@ class Model:
 
     def graph_safe(self) -> bool:
         """Whether every part may be captured into a HIP graph."""
-        parts = [self.final_norm, *self.stream_ops]
+        parts = [self.final_norm, *self.stream_ops, *((self.token_input,) if self.token_input is not None else ())]
         for b in self.blocks:
             parts.append(b)
             parts.extend(b.parts())
@@ -173,10 +190,12 @@ class Model:
 
     # ---- weights
     def tensor_specs(self) -> Dict[str, TensorSpec]:
-        return model_tensor_specs(self.spec, self.blocks, self.final_norm, self.stream_ops)
+        return model_tensor_specs(self.spec, self.blocks, self.final_norm, self.stream_ops, self.token_input)
 
     def load(self, tensors: Dict[str, torch.Tensor]) -> None:
         self.embedding = tensors[self.spec.embedding_name]
+        if self.token_input is not None:
+            self.token_input.load(tensors)
         for b in self.blocks:
             for part in b.parts():
                 part.load(tensors)
@@ -239,7 +258,9 @@ class Model:
         first = {}              # the embedding output once more, for operations between layers that read it
         first_norm = self.blocks[self.calls[0][0].layer].first_norm() if self.calls else self.final_norm
         prep = first_norm.prepared_by_product() if first_norm is not None else None
-        if (T <= self.GATHER_PREP_MAX_ROWS and prep is not None and prep[1] == self.spec.hidden_size
+        if self.token_input is not None:
+            self.token_input.forward(batch, hidden, cache.state.get(self.token_input_slot))
+        elif (T <= self.GATHER_PREP_MAX_ROWS and prep is not None and prep[1] == self.spec.hidden_size
                 and self.dtype == torch.bfloat16 and self.embedding.dtype == torch.bfloat16
                 and self.stream_dtype == torch.bfloat16 and not self.stream_ops and S == 1
                 and self.spec.hidden_size % 8 == 0 and self.spec.embedding_scale == 1.0):

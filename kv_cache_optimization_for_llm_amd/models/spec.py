@@ -80,6 +80,8 @@ class ModelSpec:
     logit_scale: float = 1.0
     logit_softcap: float = 0.0
     eos_token_ids: Tuple[int, ...] = ()
+    # How tokens become the stream's first rows (registry EMBEDDINGS); None: a gather of the token table.
+    embedding: Optional[PartSpec] = None
     # Operations on the stream between layers (registry STREAM_OPS), named by LayerCall.before.
     stream_ops: Tuple[PartSpec, ...] = ()
     # Type the residual stream is kept in: None = the engine's compute type; "float32" keeps the

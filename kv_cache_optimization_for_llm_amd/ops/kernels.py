@@ -596,6 +596,7 @@ ACTIVATIONS = {"silu": 0, "relu": 1, "gelu_tanh": 2, "relu2": 4}        # relu2:
 # gated forms only: act(gate) * up with "swish_clamped" = g sigmoid(1.702 g) (u + 1), g = min(gate, limit),
 # u = clamp(up, -limit, limit)
 GATED_ACTIVATIONS = dict(ACTIVATIONS, swish_clamped=3)
+BIAS_ACTIVATIONS = dict(ACTIVATIONS, none=5)            # bias_act alone: a bias without an activation
 
 
 def table_gate(z: torch.Tensor, table: torch.Tensor, ids: torch.Tensor, col0: int, out: torch.Tensor, activation: str,
@@ -632,14 +633,14 @@ def act_mul(gate_up: torch.Tensor, out: torch.Tensor, activation: str, limit: fl
 
 def bias_act(x: torch.Tensor, out: torch.Tensor, activation: str, bias: Optional[torch.Tensor] = None) -> torch.Tensor:
     """``out = act(x + bias)`` element by element (``bias`` fp32, one value per column, optional); ``out``
-    may be ``x``."""
-    if activation not in ACTIVATIONS:
-        raise KernelError(f"bias_act: activation {activation!r} is not one of {sorted(ACTIVATIONS)}")
+    may be ``x``.  ``activation="none"``: the bias alone."""
+    if activation not in BIAS_ACTIVATIONS:
+        raise KernelError(f"bias_act: activation {activation!r} is not one of {sorted(BIAS_ACTIVATIONS)}")
     if x.dim() != 2 or out.shape != x.shape or out.dtype != x.dtype \
             or (bias is not None and (bias.shape != (x.shape[1],) or bias.dtype != torch.float32)):
         raise KernelError(f"bias_act: x {tuple(x.shape)} and out {tuple(out.shape)} do not fit")
     check(hip_lib().kva_bias_act(_dev(out, "out"), _dev(x, "x"), dtype_code(x.dtype), _opt(bias, "bias"), x.shape[0],
-                                 x.shape[1], ACTIVATIONS[activation], _stream()), "bias_act")
+                                 x.shape[1], BIAS_ACTIVATIONS[activation], _stream()), "bias_act")
     return out
 
 
@@ -726,6 +727,71 @@ def sandwich_step(x: torch.Tensor, *, y: Optional[torch.Tensor] = None, post=Non
     return out
 
 
+def tanh_step(x: torch.Tensor, *, y: Optional[torch.Tensor] = None, y_bias: Optional[torch.Tensor] = None, post=None,
+              pre=None, out: Optional[torch.Tensor] = None, row_idx: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
+    """What lies between two branches that have tanh norms on both sides, over a residual stream ``x`` fp32 ``[T,
+    width]``: ``x += n_post(y + y_bias)``, then ``out = n_pre(x)``.  ``post`` and ``pre`` are ``(weight, bias, alpha)``:
+    ``tanh(alpha v) * weight + bias``.  Without ``post`` the branch output enters as it is (with its bias, fp32).
+    ``row_idx``: only these rows are read out, and nothing is written back."""
+    T, width = x.shape
+    if x.dim() != 2 or x.dtype != torch.float32:
+        raise KernelError(f"tanh_step: x {tuple(x.shape)} is not an fp32 [T, width] stream")
+    if y is not None and y.shape != x.shape:
+        raise KernelError("tanh_step: the branch output has the stream's shape")
+    if y_bias is not None and (y is None or y_bias.shape != (width,) or y_bias.dtype != torch.float32):
+        raise KernelError("tanh_step: a product's bias is fp32 [width] and goes with the product")
+    for norm in (post, pre):
+        if norm is not None and (norm[0].shape != (width,) or norm[1].shape != (width,) or norm[1].dtype != norm[0].dtype):
+            raise KernelError("tanh_step: a norm has a weight [width] and a bias of its shape and type")
+    if (post is not None and y is None) or (out is None) != (pre is None):
+        raise KernelError("tanh_step: the first norm goes with a branch output, the second with an output")
+    rows = T
+    if out is not None:
+        rows = T if row_idx is None else row_idx.shape[0]
+        if out.shape != (rows, width):
+            raise KernelError(f"tanh_step: out {tuple(out.shape)} is not [{rows}, {width}]")
+    elif row_idx is not None:
+        raise KernelError("tanh_step: rows are gathered for the read-out only")
+
+    def args(norm, name):
+        if norm is None:
+            return None, None, 0, 0.0
+        w, b, alpha = norm
+        return _dev(w, name), _dev(b, name), dtype_code(w.dtype), float(alpha)
+    check(hip_lib().kva_tanh_step(
+        _dev(x, "x"), _opt(y, "y"), dtype_code(y.dtype) if y is not None else 0, _opt(y_bias, "y_bias"), *args(post, "post norm"),
+        *args(pre, "pre norm"), _opt(out, "out"), dtype_code(out.dtype) if out is not None else 0,
+        _opt(row_idx, "row_idx", torch.int32), rows, width, _stream()), "tanh_step")
+    return out
+
+
+def pair_embed(x: torch.Tensor, table: torch.Tensor, scale: float, pairs: Optional[torch.Tensor], mul_prev: int, mul_cur: int,
+               norm, ids: torch.Tensor, state: torch.Tensor, entry_q_start: torch.Tensor, entry_seat: torch.Tensor,
+               feedback: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """``x[t] = n(table[id] * scale + pairs[row])`` fp32, ``row = (previous id * mul_prev + id * mul_cur) mod (len(pairs)
+    - 1)`` or the last one for a sequence's first token.  ``norm``: ``(weight, bias, alpha)`` as :func:`tanh_step`
+    takes it, or None; ``pairs`` may be None.  ``state`` int32 ``[seats, 1]``: the last id of every seat's sequence plus
+    one (0: none yet); it is left at the entries' last ids.  A negative id ``-1 - r`` stands for ``feedback[r]``."""
+    rows, width = x.shape
+    if x.dtype != torch.float32 or table.dim() != 2 or table.shape[1] != width or ids.shape != (rows,):
+        raise KernelError(f"pair_embed: x {tuple(x.shape)} (fp32), table {tuple(table.shape)}, ids {tuple(ids.shape)} do not fit")
+    if pairs is not None and (pairs.dim() != 2 or pairs.shape[1] != width or pairs.shape[0] < 2):
+        raise KernelError(f"pair_embed: the pairs' table {tuple(pairs.shape)} needs rows of {width}, two at least")
+    if norm is not None and (norm[0].shape != (width,) or norm[1].shape != (width,) or norm[1].dtype != norm[0].dtype):
+        raise KernelError("pair_embed: the norm has a weight [width] and a bias of its shape and type")
+    if state.dim() != 2 or state.dtype != torch.int32:
+        raise KernelError("pair_embed: the state is int32 [seats, n]")
+    qs, seat, entries = _entries((entry_q_start, entry_seat), "pair_embed")
+    w, b, alpha = norm if norm is not None else (None, None, 0.0)
+    check(hip_lib().kva_pair_embed(
+        _dev(x, "x"), _dev(table, "table"), dtype_code(table.dtype), table.shape[0], float(scale), _opt(pairs, "pairs"),
+        dtype_code(pairs.dtype) if pairs is not None else 0, pairs.shape[0] - 1 if pairs is not None else 1, int(mul_prev),
+        int(mul_cur), _opt(w, "norm weight"), _opt(b, "norm bias"), dtype_code(w.dtype) if w is not None else 0, float(alpha),
+        _dev(ids, "ids", torch.int32), _opt(feedback, "feedback", torch.int32), _dev(state, "state"), state.shape[1], qs, seat,
+        entries, rows, width, _stream()), "pair_embed")
+    return x
+
+
 def head_gate(x: torch.Tensor, gates: torch.Tensor, heads: int) -> torch.Tensor:
     """In place: head h of row t of ``x`` ``[T, heads * d]`` times ``sigmoid(gates[t, h])``; ``gates``
     is a ``[T, heads]`` view whose rows may be columns of a wider buffer."""
@@ -790,6 +856,58 @@ def qk_encode_cache(qkv: torch.Tensor, positions: torch.Tensor, num_q_heads: int
         head_dim, value_dim, rot, 1 if interleaved else 0, -1.0 if unit_eps is None else float(unit_eps),
         page_size, dtype_code(qkv.dtype), _opt(bias, "bias"), _opt(q_weight, "q_weight"), _opt(k_weight, "k_weight"),
         1 if norm_first else 0, _stream()), "qk_encode_cache")
+
+
+def maps_encode_cache(qkv: torch.Tensor, q_rows: torch.Tensor, positions: torch.Tensor, heads: int, kv_heads: int, dim: int,
+                      value_dim: int, cos: Optional[torch.Tensor], sin: Optional[torch.Tensor], interleaved: bool,
+                      k_cache: Optional[torch.Tensor], v_cache: Optional[torch.Tensor], slot_mapping: Optional[torch.Tensor],
+                      bias: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """Queries and keys of heads with two maps of ``dim`` elements each, ``qkv`` ``[T, (heads 2 + kv_heads 2) dim +
+    kv_heads value_dim]`` (possibly the first columns of a wider buffer): the biases (fp32, one per column) are
+    added, the first ``2 * cos.shape[1]`` elements of every map are rotated; a query head becomes two rows of ``2
+    dim`` elements, each zero where the other map lies, in ``q_rows`` ``[T, 2 heads * 2 dim]``; keys of ``2 dim``
+    elements (both maps side by side) and values go to the paged cache.  Attention over ``2 heads`` query rows
+    and ``kv_heads`` key heads of ``2 dim`` then gives every head's two outputs side by side.  ``kv_heads = 0``:
+    queries alone, and nothing is written to a cache."""
+    tokens = qkv.shape[0]
+    width = 2 * (heads + kv_heads) * dim + kv_heads * value_dim
+    if qkv.dim() != 2 or qkv.shape[1] != width or qkv.stride(1) != 1 or positions.shape != (tokens,) \
+            or q_rows.shape != (tokens, 4 * heads * dim) or q_rows.dtype != qkv.dtype:
+        raise KernelError(f"maps_encode_cache: qkv {tuple(qkv.shape)}, q_rows {tuple(q_rows.shape)} do not fit {heads} / {kv_heads} heads of 2 x {dim}")
+    if bias is not None and (bias.shape != (width,) or bias.dtype != torch.float32):
+        raise KernelError("maps_encode_cache: the biases are fp32, one per column")
+    rot = 0
+    if cos is not None:
+        if sin is None or cos.shape != sin.shape or cos.dim() != 2:
+            raise KernelError("maps_encode_cache: cos and sin tables must be [positions, rot / 2]")
+        rot = 2 * cos.shape[1]
+    write = k_cache is not None
+    page_size = 0
+    if write:
+        if kv_heads == 0 or v_cache is None or slot_mapping is None or slot_mapping.shape != (tokens,) \
+                or k_cache.dtype != qkv.dtype or v_cache.dtype != qkv.dtype:
+            raise KernelError("maps_encode_cache: key heads, K and V cache of qkv's dtype and one slot per token are needed")
+        page_size = check_kv_cache_shapes("maps_encode_cache", k_cache, v_cache, kv_heads, 2 * dim, value_dim)
+    check(hip_lib().kva_maps_encode_cache(
+        _dev(qkv, "qkv", contiguous=False), qkv.stride(0) if tokens > 1 else width, _dev(q_rows, "q_rows"),
+        _opt(k_cache, "k_cache"), _opt(v_cache, "v_cache"), _opt(cos, "cos", torch.float32), _opt(sin, "sin", torch.float32),
+        _dev(positions, "positions", torch.int32), _opt(slot_mapping if write else None, "slot_mapping", torch.int32), tokens,
+        int(heads), int(kv_heads), int(dim), int(value_dim), rot, 1 if interleaved else 0, page_size, _opt(bias, "bias"),
+        dtype_code(qkv.dtype), _stream()), "maps_encode_cache")
+    return q_rows
+
+
+def maps_combine(x: torch.Tensor, heads: int, value_dim: int, weight: float, eps: float, out: torch.Tensor, out_off: int = 0,
+                 mul: float = 1.0) -> torch.Tensor:
+    """``o = a1 - weight * a2`` of every head's two outputs (``x`` ``[T, heads * 2 * value_dim]``), then ``o /
+    sqrt(mean(o^2) + eps) * mul`` into columns ``out_off ..`` of ``out``."""
+    rows = x.shape[0]
+    if x.shape != (rows, 2 * heads * value_dim) or out.dim() != 2 or out.shape[0] != rows or out.dtype != x.dtype \
+            or not 0 <= out_off <= out.shape[1] - heads * value_dim:
+        raise KernelError(f"maps_combine: x {tuple(x.shape)} and out {tuple(out.shape)} do not fit {heads} heads of {value_dim}")
+    check(hip_lib().kva_maps_combine(_dev(out, "out"), out.shape[1], int(out_off), _dev(x, "x"), float(weight), float(eps),
+                                     float(mul), rows, int(heads), int(value_dim), dtype_code(x.dtype), _stream()), "maps_combine")
+    return out
 
 
 def latent_encode_cache(y: torch.Tensor, kv_off: int, q_lat: Optional[torch.Tensor], cache: Optional[torch.Tensor],
@@ -1668,6 +1786,34 @@ def gated_linear_attention(y: torch.Tensor, q_off: int, k_off: int, v_off: int, 
     return out
 
 
+STATE_SPACE_MAX_STATE = 512
+
+
+def state_space_scan(xbc: torch.Tensor, y: torch.Tensor, dt_off: int, a_log: torch.Tensor, dt_bias: torch.Tensor,
+                     skip: torch.Tensor, out: torch.Tensor, state: torch.Tensor, state_off: int, entry_q_start: torch.Tensor,
+                     entry_seat: torch.Tensor, heads: int, groups: int, state_size: int, vdim: int) -> torch.Tensor:
+    """Per head and token, in order: ``dt = softplus(y[t, dt_off + h] + dt_bias[h])``, ``S <- exp(-exp(a_log[h]) dt) S
+    + dt B x^T``, ``out = S^T C + skip[h] x``.  ``xbc`` fp32 ``[T, heads vdim + 2 groups state_size]`` holds x, then B
+    and C of every group; head h uses group ``h // (heads / groups)``.  ``S`` ``[heads, state_size, vdim]`` lives at
+    ``state_off`` of the seat's fp32 state row; ``out`` is fp32 ``[T, heads * vdim]``."""
+    tokens = out.shape[0]
+    if heads % groups or xbc.shape != (tokens, heads * vdim + 2 * groups * state_size) or xbc.dtype != torch.float32 \
+            or out.shape != (tokens, heads * vdim) or out.dtype != torch.float32 or y.dim() != 2 or y.shape[0] != tokens:
+        raise KernelError(f"state_space_scan: xbc {tuple(xbc.shape)}, y {tuple(y.shape)}, out {tuple(out.shape)} do not fit")
+    if not 0 <= dt_off <= y.shape[1] - heads:
+        raise KernelError("state_space_scan: the step sizes' columns lie outside y")
+    for v in (a_log, dt_bias, skip):
+        if v.shape != (heads,) or v.dtype != torch.float32:
+            raise KernelError("state_space_scan: rates, step biases and skips are fp32, one a head")
+    seat_stride = _state_row(state, state_off, heads * state_size * vdim, "state_space_scan")
+    qs, seat, entries = _entries((entry_q_start, entry_seat), "state_space_scan")
+    check(hip_lib().kva_state_space_scan(
+        _dev(out, "out"), _dev(state, "state"), seat_stride, int(state_off), _dev(xbc, "xbc"), xbc.shape[1], _dev(y, "y"),
+        dtype_code(y.dtype), y.shape[1], int(dt_off), _dev(a_log, "a_log"), _dev(dt_bias, "dt_bias"), _dev(skip, "skip"), qs,
+        seat, entries, int(heads), int(groups), int(state_size), int(vdim), _stream()), "state_space_scan")
+    return out
+
+
 def block_gates(u: torch.Tensor, w_a: torch.Tensor, w_i: torch.Tensor, bias_a: torch.Tensor, bias_i: torch.Tensor,
                 rate: torch.Tensor, a_out: torch.Tensor, b_out: torch.Tensor) -> None:
     """The decays and inputs of a real-gated linear recurrent unit for all tokens: with the channels of ``u``
@@ -1743,13 +1889,17 @@ HEAD_GATES = {"silu": 0, "sigmoid": 1}
 
 
 def head_norm_gate(x: torch.Tensor, weight: Optional[torch.Tensor], eps: float, gate: Optional[torch.Tensor], gate_off: int,
-                   out: torch.Tensor, out_off: int, heads: int, vdim: int, activation: Optional[str], mul: float = 1.0) -> torch.Tensor:
+                   out: torch.Tensor, out_off: int, heads: int, vdim: int, activation: Optional[str], mul: float = 1.0,
+                   gate_first: bool = False) -> torch.Tensor:
     """``out[t, out_off + h vdim + j] = n(x)[t, h, j] * act(gate[t, gate_off + h vdim + j]) * mul`` where
     ``n`` divides every head by its root mean square (``sqrt(mean_j x^2 + eps)``) and multiplies by
     ``weight[j]`` (fp32 ``[vdim]``, shared by the heads) or ``weight[h vdim + j]`` (fp32 ``[heads * vdim]``),
     or leaves x as it is without a weight.  ``gate`` and ``out`` may be wider buffers; ``act`` is silu or
-    sigmoid; without a ``gate`` the rows are only normed and multiplied."""
+    sigmoid; without a ``gate`` the rows are only normed and multiplied.  ``gate_first``: the gate multiplies what is
+    normed, ``n(x * act(gate))``."""
     rows = x.shape[0]
+    if gate_first and gate is None:
+        raise KernelError("head_norm_gate: a gate in front of the norm needs the gate")
     if x.shape != (rows, heads * vdim) or out.dim() != 2 \
             or out.shape[0] != rows or not 0 <= out_off <= out.shape[1] - heads * vdim:
         raise KernelError(f"head_norm_gate: x {tuple(x.shape)} and out {tuple(out.shape)} do not fit")
@@ -1764,7 +1914,7 @@ def head_norm_gate(x: torch.Tensor, weight: Optional[torch.Tensor], eps: float, 
         _dev(out, "out"), dtype_code(out.dtype), out.shape[1], int(out_off), _dev(x, "x"), dtype_code(x.dtype),
         _opt(weight, "weight"), float(eps), _opt(gate, "gate"), dtype_code(gate.dtype) if gate is not None else 0,
         gate.shape[1] if gate is not None else 0, int(gate_off),
-        rows, heads, vdim, HEAD_GATES.get(activation, 0), float(mul), w_stride, _stream()), "head_norm_gate")
+        rows, heads, vdim, HEAD_GATES.get(activation, 0), 1 if gate_first else 0, float(mul), w_stride, _stream()), "head_norm_gate")
     return out
 
 
@@ -1871,10 +2021,10 @@ def moe_expert_rows(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, sorted_
                     slot_weight: Optional[torch.Tensor] = None, gated: bool = False, limit: float = 0.0,
                     group: int = 1, tiled: bool = False) -> torch.Tensor:
     """One product per tile against its expert's matrix ``w[e]`` ``[N, K]``.  With an ``activation``
-    (the first product): row ``slot // top`` of ``x`` ``[T, K]``, activated, goes to the slot's sorted
-    place of ``out`` ``[places, N]`` (x's type).  With ``slot_weight`` (the second): the row at the
-    sorted place of ``x`` ``[places, K]``, times the slot's weight, goes to row ``slot`` of ``out`` fp32
-    ``[slots, N]``.  ``gated`` (first product): rows ``2 j`` and ``2 j + 1`` of an expert's matrix are
+    (the first product): row ``slot // top`` of ``x`` ``[T, K]`` - times the slot's ``slot_weight`` if given: a
+    weight on the expert's input - goes through the product and the activation to the slot's sorted place of
+    ``out`` ``[places, N]`` (x's type).  Without one (the second): the row at the sorted place of ``x`` ``[places,
+    K]`` goes, times the slot's ``slot_weight`` if given, to row ``slot`` of ``out`` fp32 ``[slots, N]``.  ``gated`` (first product): rows ``2 j`` and ``2 j + 1`` of an expert's matrix are
     output j's gate and up rows, and ``out`` ``[places, N / 2]`` gets ``act(gate) * up``.  ``group`` (as the list
     was sorted, :func:`moe_group`): so many tiles at a time, through LDS.  ``tiled``: the matrices are
     stored in operand order (:func:`moe_tiled_weight`)."""
@@ -1882,8 +2032,8 @@ def moe_expert_rows(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, sorted_
     n_out = w.shape[1] // 2 if gated else w.shape[1]
     if gated and (activation is None or w.shape[1] % 2):
         raise KernelError("moe_expert_rows: gate and up rows come in pairs, in the first product")
-    if (activation is None) == (slot_weight is None):
-        raise KernelError("moe_expert_rows: either an activation (first product) or slot weights (second)")
+    if slot_weight is not None and slot_weight.dtype != torch.float32:
+        raise KernelError("moe_expert_rows: the slots' weights are fp32")
     if w.dim() != 3 or w.dtype != x.dtype or x.dim() != 2 or x.shape[1] != w.shape[2] or out.dim() != 2 \
             or out.shape[1] != n_out or sorted_slot.shape != (tiles * MOE_TILE,):
         raise KernelError(f"moe_expert_rows: x {tuple(x.shape)}, w {tuple(w.shape)}, out {tuple(out.shape)} do not fit")
@@ -1892,9 +2042,11 @@ def moe_expert_rows(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, sorted_
             raise KernelError(f"moe_expert_rows: activation {activation!r} is not one of {sorted(EXPERT_ACTIVATIONS)}")
         if out.shape[0] != tiles * MOE_TILE or out.dtype != x.dtype:
             raise KernelError("moe_expert_rows: the first product writes one row of x's type per sorted place")
+        if slot_weight is not None and slot_weight.numel() != x.shape[0] * int(top):
+            raise KernelError("moe_expert_rows: one weight per (token, choice) slot")
     else:
-        if x.shape[0] != tiles * MOE_TILE or out.dtype != torch.float32 or slot_weight.numel() != out.shape[0] \
-                or slot_weight.dtype != torch.float32:
+        if x.shape[0] != tiles * MOE_TILE or out.dtype != torch.float32 \
+                or (slot_weight is not None and slot_weight.numel() != out.shape[0]):
             raise KernelError("moe_expert_rows: the second product reads sorted places and writes fp32 rows per slot")
     check(hip_lib().kva_moe_expert_rows(
         _dev(out, "out"), dtype_code(out.dtype), _dev(x, "x"), _dev(w, "w"), dtype_code(x.dtype),
@@ -1984,6 +2136,8 @@ KERNEL_CLASSES = {
     "moe_combine": "routed experts", "small_product_f32": "small fp32 products",
     "norm_into_stream": "norm", "table_gate": "elementwise",
     "hyper_step": "norm", "sandwich_step": "norm", "hyper_fill": "embedding", "bias_act": "activation",
+    "tanh_step": "norm", "pair_embed": "embedding", "maps_encode_cache": "rope + cache write", "maps_combine": "elementwise",
+    "state_space_scan": "recurrent mixers",
     "block_gates": "recurrent mixers", "linear_scan_gate": "recurrent mixers", "matrix_memory": "recurrent mixers",
 }
 

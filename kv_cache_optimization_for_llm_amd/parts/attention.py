@@ -376,3 +376,101 @@ class NormedGQAAttention(Mixer):
         attn_ops.paged_attention(y, heads, kv, batch, self.num_heads, self.num_kv_heads, self.head_dim, self.scale,
                                  self.window, keep_first=self.keep_first, value_dim=self.value_dim, chunk=self.chunk)
         return self.o(heads)
+
+
+@MIXERS.register("differential_attention")
+class DifferentialAttention(ProjectedMixer):
+    """Attention of heads with two maps: a query head has two queries of ``head_dim`` and a key head two keys, ``[map
+    1, map 2]``; each map is a causal softmax of its own over the head's values (``value_dim``), and with their
+    outputs ``a1``, ``a2`` a head is ``o = a1 - weight * a2``, divided by its root mean square (``sqrt(mean(o^2) +
+    norm_eps)``, no weight) and multiplied by ``1 - diff``.  ``weight = exp(lq1 . lk1) - exp(lq2 . lk2) + diff`` is one
+    number a layer, formed once from the stored vectors.  The position encoding turns every map's first elements.
+    ``bias``: q, k, v and the output projection have biases, named like their matrices with ``bias_suffix``.
+
+    The cache holds a key head's two keys side by side as one key of ``2 head_dim``; a query head goes to the
+    attention kernels as two rows whose other half is zero (``ops.kernels.maps_encode_cache``), so keys and values
+    are stored and read once for both maps.  ``shared_kv``: the mixer has no key and value tensors and attends over
+    what another layer call wrote to the cache slot it is given."""
+
+    graph_safe = True
+
+    def __init__(self, prefix: str, *, hidden_size: int, num_heads: int, num_kv_heads: int, head_dim: int, scale: float,
+                 diff: float, norm_eps: float, position: Optional[PartSpec] = None, value_dim: Optional[int] = None,
+                 bias: bool = False, shared_kv: bool = False, tensor_names: Optional[Dict[str, str]] = None):
+        """``tensor_names`` maps ``q k v o lq1 lk1 lq2 lk2`` and ``bias_suffix`` to names behind ``prefix``."""
+        super().__init__(prefix)
+        if num_heads % num_kv_heads:
+            raise ValueError(f"{num_heads} heads is not a multiple of {num_kv_heads} kv heads")
+        if head_dim % 2:
+            raise ValueError(f"{prefix}: maps of {head_dim} elements (keys of two maps lie in the cache in chunks of 4 or 8)")
+        self.hidden_size, self.num_heads, self.num_kv_heads = int(hidden_size), int(num_heads), int(num_kv_heads)
+        self.head_dim, self.scale, self.diff, self.norm_eps = int(head_dim), float(scale), float(diff), float(norm_eps)
+        self.value_dim = int(head_dim if value_dim is None else value_dim)
+        self.bias, self.shared_kv = bool(bias), bool(shared_kv)
+        names = dict(q="q", k="k", v="v", o="o", lq1="lq1", lk1="lk1", lq2="lq2", lk2="lk2", bias_suffix=".b")
+        names.update(tensor_names or {})
+        self.bias_suffix = names.pop("bias_suffix")
+        self.names = {key: prefix + name for key, name in names.items()}
+        position = position or PartSpec("none")
+        self.position = POSITION_ENCODINGS.get(position.kind)(**position.params)
+        self.inner_width = self.num_heads * self.value_dim
+        self.own_kv_heads = 0 if self.shared_kv else self.num_kv_heads
+        self.qkv_width = 2 * (self.num_heads + self.own_kv_heads) * self.head_dim + self.own_kv_heads * self.value_dim
+        self.map_weight = 0.0
+
+    def tensor_specs(self) -> Dict[str, TensorSpec]:
+        n, d, dv, W = self.names, self.head_dim, self.value_dim, self.hidden_size
+        specs = {n["q"]: TensorSpec((2 * self.num_heads * d, W)), n["o"]: TensorSpec((W, self.inner_width))}
+        if not self.shared_kv:
+            specs[n["k"]] = TensorSpec((2 * self.num_kv_heads * d, W))
+            specs[n["v"]] = TensorSpec((self.num_kv_heads * dv, W))
+        if self.bias:
+            for key in ("q", "o") if self.shared_kv else ("q", "k", "v", "o"):
+                specs[n[key] + self.bias_suffix] = TensorSpec((specs[n[key]].shape[0],), init="normal", role="vector")
+        for key in ("lq1", "lk1", "lq2", "lk2"):
+            specs[n[key]] = TensorSpec((d,), init="normal", role="vector")
+        return specs
+
+    def load(self, tensors: Dict[str, torch.Tensor]) -> None:
+        n = self.names
+        keys = "q" if self.shared_kv else "qkv"
+        self._w_in = torch.cat([tensors[n[key]] for key in keys], dim=0).contiguous()
+        self._w_out = tensors[n["o"]]
+        self.qkv_bias = self.out_bias = None
+        if self.bias:
+            self.qkv_bias = torch.cat([tensors[n[key] + self.bias_suffix] for key in keys]).float().contiguous()
+            self.out_bias = tensors[n["o"] + self.bias_suffix].float().contiguous()
+        l1, l2 = ((tensors[n["lq" + i]].float() * tensors[n["lk" + i]].float()).sum() for i in "12")
+        self.map_weight = float(torch.exp(l1) - torch.exp(l2)) + self.diff
+        self.load_projections()
+
+    def input_weight(self) -> torch.Tensor:
+        return self._w_in
+
+    def output_weight(self) -> torch.Tensor:
+        return self._w_out
+
+    def kv_cache_spec(self) -> KVCacheSpec:
+        return attention_cache_spec(self.num_kv_heads, 2 * self.head_dim, value_dim=self.value_dim)
+
+    def activation_elements(self) -> int:
+        return self.qkv_width + 4 * self.num_heads * self.head_dim + 3 * self.inner_width + self.hidden_size
+
+    def forward_inner(self, y, col0, ctx: MixerContext, state_off, out, out_col0, mul) -> None:
+        batch, kv = ctx.batch, ctx.kv
+        if kv is None:
+            raise K.KernelError(f"{self.prefix}: the mixer has no cache view")
+        if self.shared_kv and kv.writes:
+            raise K.KernelError(f"{self.prefix}: a layer without keys and values of its own only reads its cache slot")
+        write = kv.writes and not self.shared_kv
+        T, H = y.shape[0], self.num_heads
+        cos, sin = self.position.tables(y.device) if hasattr(self.position, "tables") else (None, None)
+        q = torch.empty((T, 4 * H * self.head_dim), dtype=y.dtype, device=y.device)
+        K.maps_encode_cache(y[:, col0:col0 + self.qkv_width], q, batch.positions, H, self.own_kv_heads, self.head_dim,
+                            self.value_dim, cos, sin, getattr(self.position, "pairing", "half") == "interleaved",
+                            kv.k_cache if write else None, kv.v_cache if write else None,
+                            kv.slot_mapping if write else None, bias=self.qkv_bias)
+        both = torch.empty((T, 2 * self.inner_width), dtype=y.dtype, device=y.device)
+        attn_ops.paged_attention(q, both, kv, batch, 2 * H, self.num_kv_heads, 2 * self.head_dim, self.scale,
+                                 value_dim=self.value_dim)
+        K.maps_combine(both, H, self.value_dim, self.map_weight, self.norm_eps, out, out_col0, (1.0 - self.diff) * mul)

@@ -212,11 +212,13 @@ class PendingNorm:
     """A branch output that has not entered the residual stream yet and does so under a norm of its own
     (``x <- x + norm(y)``), with ``addend`` (fp32, the stream's shape; optional) behind it: whoever reads the
     stream next lets both in, in the pass that reads (``ops.kernels.sandwich_step``).  ``norm`` None: ``y`` enters
-    as it is; ``y`` None: only the addend does."""
+    as it is; ``y`` None: only the addend does.  ``bias`` (fp32 per column): what is still to be added to ``y``
+    before its norm, the bias of the product that made it."""
 
     y: Optional[torch.Tensor]
     norm: object = None
     addend: Optional[torch.Tensor] = None
+    bias: Optional[torch.Tensor] = None
 
 
 @dataclass
@@ -273,6 +275,20 @@ class Norm(Part):
         """``stream += norm(y)`` in place, for arrangements that norm a branch's OUTPUT; ``copy``
         receives the new stream in another type.  Norms that cannot be used this way do not have it."""
         raise NotImplementedError(f"{type(self).__name__} cannot norm a branch output into the stream")
+
+
+class Embedding(Part):
+    """How a step's tokens become the first rows of the residual stream.  It owns the token table
+    (``table_name``, which a tied output matrix reads too) and may keep a state per request."""
+
+    table_name: str = ""
+
+    def state_spec(self) -> Optional["StateSpec"]:
+        return None
+
+    def forward(self, batch, out: torch.Tensor, state: Optional[torch.Tensor] = None) -> torch.Tensor:
+        """Fills ``out`` ``[T, width]`` (the stream) for the batch's tokens; ``state`` as :class:`Mixer`'s."""
+        raise NotImplementedError
 
 
 class PositionEncoding(Part):
@@ -332,6 +348,10 @@ class ProjectedMixer(Mixer):
 
     hidden_size: int = 0
     inner_width: int = 0
+    # Bias of the output projection (fp32 [hidden]) or None.  An arrangement whose next pass over the output can
+    # add it sets ``leaves_out_bias`` and takes it along; otherwise it is added here.
+    out_bias: Optional[torch.Tensor] = None
+    leaves_out_bias: bool = False
 
     def input_weight(self) -> torch.Tensor:
         """``[input columns, hidden]``: every matrix that reads the mixer's input, joined by rows."""
@@ -366,7 +386,11 @@ class ProjectedMixer(Mixer):
         ctx.x = x
         inner = torch.empty((x.shape[0], self.inner_width), dtype=x.dtype, device=x.device)
         self.forward_inner(y, 0, ctx, 0, inner, 0, 1.0)
-        return self._out(inner)
+        y = self._out(inner)
+        if self.out_bias is not None and not self.leaves_out_bias:
+            from ..ops import kernels as K
+            K.bias_act(y, y, "none", self.out_bias)
+        return y
 
 
 class FeedForward(Part):

@@ -15,7 +15,8 @@ from ..config.registry import BLOCKS, LAYER_INPUTS
 from ..models.spec import PartSpec
 from ..ops import kernels as K
 from ..models.spec import TensorSpec
-from .base import Block, BranchTail, MixerContext, Norm, NormedRows, Part, PendingMix, PendingNorm, PendingSum, StreamCopy
+from .base import (Block, BranchTail, MixerContext, Norm, NormedRows, Part, PendingMix, PendingNorm, PendingSum, ProjectedMixer,
+                   StreamCopy)
 
 
 @BLOCKS.register("pre_norm")
@@ -163,8 +164,8 @@ class PostNormBlock(Block):
 @BLOCKS.register("sandwich_norm")
 class SandwichNormBlock(Block):
     """A norm in front of every branch and another on its output: ``h += norm_mo(mixer(norm_m(h))); h +=
-    norm_fo(ffn(norm_f(h)))``, over a residual stream kept in 32-bit.  The norms are of kind ``"layernorm"``
-    (weight, optional bias, with or without the mean taken off).  What lies between two branches - the
+    norm_fo(ffn(norm_f(h)))``, over a residual stream kept in 32-bit.  The norms are all of kind ``"layernorm"``
+    (weight, optional bias, with or without the mean taken off) or all of kind ``"dynamic_tanh"``.  What lies between two branches - the
     output's norm, the sum, the next branch's norm - is one launch: the block hands its last output on as
     :class:`~.base.PendingNorm`, and whoever reads the stream next lets it in in its own pass.  A layer without
     a feed-forward (``"none"``) names only the mixer's two norms."""
@@ -180,6 +181,12 @@ class SandwichNormBlock(Block):
         for name, norm in self.norms.items():
             if not hasattr(norm, "pass_args"):
                 raise ValueError(f"this arrangement runs its norms inside its own pass; {name!r} is a {type(norm).__name__}")
+        kinds = {norm.pass_kind for norm in self.norms.values()}
+        if len(kinds) != 1:
+            raise ValueError(f"this arrangement's norms share a pass and are of one kind, not {sorted(kinds)}")
+        # a pass of tanh norms adds the bias of the product whose output it lets in
+        if kinds == {"tanh"} and isinstance(mixer, ProjectedMixer):
+            mixer.leaves_out_bias = True
 
     def first_norm(self) -> Optional[Norm]:
         return None
@@ -191,7 +198,8 @@ class SandwichNormBlock(Block):
             raise TypeError("this arrangement takes a 32-bit stream and a pending output with the norm it enters under")
         n = self.norms
         a = self.mixer.forward(n["mixer"].forward(hidden, delta=delta), ctx)
-        delta = PendingNorm(a, n["mixer_out"])
+        left = self.mixer.out_bias if getattr(self.mixer, "leaves_out_bias", False) else None
+        delta = PendingNorm(a, n["mixer_out"], bias=left)
         if self.has_ffn:
             f = self.feed_forward.forward(n["feed_forward"].forward(hidden, delta=delta), ctx)
             delta = PendingNorm(f, n["feed_forward_out"])

@@ -60,6 +60,8 @@ class SideBySide(Mixer):
         ins, outs = [], []
         for c in self.children:
             c.load(tensors)
+            if c.out_bias is not None:
+                raise ValueError(f"{self.prefix}: the joined output projection has no bias, a child has one")
             w = c.input_weight()
             pad = -w.shape[0] % self.COLUMN_ALIGN
             if pad:         # every child's columns start at a multiple of 16 (or 32) bytes of a row

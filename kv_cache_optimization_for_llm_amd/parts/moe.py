@@ -7,6 +7,7 @@ are chosen; their weights are the plain scores (``renormalise``: divided by thei
 ``identity`` router outputs stand for experts that return their input: they have no tensors.
 ``router_bias``: a stored vector added to the logits themselves; ``softmax_over="chosen"``: the
 largest logits are chosen and the weights are the softmax over the chosen logits alone.
+``weight_on="input"``: a weight multiplies what its expert reads instead of what it returns.
 ``gated``: an expert is ``W_down (act(W_gate x) * (W_up x))``; its gate and up matrices are stacked
 row by row in turns at load time, so that one product's epilogue has both halves of every output.
 ``router="table"``: no router at all; an integer table ``[token ids, top]`` names every token id's
@@ -46,7 +47,7 @@ class RoutedExperts(FeedForward):
                  shared_intermediate: int = 0, scores: str = "softmax", groups: int = 1, keep_groups: int = 1,
                  group_top: int = 2, weight_scale: float = 1.0, sum_eps: float = 0.0, limit: float = 0.0,
                  shared_limit: Optional[float] = None, shared_gate: bool = False, router: str = "learned",
-                 table_rows: int = 0, tensor_names: Optional[Dict[str, str]] = None):
+                 table_rows: int = 0, weight_on: str = "output", tensor_names: Optional[Dict[str, str]] = None):
         """``scores="sigmoid"``: every router output's score is its own sigmoid.  ``groups`` > 1: the outputs
         form so many equal runs of neighbours, a run's score is the sum of its ``group_top`` largest choice
         scores (score + correction), and only outputs of the ``keep_groups`` best runs can be chosen.
@@ -55,6 +56,8 @@ class RoutedExperts(FeedForward):
         (u + 1)``, ``g = min(gate, limit)``, ``u = clamp(up, -limit, limit)``; ``shared_limit``: the limit of the
         expert every token uses (default: ``limit``).  ``shared_gate``: that expert's result enters times
         ``sigmoid(w . x)``, one number a token, ``w`` stored as ``[1, hidden]``.
+        ``weight_on="input"``: a choice's weight multiplies the row its expert reads, ``expert(w x)``, and what the
+        experts return is added as it is.
         ``router="table"``: experts by token id (``table``, int32 ``[table_rows, top]``).
         ``tensor_names`` maps ``router``, ``table``, ``router_bias``, ``correction``, ``gate``, ``up``, ``down``,
         ``shared`` (a prefix) and ``shared_gate`` to names behind ``prefix``; the experts' names hold ``{e}`` for
@@ -66,6 +69,9 @@ class RoutedExperts(FeedForward):
         self.weight_scale, self.sum_eps, self.limit = float(weight_scale), float(sum_eps), float(limit)
         self.shared_limit = self.limit if shared_limit is None else float(shared_limit)
         self.has_shared_gate = bool(shared_gate)
+        if weight_on not in ("input", "output"):
+            raise ValueError(f"{prefix}: weight_on {weight_on!r} is neither 'input' nor 'output'")
+        self.weight_input = weight_on == "input"
         if self.groups < 1 or not 1 <= self.keep_groups <= self.groups or (int(experts) + int(identity)) % self.groups:
             raise ValueError(f"{prefix}: {groups} groups (of which {keep_groups} are kept) do not divide the router's outputs")
         if activation == "swish_clamped" and not gated:
@@ -201,9 +207,10 @@ class RoutedExperts(FeedForward):
                 sorted_slot, tile_expert = self._sorted(slots, group, dev)
                 K.moe_align(idx, self.experts, sorted_slot, tile_expert, group)
             act = torch.empty((sorted_slot.shape[0], self.intermediate_size), dtype=x.dtype, device=dev)
+            first, second = (wgt, None) if self.weight_input else (None, wgt)
             K.moe_expert_rows(x, self.w_up, act, sorted_slot, tile_expert, self.top, activation=self.activation,
-                              gated=self.gated, limit=self.limit, group=group, tiled=self.tiled)
-            K.moe_expert_rows(act, self.w_down, rows, sorted_slot, tile_expert, self.top, slot_weight=wgt, group=group,
+                              slot_weight=first, gated=self.gated, limit=self.limit, group=group, tiled=self.tiled)
+            K.moe_expert_rows(act, self.w_down, rows, sorted_slot, tile_expert, self.top, slot_weight=second, group=group,
                               tiled=self.tiled)
         out = torch.empty_like(x)
         extra = self.shared.forward(x, ctx) if self.shared is not None else None

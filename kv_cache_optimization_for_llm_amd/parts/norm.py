@@ -1,4 +1,4 @@
-"""RMSNorm: ``y = x / sqrt(mean(x^2) + eps) * w`` (reference: ``base/src/kernels.cu:10-36``).
+"""RMSNorm, layer norm and a norm without statistics.  RMSNorm: ``y = x / sqrt(mean(x^2) + eps) * w`` (reference: ``base/src/kernels.cu:10-36``).
 
 The weight multiplies as stored (no ``1 + w``).  ``forward`` can fuse the residual add that
 comes before the norm (``delta``) and a gather of rows (``row_idx``).
@@ -119,8 +119,11 @@ class LayerNorm(Norm):
         # the products behind a norm take the weights' type; a 32-bit stream of a bf16 model is normalised into bf16
         return torch.empty((rows, self.width), dtype=self.out_dtype or self.weight.dtype, device=x.device)
 
+    pass_kind = "moments"
+
     def pass_args(self) -> tuple:
-        """``(weight, bias, eps, center)`` as a kernel that norms inside its own pass takes them."""
+        """``(weight, bias, eps, center)`` as a kernel that norms inside its own pass takes them (one kind of
+        norm a pass: ``pass_kind``)."""
         return self.weight, self.bias, self.eps, self.center
 
     def forward(self, x, out=None, delta=None, row_idx=None):
@@ -128,6 +131,8 @@ class LayerNorm(Norm):
         if isinstance(delta, PendingNorm):
             if self.streams > 1:
                 raise TypeError(f"{self.prefix}: a branch output under a norm enters a stream of one copy")
+            if delta.bias is not None or (delta.norm is not None and delta.norm.pass_kind != self.pass_kind):
+                raise TypeError(f"{self.prefix}: this pass lets a branch output in under a norm of its own kind, without a bias")
             return K.sandwich_step(x, y=delta.y, post=delta.norm.pass_args() if delta.norm is not None else None,
                                    addend=delta.addend, pre=self.pass_args(), out=out, row_idx=row_idx)
         if self.bias is not None or self.streams > 1 or isinstance(delta, PendingMix):
@@ -154,3 +159,59 @@ class LayerNorm(Norm):
         K.layernorm(x, self.weight, self.eps, out, deltas=self._deltas(delta), weight2=twin.weight, out2=out2,
                     rms=not self.center, delta_scale=self._scale(delta))
         return out, out2
+
+
+@NORMS.register("dynamic_tanh")
+class DynamicTanh(Norm):
+    """``y = tanh(alpha x) * w + b`` with one stored number ``alpha``: no mean, no variance, every element by
+    itself.  It reads a 32-bit stream and writes rows of the type the products behind it take (the weight's); a
+    pending :class:`~.base.PendingNorm` enters the stream first, under a norm of this kind and with the bias of
+    its product (``ops.kernels.tanh_step``)."""
+
+    graph_safe = True
+    pass_kind = "tanh"
+
+    def __init__(self, prefix: str, *, width: int, weight_name: str = "weight", bias_name: Optional[str] = None,
+                 alpha_name: Optional[str] = None):
+        """``bias_name`` and ``alpha_name``: by default the weight's name with ``.b`` and ``.alpha`` behind it."""
+        super().__init__(prefix)
+        self.width = int(width)
+        self.weight_name = prefix + weight_name
+        self.bias_name = prefix + (bias_name or weight_name + ".b")
+        self.alpha_name = prefix + (alpha_name or weight_name + ".alpha")
+        self.weight: Optional[torch.Tensor] = None
+        self.bias: Optional[torch.Tensor] = None
+        self.alpha = 1.0
+
+    def tensor_specs(self) -> Dict[str, TensorSpec]:
+        return {self.weight_name: TensorSpec((self.width,), init="norm", role="vector"),
+                self.bias_name: TensorSpec((self.width,), init="normal", role="vector"),
+                self.alpha_name: TensorSpec((), init="norm", role="vector")}
+
+    def load(self, tensors: Dict[str, torch.Tensor]) -> None:
+        self.weight = tensors[self.weight_name].contiguous()
+        self.bias = tensors[self.bias_name].to(self.weight.dtype).contiguous()
+        self.alpha = float(tensors[self.alpha_name])
+
+    def activation_elements(self) -> int:
+        return self.width
+
+    def pass_args(self) -> tuple:
+        """``(weight, bias, alpha)`` as a kernel that norms inside its own pass takes them."""
+        return self.weight, self.bias, self.alpha
+
+    def forward(self, x, out=None, delta=None, row_idx=None):
+        if out is None:
+            rows = x.shape[0] if row_idx is None else row_idx.shape[0]
+            out = torch.empty((rows, self.width), dtype=self.weight.dtype, device=x.device)
+        enter = {}
+        if isinstance(delta, PendingNorm):
+            if delta.addend is not None or (delta.norm is not None and delta.norm.pass_kind != self.pass_kind):
+                raise TypeError(f"{self.prefix}: this pass lets a branch output in under a norm of its own kind, without an addend")
+            if delta.y is not None:
+                enter = dict(y=delta.y, y_bias=delta.bias, post=delta.norm.pass_args() if delta.norm is not None else None)
+        elif isinstance(delta, torch.Tensor):
+            enter = dict(y=delta)
+        elif delta is not None:
+            raise TypeError(f"{self.prefix}: this norm takes one branch output, plain or under a norm of its own kind")
+        return K.tanh_step(x, pre=self.pass_args(), out=out, row_idx=row_idx, **enter)

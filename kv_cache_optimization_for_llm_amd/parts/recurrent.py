@@ -24,6 +24,9 @@ order of every sum depends on the sizes alone.
   e^(i - m') k v^T``, ``n`` likewise with ``k`` alone, ``o = S^T q / (max(|n . q|, e^(-m')) + 1e-6)``.
 * :class:`RealGatedLRU` (``"real_gated_lru"``): per channel ``S_t = a_t S_(t-1) + sqrt(1 - a_t^2) i_t u_t``
   behind a short causal convolution, with gates made by block-diagonal matrices, times a gelu branch.
+* :class:`StateSpaceDuality` (``"state_space_duality"``): ``S_t = exp(-rate_h dt_t) S_(t-1) + dt_t B_t x_t^T``, ``y_t =
+  S_t^T C_t + D_h x_t`` with one step size per head and token, behind a short causal convolution; the gate stands
+  in front of the norm.
 """
 from __future__ import annotations
 
@@ -470,3 +473,85 @@ class RealGatedLRU(ProjectedMixer):
         K.block_gates(u, self.w_a, self.w_i, self.a_bias, self.i_bias, self.rate, a, b)
         K.linear_scan_gate(a, b, y, col0 + self.y_off, self.y_bias, out, out_col0, ctx.state, state_off,
                            batch.entry_q_start, batch.entry_seat, mul)
+
+
+@MIXERS.register("state_space_duality")
+class StateSpaceDuality(ProjectedMixer):
+    """A state-space mixer whose decay is one number per head and token (Mamba-2).  One input matrix makes ``[z | x | B
+    | C | dt]``: z and x of ``heads * value_dim``, B and C of ``groups * state_size``, dt of ``heads``.  x, B and C pass a
+    causal convolution per channel over ``conv_taps`` tokens (a bias, silu; zeros before a request's start);
+    ``dt <- softplus(dt + dt_bias)``; per head (head h uses group ``h // (heads / groups)``) ``S_t = exp(-exp(A_log) dt)
+    S_(t-1) + dt B_t x_t^T``, ``y_t = S_t^T C_t + D x_t``.  The heads' read-outs, joined, are multiplied by
+    ``silu(z)`` and then RMS-normed in ``norm_groups`` equal parts with a weight of the whole width, and
+    projected.  Decays, step sizes and the recurrence are 32-bit; the state row holds S of every head, then the
+    convolution's last ``taps - 1`` inputs."""
+
+    graph_safe = True
+    COLUMN_ALIGN = 8            # the joined projection's rows start at a multiple of 16 (or 32) bytes
+
+    def __init__(self, prefix: str, *, hidden_size: int, num_heads: int, value_dim: int, state_size: int, groups: int,
+                 conv_taps: int, norm_groups: int, norm_eps: float, tensor_names: Optional[Dict[str, str]] = None):
+        """``tensor_names`` maps ``in conv conv_bias dt_bias A_log D norm o`` to names behind ``prefix``."""
+        super().__init__(prefix)
+        self.hidden_size, self.num_heads, self.value_dim = int(hidden_size), int(num_heads), int(value_dim)
+        self.state_size, self.groups, self.conv_taps = int(state_size), int(groups), int(conv_taps)
+        self.norm_groups, self.norm_eps = int(norm_groups), float(norm_eps)
+        self.inner_width = self.num_heads * self.value_dim
+        if self.groups <= 0 or self.num_heads % self.groups:
+            raise ValueError(f"{prefix}: {num_heads} heads do not come in {groups} equal groups")
+        if self.norm_groups <= 0 or self.inner_width % self.norm_groups:
+            raise ValueError(f"{prefix}: {self.inner_width} elements are not normed in {norm_groups} equal parts")
+        if not 1 <= self.conv_taps <= 17:
+            raise ValueError(f"{prefix}: a convolution of {conv_taps} taps (1..17 are built)")
+        if not 1 <= self.state_size <= K.STATE_SPACE_MAX_STATE:
+            raise ValueError(f"{prefix}: a state of {state_size} (1..{K.STATE_SPACE_MAX_STATE} are built)")
+        self.conv_channels = self.inner_width + 2 * self.groups * self.state_size
+        self.names = _names(dict(conv="conv", conv_bias="conv.b", dt_bias="dt_bias", A_log="A_log", D="D", norm="norm", o="o",
+                                 **{"in": "in"}), tensor_names, prefix)
+
+    def tensor_specs(self) -> Dict[str, TensorSpec]:
+        n, W, H, C = self.names, self.hidden_size, self.num_heads, self.conv_channels
+        return {n["in"]: TensorSpec((self.inner_width + C + H, W)),
+                n["conv"]: TensorSpec((C, self.conv_taps), init="norm", role="vector"),
+                n["conv_bias"]: TensorSpec((C,), init="normal", role="vector"),
+                n["dt_bias"]: TensorSpec((H,), init="zeros", role="vector"), n["A_log"]: TensorSpec((H,), init="zeros", role="vector"),
+                n["D"]: TensorSpec((H,), init="norm", role="vector"),
+                n["norm"]: TensorSpec((self.inner_width,), init="norm", role="vector"),
+                n["o"]: TensorSpec((W, self.inner_width))}
+
+    def load(self, tensors: Dict[str, torch.Tensor]) -> None:
+        t = {key: tensors[name] for key, name in self.names.items()}
+        w = t["in"]
+        pad = -w.shape[0] % self.COLUMN_ALIGN
+        self._w_in = (torch.cat([w, w.new_zeros((pad, w.shape[1]))]) if pad else w).contiguous()
+        self._w_out = t["o"]
+        self.z_off, self.conv_off, self.dt_off = 0, self.inner_width, self.inner_width + self.conv_channels
+        self.conv_weight, self.conv_bias = t["conv"].float().contiguous(), t["conv_bias"].float().contiguous()
+        self.dt_bias, self.a_log, self.skip = (t[key].float().contiguous() for key in ("dt_bias", "A_log", "D"))
+        self.norm_weight = t["norm"].float().contiguous()
+        self.load_projections()
+
+    def input_weight(self) -> torch.Tensor:
+        return self._w_in
+
+    def output_weight(self) -> torch.Tensor:
+        return self._w_out
+
+    def state_elements(self) -> int:
+        return self.num_heads * self.state_size * self.value_dim + self.conv_channels * (self.conv_taps - 1)
+
+    def activation_elements(self) -> int:
+        return 3 * self.conv_channels + 4 * self.inner_width + self.hidden_size
+
+    def forward_inner(self, y, col0, ctx: MixerContext, state_off, out, out_col0, mul) -> None:
+        batch, T = ctx.batch, y.shape[0]
+        s_elems = self.num_heads * self.state_size * self.value_dim
+        xbc = torch.empty((T, self.conv_channels), dtype=torch.float32, device=y.device)
+        K.causal_conv_act(y, col0 + self.conv_off, self.conv_weight, xbc, ctx.state, state_off + s_elems, batch.entry_q_start,
+                          batch.entry_seat, batch.max_q_len, out_bias=self.conv_bias)
+        o = torch.empty((T, self.inner_width), dtype=torch.float32, device=y.device)
+        K.state_space_scan(xbc, y, col0 + self.dt_off, self.a_log, self.dt_bias, self.skip, o, ctx.state, state_off,
+                           batch.entry_q_start, batch.entry_seat, self.num_heads, self.groups, self.state_size, self.value_dim)
+        # a part of the row is a "head" of its own for the norm, and z multiplies what is normed
+        K.head_norm_gate(o, self.norm_weight, self.norm_eps, y, col0 + self.z_off, out, out_col0, self.norm_groups,
+                         self.inner_width // self.norm_groups, "silu", mul, gate_first=True)

@@ -70,6 +70,17 @@ def linear_frequencies_f64(rot_dim: int, theta: float, *, factor: float) -> np.n
     return plain_frequencies_f64(rot_dim, theta) / np.float64(factor)
 
 
+def llama3_frequencies_f64(rot_dim: int, theta: float, *, factor: float, low: float, high: float, original: float) -> np.ndarray:
+    """The llama3 rule in float64: with wavelength ``l = 2 pi / f`` a pair keeps ``f`` below ``original / high``, takes
+    ``f / factor`` above ``original / low`` and between them ``(1 - s) f / factor + s f``, ``s = (original / l - low) /
+    (high - low)``."""
+    f = plain_frequencies_f64(rot_dim, theta)
+    wave = 2.0 * math.pi / f
+    slow, fast = wave > float(original) / float(low), wave < float(original) / float(high)
+    s = (float(original) / wave - float(low)) / (float(high) - float(low)) if high != low else np.zeros_like(f)
+    return np.where(fast, f, np.where(slow, f / float(factor), (1.0 - s) * f / float(factor) + s * f))
+
+
 def yarn_frequencies(rot_dim: int, theta: float, *, factor: float, original: float, fast: float,
                      slow: float) -> np.ndarray:
     """YaRN: pair i keeps its plain frequency ``f_i`` where it turns fast and takes ``f_i / factor``
@@ -101,6 +112,7 @@ ROTARY_FREQUENCIES.register("plain", plain_frequencies, replace=True)
 ROTARY_FREQUENCIES.register("llama3", llama3_frequencies, replace=True)
 ROTARY_FREQUENCIES.register("plain_f64", plain_frequencies_f64, replace=True)
 ROTARY_FREQUENCIES.register("yarn", yarn_frequencies, replace=True)
+ROTARY_FREQUENCIES.register("llama3_f64", llama3_frequencies_f64, replace=True)
 ROTARY_FREQUENCIES.register("linear_f64", linear_frequencies_f64, replace=True)
 
 
