@@ -15,7 +15,7 @@ tokens, each with its step time, bytes and fraction of the HBM peak, and the ser
 (``kclass_...``; ``--no-kernel-classes`` leaves them out) and, for the serving runs, pages reused,
 preemptions and fragmentation failures.
 
-    python bench.py --design gadopel|radilix|lomodra|bonusun|bilolorn [--layers 8]
+    python bench.py --design gadopel|radilix|lomodra|bonusun|bilolorn|gokinex [--layers 8]
 
 is another measurement with a JSON line of its own (the default run above is untouched): prefill
 and decode throughput of a Gadopel model at layer sizes of a served model (random weights), beside
@@ -175,6 +175,29 @@ def bilolorn_config(layers: int, vocab: int, width: int = 2048) -> dict:
                        for i in range(layers)], "max_positions": 8192}
 
 
+# --design gokinex: layers of width W in runs of four - differential attention (W / 128 heads of two maps of 64 and
+# values of 128 over W / 512 kv heads: the projections of W / 64 heads of 64 over W / 256), two state-space mixers
+# (W / 64 heads of 64 with a state of 128 in W / 512 groups, four taps), and a differential attention layer that
+# reads the first one's keys and values - between tanh norms on both sides.  The first layer has a dense
+# feed-forward of 4 W (gate, up, down), the others 16 gated experts of width 3 W / 8, 4 choices a token weighted on
+# their inputs, and one more expert of that width that every token uses under a gate.  The embedding has a second
+# table for pairs of tokens.  Beside it run the closest designs, Lomodra (attention that shares keys and values,
+# recurrences with decays behind a convolution, experts of the same sizes under a router) and Bilolorn (norms on
+# both sides), and the Llama model, all at the same width.
+def gokinex_config(layers: int, vocab: int, width: int = 2048) -> dict:
+    W = width
+    moe = {"kind": "moe", "expert": {"ff": 3 * W // 8}, "router": {"experts": 16, "top": 4}, "shared": {"ff": 3 * W // 8}}
+    attn = {"heads": W // 128, "kv_heads": W // 512, "dim": 64, "vdim": 128, "scale": 0.125, "diff": 0.35,
+            "rot": {"base": 500000.0, "dims": 64, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}}
+    ssm = {"heads": W // 64, "vdim": 64, "state": 128, "groups": W // 512, "conv": 4, "norm_groups": W // 512}
+    kinds = [lambda i: ("attention", dict(attn)), lambda i: ("mamba2", ssm), lambda i: ("mamba2", ssm),
+             lambda i: ("attention", dict(attn, kv_from=i - 3))]
+    return {"architecture": "Gokinex", "vocab": vocab, "width": W, "norm": {"eps": 1e-6},
+            "embedding": {"scale": 4.0, "bigram": {"buckets": 65521, "mul_prev": 1543, "mul_cur": 769}},
+            "layers": [dict(zip(("type", "mixer"), kinds[i % 4](i)), mlp=moe if i else {"kind": "dense", "ff": 4 * W})
+                       for i in range(layers)], "max_positions": 8192}
+
+
 def design_comparison(args) -> int:
     import torch
     from kv_cache_optimization_for_llm_amd.engine.batch import StepEntry
@@ -197,6 +220,9 @@ def design_comparison(args) -> int:
     elif design == "bilolorn":
         configs = {design: bilolorn_config(layers, vocab, width), "gadopel": gadopel_config(layers, vocab, width),
                    "bonusun": bonusun_config(layers, vocab, width), "llama": llama}
+    elif design == "gokinex":
+        configs = {design: gokinex_config(layers, vocab, width), "lomodra": lomodra_config(layers, vocab, width),
+                   "bilolorn": bilolorn_config(layers, vocab, width), "llama": llama}
     elif design == "radilix":
         configs = {design: radilix_config(layers, vocab, width), "llama": llama}
     else:
@@ -285,7 +311,7 @@ def design_comparison(args) -> int:
 
 def main():
     ap = argparse.ArgumentParser()
-    ap.add_argument("--design", choices=["gadopel", "radilix", "lomodra", "bonusun", "bilolorn"], default=None,
+    ap.add_argument("--design", choices=["gadopel", "radilix", "lomodra", "bonusun", "bilolorn", "gokinex"], default=None,
                     help="another measurement (its own JSON line): a model of this design at the layer sizes of a "
                          "served model beside a Llama model of equal size; the default run is left as it is")
     ap.add_argument("--width", type=int, default=2048, help="--design: the models' width (head counts and "

@@ -1,6 +1,6 @@
 // Mixers that carry a fixed-size state per request instead of keys and values:
 //
-//  * kva_causal_conv_act / kva_conv_state_update: a short causal convolution over time per channel
+//  * kva_causal_conv_act: a short causal convolution over time per channel
 //    followed by silu; the last taps - 1 inputs of a request are part of its state.
 //  * kva_gated_delta_rule: per head S <- g S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q with
 //    unit-norm q and k, one decay g = exp(-exp(A_log) softplus(a + dt_bias)) per head and token - or a
@@ -49,75 +49,194 @@ __device__ inline float rec_column_sum(float v) {
 
 // ---- short causal convolution + silu -----------------------------------------------------
 // out[row, c] = act(sum_j w[c, j] * in(row - taps + 1 + j)[c] + out_bias[c]) with act = silu or none and
-// in = y + in_bias (both biases optional); inputs before the step's first
-// token of the request come from the seat's state [channels, taps - 1] (slot taps - 2 newest).
+// in = y + in_bias (both biases optional); inputs before the step's first token of the request come from the
+// seat's state [channels, taps - 1] (slot taps - 2 newest; it holds inputs with their bias already added, zeros
+// before a request's start), which then takes the entry's last ones.
+//
+// A thread takes VEC neighbouring channels and CONV_TOKENS tokens of an entry: all inputs it needs are asked for
+// at once, every one is loaded once.  The workgroups of an entry's first tokens are the only ones that touch its
+// state (they read it before they write it; CONV_TOKENS covers taps - 1).  TAPS = 0: any number, at run time.
+#define CONV_TOKENS 8
+#define CONV_MAX_TAPS 17
+
+struct ConvArgs {
+    void *out;
+    const void *y, *w;
+    float *state;
+    size_t seat_stride;
+    const int *entry_q_start, *entry_seat;
+    const float *in_bias, *out_bias;
+    int out_dtype, out_stride, y_dtype, y_stride, col_off, w_dtype, conv_off, channels, taps, act;
+};
+
+template <int VEC>
+__device__ inline void conv_ld(const void *p, int dtype, size_t i, float (&f)[VEC]) {
+    if constexpr (VEC == 4) {
+        if (dtype == KVA_BF16) {
+            const uint2 v = *reinterpret_cast<const uint2 *>(reinterpret_cast<const uint16_t *>(p) + i);
+            f[0] = __uint_as_float(v.x << 16); f[1] = __uint_as_float(v.x & 0xffff0000u);
+            f[2] = __uint_as_float(v.y << 16); f[3] = __uint_as_float(v.y & 0xffff0000u);
+        } else {
+            const float4 v = *reinterpret_cast<const float4 *>(reinterpret_cast<const float *>(p) + i);
+            f[0] = v.x; f[1] = v.y; f[2] = v.z; f[3] = v.w;
+        }
+    } else {
+        f[0] = rec_ld(p, dtype, i);
+    }
+}
+
+template <int VEC>
+__device__ inline void conv_store(const ConvArgs &a, size_t row, int c, float (&acc)[VEC]) {
+#pragma unroll
+    for (int v = 0; v < VEC; ++v) acc[v] = rec_act(acc[v] + (a.out_bias ? a.out_bias[c + v] : 0.f), a.act);
+    const size_t at = row * a.out_stride + c;
+    if constexpr (VEC == 4) {
+        if (a.out_dtype == KVA_BF16)
+            *reinterpret_cast<uint2 *>(reinterpret_cast<uint16_t *>(a.out) + at) =
+                make_uint2((uint32_t)float_to_bf16_bits(acc[0]) | ((uint32_t)float_to_bf16_bits(acc[1]) << 16),
+                           (uint32_t)float_to_bf16_bits(acc[2]) | ((uint32_t)float_to_bf16_bits(acc[3]) << 16));
+        else
+            *reinterpret_cast<float4 *>(reinterpret_cast<float *>(a.out) + at) = make_float4(acc[0], acc[1], acc[2], acc[3]);
+    } else {
+        rec_st(a.out, a.out_dtype, at, acc[0]);
+    }
+}
+
+template <int TAPS, int VEC>
 __global__ void __launch_bounds__(256)
-causal_conv_act_kernel(float *__restrict__ out, int out_stride, const void *__restrict__ y, int y_dtype, int y_stride,
-                       int col_off, const void *__restrict__ w, int w_dtype, const float *__restrict__ state,
-                       size_t seat_stride, int conv_off, const int *__restrict__ entry_q_start,
-                       const int *__restrict__ entry_seat, int channels, int taps, int tokens_per_block,
-                       const float *__restrict__ in_bias, const float *__restrict__ out_bias, int act) {
-    const int e = blockIdx.y;
-    const int q0 = entry_q_start[e], n = entry_q_start[e + 1] - q0;
-    const int first = blockIdx.x * tokens_per_block;
-    if (first >= n) return;
-    const int last = min(n, first + tokens_per_block);
-    const float *st = state + (size_t)entry_seat[e] * seat_stride + conv_off;
-    for (int c = threadIdx.x; c < channels; c += blockDim.x) {
-        for (int i = first; i < last; ++i) {
-            float acc = 0.f;
-            for (int j = 0; j < taps; ++j) {
-                const int src = i - (taps - 1) + j;
-                // (the state holds inputs with their bias already added; before a request's start it holds zeros)
-                const float x = src >= 0 ? rec_ld(y, y_dtype, (size_t)(q0 + src) * y_stride + col_off + c) + (in_bias ? in_bias[c] : 0.f)
-                                         : st[(size_t)c * (taps - 1) + (taps - 1) + src];
-                acc += rec_ld(w, w_dtype, (size_t)c * taps + j) * x;
-            }
-            if (out_bias) acc += out_bias[c];
-            out[(size_t)(q0 + i) * out_stride + c] = rec_act(acc, act);
+causal_conv_act_kernel(ConvArgs a) {
+    constexpr int KEEP = TAPS > 0 ? TAPS - 1 : CONV_MAX_TAPS - 1, TOKENS = TAPS > 0 ? CONV_TOKENS : 2 * CONV_TOKENS;
+    const int taps = TAPS > 0 ? TAPS : a.taps, back = taps - 1;
+    const int e = blockIdx.z;
+    const int q0 = a.entry_q_start[e], n = a.entry_q_start[e + 1] - q0;
+    const int first = blockIdx.y * TOKENS, c = (blockIdx.x * blockDim.x + threadIdx.x) * VEC;
+    if (first >= n || c >= a.channels) return;
+    const int count = min(TOKENS, n - first);
+    float bias[VEC];
+#pragma unroll
+    for (int v = 0; v < VEC; ++v) bias[v] = a.in_bias ? a.in_bias[c + v] : 0.f;
+    float *st = a.state + (size_t)a.entry_seat[e] * a.seat_stride + a.conv_off + (size_t)c * back;
+    auto input = [&](int i, float (&f)[VEC]) {                   // the entry's token i
+        conv_ld<VEC>(a.y, a.y_dtype, (size_t)(q0 + i) * a.y_stride + a.col_off + c, f);
+#pragma unroll
+        for (int v = 0; v < VEC; ++v) f[v] += bias[v];
+    };
+    // the inputs in front of the first token: the state's, or the tokens of the workgroup before
+    float old[KEEP > 0 ? KEEP : 1][VEC];
+#pragma unroll
+    for (int j = 0; j < KEEP; ++j) {
+        if (j >= back) break;
+        if (first == 0) {
+#pragma unroll
+            for (int v = 0; v < VEC; ++v) old[j][v] = st[(size_t)v * back + j];
+        } else {
+            input(first - back + j, old[j]);
         }
     }
-}
-
-// the seat's last taps - 1 inputs after this step; a thread owns a channel (reads all, then writes)
-__global__ void __launch_bounds__(256)
-conv_state_update_kernel(float *__restrict__ state, size_t seat_stride, int conv_off, const void *__restrict__ y,
-                         int y_dtype, int y_stride, int col_off, const int *__restrict__ entry_q_start,
-                         const int *__restrict__ entry_seat, int channels, int taps, const float *__restrict__ in_bias) {
-    const int e = blockIdx.y;
-    const int q0 = entry_q_start[e], n = entry_q_start[e + 1] - q0;
-    const int c = blockIdx.x * blockDim.x + threadIdx.x;
-    if (c >= channels || n <= 0) return;
-    float *st = state + (size_t)entry_seat[e] * seat_stride + conv_off + (size_t)c * (taps - 1);
-    float keep[16];
-    for (int s = 0; s < taps - 1; ++s) {
-        const int src = n - (taps - 1) + s;
-        keep[s] = src >= 0 ? rec_ld(y, y_dtype, (size_t)(q0 + src) * y_stride + col_off + c) + (in_bias ? in_bias[c] : 0.f) : st[s + n];
+    if constexpr (TAPS > 0) {
+        float in[TOKENS][VEC], w[TAPS][VEC];
+#pragma unroll
+        for (int i = 0; i < TOKENS; ++i) {
+#pragma unroll
+            for (int v = 0; v < VEC; ++v) in[i][v] = 0.f;
+            if (i < count) input(first + i, in[i]);
+        }
+#pragma unroll
+        for (int j = 0; j < TAPS; ++j)
+#pragma unroll
+            for (int v = 0; v < VEC; ++v) w[j][v] = rec_ld(a.w, a.w_dtype, (size_t)(c + v) * TAPS + j);
+#pragma unroll
+        for (int i = 0; i < TOKENS; ++i) {
+            if (i >= count) break;
+            float acc[VEC];
+#pragma unroll
+            for (int v = 0; v < VEC; ++v) {
+                acc[v] = 0.f;
+#pragma unroll
+                for (int j = 0; j < TAPS; ++j) {
+                    const int src = i - (TAPS - 1) + j;
+                    acc[v] += w[j][v] * (src >= 0 ? in[src >= 0 ? src : 0][v] : old[src < 0 ? TAPS - 1 + src : 0][v]);
+                }
+            }
+            conv_store<VEC>(a, (size_t)(q0 + first + i), c, acc);
+        }
+    } else {
+        for (int i = 0; i < count; ++i) {
+            float acc[VEC];
+#pragma unroll
+            for (int v = 0; v < VEC; ++v) acc[v] = 0.f;
+#pragma unroll
+            for (int j = 0; j < CONV_MAX_TAPS; ++j) {
+                if (j >= taps) break;
+                const int src = i - back + j;
+                float f[VEC];
+                if (src >= 0 || first > 0) input(first + src, f);
+                else
+#pragma unroll
+                    for (int v = 0; v < VEC; ++v) f[v] = st[(size_t)v * back + back + src];
+#pragma unroll
+                for (int v = 0; v < VEC; ++v) acc[v] += rec_ld(a.w, a.w_dtype, (size_t)(c + v) * taps + j) * f[v];
+            }
+            conv_store<VEC>(a, (size_t)(q0 + first + i), c, acc);
+        }
     }
-    for (int s = 0; s < taps - 1; ++s) st[s] = keep[s];
+    if (first > 0) return;
+    // the state behind the entry: its last taps - 1 inputs, older ones moved up
+    float keep[KEEP > 0 ? KEEP : 1][VEC];
+#pragma unroll
+    for (int j = 0; j < KEEP; ++j) {
+        if (j >= back) break;
+        const int src = n - back + j;
+        if (src >= 0) {
+            input(src, keep[j]);
+        } else {
+#pragma unroll
+            for (int k = 0; k < KEEP; ++k)              // (an index known when the code is compiled)
+                if (k == j + n)
+#pragma unroll
+                    for (int v = 0; v < VEC; ++v) keep[j][v] = old[k][v];
+        }
+    }
+#pragma unroll
+    for (int j = 0; j < KEEP; ++j) {
+        if (j >= back) break;
+#pragma unroll
+        for (int v = 0; v < VEC; ++v) st[(size_t)v * back + j] = keep[j][v];
+    }
 }
 
-extern "C" int kva_causal_conv_act(float *out, int out_stride, const void *y, int y_dtype, int y_stride, int col_off,
+extern "C" int kva_causal_conv_act(void *out, int out_dtype, int out_stride, const void *y, int y_dtype, int y_stride, int col_off,
                                    const void *w, int w_dtype, float *state, long long seat_stride, int conv_off,
                                    const int *entry_q_start, const int *entry_seat, int entries, int max_q_len,
                                    int channels, int taps, const float *in_bias, const float *out_bias, int act,
                                    hipStream_t stream) {
     KVA_REQUIRE(act == 0 || act == 1, "causal_conv_act: activation %d is neither none (0) nor silu (1)", act);
     KVA_REQUIRE(out && y && w && state && entry_q_start && entry_seat, "causal_conv_act: missing operand");
-    KVA_REQUIRE(channels > 0 && taps >= 1 && taps <= 17, "causal_conv_act: taps %d must lie in 1..17", taps);
+    KVA_REQUIRE(out_dtype == KVA_F32 || out_dtype == KVA_BF16, "causal_conv_act: unsupported dtype %d", out_dtype);
+    KVA_REQUIRE(channels > 0 && taps >= 1 && taps <= CONV_MAX_TAPS, "causal_conv_act: taps %d must lie in 1..%d", taps, CONV_MAX_TAPS);
     KVA_REQUIRE(entries >= 0 && entries <= 65535 && max_q_len >= 0, "causal_conv_act: bad batch");
     if (entries == 0 || max_q_len == 0) return KVA_OK;
-    const int per = 8;
-    hipLaunchKernelGGL(causal_conv_act_kernel, dim3((max_q_len + per - 1) / per, entries), dim3(256), 0, stream, out,
-                       out_stride, y, y_dtype, y_stride, col_off, w, w_dtype, state, (size_t)seat_stride, conv_off,
-                       entry_q_start, entry_seat, channels, taps, per, in_bias, out_bias, act);
+    const ConvArgs a{out, y, w, state, (size_t)seat_stride, entry_q_start, entry_seat, in_bias, out_bias, out_dtype, out_stride,
+                     y_dtype, y_stride, col_off, w_dtype, conv_off, channels, taps, act};
+    const bool vec = channels % 4 == 0 && y_stride % 4 == 0 && col_off % 4 == 0 && out_stride % 4 == 0 &&
+                     ((reinterpret_cast<uintptr_t>(y) | reinterpret_cast<uintptr_t>(out)) & 15) == 0;
+    const bool fixed = taps >= 2 && taps <= 4;
+    const int tokens = fixed ? CONV_TOKENS : 2 * CONV_TOKENS;
+    // (a decoded token: narrower workgroups, so that more of them share the work)
+    const int width = vec ? 4 : 1, threads = max_q_len == 1 ? 64 : 256;
+    const dim3 grid((channels + threads * width - 1) / (threads * width), (max_q_len + tokens - 1) / tokens, entries);
+    KVA_REQUIRE(grid.y <= 65535, "causal_conv_act: portions of %d tokens", max_q_len);
+#define KVA_CONV(TAPS)                                                                                        \
+    do {                                                                                                      \
+        if (vec) hipLaunchKernelGGL((causal_conv_act_kernel<TAPS, 4>), grid, dim3(threads), 0, stream, a);    \
+        else hipLaunchKernelGGL((causal_conv_act_kernel<TAPS, 1>), grid, dim3(threads), 0, stream, a);        \
+    } while (0)
+    if (taps == 2) KVA_CONV(2);
+    else if (taps == 3) KVA_CONV(3);
+    else if (taps == 4) KVA_CONV(4);
+    else KVA_CONV(0);
+#undef KVA_CONV
     KVA_CHECK_LAUNCH("causal_conv_act");
-    if (taps > 1) {
-        hipLaunchKernelGGL(conv_state_update_kernel, dim3((channels + 255) / 256, entries), dim3(256), 0, stream, state,
-                           (size_t)seat_stride, conv_off, y, y_dtype, y_stride, col_off, entry_q_start, entry_seat,
-                           channels, taps, in_bias);
-        KVA_CHECK_LAUNCH("conv_state_update");
-    }
     return KVA_OK;
 }
 
@@ -780,6 +899,92 @@ head_norm_gate_wide_kernel(void *__restrict__ out, int out_dtype, int out_stride
     }
 }
 
+// The same with a head's elements in registers, 8 neighbouring ones a lane at a time: `lanes` (a power of two up to
+// 64) lanes take a head, or (WIDE) a workgroup does.  For heads of a multiple of 8 elements, up to HNG_KEEP * 8 *
+// lanes of them, with every row at a multiple of 16 bytes.
+#define HNG_KEEP 4
+
+__device__ inline void hng_ld8(const void *p, int dtype, size_t i, float (&f)[8]) {
+    if (dtype == KVA_BF16) {
+        const uint4 v = *reinterpret_cast<const uint4 *>(reinterpret_cast<const uint16_t *>(p) + i);
+        const uint32_t u[4] = {v.x, v.y, v.z, v.w};
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            f[2 * j] = __uint_as_float(u[j] << 16);
+            f[2 * j + 1] = __uint_as_float(u[j] & 0xffff0000u);
+        }
+    } else {
+        const float4 a = *reinterpret_cast<const float4 *>(reinterpret_cast<const float *>(p) + i);
+        const float4 b = *reinterpret_cast<const float4 *>(reinterpret_cast<const float *>(p) + i + 4);
+        f[0] = a.x; f[1] = a.y; f[2] = a.z; f[3] = a.w; f[4] = b.x; f[5] = b.y; f[6] = b.z; f[7] = b.w;
+    }
+}
+
+template <bool WIDE>
+__global__ void __launch_bounds__(256)
+head_norm_gate_vec_kernel(void *__restrict__ out, int out_dtype, int out_stride, int out_off, const void *__restrict__ x,
+                          int x_dtype, const float *__restrict__ w, float eps, HeadGate gate, int rows, int heads, int dv,
+                          float mul, int w_stride, int lanes) {
+    __shared__ float red_s[4];
+    const int lane = threadIdx.x % lanes;                                   // (WIDE: lanes = 256)
+    const int unit = WIDE ? blockIdx.x : (blockIdx.x * blockDim.x + threadIdx.x) / lanes;
+    const bool live = unit < rows * heads;
+    const int u = live ? unit : rows * heads - 1;                           // idle lanes repeat the last head
+    const size_t t = u / heads;
+    const int h = u % heads, step = 8 * lanes;
+    float v[HNG_KEEP][8], gt[HNG_KEEP][8];
+    float sq = 0.f;
+#pragma unroll
+    for (int k = 0; k < HNG_KEEP; ++k) {
+        const int j = 8 * lane + k * step;
+#pragma unroll
+        for (int i = 0; i < 8; ++i) { v[k][i] = 0.f; gt[k][i] = 1.f; }
+        if (j >= dv) continue;
+        hng_ld8(x, x_dtype, (size_t)u * dv + j, v[k]);
+        if (gate.p) hng_ld8(gate.p, gate.dtype, t * gate.stride + gate.off + (size_t)h * dv + j, gt[k]);
+    }
+#pragma unroll
+    for (int k = 0; k < HNG_KEEP; ++k) {
+        if (8 * lane + k * step >= dv) continue;
+#pragma unroll
+        for (int i = 0; i < 8; ++i) {
+            if (gate.p) gt[k][i] = gate.act == 1 ? rec_sigmoid(gt[k][i]) : rec_silu(gt[k][i]);
+            if (gate.first) v[k][i] *= gt[k][i];
+            sq += v[k][i] * v[k][i];
+        }
+    }
+    float inv = 1.f;
+    if (w) {
+        if constexpr (WIDE) sq = block_sum(sq, red_s, 4);
+        else for (int o = lanes / 2; o > 0; o >>= 1) sq += __shfl_xor(sq, o, KVA_WAVE);
+        inv = 1.0f / sqrtf(sq / (float)dv + eps);
+    }
+    if (!live) return;
+#pragma unroll
+    for (int k = 0; k < HNG_KEEP; ++k) {
+        const int j = 8 * lane + k * step;
+        if (j >= dv) continue;
+        float wv[8];
+#pragma unroll
+        for (int i = 0; i < 8; ++i) wv[i] = 1.f;
+        if (w) hng_ld8(w, KVA_F32, (size_t)h * w_stride + j, wv);
+#pragma unroll
+        for (int i = 0; i < 8; ++i) v[k][i] = v[k][i] * inv * wv[i] * (gate.first ? 1.f : gt[k][i]) * mul;
+        const size_t at = t * out_stride + out_off + (size_t)h * dv + j;
+        if (out_dtype == KVA_BF16) {
+            uint32_t o[4];
+#pragma unroll
+            for (int i = 0; i < 4; ++i)
+                o[i] = (uint32_t)float_to_bf16_bits(v[k][2 * i]) | ((uint32_t)float_to_bf16_bits(v[k][2 * i + 1]) << 16);
+            *reinterpret_cast<uint4 *>(reinterpret_cast<uint16_t *>(out) + at) = make_uint4(o[0], o[1], o[2], o[3]);
+        } else {
+            float4 *dst = reinterpret_cast<float4 *>(reinterpret_cast<float *>(out) + at);
+            dst[0] = make_float4(v[k][0], v[k][1], v[k][2], v[k][3]);
+            dst[1] = make_float4(v[k][4], v[k][5], v[k][6], v[k][7]);
+        }
+    }
+}
+
 extern "C" int kva_head_norm_gate(void *out, int out_dtype, int out_stride, int out_off, const void *x, int x_dtype,
                                   const float *w, float eps, const void *gate, int gate_dtype, int gate_stride,
                                   int gate_off, int rows, int heads, int dv, int act, int gate_first, float mul, int w_stride,
@@ -791,7 +996,21 @@ extern "C" int kva_head_norm_gate(void *out, int out_dtype, int out_stride, int 
     KVA_REQUIRE(!gate_first || gate, "head_norm_gate: a gate in front of the norm needs the gate");
     if (rows == 0) return KVA_OK;
     const HeadGate hg{gate, gate_dtype, gate_stride, gate_off, act, gate_first};
-    if (heads < 4 && dv >= 256)
+    // (which kernel runs depends on sizes and alignment alone, never on the rows: a row's numbers are the same in any batch)
+    const bool vec = dv % 8 == 0 && dv <= 256 * 8 * HNG_KEEP && out_stride % 8 == 0 && out_off % 8 == 0 && w_stride % 8 == 0 &&
+                     (!gate || (gate_stride % 8 == 0 && gate_off % 8 == 0)) && (long long)rows * heads < (1LL << 24) &&
+                     ((reinterpret_cast<uintptr_t>(out) | reinterpret_cast<uintptr_t>(x) | reinterpret_cast<uintptr_t>(gate) |
+                       reinterpret_cast<uintptr_t>(w)) & 15) == 0;
+    if (vec && dv > 512) {
+        hipLaunchKernelGGL(head_norm_gate_vec_kernel<true>, dim3((unsigned)(rows * heads)), dim3(256), 0, stream, out, out_dtype,
+                           out_stride, out_off, x, x_dtype, w, eps, hg, rows, heads, dv, mul, w_stride, 256);
+    } else if (vec) {
+        int lanes = 1;
+        while (lanes < dv / 8) lanes *= 2;
+        hipLaunchKernelGGL(head_norm_gate_vec_kernel<false>, dim3((unsigned)(((long long)rows * heads * lanes + 255) / 256)),
+                           dim3(256), 0, stream, out, out_dtype, out_stride, out_off, x, x_dtype, w, eps, hg, rows, heads, dv,
+                           mul, w_stride, lanes);
+    } else if (heads < 4 && dv >= 256)
         hipLaunchKernelGGL(head_norm_gate_wide_kernel, dim3(rows), dim3(256), 0, stream, out, out_dtype, out_stride, out_off,
                            x, x_dtype, w, eps, hg, heads, dv, mul, w_stride);
     else

@@ -1691,7 +1691,7 @@ def causal_conv_act(y: torch.Tensor, col_off: int, weight: torch.Tensor, out: to
     weight[c, j] * in[t - taps + 1 + j, c])`` with ``in`` the columns ``col_off ..`` of ``y``; the inputs
     before an entry's first token come from the seat's state (``taps - 1`` values per channel at
     ``state_off``, oldest first; zero for a fresh seat), which afterwards holds the entry's last ones.
-    ``out`` is fp32 ``[T, channels]``.  ``in_bias`` (fp32 per channel) is added to every input (the state
+    ``out`` is ``[T, channels]``, fp32 or bf16.  ``in_bias`` (fp32 per channel) is added to every input (the state
     holds inputs with it), ``out_bias`` to every sum; ``activation`` is ``"silu"`` or ``None``."""
     tokens, channels = out.shape
     for bias in (in_bias, out_bias):
@@ -1699,14 +1699,14 @@ def causal_conv_act(y: torch.Tensor, col_off: int, weight: torch.Tensor, out: to
             raise KernelError("causal_conv_act: a bias is fp32, one value per channel")
     if activation not in (None, "silu"):
         raise KernelError(f"causal_conv_act: activation {activation!r} is neither None nor 'silu'")
-    if weight.dim() != 2 or weight.shape[0] != channels or out.dtype != torch.float32 or y.dim() != 2 \
+    if weight.dim() != 2 or weight.shape[0] != channels or y.dim() != 2 \
             or y.shape[0] != tokens or col_off < 0 or col_off + channels > y.shape[1]:
         raise KernelError(f"causal_conv_act: y {tuple(y.shape)}, weight {tuple(weight.shape)}, out {tuple(out.shape)} do not fit")
     taps = weight.shape[1]
     seat_stride = _state_row(state, state_off, channels * (taps - 1), "causal_conv_act")
     qs, seat, entries = _entries((entry_q_start, entry_seat), "causal_conv_act")
     check(hip_lib().kva_causal_conv_act(
-        _dev(out, "out"), channels, _dev(y, "y"), dtype_code(y.dtype), y.shape[1], int(col_off), _dev(weight, "weight"),
+        _dev(out, "out"), dtype_code(out.dtype), channels, _dev(y, "y"), dtype_code(y.dtype), y.shape[1], int(col_off), _dev(weight, "weight"),
         dtype_code(weight.dtype), _dev(state, "state"), seat_stride, int(state_off), qs, seat, entries, int(max_q_len),
         channels, taps, _opt(in_bias, "in_bias"), _opt(out_bias, "out_bias"), 1 if activation == "silu" else 0,
         _stream()), "causal_conv_act")
@@ -1787,30 +1787,52 @@ def gated_linear_attention(y: torch.Tensor, q_off: int, k_off: int, v_off: int, 
 
 
 STATE_SPACE_MAX_STATE = 512
+STATE_SPACE_KERNELS = {"scan": 0, "token": 1, "chunks": 2}
+STATE_SPACE_CHUNK_FROM = 24         # entries of so many tokens and more go in chunks on the matrix cores
 
 
-def state_space_scan(xbc: torch.Tensor, y: torch.Tensor, dt_off: int, a_log: torch.Tensor, dt_bias: torch.Tensor,
-                     skip: torch.Tensor, out: torch.Tensor, state: torch.Tensor, state_off: int, entry_q_start: torch.Tensor,
-                     entry_seat: torch.Tensor, heads: int, groups: int, state_size: int, vdim: int) -> torch.Tensor:
+def state_space_plan(lengths, heads: int, groups: int, state_size: int, vdim: int, dtype: torch.dtype) -> list:
+    """The launches of :func:`state_space` for entries of ``lengths`` tokens (host numbers): ``(kernel, shortest,
+    longest)``.  Which kernel takes an entry depends on its own length and the sizes alone."""
+    def takes(kernel):
+        return bool(hip_lib().kva_state_space_supported(STATE_SPACE_KERNELS[kernel], int(heads), int(groups), int(state_size),
+                                                        int(vdim), dtype_code(dtype)))
+    token = 1 if takes("token") else 0
+    chunk = STATE_SPACE_CHUNK_FROM if takes("chunks") else 1 << 30
+    ranges = [("token", 1, token), ("scan", token + 1, chunk - 1), ("chunks", chunk, 1 << 30)]
+    return [(k, lo, hi) for k, lo, hi in ranges if any(lo <= int(n) <= hi for n in lengths)]
+
+
+def state_space(xbc: torch.Tensor, y: torch.Tensor, dt_off: int, a_log: torch.Tensor, dt_bias: torch.Tensor,
+                skip: torch.Tensor, out: torch.Tensor, state: torch.Tensor, state_off: int, entry_q_start: torch.Tensor,
+                entry_seat: torch.Tensor, heads: int, groups: int, state_size: int, vdim: int, lengths,
+                plan: Optional[list] = None) -> torch.Tensor:
     """Per head and token, in order: ``dt = softplus(y[t, dt_off + h] + dt_bias[h])``, ``S <- exp(-exp(a_log[h]) dt) S
-    + dt B x^T``, ``out = S^T C + skip[h] x``.  ``xbc`` fp32 ``[T, heads vdim + 2 groups state_size]`` holds x, then B
-    and C of every group; head h uses group ``h // (heads / groups)``.  ``S`` ``[heads, state_size, vdim]`` lives at
-    ``state_off`` of the seat's fp32 state row; ``out`` is fp32 ``[T, heads * vdim]``."""
+    + dt B x^T``, ``out = S^T C + skip[h] x``.  ``xbc`` (fp32 or bf16) ``[T, heads vdim + 2 groups state_size]`` holds x,
+    then B and C of every group; head h uses group ``h // (heads / groups)``.  ``S`` ``[heads, state_size, vdim]`` lives
+    at ``state_off`` of the seat's fp32 state row; ``out`` is fp32 ``[T, heads * vdim]``.  ``lengths``: the entries'
+    numbers of tokens on the host, from which the launches are chosen (``plan``: other ones)."""
     tokens = out.shape[0]
-    if heads % groups or xbc.shape != (tokens, heads * vdim + 2 * groups * state_size) or xbc.dtype != torch.float32 \
+    if heads % groups or xbc.shape != (tokens, heads * vdim + 2 * groups * state_size) \
             or out.shape != (tokens, heads * vdim) or out.dtype != torch.float32 or y.dim() != 2 or y.shape[0] != tokens:
-        raise KernelError(f"state_space_scan: xbc {tuple(xbc.shape)}, y {tuple(y.shape)}, out {tuple(out.shape)} do not fit")
+        raise KernelError(f"state_space: xbc {tuple(xbc.shape)}, y {tuple(y.shape)}, out {tuple(out.shape)} do not fit")
     if not 0 <= dt_off <= y.shape[1] - heads:
-        raise KernelError("state_space_scan: the step sizes' columns lie outside y")
+        raise KernelError("state_space: the step sizes' columns lie outside y")
     for v in (a_log, dt_bias, skip):
         if v.shape != (heads,) or v.dtype != torch.float32:
-            raise KernelError("state_space_scan: rates, step biases and skips are fp32, one a head")
-    seat_stride = _state_row(state, state_off, heads * state_size * vdim, "state_space_scan")
-    qs, seat, entries = _entries((entry_q_start, entry_seat), "state_space_scan")
-    check(hip_lib().kva_state_space_scan(
-        _dev(out, "out"), _dev(state, "state"), seat_stride, int(state_off), _dev(xbc, "xbc"), xbc.shape[1], _dev(y, "y"),
-        dtype_code(y.dtype), y.shape[1], int(dt_off), _dev(a_log, "a_log"), _dev(dt_bias, "dt_bias"), _dev(skip, "skip"), qs,
-        seat, entries, int(heads), int(groups), int(state_size), int(vdim), _stream()), "state_space_scan")
+            raise KernelError("state_space: rates, step biases and skips are fp32, one a head")
+    seat_stride = _state_row(state, state_off, heads * state_size * vdim, "state_space")
+    qs, seat, entries = _entries((entry_q_start, entry_seat), "state_space")
+    if plan is None:
+        # (the walk over the tokens takes any state; the other kernels want it at multiples of 16 bytes)
+        plan = [("scan", 1, 1 << 30)] if state_off % 4 or seat_stride % 4 else \
+            state_space_plan(lengths, heads, groups, state_size, vdim, xbc.dtype)
+    for kernel, lo, hi in plan:
+        check(hip_lib().kva_state_space(
+            STATE_SPACE_KERNELS[kernel], int(lo), int(hi), _dev(out, "out"), _dev(state, "state"), seat_stride, int(state_off),
+            _dev(xbc, "xbc"), dtype_code(xbc.dtype), xbc.shape[1], _dev(y, "y"), dtype_code(y.dtype), y.shape[1], int(dt_off),
+            _dev(a_log, "a_log"), _dev(dt_bias, "dt_bias"), _dev(skip, "skip"), qs, seat, entries, int(heads), int(groups),
+            int(state_size), int(vdim), _stream()), "state_space")
     return out
 
 
@@ -2137,7 +2159,7 @@ KERNEL_CLASSES = {
     "norm_into_stream": "norm", "table_gate": "elementwise",
     "hyper_step": "norm", "sandwich_step": "norm", "hyper_fill": "embedding", "bias_act": "activation",
     "tanh_step": "norm", "pair_embed": "embedding", "maps_encode_cache": "rope + cache write", "maps_combine": "elementwise",
-    "state_space_scan": "recurrent mixers",
+    "state_space": "recurrent mixers",
     "block_gates": "recurrent mixers", "linear_scan_gate": "recurrent mixers", "matrix_memory": "recurrent mixers",
 }
 

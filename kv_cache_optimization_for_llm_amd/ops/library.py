@@ -91,7 +91,7 @@ _HIP_SIGNATURES = {
     "kva_host_memory_is_mapped": [P],
     "kva_sample": [P, P, I, I, I, P, P, F, P, U, P, P, I, P, P, P, P, P],
     "kva_mark_tokens": [P, P, P, I, I, P],
-    "kva_causal_conv_act": [P, I, P, I, I, I, P, I, P, LL, I, P, P, I, I, I, I, P, P, I, P],
+    "kva_causal_conv_act": [P, I, I, P, I, I, I, P, I, P, LL, I, P, P, I, I, I, I, P, P, I, P],
     "kva_gated_delta_rule": [P, P, LL, I, P, I, P, I, I, I, I, P, P, F, P, I, P, P, I, I, I, I, I, P],
     "kva_gated_linear_attention": [P, P, LL, I, P, I, I, I, I, I, P, I, F, P, I, P, P, I, I, I, I, P],
     "kva_head_norm_gate": [P, I, I, I, P, I, P, F, P, I, I, I, I, I, I, I, I, F, I, P],
@@ -112,7 +112,8 @@ _HIP_SIGNATURES = {
     "kva_pair_embed": [P, P, I, I, F, P, I, I, I, I, P, P, I, F, P, P, P, I, P, P, I, I, I, P],
     "kva_maps_encode_cache": [P, I, P, P, P, P, P, P, P, I, I, I, I, I, I, I, I, P, I, P],
     "kva_maps_combine": [P, I, I, P, F, F, F, I, I, I, I, P],
-    "kva_state_space_scan": [P, P, LL, I, P, I, P, I, I, I, P, P, P, P, P, I, I, I, I, I, P],
+    "kva_state_space": [I, I, I, P, P, LL, I, P, I, I, P, I, I, I, P, P, P, P, P, I, I, I, I, I, P],
+    "kva_state_space_supported": [I, I, I, I, I, I],
     "kva_hyper_fill": [P, P, I, I, I, I, P],
     "kva_block_gates": [P, P, P, I, I, I, P, P, I, P, P, P, P],
     "kva_linear_scan_gate": [P, I, I, I, P, P, I, P, I, I, I, P, P, LL, I, P, P, I, F, P],

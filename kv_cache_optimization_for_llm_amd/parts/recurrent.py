@@ -32,6 +32,7 @@ from __future__ import annotations
 
 from typing import Dict, Optional
 
+import numpy as np
 import torch
 
 from ..config.registry import MIXERS
@@ -538,7 +539,8 @@ class StateSpaceDuality(ProjectedMixer):
         return self._w_out
 
     def state_elements(self) -> int:
-        return self.num_heads * self.state_size * self.value_dim + self.conv_channels * (self.conv_taps - 1)
+        n = self.num_heads * self.state_size * self.value_dim + self.conv_channels * (self.conv_taps - 1)
+        return (n + 3) // 4 * 4          # (every seat's row starts at a multiple of 16 bytes)
 
     def activation_elements(self) -> int:
         return 3 * self.conv_channels + 4 * self.inner_width + self.hidden_size
@@ -546,12 +548,13 @@ class StateSpaceDuality(ProjectedMixer):
     def forward_inner(self, y, col0, ctx: MixerContext, state_off, out, out_col0, mul) -> None:
         batch, T = ctx.batch, y.shape[0]
         s_elems = self.num_heads * self.state_size * self.value_dim
-        xbc = torch.empty((T, self.conv_channels), dtype=torch.float32, device=y.device)
+        xbc = torch.empty((T, self.conv_channels), dtype=y.dtype, device=y.device)
         K.causal_conv_act(y, col0 + self.conv_off, self.conv_weight, xbc, ctx.state, state_off + s_elems, batch.entry_q_start,
                           batch.entry_seat, batch.max_q_len, out_bias=self.conv_bias)
         o = torch.empty((T, self.inner_width), dtype=torch.float32, device=y.device)
-        K.state_space_scan(xbc, y, col0 + self.dt_off, self.a_log, self.dt_bias, self.skip, o, ctx.state, state_off,
-                           batch.entry_q_start, batch.entry_seat, self.num_heads, self.groups, self.state_size, self.value_dim)
+        K.state_space(xbc, y, col0 + self.dt_off, self.a_log, self.dt_bias, self.skip, o, ctx.state, state_off,
+                      batch.entry_q_start, batch.entry_seat, self.num_heads, self.groups, self.state_size, self.value_dim,
+                      np.diff(batch.h_entry_q_start))
         # a part of the row is a "head" of its own for the norm, and z multiplies what is normed
         K.head_norm_gate(o, self.norm_weight, self.norm_eps, y, col0 + self.z_off, out, out_col0, self.norm_groups,
                          self.inner_width // self.norm_groups, "silu", mul, gate_first=True)
