@@ -5,7 +5,7 @@
 // S [state, value] per head, dt_t = softplus(y[t, dt_off + h] + dt_bias_h), rate_h = exp(A_log_h).  B and C
 // belong to groups of heads.  S is fp32, starts at zero and lives in the seat's state row between steps.
 //
-// Three kernels; each takes the entries whose number of tokens lies in a range the caller names.
+// Kernels for three kinds of entries; each takes the entries whose number of tokens lies in a range the caller names.
 //
 //  * state_space_scan_kernel walks the tokens.  Value columns of S are independent of each other: a workgroup
 //    of four wavefronts takes 16 of a head's, a wavefront 4, the 16 lanes of a row of the wavefront share a
@@ -13,7 +13,7 @@
 //    C, the 16 columns of x, the two numbers of every token - is staged in LDS for the four wavefronts while
 //    the one before is walked.  The order of every sum depends on the sizes alone.
 //  * state_space_token_kernel is a single token: S passes through registers once, 16 bytes a lane.
-//  * state_space_chunk_kernel (bf16 rows) takes chunks of 64 tokens on the matrix cores.  With c_t the sum of
+//  * state_space_states_kernel and state_space_outputs_kernel (bf16 rows) take chunks of 64 tokens on the matrix cores.  With c_t the sum of
 //    -rate dt up to t inside the chunk and S_0 the state in front of it,
 //        y_t = sum_(s <= t) (C_t . B_s) e^(c_t - c_s) dt_s x_s + e^(c_t) S_0^T C_t + D x_t,
 //        S   = e^(c_64) S_0 + sum_s B_s (e^(c_64 - c_s) dt_s x_s)^T.
@@ -247,24 +247,18 @@ state_space_token_kernel(SsmArgs a) {
 }
 
 // ---- chunks of 64 tokens on the matrix cores -------------------------------------------------------------
-// A workgroup takes 16 value columns of a head and walks the entry's chunks; NK = state size / 32 (rounded up,
-// the rest is zero).  Everything is computed transposed: lane (r = lane % 16, g = lane / 16) of a product's result
-// holds rows 4 g .. + 3 of column r.  Wavefront w takes the chunk's tokens t = 16 w .. + 15 as columns:
-//   (1) G^T[s, t] = B_s . C_t for the tiles s <= t;
-//   (2) the weights e^(c_t - c_s) dt_s G, in registers the second operand of y^T[p, t] = sum_s x^T[p, s] W^T[s, t],
-//       whose first operand is x read from LDS with the transposing load (k index: the permutation of 32 tokens
-//       in which (1) left them);
-//   (3) e^(c_t) S_0^T C with S_0^T [p, state] in LDS;
-//   (4) the wavefront's part of the state, tiles of 16 state rows w, w + 4, ..: S^T[p, n] = e^(c_64) S^T + sum_s
-//       (weighted x)^T[p, s] B[s, n], both operands by transposing loads.
-// S lives in registers and lies, as two bf16 numbers, in LDS for (3), two buffers deep: two barriers a chunk.  The
-// next chunk's rows are loaded while this one is worked on.
+// Two kernels.  state_space_states_kernel walks an entry's chunks and does nothing but hand S on: for every chunk it
+// leaves the state in front of it in a workspace.  state_space_outputs_kernel takes the chunks side by side.
+//
+// Lane (r = lane % 16, g = lane / 16) of a product's result holds rows 4 g .. + 3 of column r.  S [state, value] is kept
+// so - a value column a lane, NK = state size / 32 (rounded up, the rest is zero) pairs of tiles of 16 state rows -
+// and a pair of tiles is then, as it lies in the registers, an operand whose k index is the permutation (j / 4) 16 +
+// 4 g + j % 4 of 32 state rows; C and B are read in the same permutation (two pieces of 4 elements).
 #define SSM_CHUNK 64
-#define SSM_XS 24                // LDS stride of rows of 16 columns of x
 
 typedef __attribute__((address_space(3))) s16x4 ssm_lds_s16x4;
 
-// row stride in LDS, in elements, of rows of n (a multiple of 32): an odd multiple of 4 words whose first three
+// row stride in LDS, in elements, of rows of n (a multiple of 16): an odd multiple of 4 words whose first three
 // multiples stay 8 banks away from each other
 constexpr int ssm_stride(int n) {
     for (int words = n / 2;; ++words) {
@@ -286,213 +280,321 @@ __device__ __forceinline__ Frag8 ssm_transposed(const bf16_t *at, int stride) {
     return u.f;
 }
 
-__device__ __forceinline__ void ssm_split(float v, uint16_t &hi, uint16_t &lo) {
-    hi = float_to_bf16_bits(v);
-    lo = float_to_bf16_bits(v - bf16_bits_to_float(hi));
+// two numbers as the sums of two bf16 numbers each
+__device__ __forceinline__ void ssm_split2(float a, float b, b16x2 &hi, b16x2 &lo) {
+    union { b16x2 p; uint32_t u; } h;
+    h.p = pack_bf16(a, b);
+    hi = h.p;
+    lo = pack_bf16(a - __uint_as_float(h.u << 16), b - __uint_as_float(h.u & 0xffff0000u));
 }
 
+// inclusive sum over the wavefront's lanes: rotations' kin inside rows of 16 lanes, then the rows' totals
+template <int SHIFT>
+__device__ __forceinline__ float ssm_shifted(float v) {                  // lane - SHIFT of the row of 16, 0 in front of it
+    return __uint_as_float(__builtin_amdgcn_update_dpp(0u, __float_as_uint(v), 0x110 | SHIFT, 0xf, 0xf, false));
+}
+__device__ __forceinline__ float ssm_lane(float v, int lane) { return __uint_as_float(__builtin_amdgcn_readlane(__float_as_uint(v), lane)); }
+__device__ __forceinline__ float ssm_prefix(float v) {
+    v += ssm_shifted<1>(v);
+    v += ssm_shifted<2>(v);
+    v += ssm_shifted<4>(v);
+    v += ssm_shifted<8>(v);
+    const float r0 = ssm_lane(v, 15), r1 = ssm_lane(v, 31), r2 = ssm_lane(v, 47);
+    const int row = (threadIdx.x % KVA_WAVE) / 16;
+    return v + (row > 0 ? r0 : 0.f) + (row > 1 ? r1 : 0.f) + (row > 2 ? r2 : 0.f);
+}
+
+// a chunk's place in the workspace: entries' chunks lie one behind the other with room for a part-filled one each
+__device__ __forceinline__ size_t ssm_chunk_at(int q0, int e, int chunk) { return (size_t)q0 / SSM_CHUNK + e + chunk; }
+
+struct SsmChunks {
+    SsmArgs a;
+    uint4 *work;            // [chunk][head][tile of 16 value columns][NK][high, low part][lane]
+    int max_chunks;         // chunks of the longest entry
+};
+
+// A workgroup takes 16 value columns of a head, wavefront w the state rows of the pairs of tiles w, w + 4, ..:
+//     S[n, p] = e^(c_64) S + sum_s B^T[n, s] (e^(c_64 - c_s) dt_s x[s, p]),
+// both operands by transposing loads from LDS, the second one as the sum of two bf16 numbers.  Two buffers in LDS: a
+// barrier a chunk, and the next chunk's rows are loaded while this one is worked on.
 template <int NK>
-struct SsmChunkLds {
-    static constexpr int ST = ssm_stride(32 * NK);
-    bf16_t b[SSM_CHUNK * ST], c[SSM_CHUNK * ST];
-    bf16_t s[2][2][16 * ST];                            // [buffer][high, low part][p][state]
-    bf16_t x[SSM_CHUNK * SSM_XS], wx[2][SSM_CHUNK * SSM_XS];
-    float cum[SSM_CHUNK], dt[SSM_CHUNK];
+struct SsmStatesLds {
+    static constexpr int ST = ssm_stride(32 * NK), XS = ssm_stride(16);
+    bf16_t b[2][SSM_CHUNK * ST], wx[2][2][SSM_CHUNK * XS];
 };
 
 template <int NK>
 __global__ void __launch_bounds__(256)
-state_space_chunk_kernel(SsmArgs a) {
-    constexpr int NP = 32 * NK, ST = SsmChunkLds<NK>::ST, TILES = (2 * NK + 3) / 4;      // tiles of 16 state rows a wavefront
-    constexpr int PIECES = SSM_CHUNK * NP / 8 / 256;                                     // 16-byte pieces of B (and of C) a thread
+state_space_states_kernel(SsmChunks k) {
+    using Lds = SsmStatesLds<NK>;
+    constexpr int NP = 32 * NK, ST = Lds::ST, XS = Lds::XS, PAIRS = (NK + 3) / 4;
+    constexpr int PIECES = SSM_CHUNK * NP / 8 / 256;                     // 16-byte pieces of B a thread
     constexpr float LOG2E = 1.44269504088896340736f;
     extern __shared__ __attribute__((aligned(16))) unsigned char lds_raw[];
-    SsmChunkLds<NK> &L = *reinterpret_cast<SsmChunkLds<NK> *>(lds_raw);
+    Lds &L = *reinterpret_cast<Lds *>(lds_raw);
+    const SsmArgs &a = k.a;
     const int tid = threadIdx.x, lane = tid % KVA_WAVE, w = tid / KVA_WAVE, r = lane & 15, g = lane >> 4;
     const int slices = (a.vdim + 15) / 16, id = die_order(blockIdx.x, gridDim.x);
-    const int head = id / slices, p0 = (id % slices) * 16, e = blockIdx.y;
+    const int head = id / slices, slice = id % slices, p0 = 16 * slice, e = blockIdx.y;
     const int q0 = a.entry_q_start[e], len = a.entry_q_start[e + 1] - q0;
     if (len < a.len_lo || len > a.len_hi) return;
     const int n = a.n, dv = a.vdim, grp = head / (a.heads / a.groups);
     const bf16_t *xbc = reinterpret_cast<const bf16_t *>(a.xbc);
-    const int x_col = head * dv + p0, b_col = a.heads * dv + grp * n, c_col = b_col + a.groups * n;
-    const float rate = expf(a.a_log[head]) * LOG2E, bias = a.dt_bias[head], skip = a.d_skip[head];
-    float *Sg = a.state + (size_t)a.entry_seat[e] * a.seat_stride + a.state_off + (size_t)head * n * dv + p0 + 4 * g;
-    const bool p_on = p0 + 4 * g < dv;                                   // (dv is a multiple of 4)
-    // S^T tile k of this wavefront: rows p = 4 g .. + 3, column 16 (w + 4 k) + r
-    f32x4 S[TILES];
+    const int x_col = head * dv + p0, b_col = a.heads * dv + grp * n;
+    const float rate = expf(a.a_log[head]) * LOG2E, bias = a.dt_bias[head];
+    float *Sg = a.state + (size_t)a.entry_seat[e] * a.seat_stride + a.state_off + (size_t)head * n * dv + p0 + r;
+    const bool p_on = p0 + r < dv;
+    f32x4 S[PAIRS][2];
 #pragma unroll
-    for (int k = 0; k < TILES; ++k) {
-        const int i = 16 * (w + 4 * k) + r;
-        S[k] = f32x4{0.f, 0.f, 0.f, 0.f};
-        if (p_on && i < n) {
-            const float4 v = *reinterpret_cast<const float4 *>(Sg + (size_t)i * dv);
-            S[k] = f32x4{v.x, v.y, v.z, v.w};
-        }
-    }
-    auto leave_state = [&](int buf) {
+    for (int j = 0; j < PAIRS; ++j)
 #pragma unroll
-        for (int k = 0; k < TILES; ++k) {
-            const int i = 16 * (w + 4 * k) + r;
-            if (i >= NP) continue;
+        for (int h = 0; h < 2; ++h)
 #pragma unroll
             for (int q = 0; q < 4; ++q) {
-                uint16_t hi, lo;
-                ssm_split(S[k][q], hi, lo);
-                L.s[buf][0][(4 * g + q) * ST + i].bits = hi;
-                L.s[buf][1][(4 * g + q) * ST + i].bits = lo;
+                const int i = 32 * (w + 4 * j) + 16 * h + 4 * g + q;
+                S[j][h][q] = p_on && i < n ? Sg[(size_t)i * dv] : 0.f;
             }
-        }
-    };
-    leave_state(0);
-
-    uint4 pb[PIECES], pc[PIECES];
+    uint4 pb[PIECES];
     uint2 px;
     float pd;
     auto fetch = [&](int t0, int m) {
 #pragma unroll
         for (int j = 0; j < PIECES; ++j) {
-            const int i = tid + 256 * j, tt = i / (NP / 8), k = 8 * (i % (NP / 8));
-            const bool in = tt < m && k < n;                             // (n is a multiple of 8)
-            const bf16_t *row = xbc + (size_t)(q0 + t0 + (in ? tt : 0)) * a.xbc_stride;
-            pb[j] = in ? *reinterpret_cast<const uint4 *>(row + b_col + k) : make_uint4(0u, 0u, 0u, 0u);
-            pc[j] = in ? *reinterpret_cast<const uint4 *>(row + c_col + k) : make_uint4(0u, 0u, 0u, 0u);
+            const int i = tid + 256 * j, tt = i / (NP / 8), c = 8 * (i % (NP / 8));
+            const bool in = tt < m && c < n;                             // (n is a multiple of 8)
+            pb[j] = in ? *reinterpret_cast<const uint4 *>(xbc + (size_t)(q0 + t0 + tt) * a.xbc_stride + b_col + c)
+                       : make_uint4(0u, 0u, 0u, 0u);
         }
-        const int tt = tid / 4, p = 4 * (tid % 4);
-        px = (tt < m && p0 + p < dv) ? *reinterpret_cast<const uint2 *>(xbc + (size_t)(q0 + t0 + tt) * a.xbc_stride + x_col + p)
-                                     : make_uint2(0u, 0u);
+        // x: lane = token, wavefront w the columns 4 w .. + 3 (dv is a multiple of 4)
+        px = (lane < m && p0 + 4 * w < dv) ? *reinterpret_cast<const uint2 *>(xbc + (size_t)(q0 + t0 + lane) * a.xbc_stride + x_col + 4 * w)
+                                           : make_uint2(0u, 0u);
         pd = lane < m ? ssm_ld(a.y, a.y_dtype, (size_t)(q0 + t0 + lane) * a.y_stride + a.dt_off + head) : 0.f;
     };
     fetch(0, min(SSM_CHUNK, len));
+    const int lane_row = 4 * g + r / 4, lane_col = 4 * (r % 4);
     int buf = 0;
     for (int t0 = 0; t0 < len; t0 += SSM_CHUNK, buf ^= 1) {
         const int m = min(SSM_CHUNK, len - t0);
-        // lane = token: its step size, the sum of the logarithms (base 2) up to it, its weight in the new state
-        const float dt = lane < m ? ssm_softplus(pd + bias) : 0.f;
-        float cum = -rate * dt;
+        // the state in front of the chunk, as the operand that the outputs' kernel reads
+        uint4 *work = k.work + (((ssm_chunk_at(q0, e, t0 / SSM_CHUNK) * a.heads + head) * slices + slice) * NK * 2) * KVA_WAVE + lane;
 #pragma unroll
-        for (int o = 1; o < SSM_CHUNK; o <<= 1) {
-            const float up = __shfl_up(cum, o, KVA_WAVE);
-            if (lane >= o) cum += up;
-        }
-        const float total = __shfl(cum, SSM_CHUNK - 1, KVA_WAVE);
-        const float into = dt * __builtin_amdgcn_exp2f(total - cum);
-        const float xw = __shfl(into, 16 * w + lane / 4, KVA_WAVE);      // of the token whose x this thread stages
-        __syncthreads();                                                  // whoever still reads the chunk before is done
-#pragma unroll
-        for (int j = 0; j < PIECES; ++j) {
-            const int i = tid + 256 * j, at = (i / (NP / 8)) * ST + 8 * (i % (NP / 8));
-            *reinterpret_cast<uint4 *>(&L.b[at]) = pb[j];
-            *reinterpret_cast<uint4 *>(&L.c[at]) = pc[j];
-        }
-        {
-            const int at = (tid / 4) * SSM_XS + 4 * (tid % 4);
-            *reinterpret_cast<uint2 *>(&L.x[at]) = px;
-            const float f[4] = {__uint_as_float(px.x << 16), __uint_as_float(px.x & 0xffff0000u), __uint_as_float(px.y << 16),
-                                __uint_as_float(px.y & 0xffff0000u)};
-            Frag4 hi, lo;
-#pragma unroll
-            for (int q = 0; q < 4; ++q) ssm_split(f[q] * xw, hi.h[q], lo.h[q]);
-            *reinterpret_cast<uint2 *>(&L.wx[0][at]) = hi.u2;
-            *reinterpret_cast<uint2 *>(&L.wx[1][at]) = lo.u2;
-        }
-        if (w == 0) {
-            L.cum[lane] = cum;
-            L.dt[lane] = dt;
-        }
-        __syncthreads();
-        if (t0 + SSM_CHUNK < len) fetch(t0 + SSM_CHUNK, min(SSM_CHUNK, len - t0 - SSM_CHUNK));
-        const int t = 16 * w + r;
-        const float cum_t = L.cum[t];
-        Frag8 cf[NK];
-#pragma unroll
-        for (int ks = 0; ks < NK; ++ks) cf[ks].u4 = *reinterpret_cast<const uint4 *>(&L.c[t * ST + 32 * ks + 8 * g]);
-        // (3) what the state in front of the chunk says
-        f32x4 y = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-        for (int part = 0; part < 2; ++part)
-#pragma unroll
-            for (int ks = 0; ks < NK; ++ks) {
-                Frag8 sf;
-                sf.u4 = *reinterpret_cast<const uint4 *>(&L.s[buf][part][r * ST + 32 * ks + 8 * g]);
-                y = __builtin_amdgcn_mfma_f32_16x16x32_bf16(sf.v, cf[ks].v, y, 0, 0, 0);
-            }
-        const float from_start = __builtin_amdgcn_exp2f(cum_t);
-#pragma unroll
-        for (int q = 0; q < 4; ++q) y[q] *= from_start;
-        // (1), (2): pairs of tiles of 16 earlier tokens
-        const int lane_row = (4 * g + r / 4), lane_col = 4 * (r % 4);
-        for (int u = 0; u <= w / 2; ++u) {
+        for (int j = 0; j < PAIRS; ++j) {
+            const int ks = w + 4 * j;
+            if (ks >= NK) continue;
             Frag8 hi, lo;
 #pragma unroll
             for (int h = 0; h < 2; ++h) {
-                const int st = 2 * u + h;
-                f32x4 gt = {0.f, 0.f, 0.f, 0.f};
-                if (st <= w) {
-#pragma unroll
-                    for (int ks = 0; ks < NK; ++ks) {
-                        Frag8 bf;
-                        bf.u4 = *reinterpret_cast<const uint4 *>(&L.b[(16 * st + r) * ST + 32 * ks + 8 * g]);
-                        gt = __builtin_amdgcn_mfma_f32_16x16x32_bf16(bf.v, cf[ks].v, gt, 0, 0, 0);
-                    }
-                }
-                const float4 cs = *reinterpret_cast<const float4 *>(&L.cum[16 * st + 4 * g]);
-                const float4 ds = *reinterpret_cast<const float4 *>(&L.dt[16 * st + 4 * g]);
-                const float cum_s[4] = {cs.x, cs.y, cs.z, cs.w}, dt_s[4] = {ds.x, ds.y, ds.z, ds.w};
-#pragma unroll
-                for (int q = 0; q < 4; ++q) {
-                    const bool seen = 16 * st + 4 * g + q <= t;
-                    const float wgt = seen ? gt[q] * (__builtin_amdgcn_exp2f(cum_t - cum_s[q]) * dt_s[q]) : 0.f;
-                    ssm_split(wgt, hi.h[4 * h + q], lo.h[4 * h + q]);
-                }
+                ssm_split2(S[j][h][0], S[j][h][1], hi.p2[2 * h], lo.p2[2 * h]);
+                ssm_split2(S[j][h][2], S[j][h][3], hi.p2[2 * h + 1], lo.p2[2 * h + 1]);
             }
-            const Frag8 xf = ssm_transposed(&L.x[(32 * u + lane_row) * SSM_XS + lane_col], SSM_XS);
-            y = __builtin_amdgcn_mfma_f32_16x16x32_bf16(xf.v, hi.v, y, 0, 0, 0);
-            y = __builtin_amdgcn_mfma_f32_16x16x32_bf16(xf.v, lo.v, y, 0, 0, 0);
+            work[(2 * ks) * KVA_WAVE] = hi.u4;
+            work[(2 * ks + 1) * KVA_WAVE] = lo.u4;
         }
-        if (t < m && p_on) {
-            const uint2 xv = *reinterpret_cast<const uint2 *>(&L.x[t * SSM_XS + 4 * g]);
-            *reinterpret_cast<float4 *>(a.out + (size_t)(q0 + t0 + t) * a.heads * dv + x_col + 4 * g) =
-                make_float4(y[0] + skip * __uint_as_float(xv.x << 16), y[1] + skip * __uint_as_float(xv.x & 0xffff0000u),
-                            y[2] + skip * __uint_as_float(xv.y << 16), y[3] + skip * __uint_as_float(xv.y & 0xffff0000u));
+        // lane = token: its step size, the sum of the logarithms (base 2) up to it, its weight in the new state
+        const float dt = lane < m ? ssm_softplus(pd + bias) : 0.f;
+        const float cum = ssm_prefix(-rate * dt), total = ssm_lane(cum, SSM_CHUNK - 1);
+        const float into = dt * __builtin_amdgcn_exp2f(total - cum);
+#pragma unroll
+        for (int j = 0; j < PIECES; ++j) {
+            const int i = tid + 256 * j;
+            *reinterpret_cast<uint4 *>(&L.b[buf][(i / (NP / 8)) * ST + 8 * (i % (NP / 8))]) = pb[j];
         }
-        // (4) the state behind the chunk
+        union { b16x2 p[2]; uint2 u; } hi, lo;
+        ssm_split2(__uint_as_float(px.x << 16) * into, __uint_as_float(px.x & 0xffff0000u) * into, hi.p[0], lo.p[0]);
+        ssm_split2(__uint_as_float(px.y << 16) * into, __uint_as_float(px.y & 0xffff0000u) * into, hi.p[1], lo.p[1]);
+        *reinterpret_cast<uint2 *>(&L.wx[buf][0][lane * XS + 4 * w]) = hi.u;
+        *reinterpret_cast<uint2 *>(&L.wx[buf][1][lane * XS + 4 * w]) = lo.u;
+        if (t0 + SSM_CHUNK < len) fetch(t0 + SSM_CHUNK, min(SSM_CHUNK, len - t0 - SSM_CHUNK));
+        __syncthreads();            // (a buffer was read last two turns ago: every wavefront has passed the barrier between)
         const float keep = __builtin_amdgcn_exp2f(total);
         Frag8 wx[2][2];
 #pragma unroll
         for (int u = 0; u < 2; ++u)
 #pragma unroll
             for (int part = 0; part < 2; ++part)
-                wx[u][part] = ssm_transposed(&L.wx[part][(32 * u + lane_row) * SSM_XS + lane_col], SSM_XS);
+                wx[u][part] = ssm_transposed(&L.wx[buf][part][(32 * u + lane_row) * XS + lane_col], XS);
 #pragma unroll
-        for (int k = 0; k < TILES; ++k) {
-            const int i0 = 16 * (w + 4 * k);
-            if (i0 >= NP) continue;
+        for (int j = 0; j < PAIRS; ++j) {
+            if (w + 4 * j >= NK) continue;
+            Frag8 bf[2][2];
 #pragma unroll
-            for (int q = 0; q < 4; ++q) S[k][q] *= keep;
+            for (int h = 0; h < 2; ++h)
 #pragma unroll
-            for (int u = 0; u < 2; ++u) {
-                const Frag8 bf = ssm_transposed(&L.b[(32 * u + lane_row) * ST + i0 + lane_col], ST);
-                S[k] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wx[u][0].v, bf.v, S[k], 0, 0, 0);
-                S[k] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wx[u][1].v, bf.v, S[k], 0, 0, 0);
-            }
+                for (int u = 0; u < 2; ++u)
+                    bf[h][u] = ssm_transposed(&L.b[buf][(32 * u + lane_row) * ST + 32 * (w + 4 * j) + 16 * h + lane_col], ST);
+#pragma unroll
+            for (int h = 0; h < 2; ++h)
+#pragma unroll
+                for (int q = 0; q < 4; ++q) S[j][h][q] *= keep;
+#pragma unroll
+            for (int u = 0; u < 2; ++u)
+#pragma unroll
+                for (int part = 0; part < 2; ++part)
+#pragma unroll
+                    for (int h = 0; h < 2; ++h)
+                        S[j][h] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(bf[h][u].v, wx[u][part].v, S[j][h], 0, 0, 0);
         }
-        leave_state(buf ^ 1);
     }
 #pragma unroll
-    for (int k = 0; k < TILES; ++k) {
-        const int i = 16 * (w + 4 * k) + r;
-        if (p_on && i < n) *reinterpret_cast<float4 *>(Sg + (size_t)i * dv) = make_float4(S[k][0], S[k][1], S[k][2], S[k][3]);
+    for (int j = 0; j < PAIRS; ++j)
+#pragma unroll
+        for (int h = 0; h < 2; ++h)
+#pragma unroll
+            for (int q = 0; q < 4; ++q) {
+                const int i = 32 * (w + 4 * j) + 16 * h + 4 * g + q;
+                if (p_on && i < n) Sg[(size_t)i * dv] = S[j][h][q];
+            }
+}
+
+// A workgroup takes a chunk, a head and up to 64 of its value columns.  Everything is computed transposed, wavefront w
+// the tokens t = 16 w .. + 15 as columns: G^T[s, t] = B_s . C_t for the tiles s <= t (B in LDS, C from memory); the
+// weights e^(c_t - c_s) dt_s G, in registers the second operand of y^T[p, t] = sum_s x^T[p, s] W^T[s, t] (x in LDS, by
+// transposing loads); and per tile of 16 value columns e^(c_t) S_0^T C + that + D x.
+template <int NK>
+struct SsmOutputsLds {
+    static constexpr int ST = ssm_stride(32 * NK), XS = ssm_stride(64);
+    bf16_t b[SSM_CHUNK * ST], x[SSM_CHUNK * XS];
+    float cum[SSM_CHUNK], dt[SSM_CHUNK];
+};
+
+template <int NK>
+__global__ void __launch_bounds__(256)
+state_space_outputs_kernel(SsmChunks k) {
+    using Lds = SsmOutputsLds<NK>;
+    constexpr int NP = 32 * NK, ST = Lds::ST, XS = Lds::XS, PIECES = SSM_CHUNK * NP / 8 / 256;
+    constexpr float LOG2E = 1.44269504088896340736f;
+    __shared__ __attribute__((aligned(16))) Lds L;
+    const SsmArgs &a = k.a;
+    const int tid = threadIdx.x, lane = tid % KVA_WAVE, w = tid / KVA_WAVE, r = lane & 15, g = lane >> 4;
+    const int slices = (a.vdim + 15) / 16, blocks = (a.vdim + 63) / 64, per_chunk = a.heads * blocks;
+    const int id = die_order(blockIdx.x, gridDim.x), chunk = id / per_chunk, head = id % per_chunk / blocks, block = id % blocks;
+    const int e = blockIdx.y;
+    const int q0 = a.entry_q_start[e], len = a.entry_q_start[e + 1] - q0, t0 = chunk * SSM_CHUNK;
+    if (len < a.len_lo || len > a.len_hi || t0 >= len) return;
+    const int n = a.n, dv = a.vdim, grp = head / (a.heads / a.groups), m = min(SSM_CHUNK, len - t0), p0 = 64 * block;
+    const bf16_t *rows = reinterpret_cast<const bf16_t *>(a.xbc) + (size_t)(q0 + t0) * a.xbc_stride;
+    const int x_col = head * dv + p0, b_col = a.heads * dv + grp * n, c_col = b_col + a.groups * n;
+    const float rate = expf(a.a_log[head]) * LOG2E, skip = a.d_skip[head];
+    const float pd = lane < m ? ssm_ld(a.y, a.y_dtype, (size_t)(q0 + t0 + lane) * a.y_stride + a.dt_off + head) : 0.f;
+    uint4 pb[PIECES];
+#pragma unroll
+    for (int j = 0; j < PIECES; ++j) {
+        const int i = tid + 256 * j, tt = i / (NP / 8), c = 8 * (i % (NP / 8));
+        pb[j] = tt < m && c < n ? *reinterpret_cast<const uint4 *>(rows + (size_t)tt * a.xbc_stride + b_col + c) : make_uint4(0u, 0u, 0u, 0u);
+    }
+    uint2 px[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+        const int i = tid + 256 * j, tt = i / 16, p = 4 * (i % 16);
+        px[j] = tt < m && p0 + p < dv ? *reinterpret_cast<const uint2 *>(rows + (size_t)tt * a.xbc_stride + x_col + p) : make_uint2(0u, 0u);
+    }
+    const int t = 16 * w + r;
+    Frag8 cf[NK];
+#pragma unroll
+    for (int ks = 0; ks < NK; ++ks)
+#pragma unroll
+        for (int h = 0; h < 2; ++h) {
+            const int c = 32 * ks + 16 * h + 4 * g;
+            cf[ks].u2[h] = t < m && c < n ? *reinterpret_cast<const uint2 *>(rows + (size_t)t * a.xbc_stride + c_col + c) : make_uint2(0u, 0u);
+        }
+    const float dt = lane < m ? ssm_softplus(pd + a.dt_bias[head]) : 0.f;
+    const float cum = ssm_prefix(-rate * dt);
+#pragma unroll
+    for (int j = 0; j < PIECES; ++j) {
+        const int i = tid + 256 * j;
+        *reinterpret_cast<uint4 *>(&L.b[(i / (NP / 8)) * ST + 8 * (i % (NP / 8))]) = pb[j];
+    }
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+        const int i = tid + 256 * j;
+        *reinterpret_cast<uint2 *>(&L.x[(i / 16) * XS + 4 * (i % 16)]) = px[j];
+    }
+    if (w == 0) {
+        L.cum[lane] = cum;
+        L.dt[lane] = dt;
+    }
+    __syncthreads();
+    const float cum_t = L.cum[t];
+    Frag8 hi[2], lo[2];
+#pragma unroll
+    for (int u = 0; u < 2; ++u) {
+        hi[u].u4 = lo[u].u4 = make_uint4(0u, 0u, 0u, 0u);
+#pragma unroll
+        for (int h = 0; h < 2; ++h) {
+            const int st = 2 * u + h;
+            if (st > w) continue;                                           // (the whole wavefront: later tokens)
+            f32x4 gt = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int ks = 0; ks < NK; ++ks) {
+                Frag8 bf;
+                const bf16_t *brow = &L.b[(16 * st + r) * ST + 32 * ks + 4 * g];
+                bf.u2[0] = *reinterpret_cast<const uint2 *>(brow);
+                bf.u2[1] = *reinterpret_cast<const uint2 *>(brow + 16);
+                gt = __builtin_amdgcn_mfma_f32_16x16x32_bf16(bf.v, cf[ks].v, gt, 0, 0, 0);
+            }
+            const float4 cs = *reinterpret_cast<const float4 *>(&L.cum[16 * st + 4 * g]);
+            const float4 ds = *reinterpret_cast<const float4 *>(&L.dt[16 * st + 4 * g]);
+            const float cum_s[4] = {cs.x, cs.y, cs.z, cs.w}, dt_s[4] = {ds.x, ds.y, ds.z, ds.w};
+            float wgt[4];
+#pragma unroll
+            for (int q = 0; q < 4; ++q)
+                wgt[q] = 16 * st + 4 * g + q <= t ? gt[q] * (__builtin_amdgcn_exp2f(cum_t - cum_s[q]) * dt_s[q]) : 0.f;
+            ssm_split2(wgt[0], wgt[1], hi[u].p2[2 * h], lo[u].p2[2 * h]);
+            ssm_split2(wgt[2], wgt[3], hi[u].p2[2 * h + 1], lo[u].p2[2 * h + 1]);
+        }
+    }
+    const float from_start = __builtin_amdgcn_exp2f(cum_t);
+    const int lane_row = 4 * g + r / 4, lane_col = 4 * (r % 4);
+    const uint4 *work = k.work + (((ssm_chunk_at(q0, e, chunk) * a.heads + head) * slices + 4 * block) * NK * 2) * KVA_WAVE + lane;
+    float *orow = a.out + (size_t)(q0 + t0 + t) * a.heads * dv + x_col + 4 * g;
+#pragma unroll
+    for (int pt = 0; pt < 4; ++pt) {
+        if (p0 + 16 * pt >= dv) break;
+        f32x4 y = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int ks = 0; ks < NK; ++ks)
+#pragma unroll
+            for (int part = 0; part < 2; ++part) {
+                Frag8 sf;
+                sf.u4 = work[((pt * NK + ks) * 2 + part) * KVA_WAVE];
+                y = __builtin_amdgcn_mfma_f32_16x16x32_bf16(sf.v, cf[ks].v, y, 0, 0, 0);
+            }
+#pragma unroll
+        for (int q = 0; q < 4; ++q) y[q] *= from_start;
+#pragma unroll
+        for (int u = 0; u < 2; ++u) {
+            if (2 * u > w) continue;
+            const Frag8 xf = ssm_transposed(&L.x[(32 * u + lane_row) * XS + 16 * pt + lane_col], XS);
+            y = __builtin_amdgcn_mfma_f32_16x16x32_bf16(xf.v, hi[u].v, y, 0, 0, 0);
+            y = __builtin_amdgcn_mfma_f32_16x16x32_bf16(xf.v, lo[u].v, y, 0, 0, 0);
+        }
+        if (t < m && p0 + 16 * pt + 4 * g < dv) {                           // (dv is a multiple of 4)
+            const uint2 xv = *reinterpret_cast<const uint2 *>(&L.x[t * XS + 16 * pt + 4 * g]);
+            *reinterpret_cast<float4 *>(orow + 16 * pt) =
+                make_float4(y[0] + skip * __uint_as_float(xv.x << 16), y[1] + skip * __uint_as_float(xv.x & 0xffff0000u),
+                            y[2] + skip * __uint_as_float(xv.y << 16), y[3] + skip * __uint_as_float(xv.y & 0xffff0000u));
+        }
     }
 }
 
+static int ssm_pairs(int n) { return n <= 32 ? 1 : n <= 64 ? 2 : n <= 128 ? 4 : 8; }
+
+// bytes of workspace the chunks of a step of so many tokens and entries need
+extern "C" long long kva_state_space_workspace(int tokens, int entries, int heads, int n, int vdim) {
+    return ((long long)tokens / SSM_CHUNK + entries + 1) * heads * ((vdim + 15) / 16) * ssm_pairs(n) * 2 * KVA_WAVE * 16;
+}
+
 template <int NK>
-static int ssm_chunk_launch(const SsmArgs &a, int entries, hipStream_t stream) {
-    const int lds = (int)sizeof(SsmChunkLds<NK>);
+static int ssm_chunk_launch(const SsmChunks &k, int entries, hipStream_t stream) {
+    const SsmArgs &a = k.a;
+    const int lds = (int)sizeof(SsmStatesLds<NK>);
     if (lds > 64 * 1024)
-        hipFuncSetAttribute(reinterpret_cast<const void *>(state_space_chunk_kernel<NK>), hipFuncAttributeMaxDynamicSharedMemorySize, lds);
-    hipLaunchKernelGGL(state_space_chunk_kernel<NK>, dim3(a.heads * ((a.vdim + 15) / 16), entries), dim3(256), lds, stream, a);
-    KVA_CHECK_LAUNCH("state_space_chunk");
+        hipFuncSetAttribute(reinterpret_cast<const void *>(state_space_states_kernel<NK>), hipFuncAttributeMaxDynamicSharedMemorySize, lds);
+    hipLaunchKernelGGL(state_space_states_kernel<NK>, dim3(a.heads * ((a.vdim + 15) / 16), entries), dim3(256), lds, stream, k);
+    KVA_CHECK_LAUNCH("state_space_states");
+    hipLaunchKernelGGL(state_space_outputs_kernel<NK>, dim3((unsigned)((long long)k.max_chunks * a.heads * ((a.vdim + 63) / 64)), entries),
+                       dim3(256), 0, stream, k);
+    KVA_CHECK_LAUNCH("state_space_outputs");
     return KVA_OK;
 }
 
@@ -509,7 +611,7 @@ extern "C" int kva_state_space(int kernel, int len_lo, int len_hi, float *out, f
                                int state_off, const void *xbc, int xbc_dtype, int xbc_stride, const void *y, int y_dtype,
                                int y_stride, int dt_off, const float *a_log, const float *dt_bias, const float *d_skip,
                                const int *entry_q_start, const int *entry_seat, int entries, int heads, int groups, int n,
-                               int vdim, hipStream_t stream) {
+                               int vdim, void *work, long long work_bytes, int tokens, int max_len, hipStream_t stream) {
     KVA_REQUIRE(out && state && xbc && y && a_log && dt_bias && d_skip && entry_q_start && entry_seat,
                 "state_space: missing operand");
     KVA_REQUIRE(heads > 0 && groups > 0 && heads % groups == 0 && vdim > 0, "state_space: %d heads in %d groups", heads, groups);
@@ -528,10 +630,17 @@ extern "C" int kva_state_space(int kernel, int len_lo, int len_hi, float *out, f
     const SsmArgs a{out, state, (size_t)seat_stride, state_off, entry_q_start, entry_seat, xbc, xbc_dtype, xbc_stride, y,
                     y_dtype, y_stride, dt_off, a_log, dt_bias, d_skip, heads, groups, n, vdim, len_lo, len_hi};
     if (kernel == SSM_CHUNKS) {
-        if (n <= 32) return ssm_chunk_launch<1>(a, entries, stream);
-        if (n <= 64) return ssm_chunk_launch<2>(a, entries, stream);
-        if (n <= 128) return ssm_chunk_launch<4>(a, entries, stream);
-        return ssm_chunk_launch<8>(a, entries, stream);
+        KVA_REQUIRE(work && (reinterpret_cast<uintptr_t>(work) & 15) == 0 && tokens > 0 && max_len > 0 && max_len <= tokens &&
+                        work_bytes >= kva_state_space_workspace(tokens, entries, heads, n, vdim),
+                    "state_space: %lld bytes of workspace are too few for %d tokens in %d entries", work_bytes, tokens, entries);
+        const SsmChunks k{a, (uint4 *)work, (max_len + SSM_CHUNK - 1) / SSM_CHUNK};
+        KVA_REQUIRE((long long)k.max_chunks * heads * ((vdim + 63) / 64) < (1LL << 31), "state_space: too many chunks for one launch");
+        switch (ssm_pairs(n)) {
+        case 1: return ssm_chunk_launch<1>(k, entries, stream);
+        case 2: return ssm_chunk_launch<2>(k, entries, stream);
+        case 4: return ssm_chunk_launch<4>(k, entries, stream);
+        default: return ssm_chunk_launch<8>(k, entries, stream);
+        }
     }
     if (kernel == SSM_TOKEN) {
         hipLaunchKernelGGL(state_space_token_kernel, dim3(heads * ((vdim + 63) / 64), entries), dim3(256), 0, stream, a);

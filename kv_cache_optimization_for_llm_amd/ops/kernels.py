@@ -1803,6 +1803,11 @@ def state_space_plan(lengths, heads: int, groups: int, state_size: int, vdim: in
     return [(k, lo, hi) for k, lo, hi in ranges if any(lo <= int(n) <= hi for n in lengths)]
 
 
+def state_space_workspace(tokens: int, entries: int, heads: int, state_size: int, vdim: int) -> int:
+    """Bytes of workspace :func:`state_space` takes for a step whose entries go in chunks: the state in front of each."""
+    return int(hip_lib().kva_state_space_workspace(int(tokens), int(entries), int(heads), int(state_size), int(vdim)))
+
+
 def state_space(xbc: torch.Tensor, y: torch.Tensor, dt_off: int, a_log: torch.Tensor, dt_bias: torch.Tensor,
                 skip: torch.Tensor, out: torch.Tensor, state: torch.Tensor, state_off: int, entry_q_start: torch.Tensor,
                 entry_seat: torch.Tensor, heads: int, groups: int, state_size: int, vdim: int, lengths,
@@ -1827,12 +1832,19 @@ def state_space(xbc: torch.Tensor, y: torch.Tensor, dt_off: int, a_log: torch.Te
         # (the walk over the tokens takes any state; the other kernels want it at multiples of 16 bytes)
         plan = [("scan", 1, 1 << 30)] if state_off % 4 or seat_stride % 4 else \
             state_space_plan(lengths, heads, groups, state_size, vdim, xbc.dtype)
+    lengths = [int(m) for m in lengths]
+    if len(lengths) != entries or sum(lengths) != tokens:
+        raise KernelError("state_space: one length per entry, of all the rows together")
+    work = None
+    if any(kernel == "chunks" for kernel, _, _ in plan):
+        work = torch.empty(state_space_workspace(tokens, entries, heads, state_size, vdim), dtype=torch.uint8, device=out.device)
     for kernel, lo, hi in plan:
         check(hip_lib().kva_state_space(
             STATE_SPACE_KERNELS[kernel], int(lo), int(hi), _dev(out, "out"), _dev(state, "state"), seat_stride, int(state_off),
             _dev(xbc, "xbc"), dtype_code(xbc.dtype), xbc.shape[1], _dev(y, "y"), dtype_code(y.dtype), y.shape[1], int(dt_off),
             _dev(a_log, "a_log"), _dev(dt_bias, "dt_bias"), _dev(skip, "skip"), qs, seat, entries, int(heads), int(groups),
-            int(state_size), int(vdim), _stream()), "state_space")
+            int(state_size), int(vdim), _opt(work, "work"), 0 if work is None else work.numel(), tokens, max(lengths, default=0),
+            _stream()), "state_space")
     return out
 
 

@@ -112,7 +112,7 @@ _HIP_SIGNATURES = {
     "kva_pair_embed": [P, P, I, I, F, P, I, I, I, I, P, P, I, F, P, P, P, I, P, P, I, I, I, P],
     "kva_maps_encode_cache": [P, I, P, P, P, P, P, P, P, I, I, I, I, I, I, I, I, P, I, P],
     "kva_maps_combine": [P, I, I, P, F, F, F, I, I, I, I, P],
-    "kva_state_space": [I, I, I, P, P, LL, I, P, I, I, P, I, I, I, P, P, P, P, P, I, I, I, I, I, P],
+    "kva_state_space": [I, I, I, P, P, LL, I, P, I, I, P, I, I, I, P, P, P, P, P, I, I, I, I, I, P, LL, I, I, P],
     "kva_state_space_supported": [I, I, I, I, I, I],
     "kva_hyper_fill": [P, P, I, I, I, I, P],
     "kva_block_gates": [P, P, P, I, I, I, P, P, I, P, P, P, P],
@@ -146,6 +146,8 @@ def hip_lib():
         lib.kva_last_error.restype = c_char_p
         lib.kva_sample_workspace_bytes.argtypes = [I, I]
         lib.kva_sample_workspace_bytes.restype = LL
+        lib.kva_state_space_workspace.argtypes = [I, I, I, I, I]
+        lib.kva_state_space_workspace.restype = LL
         lib._path = path
         _hip = lib
         return _hip

@@ -543,7 +543,9 @@ class StateSpaceDuality(ProjectedMixer):
         return (n + 3) // 4 * 4          # (every seat's row starts at a multiple of 16 bytes)
 
     def activation_elements(self) -> int:
-        return 3 * self.conv_channels + 4 * self.inner_width + self.hidden_size
+        # (and the state in front of every chunk of 64 tokens, as two numbers of 16 bits an element)
+        chunk_states = self.num_heads * self.state_size * self.value_dim // 32
+        return 3 * self.conv_channels + 4 * self.inner_width + self.hidden_size + chunk_states
 
     def forward_inner(self, y, col0, ctx: MixerContext, state_off, out, out_col0, mul) -> None:
         batch, T = ctx.batch, y.shape[0]
