@@ -280,6 +280,14 @@ __device__ __forceinline__ Frag8 ssm_transposed(const bf16_t *at, int stride) {
     return u.f;
 }
 
+// softplus as a chain of few instructions: log(1 + e) with e = exp(-|z|) by the hardware's logarithm, or where that
+// would lose digits by the series (the sixth term is below 2e-8 of the sum there)
+__device__ __forceinline__ float ssm_softplus_short(float z) {
+    const float e = __builtin_amdgcn_exp2f(-fabsf(z) * 1.44269504088896340736f);
+    const float series = e * (1.f - e * (0.5f - e * (1.f / 3.f - e * (0.25f - e * 0.2f))));
+    return fmaxf(z, 0.f) + (e < 0.04f ? series : 0.69314718055994530942f * __builtin_amdgcn_logf(1.f + e));
+}
+
 // two numbers as the sums of two bf16 numbers each
 __device__ __forceinline__ void ssm_split2(float a, float b, b16x2 &hi, b16x2 &lo) {
     union { b16x2 p; uint32_t u; } h;
@@ -316,7 +324,7 @@ struct SsmChunks {
 // A workgroup takes 16 value columns of a head, wavefront w the state rows of the pairs of tiles w, w + 4, ..:
 //     S[n, p] = e^(c_64) S + sum_s B^T[n, s] (e^(c_64 - c_s) dt_s x[s, p]),
 // both operands by transposing loads from LDS, the second one as the sum of two bf16 numbers.  Two buffers in LDS: a
-// barrier a chunk, and the next chunk's rows are loaded while this one is worked on.
+// barrier a chunk; the rows of the two chunks behind this one are on their way while it is worked on.
 template <int NK>
 struct SsmStatesLds {
     static constexpr int ST = ssm_stride(32 * NK), XS = ssm_stride(16);
@@ -340,7 +348,7 @@ state_space_states_kernel(SsmChunks k) {
     if (len < a.len_lo || len > a.len_hi) return;
     const int n = a.n, dv = a.vdim, grp = head / (a.heads / a.groups);
     const bf16_t *xbc = reinterpret_cast<const bf16_t *>(a.xbc);
-    const int x_col = head * dv + p0, b_col = a.heads * dv + grp * n;
+    const int b_col = a.heads * dv + grp * n;
     const float rate = expf(a.a_log[head]) * LOG2E, bias = a.dt_bias[head];
     float *Sg = a.state + (size_t)a.entry_seat[e] * a.seat_stride + a.state_off + (size_t)head * n * dv + p0 + r;
     const bool p_on = p0 + r < dv;
@@ -354,26 +362,28 @@ state_space_states_kernel(SsmChunks k) {
                 const int i = 32 * (w + 4 * j) + 16 * h + 4 * g + q;
                 S[j][h][q] = p_on && i < n ? Sg[(size_t)i * dv] : 0.f;
             }
-    uint4 pb[PIECES];
-    uint2 px;
-    float pd;
-    auto fetch = [&](int t0, int m) {
+    struct Ahead {                      // a chunk's rows on their way
+        kva_u32x4 b[PIECES];
+        kva_u32x2 x;
+        uint16_t d;
+    } ahead0, ahead1;
+    // (no branch around a load, nothing formed from it here: tokens past the chunk's last one repeat that one, with
+    // weight zero; columns past the last one repeat others, into rows and columns of S that nobody stores)
+    auto fetch = [&](Ahead &f, int t0) {
+        const int last = min(SSM_CHUNK, len - t0) - 1;
+        const bf16_t *first = xbc + (size_t)(q0 + t0) * a.xbc_stride;
 #pragma unroll
         for (int j = 0; j < PIECES; ++j) {
-            const int i = tid + 256 * j, tt = i / (NP / 8), c = 8 * (i % (NP / 8));
-            const bool in = tt < m && c < n;                             // (n is a multiple of 8)
-            pb[j] = in ? *reinterpret_cast<const uint4 *>(xbc + (size_t)(q0 + t0 + tt) * a.xbc_stride + b_col + c)
-                       : make_uint4(0u, 0u, 0u, 0u);
+            const int i = tid + 256 * j, tt = min(i / (NP / 8), last), c = min(8 * (i % (NP / 8)), n - 8);      // (n is a multiple of 8)
+            f.b[j] = *reinterpret_cast<const kva_u32x4 *>(first + (size_t)tt * a.xbc_stride + b_col + c);
         }
         // x: lane = token, wavefront w the columns 4 w .. + 3 (dv is a multiple of 4)
-        px = (lane < m && p0 + 4 * w < dv) ? *reinterpret_cast<const uint2 *>(xbc + (size_t)(q0 + t0 + lane) * a.xbc_stride + x_col + 4 * w)
-                                           : make_uint2(0u, 0u);
-        pd = lane < m ? ssm_ld(a.y, a.y_dtype, (size_t)(q0 + t0 + lane) * a.y_stride + a.dt_off + head) : 0.f;
+        const int tt = min(lane, last);
+        f.x = *reinterpret_cast<const kva_u32x2 *>(first + (size_t)tt * a.xbc_stride + head * dv + min(p0 + 4 * w, dv - 4));
+        f.d = reinterpret_cast<const uint16_t *>(a.y)[(size_t)(q0 + t0 + tt) * a.y_stride + a.dt_off + head];
     };
-    fetch(0, min(SSM_CHUNK, len));
     const int lane_row = 4 * g + r / 4, lane_col = 4 * (r % 4);
-    int buf = 0;
-    for (int t0 = 0; t0 < len; t0 += SSM_CHUNK, buf ^= 1) {
+    auto turn = [&](Ahead &f, int t0, int buf) {
         const int m = min(SSM_CHUNK, len - t0);
         // the state in front of the chunk, as the operand that the outputs' kernel reads
         uint4 *work = k.work + (((ssm_chunk_at(q0, e, t0 / SSM_CHUNK) * a.heads + head) * slices + slice) * NK * 2) * KVA_WAVE + lane;
@@ -391,20 +401,20 @@ state_space_states_kernel(SsmChunks k) {
             work[(2 * ks + 1) * KVA_WAVE] = lo.u4;
         }
         // lane = token: its step size, the sum of the logarithms (base 2) up to it, its weight in the new state
-        const float dt = lane < m ? ssm_softplus(pd + bias) : 0.f;
+        const float dt = lane < m ? ssm_softplus_short(bf16_bits_to_float(f.d) + bias) : 0.f;
         const float cum = ssm_prefix(-rate * dt), total = ssm_lane(cum, SSM_CHUNK - 1);
         const float into = dt * __builtin_amdgcn_exp2f(total - cum);
 #pragma unroll
         for (int j = 0; j < PIECES; ++j) {
             const int i = tid + 256 * j;
-            *reinterpret_cast<uint4 *>(&L.b[buf][(i / (NP / 8)) * ST + 8 * (i % (NP / 8))]) = pb[j];
+            *reinterpret_cast<kva_u32x4 *>(&L.b[buf][(i / (NP / 8)) * ST + 8 * (i % (NP / 8))]) = f.b[j];
         }
         union { b16x2 p[2]; uint2 u; } hi, lo;
-        ssm_split2(__uint_as_float(px.x << 16) * into, __uint_as_float(px.x & 0xffff0000u) * into, hi.p[0], lo.p[0]);
-        ssm_split2(__uint_as_float(px.y << 16) * into, __uint_as_float(px.y & 0xffff0000u) * into, hi.p[1], lo.p[1]);
+        ssm_split2(__uint_as_float(f.x.x << 16) * into, __uint_as_float(f.x.x & 0xffff0000u) * into, hi.p[0], lo.p[0]);
+        ssm_split2(__uint_as_float(f.x.y << 16) * into, __uint_as_float(f.x.y & 0xffff0000u) * into, hi.p[1], lo.p[1]);
         *reinterpret_cast<uint2 *>(&L.wx[buf][0][lane * XS + 4 * w]) = hi.u;
         *reinterpret_cast<uint2 *>(&L.wx[buf][1][lane * XS + 4 * w]) = lo.u;
-        if (t0 + SSM_CHUNK < len) fetch(t0 + SSM_CHUNK, min(SSM_CHUNK, len - t0 - SSM_CHUNK));
+        if (t0 + 2 * SSM_CHUNK < len) fetch(f, t0 + 2 * SSM_CHUNK);
         __syncthreads();            // (a buffer was read last two turns ago: every wavefront has passed the barrier between)
         const float keep = __builtin_amdgcn_exp2f(total);
         Frag8 wx[2][2];
@@ -434,6 +444,12 @@ state_space_states_kernel(SsmChunks k) {
                     for (int h = 0; h < 2; ++h)
                         S[j][h] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(bf[h][u].v, wx[u][part].v, S[j][h], 0, 0, 0);
         }
+    };
+    fetch(ahead0, 0);
+    if (SSM_CHUNK < len) fetch(ahead1, SSM_CHUNK);
+    for (int t0 = 0; t0 < len; t0 += 2 * SSM_CHUNK) {
+        turn(ahead0, t0, 0);
+        if (t0 + SSM_CHUNK < len) turn(ahead1, t0 + SSM_CHUNK, 1);
     }
 #pragma unroll
     for (int j = 0; j < PAIRS; ++j)
@@ -475,29 +491,35 @@ state_space_outputs_kernel(SsmChunks k) {
     const bf16_t *rows = reinterpret_cast<const bf16_t *>(a.xbc) + (size_t)(q0 + t0) * a.xbc_stride;
     const int x_col = head * dv + p0, b_col = a.heads * dv + grp * n, c_col = b_col + a.groups * n;
     const float rate = expf(a.a_log[head]) * LOG2E, skip = a.d_skip[head];
-    const float pd = lane < m ? ssm_ld(a.y, a.y_dtype, (size_t)(q0 + t0 + lane) * a.y_stride + a.dt_off + head) : 0.f;
+    // (no branch around a load: tokens past the chunk's last one repeat that one - nobody sees them or stores what they
+    // see - and columns of B and x past the last one repeat others, which meet zeros of C or are not stored)
+    const uint16_t pd = reinterpret_cast<const uint16_t *>(a.y)[(size_t)(q0 + t0 + min(lane, m - 1)) * a.y_stride + a.dt_off + head];
     uint4 pb[PIECES];
 #pragma unroll
     for (int j = 0; j < PIECES; ++j) {
-        const int i = tid + 256 * j, tt = i / (NP / 8), c = 8 * (i % (NP / 8));
-        pb[j] = tt < m && c < n ? *reinterpret_cast<const uint4 *>(rows + (size_t)tt * a.xbc_stride + b_col + c) : make_uint4(0u, 0u, 0u, 0u);
+        const int i = tid + 256 * j, tt = min(i / (NP / 8), m - 1), c = min(8 * (i % (NP / 8)), n - 8);
+        pb[j] = *reinterpret_cast<const uint4 *>(rows + (size_t)tt * a.xbc_stride + b_col + c);
     }
     uint2 px[4];
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
-        const int i = tid + 256 * j, tt = i / 16, p = 4 * (i % 16);
-        px[j] = tt < m && p0 + p < dv ? *reinterpret_cast<const uint2 *>(rows + (size_t)tt * a.xbc_stride + x_col + p) : make_uint2(0u, 0u);
+        const int i = tid + 256 * j, tt = min(i / 16, m - 1), p = min(p0 + 4 * (i % 16), dv - 4);
+        px[j] = *reinterpret_cast<const uint2 *>(rows + (size_t)tt * a.xbc_stride + head * dv + p);
     }
     const int t = 16 * w + r;
     Frag8 cf[NK];
 #pragma unroll
     for (int ks = 0; ks < NK; ++ks)
 #pragma unroll
-        for (int h = 0; h < 2; ++h) {
-            const int c = 32 * ks + 16 * h + 4 * g;
-            cf[ks].u2[h] = t < m && c < n ? *reinterpret_cast<const uint2 *>(rows + (size_t)t * a.xbc_stride + c_col + c) : make_uint2(0u, 0u);
-        }
-    const float dt = lane < m ? ssm_softplus(pd + a.dt_bias[head]) : 0.f;
+        for (int h = 0; h < 2; ++h)
+            cf[ks].u2[h] = *reinterpret_cast<const uint2 *>(rows + (size_t)min(t, m - 1) * a.xbc_stride + c_col +
+                                                            min(32 * ks + 16 * h + 4 * g, n - 4));
+#pragma unroll
+    for (int ks = 0; ks < NK; ++ks)
+#pragma unroll
+        for (int h = 0; h < 2; ++h)
+            if (32 * ks + 16 * h + 4 * g >= n) cf[ks].u2[h] = make_uint2(0u, 0u);
+    const float dt = lane < m ? ssm_softplus_short(bf16_bits_to_float(pd) + a.dt_bias[head]) : 0.f;
     const float cum = ssm_prefix(-rate * dt);
 #pragma unroll
     for (int j = 0; j < PIECES; ++j) {
@@ -624,8 +646,8 @@ extern "C" int kva_state_space(int kernel, int len_lo, int len_hi, float *out, f
     KVA_REQUIRE(kernel != SSM_TOKEN || (len_lo == 1 && len_hi == 1), "state_space: the kernel of a single token takes entries of one");
     const bool rows16 = seat_stride % 4 == 0 && state_off % 4 == 0 && ((reinterpret_cast<uintptr_t>(state) | reinterpret_cast<uintptr_t>(out)) & 15) == 0;
     KVA_REQUIRE(kernel == SSM_SCAN || rows16, "state_space: states and results must start at multiples of 16 bytes");
-    KVA_REQUIRE(kernel != SSM_CHUNKS || (xbc_stride % 8 == 0 && (reinterpret_cast<uintptr_t>(xbc) & 15) == 0),
-                "state_space: rows must start at multiples of 16 bytes");
+    KVA_REQUIRE(kernel != SSM_CHUNKS || (y_dtype == KVA_BF16 && xbc_stride % 8 == 0 && (reinterpret_cast<uintptr_t>(xbc) & 15) == 0),
+                "state_space: bf16 rows that start at multiples of 16 bytes");
     if (entries == 0) return KVA_OK;
     const SsmArgs a{out, state, (size_t)seat_stride, state_off, entry_q_start, entry_seat, xbc, xbc_dtype, xbc_stride, y,
                     y_dtype, y_stride, dt_off, a_log, dt_bias, d_skip, heads, groups, n, vdim, len_lo, len_hi};
