@@ -5,6 +5,7 @@
 //  * kva_moe_route:  scores = softmax(logits) over all router outputs; the `top` largest of
 //    scores + correction are chosen; their weights are the plain scores (optionally renormalised).
 //    Or (`over_chosen`) the largest logits are chosen and the weights are the softmax over them alone.
+//  * kva_moe_router: the router's product (bf16 operands), that choice and, for up to 16 tokens, the list below in one launch.
 //  * kva_moe_align:  the (token, choice) slots of real experts sorted by expert into a list padded
 //    so that every tile of 16 rows belongs to one expert (`sorted_slot`, -1 = padding), with the
 //    expert of every tile (`tile_expert`, -1 = unused tile).  Without a router (`table`): the experts of a
@@ -38,22 +39,22 @@ __device__ inline float moe_activate(float z, int act) {
 }
 
 // ---- router ------------------------------------------------------------------------------
-__global__ void __launch_bounds__(256)
-moe_route_kernel(int *__restrict__ idx, float *__restrict__ wgt, const float *__restrict__ logits,
-                 const float *__restrict__ correction, int tokens, int outputs, int top, int renormalise,
-                 int over_chosen, int sigmoid_scores, int groups, int keep_groups, int group_top, float weight_scale,
-                 float sum_eps, int logits_stride) {
-    __shared__ float choice_s[4][KVA_WAVE * MOE_ROUTE_PER_LANE];
+struct MoeRoute {
+    const float *correction;
+    int outputs, top, renormalise, over_chosen, sigmoid_scores, groups, keep_groups, group_top;
+    float weight_scale, sum_eps;
+};
+
+// one token by one wavefront: `logits` [outputs] (memory or LDS) -> idx and wgt [top]; `choice` is the wavefront's own
+// piece of LDS, KVA_WAVE * MOE_ROUTE_PER_LANE floats (read with groups only)
+__device__ inline void moe_route_token(const MoeRoute &a, const float *logits, int *idx, float *wgt, float *choice) {
     const int lane = threadIdx.x % KVA_WAVE;
-    const int t = blockIdx.x * (blockDim.x / KVA_WAVE) + threadIdx.x / KVA_WAVE;
-    if (t >= tokens) return;
-    float *choice = choice_s[threadIdx.x / KVA_WAVE];
     float s[MOE_ROUTE_PER_LANE], ch[MOE_ROUTE_PER_LANE];
     float mx = -INFINITY;
 #pragma unroll
     for (int j = 0; j < MOE_ROUTE_PER_LANE; ++j) {
         const int e = lane + j * KVA_WAVE;
-        s[j] = e < outputs ? logits[(size_t)t * logits_stride + e] : -INFINITY;
+        s[j] = e < a.outputs ? logits[e] : -INFINITY;
         mx = fmaxf(mx, s[j]);
     }
     mx = wave_max(mx);
@@ -61,38 +62,38 @@ moe_route_kernel(int *__restrict__ idx, float *__restrict__ wgt, const float *__
 #pragma unroll
     for (int j = 0; j < MOE_ROUTE_PER_LANE; ++j) {
         const int e = lane + j * KVA_WAVE;
-        s[j] = e < outputs ? expf(s[j] - mx) : 0.f;
+        s[j] = e < a.outputs ? expf(s[j] - mx) : 0.f;
         sum += s[j];
     }
     sum = wave_sum(sum);
 #pragma unroll
     for (int j = 0; j < MOE_ROUTE_PER_LANE; ++j) {
         const int e = lane + j * KVA_WAVE;
-        if (over_chosen) {
+        if (a.over_chosen) {
             // the logits themselves are compared, and the weights are a softmax over the chosen ones
             // alone: exp(logit - max) here, divided by the chosen ones' sum below
-            ch[j] = e < outputs ? logits[(size_t)t * logits_stride + e] + (correction ? correction[e] : 0.f) : -INFINITY;
+            ch[j] = e < a.outputs ? logits[e] + (a.correction ? a.correction[e] : 0.f) : -INFINITY;
         } else {
             // scores: the softmax over all outputs, or every output's own sigmoid
-            s[j] = sigmoid_scores ? (e < outputs ? 1.f / (1.f + expf(-logits[(size_t)t * logits_stride + e])) : 0.f) : s[j] / sum;
-            ch[j] = e < outputs ? s[j] + (correction ? correction[e] : 0.f) : -INFINITY;
+            s[j] = a.sigmoid_scores ? (e < a.outputs ? 1.f / (1.f + expf(-logits[e])) : 0.f) : s[j] / sum;
+            ch[j] = e < a.outputs ? s[j] + (a.correction ? a.correction[e] : 0.f) : -INFINITY;
         }
     }
-    if (groups > 1) {
+    if (a.groups > 1) {
         // Outputs form `groups` equal runs of neighbours.  A group's score is the sum of its `group_top`
         // largest choice scores; only outputs of the `keep_groups` best groups (of equal ones the lowest
         // index) can be chosen: the others' choice scores become -inf.  Lane g takes group g.
-        const int per = outputs / groups;
+        const int per = a.outputs / a.groups;
 #pragma unroll
         for (int j = 0; j < MOE_ROUTE_PER_LANE; ++j)
-            if (lane + j * KVA_WAVE < outputs) choice[lane + j * KVA_WAVE] = ch[j];
+            if (lane + j * KVA_WAVE < a.outputs) choice[lane + j * KVA_WAVE] = ch[j];
         __builtin_amdgcn_wave_barrier();
         __threadfence_block();
         float gs = -INFINITY;
-        if (lane < groups) {
+        if (lane < a.groups) {
             gs = 0.f;
             unsigned long long taken = 0ull;            // (a group holds at most 64 outputs when it is scored this way; larger ones below)
-            for (int k = 0; k < group_top && k < per; ++k) {
+            for (int k = 0; k < a.group_top && k < per; ++k) {
                 float bv = -INFINITY;
                 int bi = -1;
                 for (int i = 0; i < per; ++i) {
@@ -105,9 +106,9 @@ moe_route_kernel(int *__restrict__ idx, float *__restrict__ wgt, const float *__
             }
         }
         unsigned long long allowed = 0ull;
-        for (int k = 0; k < keep_groups; ++k) {
+        for (int k = 0; k < a.keep_groups; ++k) {
             float bv = gs;
-            int bg = lane < groups && !((allowed >> lane) & 1ull) ? lane : 0x7fffffff;
+            int bg = lane < a.groups && !((allowed >> lane) & 1ull) ? lane : 0x7fffffff;
             if (bg == 0x7fffffff) bv = -INFINITY;
 #pragma unroll
             for (int off = KVA_WAVE / 2; off > 0; off >>= 1) {
@@ -120,18 +121,18 @@ moe_route_kernel(int *__restrict__ idx, float *__restrict__ wgt, const float *__
 #pragma unroll
         for (int j = 0; j < MOE_ROUTE_PER_LANE; ++j) {
             const int e = lane + j * KVA_WAVE;
-            if (e < outputs && !((allowed >> (e / per)) & 1ull)) ch[j] = -INFINITY;
+            if (e < a.outputs && !((allowed >> (e / per)) & 1ull)) ch[j] = -INFINITY;
         }
     }
     float total = 0.f;
-    for (int k = 0; k < top; ++k) {
+    for (int k = 0; k < a.top; ++k) {
         // the largest remaining choice score; of equal ones the lowest index
         float bv = -INFINITY, bs = 0.f;
         int be = 0x7fffffff;
 #pragma unroll
         for (int j = 0; j < MOE_ROUTE_PER_LANE; ++j) {
             const int e = lane + j * KVA_WAVE;
-            if (e < outputs && (ch[j] > bv || (ch[j] == bv && e < be))) { bv = ch[j]; be = e; bs = s[j]; }
+            if (e < a.outputs && (ch[j] > bv || (ch[j] == bv && e < be))) { bv = ch[j]; be = e; bs = s[j]; }
         }
 #pragma unroll
         for (int off = KVA_WAVE / 2; off > 0; off >>= 1) {
@@ -144,16 +145,40 @@ moe_route_kernel(int *__restrict__ idx, float *__restrict__ wgt, const float *__
             if (lane + j * KVA_WAVE == be) ch[j] = -INFINITY;
         total += bs;
         if (lane == 0) {
-            idx[(size_t)t * top + k] = be;
-            wgt[(size_t)t * top + k] = bs;
+            idx[k] = be;
+            wgt[k] = bs;
         }
     }
     if (lane == 0) {
-        if (renormalise || over_chosen)
-            for (int k = 0; k < top; ++k) wgt[(size_t)t * top + k] = wgt[(size_t)t * top + k] / (total + sum_eps) * weight_scale;
-        else if (weight_scale != 1.f)
-            for (int k = 0; k < top; ++k) wgt[(size_t)t * top + k] *= weight_scale;
+        if (a.renormalise || a.over_chosen)
+            for (int k = 0; k < a.top; ++k) wgt[k] = wgt[k] / (total + a.sum_eps) * a.weight_scale;
+        else if (a.weight_scale != 1.f)
+            for (int k = 0; k < a.top; ++k) wgt[k] *= a.weight_scale;
     }
+}
+
+__global__ void __launch_bounds__(256)
+moe_route_kernel(int *__restrict__ idx, float *__restrict__ wgt, const float *__restrict__ logits, MoeRoute a, int tokens,
+                 int logits_stride) {
+    __shared__ float choice_s[4][KVA_WAVE * MOE_ROUTE_PER_LANE];
+    const int t = blockIdx.x * (blockDim.x / KVA_WAVE) + threadIdx.x / KVA_WAVE;
+    if (t >= tokens) return;
+    moe_route_token(a, logits + (size_t)t * logits_stride, idx + (size_t)t * a.top, wgt + (size_t)t * a.top,
+                    choice_s[threadIdx.x / KVA_WAVE]);
+}
+
+static int moe_route_check(const MoeRoute &a) {
+    KVA_REQUIRE(a.groups >= 1 && a.groups <= KVA_WAVE && a.outputs % a.groups == 0 && a.keep_groups >= 1 &&
+                    a.keep_groups <= a.groups && a.group_top >= 1,
+                "moe_route: %d groups (at most %d, dividing the %d outputs) of which %d are kept", a.groups, KVA_WAVE, a.outputs,
+                a.keep_groups);
+    KVA_REQUIRE(a.groups == 1 || (a.outputs / a.groups <= 64 && a.top <= a.keep_groups * (a.outputs / a.groups)),
+                "moe_route: groups of at most 64 outputs, and enough outputs in the kept groups for top %d", a.top);
+    KVA_REQUIRE(!(a.sigmoid_scores && a.over_chosen), "moe_route: sigmoid scores exclude the softmax over the chosen logits");
+    KVA_REQUIRE(a.outputs > 0 && a.outputs <= KVA_WAVE * MOE_ROUTE_PER_LANE, "moe_route: %d router outputs (at most %d)",
+                a.outputs, KVA_WAVE * MOE_ROUTE_PER_LANE);
+    KVA_REQUIRE(a.top > 0 && a.top <= a.outputs, "moe_route: top %d of %d", a.top, a.outputs);
+    return KVA_OK;
 }
 
 extern "C" int kva_moe_route(int *idx, float *wgt, const float *logits, const float *correction, int tokens,
@@ -162,21 +187,11 @@ extern "C" int kva_moe_route(int *idx, float *wgt, const float *logits, const fl
                              hipStream_t stream) {
     // logits_stride: elements between two tokens' rows of logits (the logits may be the first columns of a wider product)
     KVA_REQUIRE(logits_stride >= outputs, "moe_route: a row of logits holds at least the %d outputs", outputs);
-    KVA_REQUIRE(groups >= 1 && groups <= KVA_WAVE && outputs % groups == 0 && keep_groups >= 1 && keep_groups <= groups &&
-                    group_top >= 1,
-                "moe_route: %d groups (at most %d, dividing the %d outputs) of which %d are kept", groups, KVA_WAVE, outputs,
-                keep_groups);
-    KVA_REQUIRE(groups == 1 || (outputs / groups <= 64 && top <= keep_groups * (outputs / groups)),
-                "moe_route: groups of at most 64 outputs, and enough outputs in the kept groups for top %d", top);
-    KVA_REQUIRE(!(sigmoid_scores && over_chosen), "moe_route: sigmoid scores exclude the softmax over the chosen logits");
     KVA_REQUIRE(idx && wgt && logits && tokens >= 0, "moe_route: missing operand");
-    KVA_REQUIRE(outputs > 0 && outputs <= KVA_WAVE * MOE_ROUTE_PER_LANE, "moe_route: %d router outputs (at most %d)",
-                outputs, KVA_WAVE * MOE_ROUTE_PER_LANE);
-    KVA_REQUIRE(top > 0 && top <= outputs, "moe_route: top %d of %d", top, outputs);
+    const MoeRoute a{correction, outputs, top, renormalise, over_chosen, sigmoid_scores, groups, keep_groups, group_top, weight_scale, sum_eps};
+    if (int rc = moe_route_check(a)) return rc;
     if (tokens == 0) return KVA_OK;
-    hipLaunchKernelGGL(moe_route_kernel, dim3((tokens + 3) / 4), dim3(256), 0, stream, idx, wgt, logits, correction,
-                       tokens, outputs, top, renormalise, over_chosen, sigmoid_scores, groups, keep_groups, group_top,
-                       weight_scale, sum_eps, logits_stride);
+    hipLaunchKernelGGL(moe_route_kernel, dim3((tokens + 3) / 4), dim3(256), 0, stream, idx, wgt, logits, a, tokens, logits_stride);
     KVA_CHECK_LAUNCH("moe_route");
     return KVA_OK;
 }
@@ -204,10 +219,8 @@ __device__ inline int moe_slot_expert(int *idx, int s, const MoeTable &tab) {
     return tab.table[(size_t)id * tab.top + s % tab.top];
 }
 
-__global__ void __launch_bounds__(1024)
-moe_align_kernel(int *__restrict__ sorted_slot, int *__restrict__ tile_expert, int *idx, int slots, int experts, int capacity,
-                 int max_tiles, int group, MoeTable tab) {
-    __shared__ int count[MOE_MAX_EXPERTS], start[MOE_MAX_EXPERTS];
+__device__ inline void moe_align_workgroup(int *sorted_slot, int *tile_expert, int *idx, int slots, int experts, int capacity,
+                                           int max_tiles, int group, const MoeTable &tab, int *count, int *start) {
     const bool in_registers = slots <= (int)blockDim.x * MOE_SLOTS_IN_REGISTERS;
     int ex[MOE_SLOTS_IN_REGISTERS], at[MOE_SLOTS_IN_REGISTERS];
 #pragma unroll
@@ -273,14 +286,27 @@ moe_align_kernel(int *__restrict__ sorted_slot, int *__restrict__ tile_expert, i
     }
 }
 
-static int moe_align_launch(int *sorted_slot, int *tile_expert, int *idx, int slots, int experts, int capacity, int max_tiles,
-                            int group, const MoeTable &tab, hipStream_t stream) {
+__global__ void __launch_bounds__(1024)
+moe_align_kernel(int *__restrict__ sorted_slot, int *__restrict__ tile_expert, int *idx, int slots, int experts, int capacity,
+                 int max_tiles, int group, MoeTable tab) {
+    __shared__ int count[MOE_MAX_EXPERTS], start[MOE_MAX_EXPERTS];
+    moe_align_workgroup(sorted_slot, tile_expert, idx, slots, experts, capacity, max_tiles, group, tab, count, start);
+}
+
+static int moe_align_check(const int *sorted_slot, const int *tile_expert, const int *idx, int slots, int experts, int capacity,
+                           int max_tiles, int group) {
     KVA_REQUIRE(group >= 1 && max_tiles % group == 0, "moe_align: %d tiles do not come in groups of %d", max_tiles, group);
     KVA_REQUIRE(sorted_slot && tile_expert && idx, "moe_align: missing operand");
     KVA_REQUIRE(experts > 0 && experts <= MOE_MAX_EXPERTS, "moe_align: %d experts (at most %d)", experts, MOE_MAX_EXPERTS);
     KVA_REQUIRE(capacity == max_tiles * MOE_TILE && capacity >= slots + experts * (MOE_TILE * group - 1),
                 "moe_align: a list of %d places cannot hold %d slots of %d experts in tiles of %d", capacity, slots,
                 experts, MOE_TILE);
+    return KVA_OK;
+}
+
+static int moe_align_launch(int *sorted_slot, int *tile_expert, int *idx, int slots, int experts, int capacity, int max_tiles,
+                            int group, const MoeTable &tab, hipStream_t stream) {
+    if (int rc = moe_align_check(sorted_slot, tile_expert, idx, slots, experts, capacity, max_tiles, group)) return rc;
     hipLaunchKernelGGL(moe_align_kernel, dim3(1), dim3(1024), 0, stream, sorted_slot, tile_expert, idx, slots, experts,
                        capacity, max_tiles, group, tab);
     KVA_CHECK_LAUNCH("moe_align");
@@ -300,6 +326,108 @@ extern "C" int kva_moe_table_align(int *sorted_slot, int *tile_expert, int *idx,
     KVA_REQUIRE(wgt && table && ids && table_rows > 0 && tokens >= 0 && top > 0, "moe_table_align: missing operand or bad sizes");
     return moe_align_launch(sorted_slot, tile_expert, idx, tokens * top, experts, capacity, max_tiles, group,
                             MoeTable{table, ids, feedback, table_rows, top, weight, wgt}, stream);
+}
+
+// ---- the router's product, the choice and (few tokens) the sorted list in one launch ---------------------------------
+// A workgroup of 16 wavefronts takes 16 tokens: logits^T[n, t] = W[n, :] . x[t, :] + bias[n] on the matrix cores (bf16
+// operands, whose products are exact, and fp32 sums), a tile of 16 outputs and a part of K a wavefront; the parts meet in
+// LDS in a fixed order, and wavefront i then routes token i.  Outputs past the router's (an expert's gate, say) go to
+// `rest` [tokens, N - outputs].  A single workgroup's slots are sorted by expert right behind it.  The order of every
+// sum depends on the sizes alone.
+#define MOE_ROUTER_MAX_N 512
+
+struct MoeRouter {
+    const bf16_t *x, *w;
+    const float *bias;
+    float *rest;
+    int *idx;
+    float *wgt;
+    int tokens, N, K, x_stride;
+};
+
+__global__ void __launch_bounds__(1024)
+moe_router_kernel(MoeRouter m, MoeRoute a, int *__restrict__ sorted_slot, int *__restrict__ tile_expert, int experts, int capacity,
+                  int max_tiles, int group) {
+    extern __shared__ float moe_lds[];
+    __shared__ int count[MOE_MAX_EXPERTS], start[MOE_MAX_EXPERTS];
+    __shared__ float part[16][KVA_WAVE][4];
+    const int lane = threadIdx.x % KVA_WAVE, wave = threadIdx.x / KVA_WAVE, r = lane & 15, g = lane >> 4;
+    const int t0 = blockIdx.x * 16, tiles = (m.N + 15) / 16, parts = tiles < 16 ? 16 / tiles : 1;
+    float *logits = moe_lds;                                     // [16 tokens][N]
+    const int steps = m.K / 32, per = (steps + parts - 1) / parts;
+    const bf16_t *xrow = m.x + (size_t)min(t0 + r, m.tokens - 1) * m.x_stride + 8 * g;
+    for (int tile0 = 0; tile0 < tiles; tile0 += 16) {            // (more than 256 outputs: in turns)
+        const int tile = tile0 + wave % min(tiles, 16), kp = wave / min(tiles, 16);
+        const bool on = tile < tiles && kp < parts;
+        f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+        if (on) {
+            const bf16_t *wrow = m.w + (size_t)min(16 * tile + r, m.N - 1) * m.K + 8 * g;
+            const int s1 = min(steps, (kp + 1) * per);
+#pragma unroll 8
+            for (int s = kp * per; s < s1; ++s) {
+                Frag8 xf, wf;
+                xf.u4 = *reinterpret_cast<const uint4 *>(xrow + 32 * s);
+                wf.u4 = *reinterpret_cast<const uint4 *>(wrow + 32 * s);
+                acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf.v, xf.v, acc, 0, 0, 0);
+            }
+        }
+        __syncthreads();
+#pragma unroll
+        for (int i = 0; i < 4; ++i) part[wave][lane][i] = acc[i];
+        __syncthreads();
+        if (on && kp == 0) {                                     // lane (token r, group g): outputs 16 tile + 4 g .. + 3
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                const int n = 16 * tile + 4 * g + i;
+                float v = acc[i];
+                for (int p = 1; p < parts; ++p) v += part[wave + p * min(tiles, 16)][lane][i];
+                if (n < m.N) logits[r * m.N + n] = v + (m.bias ? m.bias[n] : 0.f);
+            }
+        }
+    }
+    __syncthreads();
+    const int t = t0 + wave;
+    if (t < m.tokens) {
+        moe_route_token(a, logits + wave * m.N, m.idx + (size_t)t * a.top, m.wgt + (size_t)t * a.top,
+                        logits + 16 * m.N + (a.groups > 1 ? wave * KVA_WAVE * MOE_ROUTE_PER_LANE : 0));
+        for (int n = a.outputs + lane; n < m.N; n += KVA_WAVE) m.rest[(size_t)t * (m.N - a.outputs) + n - a.outputs] = logits[wave * m.N + n];
+    }
+    if (!sorted_slot) return;
+    __threadfence_block();
+    __syncthreads();
+    moe_align_workgroup(sorted_slot, tile_expert, m.idx, m.tokens * a.top, experts, capacity, max_tiles, group,
+                        MoeTable{nullptr, nullptr, nullptr, 0, 1, 0.f, nullptr}, count, start);
+}
+
+extern "C" int kva_moe_router_supported(int x_dtype, int w_dtype, int N, int K) {
+    return x_dtype == KVA_BF16 && w_dtype == KVA_BF16 && K > 0 && K % 32 == 0 && N > 0 && N <= MOE_ROUTER_MAX_N;
+}
+
+// sorted_slot may be null: the list is then left to kva_moe_align (it must be for more than 16 tokens)
+extern "C" int kva_moe_router(int *idx, float *wgt, float *rest, const void *x, int x_stride, const void *w, const float *bias,
+                              const float *correction, int tokens, int N, int K, int outputs, int top, int renormalise,
+                              int over_chosen, int sigmoid_scores, int groups, int keep_groups, int group_top,
+                              float weight_scale, float sum_eps, int *sorted_slot, int *tile_expert, int experts,
+                              int capacity, int max_tiles, int group, hipStream_t stream) {
+    KVA_REQUIRE(idx && wgt && x && w && tokens >= 0 && outputs <= N && (outputs == N || rest), "moe_router: missing operand");
+    KVA_REQUIRE(kva_moe_router_supported(KVA_BF16, KVA_BF16, N, K) && x_stride >= K && x_stride % 8 == 0 &&
+                    ((reinterpret_cast<uintptr_t>(x) | reinterpret_cast<uintptr_t>(w)) & 15) == 0,
+                "moe_router: no kernel for %d outputs of %d elements, or rows that do not start at multiples of 16 bytes", N, K);
+    const MoeRoute a{correction, outputs, top, renormalise, over_chosen, sigmoid_scores, groups, keep_groups, group_top, weight_scale, sum_eps};
+    if (int rc = moe_route_check(a)) return rc;
+    if (sorted_slot) {
+        KVA_REQUIRE(tokens <= 16, "moe_router: the list of more than 16 tokens is sorted by a launch of its own");
+        if (int rc = moe_align_check(sorted_slot, tile_expert, idx, tokens * top, experts, capacity, max_tiles, group)) return rc;
+    }
+    if (tokens == 0) return KVA_OK;
+    const size_t lds = (size_t)(16 * N + (groups > 1 ? 16 * KVA_WAVE * MOE_ROUTE_PER_LANE : 0)) * sizeof(float);
+    if (lds > 32 * 1024)
+        hipFuncSetAttribute(reinterpret_cast<const void *>(moe_router_kernel), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+    hipLaunchKernelGGL(moe_router_kernel, dim3((tokens + 15) / 16), dim3(1024), lds, stream,
+                       MoeRouter{(const bf16_t *)x, (const bf16_t *)w, bias, rest, idx, wgt, tokens, N, K, x_stride}, a, sorted_slot,
+                       tile_expert, experts, capacity, max_tiles, group);
+    KVA_CHECK_LAUNCH("moe_router");
+    return KVA_OK;
 }
 
 // ---- one product per tile ------------------------------------------------------------------

@@ -848,7 +848,8 @@ extern "C" int kva_sandwich_step(float *x, const void *y, int y_dtype, const voi
 // then element by element,
 //     x <- x + n_post(y + y_bias),    out = n_pre(x),
 // over the residual stream x [rows, width] fp32; y_bias (fp32, optional) is the bias of the product that made y.
-// Without y the stream is only read; without `out` it is only updated.  With row_idx only the named rows are
+// The branch output may still be the rows of routed experts: y = sum_k rows[t top + k] + sigmoid(gate[t]) extra[t] (the
+// second part optional, with or without its gate).  Without y the stream is only read; without `out` it is only updated.  With row_idx only the named rows are
 // read, and nothing is written back: the model's last norm.  A thread takes 4 neighbouring elements of a row
 // (VEC) or one.
 struct TanhNorm {
@@ -857,10 +858,15 @@ struct TanhNorm {
     float alpha;
 };
 
+struct TanhRows {
+    const float *rows, *gate;
+    int top, gate_stride;
+};
+
 template <bool VEC>
 __global__ void __launch_bounds__(256)
 tanh_step_kernel(float *__restrict__ x, const void *__restrict__ y, int y_dtype, const float *__restrict__ y_bias,
-                 TanhNorm post, TanhNorm pre, void *__restrict__ out, int out_dtype, const int *__restrict__ row_idx,
+                 TanhRows er, TanhNorm post, TanhNorm pre, void *__restrict__ out, int out_dtype, const int *__restrict__ row_idx,
                  int width, size_t n) {
     constexpr int W = VEC ? 4 : 1;
     const size_t i = ((size_t)blockIdx.x * blockDim.x + threadIdx.x) * W;
@@ -876,8 +882,24 @@ tanh_step_kernel(float *__restrict__ x, const void *__restrict__ y, int y_dtype,
 #pragma unroll
     for (int e = 0; e < W; ++e) yv[e] = yb[e] = pw[e] = pb[e] = nw[e] = nb[e] = 0.f;
     load(x, KVA_F32, at, v);
-    if (y) {
-        load(y, y_dtype, at, yv);
+    const bool enters = y || er.rows;
+    if (enters) {
+        if (y) load(y, y_dtype, at, yv);
+        if (er.rows) {
+            const size_t t = at / width;
+            const float eg = y && er.gate ? 1.f / (1.f + expf(-er.gate[t * er.gate_stride])) : 1.f;
+            float sum[W];
+#pragma unroll
+            for (int e = 0; e < W; ++e) sum[e] = 0.f;
+            for (int k = 0; k < er.top; ++k) {
+                float f[W];
+                load(er.rows, KVA_F32, (t * er.top + k) * width + j, f);
+#pragma unroll
+                for (int e = 0; e < W; ++e) sum[e] += f[e];
+            }
+#pragma unroll
+            for (int e = 0; e < W; ++e) yv[e] = sum[e] + (y ? eg * yv[e] : 0.f);
+        }
         if (y_bias) load(y_bias, KVA_F32, j, yb);
         if (post.w) {
             load(post.w, post.dtype, j, pw);
@@ -888,7 +910,7 @@ tanh_step_kernel(float *__restrict__ x, const void *__restrict__ y, int y_dtype,
         load(pre.w, pre.dtype, j, nw);
         load(pre.b, pre.dtype, j, nb);
     }
-    if (y) {
+    if (enters) {
 #pragma unroll
         for (int e = 0; e < W; ++e) v[e] += post.w ? tanhf(post.alpha * (yv[e] + yb[e])) * pw[e] + pb[e] : yv[e] + yb[e];
         if (!row_idx) {
@@ -915,25 +937,27 @@ tanh_step_kernel(float *__restrict__ x, const void *__restrict__ y, int y_dtype,
 extern "C" int kva_tanh_step(float *x, const void *y, int y_dtype, const float *y_bias, const void *post_w, const void *post_b,
                              int post_dtype, float post_alpha, const void *pre_w, const void *pre_b, int pre_dtype,
                              float pre_alpha, void *out, int out_dtype, const int *row_idx, int rows, int width,
-                             hipStream_t stream) {
+                             const float *expert_rows, const float *gate, int top, int gate_stride, hipStream_t stream) {
     KVA_REQUIRE(x && rows >= 0 && width > 0, "tanh_step: missing operand or bad sizes");
-    KVA_REQUIRE(y || (!post_w && !y_bias), "tanh_step: a norm or a bias without the branch output it goes with");
+    KVA_REQUIRE(!expert_rows || (top > 0 && gate_stride >= 0), "tanh_step: experts' rows come so many a token");
+    KVA_REQUIRE(y || expert_rows || (!post_w && !y_bias), "tanh_step: a norm or a bias without the branch output it goes with");
     KVA_REQUIRE((post_w == nullptr) == (post_b == nullptr) && (pre_w == nullptr) == (pre_b == nullptr),
                 "tanh_step: a norm has a weight and a bias");
     KVA_REQUIRE(!out || pre_w, "tanh_step: the read-out needs a norm");
-    KVA_REQUIRE(y || out, "tanh_step: nothing to do");
+    KVA_REQUIRE(y || expert_rows || out, "tanh_step: nothing to do");
     KVA_REQUIRE(!row_idx || out, "tanh_step: rows are gathered for the read-out only");
     if (rows == 0) return KVA_OK;
     const TanhNorm post{post_w, post_b, post_dtype, post_alpha}, pre{pre_w, pre_b, pre_dtype, pre_alpha};
     const size_t n = (size_t)rows * width;
-    const bool vec = width % 4 == 0 && aligned16(x) && aligned16(y) && aligned16(y_bias) && aligned16(post_w) &&
+    const TanhRows er{expert_rows, gate, top, gate_stride};
+    const bool vec = width % 4 == 0 && aligned16(x) && aligned16(y) && aligned16(y_bias) && aligned16(expert_rows) && aligned16(post_w) &&
                      aligned16(post_b) && aligned16(pre_w) && aligned16(pre_b) && aligned16(out);
     if (vec)
         hipLaunchKernelGGL(tanh_step_kernel<true>, dim3((unsigned)((n / 4 + 255) / 256)), dim3(256), 0, stream, x, y, y_dtype,
-                           y_bias, post, pre, out, out_dtype, row_idx, width, n);
+                           y_bias, er, post, pre, out, out_dtype, row_idx, width, n);
     else
         hipLaunchKernelGGL(tanh_step_kernel<false>, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, stream, x, y, y_dtype,
-                           y_bias, post, pre, out, out_dtype, row_idx, width, n);
+                           y_bias, er, post, pre, out, out_dtype, row_idx, width, n);
     KVA_CHECK_LAUNCH("tanh_step");
     return KVA_OK;
 }
@@ -956,12 +980,14 @@ __device__ inline int pair_token(const int *ids, const int *feedback, int t, int
     return id < 0 ? 0 : (id >= table_rows ? table_rows - 1 : id);
 }
 
+template <bool VEC>
 __global__ void __launch_bounds__(256)
 pair_embed_kernel(float *__restrict__ x, const void *__restrict__ table, int table_dtype, int table_rows, float scale,
                   PairTable pairs, TanhNorm norm, const int *__restrict__ ids, const int *__restrict__ feedback,
                   int *__restrict__ state, int state_stride, const int *__restrict__ entry_q_start,
                   const int *__restrict__ entry_seat, int entries, int width) {
-    __shared__ int entry_s, prev_s;
+    constexpr int W = VEC ? 4 : 1;
+    __shared__ int entry_s, id_s, row_s;
     const int t = blockIdx.x;
     if (threadIdx.x == 0) entry_s = -1;
     __syncthreads();
@@ -969,23 +995,41 @@ pair_embed_kernel(float *__restrict__ x, const void *__restrict__ table, int tab
         if (entry_q_start[e] == t && entry_q_start[e + 1] > t) entry_s = e;      // (one entry at most starts here)
     __syncthreads();
     if (threadIdx.x == 0) {
-        const int e = entry_s;
+        const int e = entry_s, id = pair_token(ids, feedback, t, table_rows);
+        int prev;
         if (e < 0) {
-            prev_s = pair_token(ids, feedback, t - 1, table_rows);
+            prev = pair_token(ids, feedback, t - 1, table_rows);
         } else {
             int *seat = state + (size_t)entry_seat[e] * state_stride;
-            prev_s = *seat - 1;
+            prev = *seat - 1;
             *seat = pair_token(ids, feedback, entry_q_start[e + 1] - 1, table_rows) + 1;
         }
+        id_s = id;
+        row_s = prev < 0 ? pairs.buckets : (int)((prev * pairs.mul_prev + id * pairs.mul_cur) % pairs.buckets);
     }
     __syncthreads();
-    const int id = pair_token(ids, feedback, t, table_rows), prev = prev_s;
-    const int row = prev < 0 ? pairs.buckets : (int)((prev * pairs.mul_prev + id * pairs.mul_cur) % pairs.buckets);
-    for (int j = threadIdx.x; j < width; j += blockDim.x) {
-        float v = ld_as_float(table, table_dtype, (size_t)id * width + j) * scale;
-        if (pairs.p) v += ld_as_float(pairs.p, pairs.dtype, (size_t)row * width + j);
-        if (norm.w) v = tanhf(norm.alpha * v) * ld_as_float(norm.w, norm.dtype, j) + ld_as_float(norm.b, norm.dtype, j);
-        x[(size_t)t * width + j] = v;
+    const size_t id = id_s, row = row_s;
+    auto load = [&](const void *p, int dtype, size_t k, float (&f)[W]) {
+        if constexpr (VEC) hyper_ld4(p, dtype, k, f);
+        else f[0] = ld_as_float(p, dtype, k);
+    };
+    for (int j = W * threadIdx.x; j < width; j += W * blockDim.x) {
+        float v[W], q[W], w[W], b[W];
+#pragma unroll
+        for (int i = 0; i < W; ++i) q[i] = 0.f;
+        load(table, table_dtype, id * width + j, v);
+        if (pairs.p) load(pairs.p, pairs.dtype, row * width + j, q);
+        if (norm.w) {
+            load(norm.w, norm.dtype, j, w);
+            load(norm.b, norm.dtype, j, b);
+        }
+#pragma unroll
+        for (int i = 0; i < W; ++i) {
+            v[i] = v[i] * scale + q[i];
+            if (norm.w) v[i] = tanhf(norm.alpha * v[i]) * w[i] + b[i];
+        }
+        if constexpr (VEC) *reinterpret_cast<float4 *>(x + (size_t)t * width + j) = make_float4(v[0], v[1], v[2], v[3]);
+        else x[(size_t)t * width + j] = v[0];
     }
 }
 
@@ -1000,8 +1044,9 @@ extern "C" int kva_pair_embed(float *x, const void *table, int table_dtype, int 
                 "pair_embed: bad sizes or negative multipliers");
     KVA_REQUIRE((norm_w == nullptr) == (norm_b == nullptr), "pair_embed: a norm has a weight and a bias");
     if (tokens == 0) return KVA_OK;
-    hipLaunchKernelGGL(pair_embed_kernel, dim3(tokens), dim3(256), 0, stream, x, table, table_dtype, table_rows, scale,
-                       PairTable{pair_table, pair_dtype, buckets, mul_prev, mul_cur},
+    const bool vec = width % 4 == 0 && aligned16(x) && aligned16(table) && aligned16(pair_table) && aligned16(norm_w) && aligned16(norm_b);
+    hipLaunchKernelGGL(vec ? pair_embed_kernel<true> : pair_embed_kernel<false>, dim3(tokens), dim3(256), 0, stream, x, table,
+                       table_dtype, table_rows, scale, PairTable{pair_table, pair_dtype, buckets, mul_prev, mul_cur},
                        TanhNorm{norm_w, norm_b, norm_dtype, norm_alpha}, ids, feedback, state, state_stride, entry_q_start,
                        entry_seat, entries, width);
     KVA_CHECK_LAUNCH("pair_embed");

@@ -732,18 +732,26 @@ def tanh_step(x: torch.Tensor, *, y: Optional[torch.Tensor] = None, y_bias: Opti
     """What lies between two branches that have tanh norms on both sides, over a residual stream ``x`` fp32 ``[T,
     width]``: ``x += n_post(y + y_bias)``, then ``out = n_pre(x)``.  ``post`` and ``pre`` are ``(weight, bias, alpha)``:
     ``tanh(alpha v) * weight + bias``.  Without ``post`` the branch output enters as it is (with its bias, fp32).
-    ``row_idx``: only these rows are read out, and nothing is written back."""
+    ``y`` may be :class:`ExpertRows`: the sum is formed on the way.  ``row_idx``: only these rows are read out, and
+    nothing is written back."""
     T, width = x.shape
     if x.dim() != 2 or x.dtype != torch.float32:
         raise KernelError(f"tanh_step: x {tuple(x.shape)} is not an fp32 [T, width] stream")
     if y is not None and y.shape != x.shape:
         raise KernelError("tanh_step: the branch output has the stream's shape")
-    if y_bias is not None and (y is None or y_bias.shape != (width,) or y_bias.dtype != torch.float32):
+    rows_of, gate, top, gate_stride = None, None, 0, 0
+    if isinstance(y, ExpertRows):
+        if y.rows.shape != (T * y.top, width) or y.rows.dtype != torch.float32:
+            raise KernelError(f"tanh_step: experts' rows {tuple(y.rows.shape)} are not fp32 [T * top, width]")
+        rows_of, top = y.rows, y.top
+        gate, gate_stride = y.gate_column()
+        y = y.extra
+    if y_bias is not None and ((y is None and rows_of is None) or y_bias.shape != (width,) or y_bias.dtype != torch.float32):
         raise KernelError("tanh_step: a product's bias is fp32 [width] and goes with the product")
     for norm in (post, pre):
         if norm is not None and (norm[0].shape != (width,) or norm[1].shape != (width,) or norm[1].dtype != norm[0].dtype):
             raise KernelError("tanh_step: a norm has a weight [width] and a bias of its shape and type")
-    if (post is not None and y is None) or (out is None) != (pre is None):
+    if (post is not None and y is None and rows_of is None) or (out is None) != (pre is None):
         raise KernelError("tanh_step: the first norm goes with a branch output, the second with an output")
     rows = T
     if out is not None:
@@ -761,7 +769,8 @@ def tanh_step(x: torch.Tensor, *, y: Optional[torch.Tensor] = None, y_bias: Opti
     check(hip_lib().kva_tanh_step(
         _dev(x, "x"), _opt(y, "y"), dtype_code(y.dtype) if y is not None else 0, _opt(y_bias, "y_bias"), *args(post, "post norm"),
         *args(pre, "pre norm"), _opt(out, "out"), dtype_code(out.dtype) if out is not None else 0,
-        _opt(row_idx, "row_idx", torch.int32), rows, width, _stream()), "tanh_step")
+        _opt(row_idx, "row_idx", torch.int32), rows, width, _opt(rows_of, "rows"),
+        None if gate is None else _dev(gate, "gate", torch.float32, contiguous=False), top, int(gate_stride), _stream()), "tanh_step")
     return out
 
 
@@ -1985,6 +1994,44 @@ def moe_route(logits: torch.Tensor, correction: Optional[torch.Tensor], top: int
                                   logits.stride(0) if tokens > 1 else outputs, _stream()), "moe_route")
 
 
+MOE_ROUTER_LIST_TOKENS = 16         # a step of up to so many tokens has its slots sorted by the router's launch
+
+
+def moe_router_supported(x: torch.Tensor, w: torch.Tensor) -> bool:
+    """Whether :func:`moe_router` takes rows like ``x`` and the router's matrix ``w``."""
+    return bool(hip_lib().kva_moe_router_supported(dtype_code(x.dtype), dtype_code(w.dtype), w.shape[0], w.shape[1]))
+
+
+def moe_router(x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor], correction: Optional[torch.Tensor], outputs: int,
+               top: int, idx: torch.Tensor, wgt: torch.Tensor, rest: Optional[torch.Tensor], renormalise: bool = False,
+               over_chosen: bool = False, *, scores: str = "softmax", groups: int = 1, keep_groups: int = 1, group_top: int = 2,
+               weight_scale: float = 1.0, sum_eps: float = 0.0, experts: int = 0, sorted_slot: Optional[torch.Tensor] = None,
+               tile_expert: Optional[torch.Tensor] = None, group: int = 1) -> None:
+    """The product ``logits = x @ w^T + bias`` of bf16 operands with fp32 sums and :func:`moe_route` over its first
+    ``outputs`` columns in one launch; the columns behind them go to ``rest`` fp32 ``[T, N - outputs]``.  With
+    ``sorted_slot`` and ``tile_expert`` (at most ``MOE_ROUTER_LIST_TOKENS`` tokens) the chosen slots are sorted as
+    :func:`moe_align` does, in the same launch."""
+    tokens, k = x.shape
+    n = w.shape[0]
+    if scores not in ("softmax", "sigmoid"):
+        raise KernelError(f"moe_router: scores {scores!r} is neither 'softmax' nor 'sigmoid'")
+    if w.dim() != 2 or w.shape[1] != k or not moe_router_supported(x, w) or idx.shape != (tokens, top) or wgt.shape != (tokens, top) \
+            or not 0 < outputs <= n or (rest is None) != (outputs == n) or (rest is not None and rest.shape != (tokens, n - outputs)) \
+            or (correction is not None and correction.shape != (outputs,)) or (bias is not None and bias.shape != (n,)):
+        raise KernelError(f"moe_router: x {tuple(x.shape)}, w {tuple(w.shape)}, idx {tuple(idx.shape)} do not fit {outputs} outputs")
+    tiles = 0
+    if sorted_slot is not None:
+        tiles = tile_expert.shape[0]
+        if tokens > MOE_ROUTER_LIST_TOKENS or sorted_slot.shape != (tiles * MOE_TILE,) or tiles < moe_tiles(tokens * top, experts, group):
+            raise KernelError(f"moe_router: {tiles} tiles cannot hold {tokens * top} slots of {experts} experts, or too many tokens")
+    check(hip_lib().kva_moe_router(
+        _dev(idx, "idx", torch.int32), _dev(wgt, "wgt", torch.float32), _opt(rest, "rest", torch.float32), _dev(x, "x"), k,
+        _dev(w, "w"), _opt(bias, "bias", torch.float32), _opt(correction, "correction", torch.float32), tokens, n, k, int(outputs),
+        int(top), 1 if renormalise else 0, 1 if over_chosen else 0, 1 if scores == "sigmoid" else 0, int(groups), int(keep_groups),
+        int(group_top), float(weight_scale), float(sum_eps), _opt(sorted_slot, "sorted_slot", torch.int32),
+        _opt(tile_expert, "tile_expert", torch.int32), int(experts), tiles * MOE_TILE, tiles, int(group), _stream()), "moe_router")
+
+
 def moe_tiles(slots: int, experts: int, group: int = 1) -> int:
     """Tiles of 16 rows that hold ``slots`` (token, choice) pairs sorted by expert, whatever the split, every
     expert's run a multiple of ``group`` tiles."""
@@ -2119,6 +2166,37 @@ def small_product_f32(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, bias:
     return out
 
 
+class ExpertRows:
+    """What routed experts returned, not added up yet: ``rows`` (fp32 ``[T * top, width]``, weighted) and, optionally, the
+    output ``extra`` of an expert every token uses, times ``sigmoid(extra_gate[t])`` (fp32, a column) if that is there.
+    Whoever reads the sum next may form it in its own pass (:func:`tanh_step`); :meth:`sum` forms it with
+    :func:`moe_combine`."""
+
+    def __init__(self, x, rows, idx, wgt, experts: int, extra=None, extra_gate=None):
+        self.x, self.rows, self.idx, self.wgt, self.experts, self.extra, self.extra_gate = x, rows, idx, wgt, experts, extra, extra_gate
+        self.top = idx.shape[1]
+
+    @property
+    def shape(self):
+        return self.x.shape
+
+    @property
+    def dtype(self):
+        return self.x.dtype
+
+    def gate_column(self):
+        """(the gate's numbers as a one-dimensional view or None, elements from one to the next)"""
+        g = self.extra_gate
+        if g is None:
+            return None, 0
+        g = g[:, 0] if g.dim() == 2 else g
+        return g, g.stride(0) if g.shape[0] > 1 else 1
+
+    def sum(self) -> torch.Tensor:
+        return moe_combine(self.x, self.rows, self.idx, self.wgt, self.experts, torch.empty_like(self.x), extra=self.extra,
+                           extra_gate=self.extra_gate)
+
+
 def moe_combine(x: torch.Tensor, rows: torch.Tensor, idx: torch.Tensor, wgt: torch.Tensor, experts: int,
                 out: torch.Tensor, extra: Optional[torch.Tensor] = None,
                 extra_gate: Optional[torch.Tensor] = None) -> torch.Tensor:
@@ -2166,7 +2244,7 @@ KERNEL_CLASSES = {
     "sample": "sampling", "mark_tokens": "sampling",
     "causal_conv_act": "recurrent mixers", "gated_delta_rule": "recurrent mixers",
     "gated_linear_attention": "recurrent mixers", "head_norm_gate": "elementwise",
-    "moe_route": "routed experts", "moe_align": "routed experts", "moe_table_align": "routed experts", "moe_expert_rows": "routed experts",
+    "moe_route": "routed experts", "moe_router": "routed experts", "moe_align": "routed experts", "moe_table_align": "routed experts", "moe_expert_rows": "routed experts",
     "moe_combine": "routed experts", "small_product_f32": "small fp32 products",
     "norm_into_stream": "norm", "table_gate": "elementwise",
     "hyper_step": "norm", "sandwich_step": "norm", "hyper_fill": "embedding", "bias_act": "activation",

@@ -96,6 +96,8 @@ _HIP_SIGNATURES = {
     "kva_gated_linear_attention": [P, P, LL, I, P, I, I, I, I, I, P, I, F, P, I, P, P, I, I, I, I, P],
     "kva_head_norm_gate": [P, I, I, I, P, I, P, F, P, I, I, I, I, I, I, I, I, F, I, P],
     "kva_moe_route": [P, P, P, P, I, I, I, I, I, I, I, I, I, F, F, I, P],
+    "kva_moe_router": [P, P, P, P, I, P, P, P, I, I, I, I, I, I, I, I, I, I, I, F, F, P, P, I, I, I, I, P],
+    "kva_moe_router_supported": [I, I, I, I],
     "kva_moe_align": [P, P, P, I, I, I, I, I, P],
     "kva_moe_group_supported": [I, I],
     "kva_moe_table_align": [P, P, P, P, P, I, P, P, I, I, F, I, I, I, I, P],
@@ -108,7 +110,7 @@ _HIP_SIGNATURES = {
     "kva_hyper_step": [P, I, P, I, P, P, F, P, P, P, I, F, P, I, P, I, I, P],
     "kva_latent_attention_merge": [P, P, P, P, I, I, I, I, P],
     "kva_sandwich_step": [P, P, I, P, P, I, I, F, P, P, P, I, I, F, P, I, P, I, I, P],
-    "kva_tanh_step": [P, P, I, P, P, P, I, F, P, P, I, F, P, I, P, I, I, P],
+    "kva_tanh_step": [P, P, I, P, P, P, I, F, P, P, I, F, P, I, P, I, I, P, P, I, I, P],
     "kva_pair_embed": [P, P, I, I, F, P, I, I, I, I, P, P, I, F, P, P, P, I, P, P, I, I, I, P],
     "kva_maps_encode_cache": [P, I, P, P, P, P, P, P, P, I, I, I, I, I, I, I, I, P, I, P],
     "kva_maps_combine": [P, I, I, P, F, F, F, I, I, I, I, P],

@@ -187,6 +187,8 @@ class SandwichNormBlock(Block):
         # a pass of tanh norms adds the bias of the product whose output it lets in
         if kinds == {"tanh"} and isinstance(mixer, ProjectedMixer):
             mixer.leaves_out_bias = True
+        if kinds == {"tanh"} and hasattr(feed_forward, "leaves_rows"):
+            feed_forward.leaves_rows = True        # ... and adds up what routed experts returned
 
     def first_norm(self) -> Optional[Norm]:
         return None

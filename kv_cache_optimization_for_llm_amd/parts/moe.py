@@ -187,6 +187,10 @@ class RoutedExperts(FeedForward):
         # the shared expert's gate: one number a token, in 32-bit; its sigmoid is taken where the rows are added
         return product[:, self.outputs] if self.shared_gate is not None else None
 
+    # an arrangement whose next pass over the output can add the experts' rows up sets this: they are then handed on
+    # as ops.kernels.ExpertRows
+    leaves_rows = False
+
     def forward(self, x, ctx: MixerContext, tail=None):
         T, dev = x.shape[0], x.device
         idx = torch.empty((T, self.top), dtype=torch.int32, device=dev)
@@ -197,21 +201,36 @@ class RoutedExperts(FeedForward):
             sorted_slot, tile_expert = self._sorted(slots, group, dev)
             K.moe_table_align(self.table, ctx.batch.token_ids, idx, wgt, self.experts, sorted_slot, tile_expert,
                               getattr(ctx.batch, "feedback", None), group)
+        elif K.moe_router_supported(x, self.router):
+            # one launch for the router's product and the choice, and for few tokens the sorted list too
+            rest = torch.empty((T, 1), dtype=torch.float32, device=dev) if self.shared_gate is not None else None
+            listed = {}
+            if self.experts:
+                sorted_slot, tile_expert = self._sorted(slots, group, dev)
+                if T <= K.MOE_ROUTER_LIST_TOKENS:
+                    listed = dict(sorted_slot=sorted_slot, tile_expert=tile_expert)
+            K.moe_router(x, self.router, self.router_bias, self.correction, self.outputs, self.top, idx, wgt, rest,
+                         self.renormalise, self.over_chosen, scores=self.scores, groups=self.groups,
+                         keep_groups=self.keep_groups, group_top=self.group_top, weight_scale=self.weight_scale,
+                         sum_eps=self.sum_eps, experts=self.experts, group=group, **listed)
+            if self.experts and not listed:
+                K.moe_align(idx, self.experts, sorted_slot, tile_expert, group)
+            gate = rest[:, 0] if rest is not None else None
         else:
             gate = self._route(x, idx, wgt)
+            if self.experts:
+                sorted_slot, tile_expert = self._sorted(slots, group, dev)
+                K.moe_align(idx, self.experts, sorted_slot, tile_expert, group)
         if RoutedExperts.on_route is not None and not torch.cuda.is_current_stream_capturing():
             RoutedExperts.on_route(self, idx)
         rows = torch.empty((slots, self.hidden_size), dtype=torch.float32, device=dev)
         if self.experts:
-            if not self.by_table:
-                sorted_slot, tile_expert = self._sorted(slots, group, dev)
-                K.moe_align(idx, self.experts, sorted_slot, tile_expert, group)
             act = torch.empty((sorted_slot.shape[0], self.intermediate_size), dtype=x.dtype, device=dev)
             first, second = (wgt, None) if self.weight_input else (None, wgt)
             K.moe_expert_rows(x, self.w_up, act, sorted_slot, tile_expert, self.top, activation=self.activation,
                               slot_weight=first, gated=self.gated, limit=self.limit, group=group, tiled=self.tiled)
             K.moe_expert_rows(act, self.w_down, rows, sorted_slot, tile_expert, self.top, slot_weight=second, group=group,
                               tiled=self.tiled)
-        out = torch.empty_like(x)
         extra = self.shared.forward(x, ctx) if self.shared is not None else None
-        return K.moe_combine(x, rows, idx, wgt, self.experts, out, extra=extra, extra_gate=gate)
+        out = K.ExpertRows(x, rows, idx, wgt, self.experts, extra, gate)
+        return out if self.leaves_rows and self.identity == 0 else out.sum()

@@ -537,6 +537,17 @@ def test_experts_weighted_on_their_inputs(T, W, ff, experts, top, shared, dtype,
     w = {k: v.double() for k, v in state.items()}
     want = plain.experts(x.double(), w, "p.", mlp)
     got = part.forward(x.to(gpu), MixerContext(batch=None)).double().cpu()
+    part.leaves_rows = True                 # the rows handed on, and added up inside the step between branches
+    left = part.forward(x.to(gpu), MixerContext(batch=None))
+    assert isinstance(left, K.ExpertRows) and left.shape == x.shape
+    stream = torch.zeros((T, W), device=gpu)
+    K.tanh_step(stream, y=left)
+    close(stream, got, TOL[dtype], "added up on the way")
+    ones, zero = torch.ones(W, device=gpu), torch.zeros(W, device=gpu)
+    out, pick = torch.empty((2, W), device=gpu), i32([T - 1, 0], gpu)
+    K.tanh_step(torch.zeros((T, W), device=gpu), y=left, post=(ones, zero, 0.5), pre=(ones, zero, 1.0), out=out, row_idx=pick)
+    close(out, torch.tanh(torch.tanh(0.5 * got[[T - 1, 0]])), TOL[dtype], "gathered rows")
+    part.leaves_rows = False
     # (a close call between two experts may go the other way in 32-bit: none is that close here)
     s = torch.sigmoid(x.double() @ w["p.router"].T).sort(-1, descending=True).values
     clear = torch.ones(T, dtype=torch.bool) if top == experts else (s[:, top - 1] - s[:, top]) > 1e-5
@@ -547,3 +558,41 @@ def test_experts_weighted_on_their_inputs(T, W, ff, experts, top, shared, dtype,
     behind.load({k: v.to(gpu) for k, v in state.items()})
     other = behind.forward(x.to(gpu), MixerContext(batch=None)).double().cpu()
     assert T == 1 or (other - got).abs().max() > 0.05 * want.abs().max()       # the two places of the weight differ
+
+
+@pytest.mark.parametrize("T, W, outputs, extra, top, kw", [
+    (1, 64, 4, 1, 1, dict(scores="sigmoid")), (8, 2048, 16, 1, 4, dict(scores="sigmoid")), (16, 96, 40, 0, 6, {}),
+    (17, 256, 5, 2, 2, dict(renormalise=True, scores="sigmoid")), (70, 32, 64, 0, 8, dict(scores="sigmoid", groups=8, keep_groups=3, renormalise=True)),
+    (5, 544, 300, 1, 9, dict(over_chosen=True)), (33, 64, 511, 1, 3, dict(scores="sigmoid"))])
+@pytest.mark.parametrize("with_bias", [False, True])
+def test_the_routers_product_the_choice_and_the_list_in_one_launch(T, W, outputs, extra, top, kw, with_bias, gpu):
+    """Against the same steps in three launches: logits, choice, weights, the other columns, the sorted list."""
+    x, w = rnd((T, W), 1, torch.bfloat16), rnd((outputs + extra, W), 2, torch.bfloat16, W ** -0.5)
+    bias = rnd((outputs + extra,), 3) if with_bias else None
+    corr = rnd((outputs,), 4, scale=0.1) if with_bias else None
+    on = lambda t: None if t is None else t.to(gpu)
+    idx, wgt = torch.empty((T, top), dtype=torch.int32, device=gpu), torch.empty((T, top), device=gpu)
+    rest = torch.empty((T, extra), device=gpu) if extra else None
+    tiles = K.moe_tiles(T * top, outputs)
+    lists = [(torch.empty(tiles * K.MOE_TILE, dtype=torch.int32, device=gpu), torch.empty(tiles, dtype=torch.int32, device=gpu)) for _ in range(2)]
+    listed = dict(sorted_slot=lists[0][0], tile_expert=lists[0][1]) if T <= K.MOE_ROUTER_LIST_TOKENS else {}
+    assert K.moe_router_supported(x, w)
+    K.moe_router(on(x), on(w), on(bias), on(corr), outputs, top, idx, wgt, rest, experts=outputs, **listed, **kw)
+    logits = x.double() @ w.double().T + (0 if bias is None else bias.double())
+    if extra:
+        close(rest, logits[:, outputs:], 1e-5, "the other columns")
+    idx2, wgt2 = torch.empty_like(idx), torch.empty_like(wgt)
+    K.moe_route(logits[:, :outputs].float().contiguous().to(gpu), on(corr), top, idx2, wgt2, **kw)
+    same = (idx == idx2).all(-1)
+    assert same.float().mean() > 0.97                                  # (a close call may go the other way)
+    close(wgt[same], wgt2[same], 1e-4, "weights")
+    if listed:
+        K.moe_align(idx, outputs, *lists[1])
+        assert torch.equal(lists[0][1], lists[1][1])
+        for tile in range(tiles):                                       # (the order inside an expert's run is free)
+            a, b = (set(l[0].view(tiles, -1)[tile].cpu().tolist()) for l in lists)
+            e = int(lists[0][1][tile])
+            assert e < 0 or all(int(idx.view(-1)[s]) == e for s in a if s >= 0)
+        assert sorted(lists[0][0].cpu().tolist()) == sorted(lists[1][0].cpu().tolist())
+    with pytest.raises(K.KernelError):
+        K.moe_router(on(x), on(w.float()), None, None, outputs, top, idx, wgt, rest)
