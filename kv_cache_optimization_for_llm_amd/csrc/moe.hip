@@ -46,13 +46,14 @@ struct MoeRoute {
 };
 
 // one token by one wavefront: `logits` [outputs] (memory or LDS) -> idx and wgt [top]; `choice` is the wavefront's own
-// piece of LDS, KVA_WAVE * MOE_ROUTE_PER_LANE floats (read with groups only)
+// piece of LDS, KVA_WAVE * PL floats (16-byte aligned; with PL > 1 read with groups only).  A lane takes PL outputs.
+template <int PL>
 __device__ inline void moe_route_token(const MoeRoute &a, const float *logits, int *idx, float *wgt, float *choice) {
     const int lane = threadIdx.x % KVA_WAVE;
-    float s[MOE_ROUTE_PER_LANE], ch[MOE_ROUTE_PER_LANE];
+    float s[PL], ch[PL];
     float mx = -INFINITY;
 #pragma unroll
-    for (int j = 0; j < MOE_ROUTE_PER_LANE; ++j) {
+    for (int j = 0; j < PL; ++j) {
         const int e = lane + j * KVA_WAVE;
         s[j] = e < a.outputs ? logits[e] : -INFINITY;
         mx = fmaxf(mx, s[j]);
@@ -60,14 +61,14 @@ __device__ inline void moe_route_token(const MoeRoute &a, const float *logits, i
     mx = wave_max(mx);
     float sum = 0.f;
 #pragma unroll
-    for (int j = 0; j < MOE_ROUTE_PER_LANE; ++j) {
+    for (int j = 0; j < PL; ++j) {
         const int e = lane + j * KVA_WAVE;
         s[j] = e < a.outputs ? expf(s[j] - mx) : 0.f;
         sum += s[j];
     }
     sum = wave_sum(sum);
 #pragma unroll
-    for (int j = 0; j < MOE_ROUTE_PER_LANE; ++j) {
+    for (int j = 0; j < PL; ++j) {
         const int e = lane + j * KVA_WAVE;
         if (a.over_chosen) {
             // the logits themselves are compared, and the weights are a softmax over the chosen ones
@@ -85,7 +86,7 @@ __device__ inline void moe_route_token(const MoeRoute &a, const float *logits, i
         // index) can be chosen: the others' choice scores become -inf.  Lane g takes group g.
         const int per = a.outputs / a.groups;
 #pragma unroll
-        for (int j = 0; j < MOE_ROUTE_PER_LANE; ++j)
+        for (int j = 0; j < PL; ++j)
             if (lane + j * KVA_WAVE < a.outputs) choice[lane + j * KVA_WAVE] = ch[j];
         __builtin_amdgcn_wave_barrier();
         __threadfence_block();
@@ -119,10 +120,37 @@ __device__ inline void moe_route_token(const MoeRoute &a, const float *logits, i
             if (bg != 0x7fffffff) allowed |= 1ull << bg;
         }
 #pragma unroll
-        for (int j = 0; j < MOE_ROUTE_PER_LANE; ++j) {
+        for (int j = 0; j < PL; ++j) {
             const int e = lane + j * KVA_WAVE;
             if (e < a.outputs && !((allowed >> (e / per)) & 1ull)) ch[j] = -INFINITY;
         }
+    }
+    if constexpr (PL == 1) {
+        // every lane counts the outputs in front of its own (of equal ones the lowest index comes first)
+        __builtin_amdgcn_wave_barrier();
+        choice[lane] = ch[0];
+        __threadfence_block();
+        __builtin_amdgcn_wave_barrier();
+        int rank = 0;
+        for (int e = 0; e < a.outputs; e += 4) {
+            const float4 c = *reinterpret_cast<const float4 *>(choice + e);
+            rank += (c.x > ch[0] || (c.x == ch[0] && e < lane)) + (c.y > ch[0] || (c.y == ch[0] && e + 1 < lane)) +
+                    (c.z > ch[0] || (c.z == ch[0] && e + 2 < lane)) + (c.w > ch[0] || (c.w == ch[0] && e + 3 < lane));
+        }
+        const bool chosen = lane < a.outputs && rank < a.top;
+        if (chosen) idx[rank] = lane;
+        if (!(a.renormalise || a.over_chosen)) {
+            if (chosen) wgt[rank] = s[0] * a.weight_scale;
+            return;
+        }
+        __builtin_amdgcn_wave_barrier();
+        if (chosen) choice[rank] = s[0];
+        __threadfence_block();
+        __builtin_amdgcn_wave_barrier();
+        float sum_chosen = 0.f;
+        for (int k = 0; k < a.top; ++k) sum_chosen += choice[k];
+        if (lane < a.top) wgt[lane] = choice[lane] / (sum_chosen + a.sum_eps) * a.weight_scale;
+        return;
     }
     float total = 0.f;
     for (int k = 0; k < a.top; ++k) {
@@ -130,7 +158,7 @@ __device__ inline void moe_route_token(const MoeRoute &a, const float *logits, i
         float bv = -INFINITY, bs = 0.f;
         int be = 0x7fffffff;
 #pragma unroll
-        for (int j = 0; j < MOE_ROUTE_PER_LANE; ++j) {
+        for (int j = 0; j < PL; ++j) {
             const int e = lane + j * KVA_WAVE;
             if (e < a.outputs && (ch[j] > bv || (ch[j] == bv && e < be))) { bv = ch[j]; be = e; bs = s[j]; }
         }
@@ -141,7 +169,7 @@ __device__ inline void moe_route_token(const MoeRoute &a, const float *logits, i
             if (ov > bv || (ov == bv && oe < be)) { bv = ov; be = oe; bs = os; }
         }
 #pragma unroll
-        for (int j = 0; j < MOE_ROUTE_PER_LANE; ++j)
+        for (int j = 0; j < PL; ++j)
             if (lane + j * KVA_WAVE == be) ch[j] = -INFINITY;
         total += bs;
         if (lane == 0) {
@@ -157,13 +185,14 @@ __device__ inline void moe_route_token(const MoeRoute &a, const float *logits, i
     }
 }
 
+template <int PL>
 __global__ void __launch_bounds__(256)
 moe_route_kernel(int *__restrict__ idx, float *__restrict__ wgt, const float *__restrict__ logits, MoeRoute a, int tokens,
                  int logits_stride) {
-    __shared__ float choice_s[4][KVA_WAVE * MOE_ROUTE_PER_LANE];
+    __shared__ __attribute__((aligned(16))) float choice_s[4][KVA_WAVE * PL];
     const int t = blockIdx.x * (blockDim.x / KVA_WAVE) + threadIdx.x / KVA_WAVE;
     if (t >= tokens) return;
-    moe_route_token(a, logits + (size_t)t * logits_stride, idx + (size_t)t * a.top, wgt + (size_t)t * a.top,
+    moe_route_token<PL>(a, logits + (size_t)t * logits_stride, idx + (size_t)t * a.top, wgt + (size_t)t * a.top,
                     choice_s[threadIdx.x / KVA_WAVE]);
 }
 
@@ -191,7 +220,7 @@ extern "C" int kva_moe_route(int *idx, float *wgt, const float *logits, const fl
     const MoeRoute a{correction, outputs, top, renormalise, over_chosen, sigmoid_scores, groups, keep_groups, group_top, weight_scale, sum_eps};
     if (int rc = moe_route_check(a)) return rc;
     if (tokens == 0) return KVA_OK;
-    hipLaunchKernelGGL(moe_route_kernel, dim3((tokens + 3) / 4), dim3(256), 0, stream, idx, wgt, logits, a, tokens, logits_stride);
+    hipLaunchKernelGGL(outputs <= KVA_WAVE ? moe_route_kernel<1> : moe_route_kernel<MOE_ROUTE_PER_LANE>, dim3((tokens + 3) / 4), dim3(256), 0, stream, idx, wgt, logits, a, tokens, logits_stride);
     KVA_CHECK_LAUNCH("moe_route");
     return KVA_OK;
 }
@@ -345,10 +374,11 @@ struct MoeRouter {
     int tokens, N, K, x_stride;
 };
 
+template <int PL>
 __global__ void __launch_bounds__(1024)
 moe_router_kernel(MoeRouter m, MoeRoute a, int *__restrict__ sorted_slot, int *__restrict__ tile_expert, int experts, int capacity,
                   int max_tiles, int group) {
-    extern __shared__ float moe_lds[];
+    extern __shared__ __attribute__((aligned(16))) float moe_lds[];
     __shared__ int count[MOE_MAX_EXPERTS], start[MOE_MAX_EXPERTS];
     __shared__ float part[16][KVA_WAVE][4];
     const int lane = threadIdx.x % KVA_WAVE, wave = threadIdx.x / KVA_WAVE, r = lane & 15, g = lane >> 4;
@@ -388,8 +418,8 @@ moe_router_kernel(MoeRouter m, MoeRoute a, int *__restrict__ sorted_slot, int *_
     __syncthreads();
     const int t = t0 + wave;
     if (t < m.tokens) {
-        moe_route_token(a, logits + wave * m.N, m.idx + (size_t)t * a.top, m.wgt + (size_t)t * a.top,
-                        logits + 16 * m.N + (a.groups > 1 ? wave * KVA_WAVE * MOE_ROUTE_PER_LANE : 0));
+        moe_route_token<PL>(a, logits + wave * m.N, m.idx + (size_t)t * a.top, m.wgt + (size_t)t * a.top,
+                            logits + 16 * m.N + (PL == 1 || a.groups > 1 ? wave * KVA_WAVE * PL : 0));
         for (int n = a.outputs + lane; n < m.N; n += KVA_WAVE) m.rest[(size_t)t * (m.N - a.outputs) + n - a.outputs] = logits[wave * m.N + n];
     }
     if (!sorted_slot) return;
@@ -420,10 +450,12 @@ extern "C" int kva_moe_router(int *idx, float *wgt, float *rest, const void *x, 
         if (int rc = moe_align_check(sorted_slot, tile_expert, idx, tokens * top, experts, capacity, max_tiles, group)) return rc;
     }
     if (tokens == 0) return KVA_OK;
-    const size_t lds = (size_t)(16 * N + (groups > 1 ? 16 * KVA_WAVE * MOE_ROUTE_PER_LANE : 0)) * sizeof(float);
+    const int per_lane = outputs <= KVA_WAVE ? 1 : MOE_ROUTE_PER_LANE;
+    const size_t lds = (size_t)(16 * N + (per_lane == 1 || groups > 1 ? 16 * KVA_WAVE * per_lane : 0)) * sizeof(float);
+    auto kernel = per_lane == 1 ? moe_router_kernel<1> : moe_router_kernel<MOE_ROUTE_PER_LANE>;
     if (lds > 32 * 1024)
-        hipFuncSetAttribute(reinterpret_cast<const void *>(moe_router_kernel), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
-    hipLaunchKernelGGL(moe_router_kernel, dim3((tokens + 15) / 16), dim3(1024), lds, stream,
+        hipFuncSetAttribute(reinterpret_cast<const void *>(kernel), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+    hipLaunchKernelGGL(kernel, dim3((tokens + 15) / 16), dim3(1024), lds, stream,
                        MoeRouter{(const bf16_t *)x, (const bf16_t *)w, bias, rest, idx, wgt, tokens, N, K, x_stride}, a, sorted_slot,
                        tile_expert, experts, capacity, max_tiles, group);
     KVA_CHECK_LAUNCH("moe_router");
