@@ -1,0 +1,179 @@
+"""Small Gokinex configurations with seeded weights, and helpers that compare an engine's rows with the plain
+implementation (``plain_gokinex``)."""
+import json
+import os
+from typing import Dict, List, Tuple
+
+import numpy as np
+import torch
+
+import plain_gokinex as plain
+from bilolorn_util import run_steps  # noqa: F401  (re-exported for the tests)
+from radilix_util import prompt, row_error  # noqa: F401
+
+
+def rot(base, dims, scaling=None):
+    r = {"base": base, "dims": dims}
+    if scaling is not None:
+        r["scaling"] = dict(zip(("factor", "low", "high", "original"), scaling))
+    return r
+
+
+def attention(heads, kv_heads, dim, vdim, diff, scale, rotation=None, kv_from=None):
+    m = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "diff": diff, "scale": scale, "rot": rotation}
+    if kv_from is not None:
+        m["kv_from"] = kv_from
+    return ("attention", m)
+
+
+def mamba2(heads, vdim, state, groups, conv, norm_groups):
+    return ("mamba2", {"heads": heads, "vdim": vdim, "state": state, "groups": groups, "conv": conv, "norm_groups": norm_groups})
+
+
+def dense(ff):
+    return {"kind": "dense", "ff": ff}
+
+
+def moe(experts, top, ff, shared=None):
+    m = {"kind": "moe", "expert": {"ff": ff}, "router": {"experts": experts, "top": top}}
+    if shared is not None:
+        m["shared"] = {"ff": shared}
+    return m
+
+
+def config(vocab, width, eps, scale, layers, bigram=None):
+    """``layers``: pairs of a mixer (:func:`attention`, :func:`mamba2`) and a feed-forward or None"""
+    emb = {"scale": scale}
+    if bigram is not None:
+        emb["bigram"] = dict(zip(("buckets", "mul_prev", "mul_cur"), bigram))
+    return {"architecture": "Gokinex", "vocab": vocab, "width": width, "norm": {"eps": eps}, "embedding": emb,
+            "layers": [{"type": kind, "mixer": m, "mlp": mlp} for (kind, m), mlp in layers]}
+
+
+# A: sizes that no matrix-core kernel has an instance for (maps of 10 and 6, values of 14 and 20, a width of 92, states
+#    of 10 and 7, three taps); a recurrence first; a layer that reads another's keys across a recurrence, with other
+#    constants and a mask of its own; a layer without a feed-forward; every expert chosen.
+CFG_A = config(211, 92, 0.003, 1.7, [
+    (mamba2(3, 12, 10, 1, 3, 2), moe(6, 2, 44, 36)),
+    (attention(6, 2, 10, 14, 0.2, 0.3, rot(300.0, 6, (4.0, 1.0, 3.0, 40))), dense(84)),
+    (mamba2(4, 6, 7, 4, 5, 3), None),
+    (attention(4, 2, 10, 14, 0.45, 0.4, rot(300.0, 6, (4.0, 1.0, 3.0, 40)), kv_from=1), moe(5, 5, 40)),
+    (attention(3, 3, 6, 20, 0.0, 0.5, rot(50.0, 6)), dense(60))], (97, 13, 5))
+# B: values that are equal or 1: one head, one group, one expert, one tap, one bucket, an embedding multiplier of 1,
+#    maps as large as values, no rotation.
+CFG_B = config(157, 72, 0.01, 1.0, [
+    (attention(2, 2, 16, 16, 0.3, 0.25), moe(1, 1, 24, 24)),
+    (mamba2(1, 8, 8, 1, 1, 1), moe(3, 1, 16)),
+    (attention(1, 1, 4, 4, 0.8, 1.0, rot(7.0, 4)), dense(72)),
+    (mamba2(4, 8, 8, 4, 2, 4), dense(40))], (1, 1, 1))
+# C: sizes at which the bf16 engine takes its matrix-core kernels: maps of 16, 32 and 64 with values of 32, 64 and 128,
+#    more heads than a tile has rows, states of 16, 64 and 128, heads of 16 and 32, two layers that read the first
+#    one's keys.
+CFG_C = config(263, 288, 0.001, 0.7, [
+    (attention(20, 4, 32, 64, 0.25, 0.2, rot(100000.0, 16, (8.0, 1.0, 4.0, 128))), moe(8, 3, 64, 96)),
+    (mamba2(6, 32, 64, 3, 4, 2), moe(10, 1, 96)),
+    (attention(8, 4, 32, 64, 0.5, 0.15, rot(100000.0, 16, (8.0, 1.0, 4.0, 128)), kv_from=0), dense(320)),
+    (mamba2(4, 16, 128, 2, 4, 1), dense(160)),
+    (attention(4, 2, 16, 32, 0.1, 0.3, rot(1000.0, 16)), moe(6, 2, 160, 64)),
+    (attention(4, 4, 32, 64, 0.35, 0.2, rot(100000.0, 16, (8.0, 1.0, 4.0, 128)), kv_from=0), dense(64))], (509, 31, 17))
+# D: a width of 512, where one or two decoded tokens take the matrix-vector kernels, maps of 64 with values of 128, a
+#    state of 256, eight norm groups, a vocabulary that is no multiple of 8, a table of pairs larger than the vocabulary.
+CFG_D = config(1003, 512, 1e-5, 3.0, [
+    (attention(4, 2, 64, 128, 0.3, 0.12, rot(40000.0, 32, (16.0, 1.0, 4.0, 64))), dense(1024)),
+    (mamba2(8, 64, 256, 2, 4, 8), moe(12, 3, 128, 192)),
+    (attention(2, 2, 64, 128, 0.6, 0.1, rot(40000.0, 32, (16.0, 1.0, 4.0, 64)), kv_from=0), moe(24, 5, 64, 64))],
+    (2039, 1543, 769))
+# E: no second table; many heads over small values; heads of 4; a recurrence alone at the end.
+CFG_E = config(131, 64, 0.02, 0.25, [
+    (attention(32, 8, 4, 8, 0.15, 0.5, rot(500.0, 2)), dense(56)),
+    (mamba2(16, 4, 24, 8, 4, 16), None)])
+CONFIGS = {"A": (CFG_A, 5), "B": (CFG_B, 6), "C": (CFG_C, 7), "D": (CFG_D, 8), "E": (CFG_E, 9)}
+
+
+def write_model(folder: str, cfg: dict, seed: int, gain: float = 1.0, edit=None) -> Tuple[str, Dict[str, torch.Tensor]]:
+    """A model folder with seeded weights: matrices N(0, gain / sqrt(in)); vectors, which the random-weights mode leaves
+    near one or tiny, are spread out so that they weigh in.  ``edit(state)`` may change the tensors before they are
+    stored.  Returns the folder and the tensors."""
+    from safetensors.torch import save_file
+    from kv_cache_optimization_for_llm_amd.models.builder import tensor_specs_for_config
+    from kv_cache_optimization_for_llm_amd.weights.random_init import random_state_dict
+
+    os.makedirs(folder, exist_ok=True)
+    with open(os.path.join(folder, "config.json"), "w") as f:
+        json.dump(cfg, f)
+    state = random_state_dict(tensor_specs_for_config(cfg), seed, torch.bfloat16, gain)
+    g = torch.Generator().manual_seed(seed)
+
+    def rnd(shape, std, mean=0.0):
+        return (torch.randn(shape, generator=g) * std + mean).to(torch.bfloat16)
+    for name, t in state.items():
+        last = name.rsplit(".", 1)[-1]
+        if last == "alpha":
+            state[name] = rnd(t.shape, 0.15, 0.8 if "b.alpha" not in name else 1.2)
+        elif name in ("embed", "bigram"):
+            state[name] = rnd(t.shape, 1.0)
+        elif last in ("lq1", "lk1", "lq2", "lk2"):
+            state[name] = rnd(t.shape, 0.8 / t.shape[0] ** 0.25)
+        elif last == "conv":
+            state[name] = rnd(t.shape, t.shape[1] ** -0.5)
+        elif last in ("dt_bias", "A_log"):
+            state[name] = rnd(t.shape, 0.8, -1.0)
+        elif last == "D":
+            state[name] = rnd(t.shape, 0.5, 1.0)
+        elif len(t.shape) == 1:
+            state[name] = rnd(t.shape, 0.3, 0.0 if last == "b" else 1.0)
+    if edit is not None:
+        edit(state)
+    save_file(state, os.path.join(folder, "model.safetensors"))
+    return folder, state
+
+
+TOLERANCE = {"float32": 1e-4, "bfloat16": 3e-2}
+LIMITS: Dict[str, List[float]] = {}      # bfloat16: per request and position
+_PLAIN: Dict[tuple, tuple] = {}
+
+
+def bf16_rounding(t):
+    return t.to(torch.bfloat16).to(t.dtype)
+
+
+def expected_rows(cfg: dict, state: Dict[str, torch.Tensor], requests: Dict[str, List[int]],
+                  dtype: str = "float32") -> Dict[str, np.ndarray]:
+    """Logits of the plain forward pass per request.  In bfloat16 a row's limit is three times what rounding
+    everything a 16-bit engine stores does to it in the plain model, where that is more than the general one (an
+    expert's choice may turn on it)."""
+    out = {}
+    LIMITS.clear()
+    for rid, toks in requests.items():
+        key = (id(state), tuple(toks), dtype)
+        if key not in _PLAIN:
+            full = _PLAIN.get((id(state), tuple(toks), "float32"), (None, None))[1]
+            full = plain.forward(cfg, state, toks).numpy() if full is None else full
+            limits = []
+            if dtype == "bfloat16":
+                moved = plain.forward(cfg, state, toks, r_=bf16_rounding).numpy()
+                limits = [3.0 * row_error(moved[p], full[p]) for p in range(len(toks))]
+            _PLAIN[key] = (state, full, limits)
+        out[rid] = _PLAIN[key][1]
+        if dtype == "bfloat16":
+            LIMITS[rid] = [max(TOLERANCE[dtype], e) for e in _PLAIN[key][2]]
+    return out
+
+
+def assert_rows(rows, expected: Dict[str, np.ndarray], dtype: str, what: str = "", tolerance=None) -> float:
+    """Every row within its limit in 32-bit; in bfloat16 (where a limit is one sample of what rounding does, and a
+    rounding that tips an expert's choice at one token moves the rows behind it) no row beyond one and a half times
+    the larger of its limit and the median limit's triple, at most one in fifty (or one) beyond its own."""
+    worst, over = 0.0, 0
+    for (rid, p), row in rows.items():
+        assert np.isfinite(row).all(), f"{what}: request {rid} position {p} has a logit that is not finite"
+        e = row_error(row, expected[rid][p])
+        limit = LIMITS[rid][p] if dtype == "bfloat16" else (tolerance or TOLERANCE[dtype])
+        hard = 1.5 * limit if dtype == "bfloat16" else limit
+        if dtype == "bfloat16":
+            hard = max(hard, 4.5 * float(np.median(LIMITS[rid])))
+        assert e <= hard, f"{what}: request {rid} position {p} is off by {e:.3g} (limit {hard:.3g})"
+        over += e > limit
+        worst = max(worst, e)
+    assert over <= max(1, len(rows) // 50), f"{what}: {over} of {len(rows)} rows are beyond their limits"
+    return worst
