@@ -8,7 +8,7 @@ import numpy as np
 import torch
 
 import plain_gokinex as plain
-from bilolorn_util import run_steps  # noqa: F401  (re-exported for the tests)
+from bonusun_util import run_steps  # noqa: F401  (re-exported for the tests)
 from radilix_util import prompt, row_error  # noqa: F401
 
 
@@ -130,48 +130,48 @@ def write_model(folder: str, cfg: dict, seed: int, gain: float = 1.0, edit=None)
 
 TOLERANCE = {"float32": 1e-4, "bfloat16": 3e-2}
 LIMITS: Dict[str, List[float]] = {}      # bfloat16: per request and position
-_PLAIN: Dict[tuple, tuple] = {}
+# a router's choice is the engine's to make where the plain implementation's own margin (a gap between two scores) is
+# below this: the engine's input to the router carries its format's rounding.  What a router does wrong shows in
+# 32-bit, where no gap is forgiven.
+CLOSE_CALL = {"float32": 1e-4, "bfloat16": 0.15}
 
 
 def bf16_rounding(t):
     return t.to(torch.bfloat16).to(t.dtype)
 
 
-def expected_rows(cfg: dict, state: Dict[str, torch.Tensor], requests: Dict[str, List[int]],
-                  dtype: str = "float32") -> Dict[str, np.ndarray]:
-    """Logits of the plain forward pass per request.  In bfloat16 a row's limit is three times what rounding
-    everything a 16-bit engine stores does to it in the plain model, where that is more than the general one (an
-    expert's choice may turn on it)."""
+def expected_rows(cfg: dict, state: Dict[str, torch.Tensor], requests: Dict[str, List[int]], dtype: str = "float32",
+                  routes=None) -> Dict[str, np.ndarray]:
+    """Logits of the plain forward pass per request.  With ``routes`` (what the engine's routers chose) the plain
+    experts are the engine's, and every choice that differs from the plain router's own must be a close call of that
+    router.  In bfloat16 a row's limit is three times what rounding everything a 16-bit engine stores does to it in the
+    plain model, where that is more than the general one."""
     out = {}
     LIMITS.clear()
     for rid, toks in requests.items():
-        key = (id(state), tuple(toks), dtype)
-        if key not in _PLAIN:
-            full = _PLAIN.get((id(state), tuple(toks), "float32"), (None, None))[1]
-            full = plain.forward(cfg, state, toks).numpy() if full is None else full
-            limits = []
-            if dtype == "bfloat16":
-                moved = plain.forward(cfg, state, toks, r_=bf16_rounding).numpy()
-                limits = [3.0 * row_error(moved[p], full[p]) for p in range(len(toks))]
-            _PLAIN[key] = (state, full, limits)
-        out[rid] = _PLAIN[key][1]
+        forced = None if routes is None else {layer: idx[:len(toks)] for layer, idx in routes[rid].items()}
+        margins: dict = {}
+        out[rid] = plain.forward(cfg, state, toks, forced=forced, margins=margins).numpy()
         if dtype == "bfloat16":
-            LIMITS[rid] = [max(TOLERANCE[dtype], e) for e in _PLAIN[key][2]]
+            moved = plain.forward(cfg, state, toks, r_=bf16_rounding, forced=forced).numpy()
+            LIMITS[rid] = [max(TOLERANCE[dtype], 3.0 * row_error(moved[p], out[rid][p])) for p in range(len(toks))]
+        for layer, (own, margin) in margins.items() if forced is not None else ():
+            differs = (forced[layer].sort(-1).values != own.sort(-1).values).any(-1)
+            assert (margin[differs] <= CLOSE_CALL[dtype]).all(), \
+                f"request {rid}, layer {layer}: the engine's router chose other experts where the choice was clear " \
+                f"(a gap of {float(margin[differs].max()):.3g}, {int(differs.sum())} of {len(differs)} tokens differ)"
     return out
 
 
 def assert_rows(rows, expected: Dict[str, np.ndarray], dtype: str, what: str = "", tolerance=None) -> float:
-    """Every row within its limit in 32-bit; in bfloat16 (where a limit is one sample of what rounding does, and a
-    rounding that tips an expert's choice at one token moves the rows behind it) no row beyond one and a half times
-    the larger of its limit and the median limit's triple, at most one in fifty (or one) beyond its own."""
+    """Every row within its limit in 32-bit.  In bfloat16 a row's limit is an estimate (one sample of what rounding
+    does at that place), so: no row beyond twice its limit, at most one in fifty (or one) beyond it."""
     worst, over = 0.0, 0
     for (rid, p), row in rows.items():
         assert np.isfinite(row).all(), f"{what}: request {rid} position {p} has a logit that is not finite"
         e = row_error(row, expected[rid][p])
         limit = LIMITS[rid][p] if dtype == "bfloat16" else (tolerance or TOLERANCE[dtype])
-        hard = 1.5 * limit if dtype == "bfloat16" else limit
-        if dtype == "bfloat16":
-            hard = max(hard, 4.5 * float(np.median(LIMITS[rid])))
+        hard = 2.0 * limit if dtype == "bfloat16" else limit
         assert e <= hard, f"{what}: request {rid} position {p} is off by {e:.3g} (limit {hard:.3g})"
         over += e > limit
         worst = max(worst, e)

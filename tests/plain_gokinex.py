@@ -163,12 +163,19 @@ def choose(scores: torch.Tensor, top: int) -> List[int]:
     return sorted(range(scores.shape[0]), key=lambda e: (-float(scores[e]), e))[:top]
 
 
-def experts(h, w, p: str, mlp: Mapping, r_=same) -> torch.Tensor:
-    """Every chosen expert reads its weight times the token's row; the outputs are added as they are."""
+def experts(h, w, p: str, mlp: Mapping, r_=same, forced=None, margins: Optional[list] = None) -> torch.Tensor:
+    """Every chosen expert reads its weight times the token's row; the outputs are added as they are.  ``forced`` [T,
+    top]: the experts that are used instead of the router's choice; ``margins`` takes the router's own choice and, per
+    token, how far apart the last score chosen and the first one not chosen are."""
+    top = mlp["router"]["top"]
     scores = torch.sigmoid(h @ w[p + "router"].T)
+    own = torch.tensor([choose(s, top) for s in scores])
+    if margins is not None:
+        ranked = scores.sort(-1, descending=True).values
+        margins.append((own, ranked[:, top - 1] - ranked[:, top] if top < scores.shape[1] else torch.zeros(h.shape[0], dtype=h.dtype)))
     out = torch.zeros_like(h)
     for t in range(h.shape[0]):
-        for e in choose(scores[t], mlp["router"]["top"]):
+        for e in (own if forced is None else forced)[t].tolist():
             u = scores[t, e] * h[t:t + 1]
             pe = f"{p}e{e}."
             out[t] += (r_(silu(u @ w[pe + "gate"].T) * (u @ w[pe + "up"].T)) @ w[pe + "down"].T)[0]
@@ -177,13 +184,15 @@ def experts(h, w, p: str, mlp: Mapping, r_=same) -> torch.Tensor:
     return r_(out)
 
 
-def feed_forward(h, w, p: str, mlp: Mapping, r_=same) -> torch.Tensor:
-    return r_(gated(h, w, p, gelu_tanh, r_)) if mlp["kind"] == "dense" else experts(h, w, p, mlp, r_)
+def feed_forward(h, w, p: str, mlp: Mapping, r_=same, forced=None, margins: Optional[list] = None) -> torch.Tensor:
+    return r_(gated(h, w, p, gelu_tanh, r_)) if mlp["kind"] == "dense" else experts(h, w, p, mlp, r_, forced, margins)
 
 
 def forward(cfg: Mapping, weights: Mapping[str, torch.Tensor], tokens, dtype=torch.float64,
-            residuals: Optional[list] = None, r_=same) -> torch.Tensor:
-    """Logits [T, vocab] of one whole sequence; ``residuals`` collects the stream after every layer."""
+            residuals: Optional[list] = None, r_=same, forced: Optional[Mapping] = None,
+            margins: Optional[dict] = None) -> torch.Tensor:
+    """Logits [T, vocab] of one whole sequence; ``residuals`` collects the stream after every layer; ``forced`` and
+    ``margins``: per layer, see :func:`experts`."""
     w: Dict[str, torch.Tensor] = {k: (v.to(dtype) if v.is_floating_point() else v) for k, v in weights.items()}
     eps = cfg["norm"]["eps"]
     x = embedding([int(t) for t in tokens], w, cfg["embedding"])
@@ -199,7 +208,11 @@ def forward(cfg: Mapping, weights: Mapping[str, torch.Tensor], tokens, dtype=tor
         x = x + dynamic_tanh(y, w, p + "norm1b")
         if layer.get("mlp"):
             h = r_(dynamic_tanh(x, w, p + "norm2"))
-            x = x + dynamic_tanh(feed_forward(h, w, p + "mlp.", layer["mlp"], r_), w, p + "norm2b")
+            took: list = []
+            y = feed_forward(h, w, p + "mlp.", layer["mlp"], r_, None if forced is None else forced.get(i), took)
+            x = x + dynamic_tanh(y, w, p + "norm2b")
+            if margins is not None and took:
+                margins[i] = took[0]
         if residuals is not None:
             residuals.append(x)
     return r_(dynamic_tanh(x, w, "final.norm")) @ w["head"].T

@@ -74,9 +74,9 @@ def test_random_models_under_random_schedules(seed, dtype, tmp_path, gpu):
     reqs = {f"q{i}": U.prompt(cfg, n, 13 * i + seed) for i, n in enumerate(lengths)}
     steps = R.mixed(reqs, seed=seed, max_live=4, chunk_sizes=(2, 3, 7, 16, 40, 70))
     eng = Engine(folder, EngineOptions(dtype=dtype, page_size=16, cache_tokens=R.max_live_tokens(steps, unit=16),
-                                       max_seqs=4, max_seq_len=160, max_batch_tokens=1024, use_graphs=seed % 2 == 1))
-    rows = U.run_steps(eng, steps)
+                                       max_seqs=4, max_seq_len=160, max_batch_tokens=1024, use_graphs=False))
+    rows, routes = U.run_steps(eng, steps, cfg)
     assert len(rows) == sum(lengths)
-    U.assert_rows(rows, U.expected_rows(cfg, state, reqs, dtype), dtype, f"model {cfg}")
+    U.assert_rows(rows, U.expected_rows(cfg, state, reqs, dtype, routes), dtype, f"model {cfg}")
     eng.cache.check()
     assert eng.cache.free_seats == 4 and all(g.free_pages() == g.num_pages for g in eng.cache.groups)
